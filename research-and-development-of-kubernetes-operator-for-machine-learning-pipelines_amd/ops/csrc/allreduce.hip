@@ -589,7 +589,9 @@ void car_destroy(long h) {
       hipIpcCloseMemHandle(s->peers.base[p]);
       if (s->split && s->peers.data[p]) hipIpcCloseMemHandle(s->peers.data[p]);
     }
-  hipFree(s->buf);
+  // uncached memory a kernel has read stays allocated until the process ends: allocations that
+  // reused it after a free have held wrong values
+  if (!s->uncached) hipFree(s->buf);
   if (s->dbuf) hipFree(s->dbuf);
   hipFree(s->epochs);
   hipHostFree(s->err_host);

@@ -438,7 +438,9 @@ void ep_destroy(long h) {
   hipDeviceSynchronize();
   for (int p = 0; p < s->world; ++p)
     if (p != s->rank && s->peers.base[p]) hipIpcCloseMemHandle(s->peers.base[p]);
-  hipFree(s->buf);
+  // uncached memory a kernel has read stays allocated until the process ends: allocations that
+  // reused it after a free have held wrong values
+  if (!s->uncached) hipFree(s->buf);
   for (void* q : {(void*)s->epoch, (void*)s->tickets, (void*)s->wcnt, (void*)s->wbase, (void*)s->lrank,
                   (void*)s->info, (void*)s->meta_l})
     hipFree(q);

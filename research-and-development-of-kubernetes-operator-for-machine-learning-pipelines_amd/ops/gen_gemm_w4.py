@@ -79,9 +79,8 @@ class Sched:
 
 
 # All 16 DMAs between the barriers (one per 4 MFMAs), next-tile reads packed at the end.
-# Measured and dropped (profiles/r03_gemm_w4.md): B2 at MFMA 86 with one DMA per 3 MFMAs, a
-# hipBLASLt-like 8 + 8 DMA split around B2 at the half boundary (both within 1 %), and
-# non-temporal weight / activation DMAs (2-8 % slower).
+# Measured and dropped (profiles/r03_gemm_w4.md): B2 at MFMA 86 with one DMA per 3 MFMAs (within
+# 1 %), and non-temporal weight / activation DMAs (2-8 % slower).
 SCHEDS = [Sched(rd1=[1 + 2 * k for k in range(16)], b1=38, dma=[40 + 4 * k for k in range(16)], b2=102,
                 rd0=[103 + round(k * 24 / 15) for k in range(16)])]
 # the half-height tile (BM = 128): 64 MFMAs, 12 fragment reads per k-half, 12 DMA pieces
