@@ -17,7 +17,7 @@ from __future__ import annotations
 
 from dataclasses import asdict, dataclass
 
-from ..models.config import ModelConfig, get_config
+from ..models.config import HybridConfig, ModelConfig, get_config
 
 GB = 1e9
 
@@ -40,6 +40,8 @@ class Placement:
 
 
 def _valid_tp(cfg: ModelConfig, tp: int) -> bool:
+    if isinstance(cfg, HybridConfig):  # one GPU (no tensor-parallel form)
+        return tp == 1
     return cfg.num_heads % tp == 0 and cfg.intermediate_size % tp == 0 and cfg.vocab_size % tp == 0
 
 

@@ -51,3 +51,14 @@ def init_weight(shape, device, dtype=torch.bfloat16, std: float = 0.02, gen: tor
 
 def init_norm(n, device, dtype=torch.bfloat16):
     return torch.ones(n, device=device, dtype=dtype)
+
+
+def fuse_rows(parts, multiple: int = 16, large: int = 256) -> torch.Tensor:
+    """Projections of one input stacked into one weight [N, K], zero rows up to a whole number of
+    GEMM tiles (``large`` from 2048 rows, where the 256-column tiles run)."""
+    n = sum(p.shape[0] for p in parts)
+    m = large if n >= 2048 else multiple
+    pad = -n % m
+    if pad:
+        parts = [*parts, parts[0].new_zeros(pad, parts[0].shape[1])]
+    return torch.cat(parts, 0).contiguous()

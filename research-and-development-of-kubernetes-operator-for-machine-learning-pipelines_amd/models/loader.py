@@ -18,6 +18,8 @@ Layout mapping (HF name -> ours; TP sharding then reuses ``load_shard_from``):
   Mixtral: block_sparse_moe.gate | mlp.gate      -> router
            experts.{e}.w1 / w3 (legacy) or experts.gate_up_proj (fused) -> w13 (interleaved)
            experts.{e}.w2 or experts.down_proj   -> w2
+Kosesun checkpoints (``"architecture": "Kosesun"``; tensors ``l<i>.mix.*`` ...) are read by the model
+itself as it is built (models/kosesun.py).
 Tensors are read lazily, one layer at a time (safetensors memory map), so a 141 GB
 checkpoint never sits in host memory at once.
 """
@@ -30,7 +32,7 @@ from pathlib import Path
 
 import torch
 
-from .config import ModelConfig, PRESETS
+from .config import AttentionSpec, GLASpec, LayerSpec, ModelConfig, PRESETS, hybrid_config
 
 _ARCH_NAMES = {"LlamaForCausalLM": "llama", "MixtralForCausalLM": "mixtral", "MistralForCausalLM": "llama"}
 
@@ -97,6 +99,48 @@ def config_from_hf(d: dict, name: str | None = None) -> ModelConfig:
         rope_scaling=scaling, eos_token_id=int(eos), extra_eos_ids=eos_all[1:])
 
 
+def _only(d: dict, known: set, where: str) -> None:
+    extra = set(d) - known
+    if extra:
+        raise ValueError(f"{where}: unsupported settings {sorted(extra)}")
+
+
+def config_from_kosesun(d: dict, shape_of, name: str | None = None, max_position: int | None = None) -> ModelConfig:
+    """HybridConfig from a Kosesun ``config.json`` dict.  ``shape_of(tensor name)``: sizes that only
+    the checkpoint's tensors give (the decay projection's inner size).  Settings this runtime does
+    not know are rejected, never dropped."""
+    _only(d, {"architecture", "embedding", "layers", "logit_softcap", "norm", "streams", "vocab", "width"}, "config")
+    layers = []
+    for i, la in enumerate(d["layers"]):
+        _only(la, {"type", "mixer", "mlp"}, f"layer {i}")
+        m, mlp = la["mixer"], la.get("mlp")
+        if la["type"] == "attention":
+            _only(m, {"dim", "heads", "kv_heads", "rot", "scale", "v_mix", "vdim"}, f"layer {i} mixer")
+            rot = m.get("rot") or {"base": 1.0, "dims": 0}
+            _only(rot, {"base", "dims"}, f"layer {i} rotation")
+            mixer = AttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]),
+                                  vdim=int(m["vdim"]), scale=float(m["scale"]), rot_base=float(rot["base"]),
+                                  rot_dims=int(rot["dims"]), v_mix=bool(m.get("v_mix", False)))
+            if mixer.scale <= 0:
+                raise ValueError(f"layer {i}: score scale must be positive")
+            if mixer.heads % mixer.kv_heads or mixer.dim % 2 or mixer.rot_dims % 2 or mixer.rot_dims > mixer.dim:
+                raise ValueError(f"layer {i}: unsupported attention sizes {m}")
+        elif la["type"] == "gla":
+            _only(m, {"dim", "heads", "tau", "vdim"}, f"layer {i} mixer")
+            mixer = GLASpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), tau=float(m["tau"]),
+                            rank=int(shape_of(f"l{i}.mix.a1")[0]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {la['type']!r}")
+        if mlp is not None:
+            _only(mlp, {"ff", "kind"}, f"layer {i} mlp")
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unsupported feed-forward {mlp['kind']!r}")
+        layers.append(LayerSpec(mixer, int(mlp["ff"]) if mlp is not None else 0))
+    kw = {} if max_position is None else {"max_position": max_position}
+    return hybrid_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers, int(d["streams"]),
+                         float(d["embedding"]["scale"]), float(d["logit_softcap"]), float(d["norm"]["eps"]), **kw)
+
+
 class _Tensors:
     """Name -> tensor over every ``*.safetensors`` shard of a directory (lazy, mmap)."""
 
@@ -108,6 +152,11 @@ class _Tensors:
 
     def has(self, k: str) -> bool:
         return k in self._where
+
+    def shape(self, k: str) -> list:
+        if k not in self._where:
+            raise KeyError(f"checkpoint has no tensor {k!r}")
+        return self._where[k].get_slice(k).get_shape()
 
     def get(self, k: str) -> torch.Tensor:
         if k not in self._where:
@@ -179,11 +228,19 @@ class HFWeights:
 
 def load_pretrained(path: str | os.PathLike, device="cuda", dtype=torch.bfloat16, pstate=None,
                     name: str | None = None, fold_norms: bool = True):
-    """Build our model for the checkpoint in ``path`` and copy its (TP-sharded) weights in."""
+    """Build our model for the checkpoint in ``path`` and copy its (TP-sharded) weights in.  The
+    model class follows from config.json: ``architecture`` (Kosesun) or HF's ``architectures``."""
     from . import build_model
 
     path = Path(path)
-    cfg = config_from_hf(json.loads((path / "config.json").read_text()), name=name or path.name)
+    d = json.loads((path / "config.json").read_text())
+    if "architecture" in d:
+        if d["architecture"] != "Kosesun":
+            raise ValueError(f"unsupported checkpoint architecture {d['architecture']!r}")
+        t = _Tensors(path)
+        cfg = config_from_kosesun(d, t.shape, name=name or path.name)
+        return build_model(cfg, device=device, dtype=dtype, pstate=pstate, weights=t)
+    cfg = config_from_hf(d, name=name or path.name)
     model = build_model(cfg, device=device, dtype=dtype, pstate=pstate)
     with torch.no_grad():
         model.load_shard_from(HFWeights(path, cfg))

@@ -203,6 +203,9 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
         x2 = x2.contiguous()
     M, K = x2.shape
     o2 = torch.empty(M, out_n, dtype=x.dtype, device=x.device) if out is None else out.view(M, out_n)
+    if x.dtype == torch.float32 and epi == EPI_NONE:  # true fp32 (library product; no reduced-precision mode)
+        torch.matmul(x2, w.t(), out=o2)
+        return o2.view(*lead, out_n) if out is None else out
     _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi)
     return o2.view(*lead, out_n) if out is None else out
 
@@ -704,6 +707,92 @@ def sample(logits, temps, top_ks, top_ps, uniform, full: bool | None = None) -> 
 
 __all__ = ["argmax", "sample", "load","available", "library_path", "rmsnorm", "add_rmsnorm", "rope_cache",
            "silu_mul", "embedding", "paged_attention", "ref"]
+
+
+# ------------------------------------------------- hybrid decoder layers --
+
+def hyper_begin(ids, table, scale: float, n_streams: int, w_in, norm_w, eps: float):
+    """Hyper-connection streams of a step, all the scaled embedding row, and the first sublayer's
+    input: (streams fp32 [T, S, W], norm(sum_s w_in[s] x_s) in the table's dtype)."""
+    T, W = ids.numel(), table.shape[1]
+    if not table.is_cuda:
+        return ref.hyper_begin(ids, table, scale, n_streams, w_in, norm_w, eps)
+    _need_gpu()
+    streams = torch.empty(T, n_streams, W, dtype=torch.float32, device=table.device)
+    xn = torch.empty(T, W, dtype=table.dtype, device=table.device)
+    torch.ops.mlop.hyper_begin(xn, streams, ids, table, scale, w_in, norm_w, eps)
+    return streams, xn
+
+
+def hyper_step(streams, y, mix, w_out, w_in, norm_w, eps: float, store: bool = True):
+    """streams[:, t] <- sum_s mix[s, t] streams[:, s] + w_out[t] y (in place, unless ``store`` is off:
+    nothing reads them again); returns the next sublayer's input norm(sum_t w_in[t] streams[:, t])."""
+    if not y.is_cuda:
+        return ref.hyper_step(streams, y, mix, w_out, w_in, norm_w, eps)
+    _need_gpu()
+    xn = torch.empty_like(y)
+    torch.ops.mlop.hyper_step(xn, streams, y, mix, w_out, w_in, norm_w, eps, store)
+    return xn
+
+
+def relu2(x):
+    """max(x, 0)^2, in place."""
+    if not x.is_cuda:
+        return x.copy_(ref.relu2(x))
+    _need_gpu()
+    torch.ops.mlop.relu2(x)
+    return x
+
+
+def softcap(x, cap: float):
+    """cap * tanh(x / cap), fp32."""
+    if not x.is_cuda:
+        return ref.softcap(x, cap)
+    _need_gpu()
+    out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    torch.ops.mlop.softcap(out, x, cap)
+    return out
+
+
+def qk_norm_rope(proj, n_heads: int, dim: int, vdim: int, q_w, k_w, eps: float, cos_sin, positions, slots, k_cache,
+                 v_cache, v_first=None, lam=None):
+    """proj [T, >= H dim + G (dim + vdim)] = [q | k | v | ...] -> q [T, H, KP]: RMS norm of the whole q
+    and k rows (``q_w`` None: none), rotation of the first cos_sin.shape[1] dims of each head in
+    pairs (2i, 2i + 1); k and v ((1 - lam) v + lam v_first) into the paged caches."""
+    if not proj.is_cuda:
+        return ref.qk_norm_rope(proj, n_heads, dim, vdim, q_w, k_w, eps, cos_sin, positions, slots, k_cache, v_cache,
+                                v_first, lam)
+    _need_gpu()
+    q = torch.empty(proj.shape[0], n_heads, k_cache.shape[3], dtype=proj.dtype, device=proj.device)
+    torch.ops.mlop.qk_norm_rope(q, k_cache, v_cache, proj, dim, vdim, q_w, k_w, eps, cos_sin, positions, slots, v_first,
+                                lam)
+    return q
+
+
+def attention_hd(q, k_cache, v_cache, meta, dim: int, vdim: int, scale: float, sink=None, gate=None):
+    """Ragged causal paged attention of any head sizes: q [T, H, KP] -> [T, H, vdim].  ``sink`` [H] joins
+    each head's softmax denominator; ``gate`` [T, H]: the head's output times sigmoid(gate)."""
+    if not q.is_cuda:
+        return ref.attention_hd(q, k_cache, v_cache, meta, dim, vdim, scale, sink, gate)
+    _need_gpu()
+    out = torch.empty(q.shape[0], q.shape[1], vdim, dtype=q.dtype, device=q.device)
+    torch.ops.mlop.attention_hd(out, meta.part_o, meta.part_ml, meta.part_sem, q, k_cache, v_cache, meta.block_tables,
+                                meta.tile_seq, meta.tile_q0, meta.ptile_seq, meta.ptile_q0, meta.q_start, meta.q_len,
+                                meta.ctx_len, dim, scale, sink, gate, meta.part_tokens, meta.nparts)
+    return out
+
+
+def gla(proj, n_heads: int, dim: int, vdim: int, a2, a2_b, norm_w, tau: float, eps: float, state, meta):
+    """Gated linear attention of a ragged step: proj [T, ...] = [q | k | v | gate | a1 | ...] -> the normed,
+    gated heads [T, H vdim]; ``state`` [slots, H, dim, vdim] fp32 (slot = sequence row) is advanced."""
+    if not proj.is_cuda:
+        return ref.gla(proj, n_heads, dim, vdim, a2, a2_b, norm_w, tau, eps, state, meta)
+    _need_gpu()
+    out = torch.empty(proj.shape[0], n_heads * vdim, dtype=proj.dtype, device=proj.device)
+    torch.ops.mlop.gla(out, state, proj, n_heads, dim, vdim, a2, a2_b, norm_w, tau, eps, meta.q_start, meta.q_len,
+                       meta.ctx_len, meta.tile_seq, meta.citem_seq, meta.citem_t0, meta.crow_seq, meta.crow_item0,
+                       meta.chunk)
+    return out
 
 
 # ------------------------------------------------------------------ MoE --

@@ -3,8 +3,8 @@
 Every ``csrc/*.hip`` file is compiled by ``hipcc --offload-arch=gfx950`` into
 its own object (parallel, incremental on CONTENT: an object is rebuilt when the
 hash of its source + every header + its command line differs from the one
-recorded beside it, never on mtimes), ``csrc/bindings.cpp`` (the torch op
-registrations) is compiled against torch's headers, and the objects are linked
+recorded beside it, never on mtimes), ``csrc/bindings*.cpp`` (the torch op
+registrations) are compiled against torch's headers, and the objects are linked
 against torch's own HIP runtime (``torch/lib/libamdhip64.so``, SONAME
 ``libamdhip64.so.7``) so the process holds exactly one HIP runtime.
 
@@ -85,7 +85,8 @@ def _stale(obj: Path, src: Path, headers, cmd) -> tuple[bool, str]:
 # KERNEL_FLAGS: no packed f32 arithmetic (v_pk_add / mul / fma_f32) from ordinary float code: some
 # forms have returned wrong results on this hardware, without an error.
 KERNEL_FLAGS = ["-ffp-contract=fast", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
-FILE_FLAGS = {"attention": ["-fno-honor-nans", "-fno-slp-vectorize"]}
+FILE_FLAGS = {"attention": ["-fno-honor-nans", "-fno-slp-vectorize"],
+              "attention_hd": ["-fno-honor-nans", "-fno-slp-vectorize"]}
 
 
 def _run(cmd):
@@ -119,16 +120,18 @@ def build(jobs: int | None = None, force: bool = False, verbose: bool = False) -
         stale, digest = _stale(obj, src, headers, cmd)
         if force or stale:
             jobs_list.append((cmd, obj, digest))
-    bsrc = CSRC / "bindings.cpp"
-    bobj = BUILD / "bindings.o"
+    # torch op registrations: csrc/bindings*.cpp
+    bindings = sorted(CSRC.glob("bindings*.cpp"))
     py_inc = sysconfig.get_paths()["include"]
-    bcmd = [hipcc, *common, "-x", "c++", f"-D_GLIBCXX_USE_CXX11_ABI={abi}", "-DUSE_ROCM=1",
-            "-DTORCH_EXTENSION_NAME=_C", *[f"-I{p}" for p in tinc], f"-I{py_inc}",
-            "-I/opt/rocm/include", "-Wno-deprecated-declarations",
-            "-c", str(bsrc), "-o", str(bobj)]
-    stale, digest = _stale(bobj, bsrc, headers, bcmd)
-    if force or stale:
-        jobs_list.append((bcmd, bobj, digest))
+    for src in bindings:
+        obj = BUILD / (src.stem + ".o")
+        cmd = [hipcc, *common, "-x", "c++", f"-D_GLIBCXX_USE_CXX11_ABI={abi}", "-DUSE_ROCM=1",
+               "-DTORCH_EXTENSION_NAME=_C", *[f"-I{p}" for p in tinc], f"-I{py_inc}",
+               "-I/opt/rocm/include", "-Wno-deprecated-declarations",
+               "-c", str(src), "-o", str(obj)]
+        stale, digest = _stale(obj, src, headers, cmd)
+        if force or stale:
+            jobs_list.append((cmd, obj, digest))
     # the tree's source hash, compiled into the library (ops.load() checks it)
     want = source_hash()
     hsrc, hobj = BUILD / "srchash.cpp", BUILD / "srchash.o"
@@ -150,7 +153,7 @@ def build(jobs: int | None = None, force: bool = False, verbose: bool = False) -
             for r in ex.map(run, jobs_list):
                 if verbose and (r.stdout or r.stderr):
                     print(r.stdout, r.stderr, file=sys.stderr)
-    objs = [BUILD / (s.stem + ".o") for s in kernels] + [BUILD / (s.stem + ".o") for s in hosts] + [bobj, hobj]
+    objs = [BUILD / (s.stem + ".o") for s in (*kernels, *hosts, *bindings)] + [hobj]
     if force or jobs_list or not OUT.exists():
         tlib = troot / "lib"
         tmp = OUT.with_suffix(".so.tmp")

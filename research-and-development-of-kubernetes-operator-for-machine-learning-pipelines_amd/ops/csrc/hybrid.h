@@ -1,0 +1,104 @@
+// Launchers of the hybrid-decoder kernels (hyper-connections, whole-projection query / key norm
+// with partial rotary positions, paged attention of any head sizes with a softmax sink and an
+// output gate, gated linear attention).  `f32` selects float operands; otherwise bf16.
+#pragma once
+
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+namespace mlop {
+
+// ---- hyper-connections (hyper.hip)
+struct HyperArgs {
+  float* streams;        // [T, S, W]
+  void* xn;              // [T, W] normed sublayer input
+  const void* y;         // [T, W] sublayer output (null: streams start from the embedding)
+  const long* ids;       // [T]     (start only)
+  const void* table;     // [vocab, W] (start only)
+  float embed_scale;
+  long vocab;
+  const float* mix;      // [S, S] (from, to)
+  const float* w_out;    // [S]
+  const float* w_in;     // [S] of the sublayer that reads next
+  const float* norm_w;   // [W]
+  float eps;
+  int T, W, S;
+  bool store;            // write the new streams back (off behind the last sublayer)
+};
+void launch_hyper(const HyperArgs& a, bool f32, hipStream_t st);
+constexpr int kMaxStreams = 64;
+
+// ---- query / key norm + rotary + value mixing + paged stores (qk_norm.hip)
+struct QkNormArgs {
+  void* q_out;           // [T, H, KP], dims past D zero
+  void* k_cache;         // [NB, G, BS, KP]
+  void* v_cache;         // [NB, G, BS, VP]
+  const void* proj;      // [T, ldp]: q (H x D) | k (G x D) | v (G x V) | ...
+  long ldp;
+  const void* v_first;   // values to mix in, row stride ldf (null: none)
+  long ldf;
+  const float* lam;      // [1] share of v_first
+  const float* q_w;      // [H * D] (null: no norm)
+  const float* k_w;      // [G * D]
+  float eps;
+  const float* cos_sin;  // [max_pos, R]: cos of the R / 2 pairs, then sin
+  int R;                 // rotated dims of a head (even; pairs 2i, 2i + 1)
+  const int* pos;
+  const int* slots;      // < 0: no cache write
+  int T, H, G, D, V, KP, VP, BS;
+};
+void launch_qk_norm(const QkNormArgs& a, bool f32, hipStream_t st);
+
+// ---- paged attention of any head sizes (attention_hd.hip)
+struct AttnHdArgs {
+  void* out;             // [T, H, V]
+  const void* q;         // [T, H, KP]
+  const void* k_cache;   // [NB, G, 16, KP]
+  const void* v_cache;   // [NB, G, 16, VP]
+  const int* bt;
+  int bt_stride;
+  const int *q_start, *q_len, *ctx_len;
+  const float* sink;     // [H] or null
+  const void* gate;      // [T, gate_stride] pre-sigmoid, one per head, or null
+  long gate_stride;
+  int H, G, D, V, KP, VP;
+  float scale_log2;
+  int num_blocks;
+};
+// one query token per tile, split over `nparts` ranges of `part_tokens` keys
+void launch_paged_hd(const AttnHdArgs& a, bool f32, float* part_o, float* part_ml, int* sem, const int* tile_seq,
+                     const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st);
+// tiles of up to 128 query tokens of one head
+void launch_flash_hd(const AttnHdArgs& a, bool f32, const int* tile_seq, const int* tile_q0, int num_tiles,
+                     hipStream_t st);
+constexpr int kHdTile = 128;      // query tokens of a flash tile
+constexpr int kHdMaxDim = 256;    // head sizes of the MFMA kernels (larger ones take the plain kernel)
+constexpr int kHdMaxV = 1024;     // value size of the plain kernel
+
+// ---- gated linear attention (gla.hip)
+struct GlaArgs {
+  void* out;             // [T, H * dv] (normed and gated)
+  const void* proj;      // [T, ldp]: q (H x dk) | k (H x dk) | v (H x dv) | g (H x dv) | a1 (rank)
+  long ldp;
+  const void* a2;        // [H * dk, rank]
+  const float* a2_b;     // [H * dk]
+  const float* norm_w;   // [dv]
+  float* state;          // [slots, H, dk, dv]
+  const int *q_start, *q_len, *ctx_len;
+  int n_slots, H, dk, dv, rank;
+  float inv_tau, q_scale, eps;
+};
+// every token of each listed row in turn (one-token rows; any sizes)
+void launch_gla_rows(const GlaArgs& a, bool f32, const int* rows, int n_rows, hipStream_t st);
+// chunks of `chunk` tokens in parallel: logd [T, H * dk], o32 [T, H, dv], cstate [items, H, dk, dv],
+// cdecay [items, H, dk] are scratch; crow_* list the sequences and their items
+void launch_gla_chunks(const GlaArgs& a, bool f32, float* logd, float* o32, float* cstate, float* cdecay, int T,
+                       const int* item_seq, const int* item_t0, int n_items, const int* crow_seq,
+                       const int* crow_item0, int n_crows, int chunk, hipStream_t st);
+constexpr int kGlaMaxDk = 256;    // key size of the chunked kernel
+
+// ---- elementwise (hyper.hip)
+void launch_relu2(void* x, long n, bool f32, hipStream_t st);                       // in place
+void launch_softcap(float* out, const void* x, long n, float cap, bool f32, hipStream_t st);
+
+}  // namespace mlop

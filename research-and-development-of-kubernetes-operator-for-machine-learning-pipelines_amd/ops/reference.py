@@ -107,6 +107,107 @@ def paged_attention(q, k_cache, v_cache, meta):
     return out
 
 
+# ------------------------------------------------- hybrid decoder layers --
+
+def _unit(x, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def hyper_begin(ids, table, scale, n_streams, w_in, norm_w, eps):
+    x = table[ids.reshape(-1).long()].float() * scale
+    streams = x[:, None, :].repeat(1, n_streams, 1)
+    return streams, (_unit(torch.einsum("s,tsw->tw", w_in, streams), eps) * norm_w).to(table.dtype)
+
+
+def hyper_step(streams, y, mix, w_out, w_in, norm_w, eps):
+    streams.copy_(torch.einsum("st,bsw->btw", mix, streams) + w_out[None, :, None] * y.float()[:, None, :])
+    return (_unit(torch.einsum("s,tsw->tw", w_in, streams), eps) * norm_w).to(y.dtype)
+
+
+def relu2(x):
+    return torch.relu(x.float()).square().to(x.dtype)
+
+
+def softcap(x, cap):
+    return cap * torch.tanh(x.float() / cap)
+
+
+def rotate_pairs(x, cos, sin):
+    """x [T, heads, D] with pairs (2i, 2i + 1), cos / sin [T, R / 2]: the first R dims turn."""
+    R = 2 * cos.shape[-1]
+    u, v = x[..., :R:2], x[..., 1:R:2]
+    c, s = cos[:, None], sin[:, None]
+    turned = torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2)
+    return torch.cat([turned, x[..., R:]], -1)
+
+
+def qk_norm_rope(proj, H, D, V, q_w, k_w, eps, cos_sin, positions, slots, k_cache, v_cache, v_first, lam):
+    T, G, BS, KP = proj.shape[0], k_cache.shape[1], k_cache.shape[2], k_cache.shape[3]
+    x = proj.float()
+    q, k, v = x[:, :H * D], x[:, H * D:(H + G) * D], x[:, (H + G) * D:(H + G) * D + G * V]
+    if q_w is not None:
+        q, k = _unit(q, eps) * q_w, _unit(k, eps) * k_w
+    half = cos_sin.shape[1] // 2
+    cs = cos_sin[positions.long()]
+    q = rotate_pairs(q.reshape(T, H, D), cs[:, :half], cs[:, half:])
+    k = rotate_pairs(k.reshape(T, G, D), cs[:, :half], cs[:, half:])
+    if v_first is not None:
+        v = (1 - lam) * v + lam * v_first.float()
+    keep = slots >= 0
+    blk, off = slots[keep].long() // BS, slots[keep].long() % BS
+    k_cache[blk, :, off, :D] = k[keep].to(k_cache.dtype)
+    v_cache[blk, :, off, :V] = v.reshape(T, G, V)[keep].to(v_cache.dtype)
+    out = torch.zeros(T, H, KP, dtype=proj.dtype, device=proj.device)
+    out[:, :, :D] = q.to(proj.dtype)
+    return out
+
+
+def _live_rows(meta):
+    rows = set(meta.tile_seq.tolist()) | set(meta.ptile_seq.tolist())
+    qs, ql, cl = meta.q_start.tolist(), meta.q_len.tolist(), meta.ctx_len.tolist()
+    return [(r, qs[r], ql[r], cl[r]) for r in sorted(rows) if ql[r] and cl[r]]
+
+
+def attention_hd(q, k_cache, v_cache, meta, D, V, scale, sink, gate):
+    T, H = q.shape[:2]
+    G = k_cache.shape[1]
+    out = torch.zeros(T, H, V, dtype=torch.float32, device=q.device)
+    for row, s, n, ctx in _live_rows(meta):
+        k, v = gather_kv(k_cache, v_cache, meta.block_tables[row], ctx)
+        k = k[..., :D].float().repeat_interleave(H // G, 1)
+        v = v[..., :V].float().repeat_interleave(H // G, 1)
+        w = torch.einsum("qhd,khd->hqk", q[s:s + n, :, :D].float(), k) * scale
+        pos = torch.arange(ctx - n, ctx, device=q.device)[:, None]
+        w = w.masked_fill((torch.arange(ctx, device=q.device)[None] > pos)[None], float("-inf"))
+        if sink is not None:
+            w = torch.cat([w, sink.float().view(H, 1, 1).expand(H, n, 1)], -1)
+        p = torch.softmax(w, -1)[..., :ctx]
+        out[s:s + n] = torch.einsum("hqk,khd->qhd", p, v)
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float())[..., None]
+    return out.to(q.dtype)
+
+
+def gla(proj, H, D, V, a2, a2_b, norm_w, tau, eps, state, meta):
+    T, hk, hv = proj.shape[0], H * D, H * V
+    x = proj.float()
+    q = x[:, :hk].reshape(T, H, D) * D ** -0.5
+    k = x[:, hk:2 * hk].reshape(T, H, D)
+    v = x[:, 2 * hk:2 * hk + hv].reshape(T, H, V)
+    g = x[:, 2 * hk + hv:2 * hk + 2 * hv]
+    z = x[:, 2 * hk + 2 * hv:2 * hk + 2 * hv + a2.shape[1]] @ a2.float().t() + a2_b
+    decay = torch.exp(torch.nn.functional.logsigmoid(z) / tau).reshape(T, H, D)
+    o = torch.zeros(T, H, V, dtype=torch.float32, device=proj.device)
+    for row, s, n, ctx in _live_rows(meta):
+        S = torch.zeros_like(state[row]) if ctx == n else state[row]
+        for t in range(s, s + n):
+            S = decay[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+            o[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[row] = S
+    o = (_unit(o, eps) * norm_w).reshape(T, hv) * torch.nn.functional.silu(g)
+    return o.to(proj.dtype)
+
+
 # ------------------------------------------------------------------ MoE --
 
 def moe_route(logits, top_k):

@@ -44,6 +44,14 @@ class AttnMeta:
     # int32 tickets (zero-initialised, re-armed by the kernel): the last partition of a
     # split-KV (tile, kv head) combines the slabs in the same launch; None -> reduce launch
     part_sem: torch.Tensor | None = None
+    # recurrent layers (None: the model has none): prompt portions cut into chunks of ``chunk``
+    # tokens (item -> row, first token of the portion) and the rows they belong to (row, first item);
+    # one-token rows are ``tile_seq``
+    citem_seq: torch.Tensor | None = None
+    citem_t0: torch.Tensor | None = None
+    crow_seq: torch.Tensor | None = None
+    crow_item0: torch.Tensor | None = None
+    chunk: int = 0
 
 
 # 128-token partitions: one 32-token page pair per wave at batch 1 (256: 312 tok/s, 128: 322,
@@ -101,12 +109,17 @@ class MetaBuffers:
     and ``max_seqs`` concurrent sequences."""
 
     def __init__(self, max_tokens: int, max_seqs: int, max_blocks_per_seq: int, group: int,
-                 n_kv: int, max_model_len: int, device, flash_min_q: int = 17):
+                 n_kv: int, max_model_len: int, device, flash_min_q: int = 17, flash_tile: int | None = None,
+                 part_dim: int = 128, chunk: int = 0, max_logits: int | None = None):
+        """``flash_tile``: query tokens of a prompt tile (default: 128 MFMA rows of the GQA group);
+        ``part_dim``: value size of the split-KV partials; ``chunk``: prompt chunk of recurrent
+        layers (0: none); ``max_logits``: logits rows of a step (default: one per sequence)."""
         self.device = torch.device(device)
         self.max_tokens, self.max_seqs, self.mb = max_tokens, max_seqs, max_blocks_per_seq
         self.G, self.n_kv, self.max_model_len = group, n_kv, max_model_len
         self.qt = 16 // group
-        self.pqt = 128 // group if group <= 8 else 0  # flash tile tokens (0: no flash kernel for G > 8)
+        # flash tile tokens (0: no flash kernel for G > 8)
+        self.pqt = flash_tile or (128 // group if group <= 8 else 0)
         self.flash_min_q = flash_min_q if self.pqt else 1 << 30
         self.max_tiles = max_tokens  # worst case: one tile per token
         self.npt = 0                 # flash tiles of the last fill
@@ -114,6 +127,12 @@ class MetaBuffers:
         sizes = [("positions", max_tokens), ("slots", max_tokens), ("tile_seq", self.max_tiles),
                  ("tile_q0", self.max_tiles), ("ptile_seq", self.max_tiles), ("ptile_q0", self.max_tiles),
                  ("q_start", max_seqs), ("q_len", max_seqs), ("ctx_len", max_seqs)]
+        self.chunk = chunk
+        self.n_items = self.n_crows = 0  # recurrent chunk items / rows of the last fill
+        if chunk:
+            ni = max_tokens // chunk + min(max_seqs, max_tokens // 2) + 1
+            sizes += [("citem_seq", ni), ("citem_t0", ni), ("crow_seq", max_seqs), ("crow_item0", max_seqs)]
+        self.max_logits = max_logits = max(max_logits or 0, max_seqs)
         # ONE int32 buffer per side: [header | int32 metadata | ids (int64) | logits index (int64) |
         # block tables], every region 64-int aligned.  One H2D ships a step; a tensor-parallel
         # step is ONE broadcast of the device buffer (engine.StepSync: header + metadata + ids
@@ -129,7 +148,7 @@ class MetaBuffers:
         ids_lo = o
         o += (2 * max_tokens + 63) // 64 * 64
         lidx_lo = o
-        o += (2 * max_seqs + 63) // 64 * 64
+        o += (2 * max_logits + 63) // 64 * 64
         self.off["block_tables"] = (o, max_seqs * max_blocks_per_seq)
         o += (max_seqs * max_blocks_per_seq + 63) // 64 * 64
         self.total = o
@@ -145,14 +164,14 @@ class MetaBuffers:
         self.ids_h = self.hbuf[ids_lo:ids_lo + 2 * max_tokens].view(torch.int64)
         self.ids_hn = self.ids_h.numpy()
         self.ids_d = self.dbuf[ids_lo:ids_lo + 2 * max_tokens].view(torch.int64)
-        self.lidx_h = self.hbuf[lidx_lo:lidx_lo + 2 * max_seqs].view(torch.int64)
+        self.lidx_h = self.hbuf[lidx_lo:lidx_lo + 2 * max_logits].view(torch.int64)
         self.lidx_hn = self.lidx_h.numpy()
-        self.lidx_d = self.dbuf[lidx_lo:lidx_lo + 2 * max_seqs].view(torch.int64)
+        self.lidx_d = self.dbuf[lidx_lo:lidx_lo + 2 * max_logits].view(torch.int64)
         # partial-softmax workspace for the split-KV path (sized for the worst launch)
         # plan_partitions only splits launches with < target/2 base workgroups, so
         # tiles * n_kv * nparts stays <= ~2 * target: size for 4096 partial tiles
         self.wp_capacity = 4096
-        self.part_o = torch.empty(self.wp_capacity * 16 * 128, dtype=torch.float32, device=self.device)
+        self.part_o = torch.empty(self.wp_capacity * 16 * part_dim, dtype=torch.float32, device=self.device)
         self.part_ml = torch.empty(self.wp_capacity * 16 * 2, dtype=torch.float32, device=self.device)
         self.part_sem = torch.zeros(self.wp_capacity, dtype=torch.int32, device=self.device)
         bt = self.view_h("block_tables").reshape(max_seqs, max_blocks_per_seq)
@@ -195,7 +214,14 @@ class MetaBuffers:
             ptile_seq=self.view_d("ptile_seq", num_ptiles), ptile_q0=self.view_d("ptile_q0", num_ptiles),
             q_start=self.view_d("q_start"), q_len=self.view_d("q_len"), ctx_len=self.view_d("ctx_len"),
             part_tokens=part_tokens, nparts=nparts, part_o=self.part_o, part_ml=self.part_ml,
-            logits_idx=self.lidx_d[:n_logits], num_tokens=num_tokens, part_sem=self.part_sem)
+            logits_idx=self.lidx_d[:n_logits], num_tokens=num_tokens, part_sem=self.part_sem, **self._chunk_views())
+
+    def _chunk_views(self) -> dict:
+        if not self.chunk:
+            return {}
+        n, r = self.n_items, self.n_crows
+        return {"citem_seq": self.view_d("citem_seq", n), "citem_t0": self.view_d("citem_t0", n),
+                "crow_seq": self.view_d("crow_seq", r), "crow_item0": self.view_d("crow_item0", r), "chunk": self.chunk}
 
     def fill(self, rows, q_lens, ctx_lens, token_ids_per_seq, want_logits=None):
         """Fill host arrays for a ragged batch.
@@ -204,7 +230,7 @@ class MetaBuffers:
         KV is written this step; ctx_lens[i] context length AFTER this step;
         token_ids_per_seq[i]: the q_len input ids. Block tables must already
         hold the pages covering ctx_lens.  want_logits[i] (default all): emit a
-        logits row for sequence i's last token.  Returns (T, num_tiles, n_logits);
+        logits row for sequence i's last token; a list of token offsets emits those.  Returns (T, num_tiles, n_logits);
         the flash-tile count is left in ``self.npt``."""
         return self._fill_ragged(0, 0, 0, rows, q_lens, ctx_lens, token_ids_per_seq, want_logits)
 
@@ -223,6 +249,7 @@ class MetaBuffers:
         ts_h, tq_h = self.view_h("tile_seq"), self.view_h("tile_q0")
         pts_h, ptq_h = self.view_h("ptile_seq"), self.view_h("ptile_q0")
         npt, pqt = 0, self.pqt
+        ni = nr = 0
         max_flash_q = 0
         qs_h, ql_h, cl_h = self.view_h("q_start"), self.view_h("q_len"), self.view_h("ctx_len")
         qt = self.qt
@@ -245,20 +272,31 @@ class MetaBuffers:
                 ts_h[nt:nt + ntile] = row
                 tq_h[nt:nt + ntile] = np.arange(ntile, dtype=np.int32) * qt
                 nt += ntile
-            t += ql
-            if want_logits is None or want_logits[i]:
-                self.lidx_hn[nl] = t - 1
+            if self.chunk and ql > 1:
+                n = -(-ql // self.chunk)
+                self.view_h("crow_seq")[nr], self.view_h("crow_item0")[nr] = row, ni
+                self.view_h("citem_seq")[ni:ni + n] = row
+                self.view_h("citem_t0")[ni:ni + n] = np.arange(n, dtype=np.int32) * self.chunk
+                ni, nr = ni + n, nr + 1
+            w = True if want_logits is None else want_logits[i]
+            if isinstance(w, (list, tuple)):
+                self.lidx_hn[nl:nl + len(w)] = np.asarray(w, dtype=np.int64) + t
+                nl += len(w)
+            elif w:
+                self.lidx_hn[nl] = t + ql - 1
                 nl += 1
+            t += ql
         if npt > 1 and FLASH_LPT and max_flash_q >= FLASH_LPT_MIN_Q:
             order_flash_tiles(pts_h[:npt], ptq_h[:npt], self._pwork[:npt])
         self.npt = npt
+        self.n_items, self.n_crows = ni, nr
         return t, nt, nl
 
     def fill_decode(self, rows: np.ndarray, ctx_lens: np.ndarray, last_tokens: np.ndarray, pad_to: int):
         """Vectorised decode fill: one query token per sequence, padded to the
         graph bucket ``pad_to`` with rows that attend to nothing."""
         B = len(rows)
-        self.npt = 0
+        self.npt = self.n_items = self.n_crows = 0
         pos_h, slot_h = self.view_h("positions"), self.view_h("slots")
         ts_h, tq_h = self.view_h("tile_seq"), self.view_h("tile_q0")
         qs_h, ql_h, cl_h = self.view_h("q_start"), self.view_h("q_len"), self.view_h("ctx_len")

@@ -37,7 +37,7 @@ import torch
 
 from .. import ops
 from .attn_meta import MetaBuffers, plan_partitions
-from .kv_cache import BLOCK_SIZE, BlockAllocator, KVCache, blocks_for_budget, blocks_needed, prefix_hashes
+from .kv_cache import BLOCK_SIZE, BlockAllocator, KVCache, StateCache, blocks_for_budget, blocks_needed, prefix_hashes
 from .sampler import Sampler, SamplingParams
 from .tracing import StepTracer, TorchProfileWindow
 
@@ -214,6 +214,7 @@ class EngineConfig:
     mixed_min_chunk: int = 64     # below this many free token slots, decode alone
     seed: int = 0
     enable_prefix_caching: bool = True  # share computed prompt pages between requests (same prefix)
+    max_step_logits: int | None = None  # logits rows of one step (None: one per sequence; ``feed`` may want more)
     # one-step-ahead scheduling (TP = EP = 1, mixed prefill): step t+1 is built and launched
     # while step t still runs on the device; step t's tokens are read back afterwards
     async_scheduling: bool = True
@@ -294,7 +295,8 @@ class Engine:
         t_kv = time.perf_counter()
         # TP ranks must all hold every page id the leader hands out: eager backing there
         self.kv = KVCache(mc.num_layers, nb, model.n_kv, mc.head_dim, self.device, model.dtype,
-                          lazy=False if tp.size > 1 else None)
+                          lazy=False if tp.size > 1 else None, layout=getattr(model, "cache_layout", None),
+                          state_shapes=self._state_shapes(), state_slots=cfg.max_num_seqs)
         if self.device.type == "cuda":
             torch.cuda.synchronize(self.device)
         kv_alloc_ms = int(1e3 * (time.perf_counter() - t_kv))
@@ -306,7 +308,13 @@ class Engine:
         self.G = model.n_q // model.n_kv
         self.meta = MetaBuffers(max(cfg.max_num_batched_tokens, cfg.max_num_seqs),
                                 cfg.max_num_seqs + self.buckets[-1], self.max_blocks_per_seq,
-                                self.G, model.n_kv, self.max_model_len, self.device)
+                                n_kv=model.n_kv, max_model_len=self.max_model_len, device=self.device,
+                                max_logits=cfg.max_step_logits,
+                                **getattr(model, "meta_kwargs", {"group": self.G}))
+        if hasattr(model, "reserve_positions"):
+            model.reserve_positions(self.max_model_len)
+        # cached pages stand for a prefix only where they are all of its state
+        self.prefix_caching = cfg.enable_prefix_caching and not self._state_shapes()
         self.free_rows = list(range(cfg.max_num_seqs - 1, -1, -1))
         self.rows_hi = 0  # high-water row + 1: the block-table rows a step's upload / broadcast moves
         # struct-of-arrays state of running rows: the decode hot path is vectorised
@@ -394,6 +402,9 @@ class Engine:
                            self.device, group=ep.handle)
 
     # ----------------------------------------------------------- sizing --
+    def _state_shapes(self):
+        return getattr(self.model, "state_shapes", ())
+
     def _auto_blocks(self) -> int:
         mc, m = self.model.cfg, self.model
         if self.cfg.kv_cache_bytes:
@@ -414,7 +425,14 @@ class Engine:
             budget = 64 * 2**20
         need = int(self.cfg.kv_fraction * self.cfg.max_num_seqs *
                    blocks_needed(min(self.cfg.max_model_len, mc.max_position))) + 2
-        nb = blocks_for_budget(budget, mc.num_layers, m.n_kv, mc.head_dim)
+        layout = getattr(m, "cache_layout", None)
+        if layout is None:
+            nb = blocks_for_budget(budget, mc.num_layers, m.n_kv, mc.head_dim)
+        else:
+            budget -= self.cfg.max_num_seqs * StateCache.bytes_per_slot(self._state_shapes())
+            esz = torch.empty(0, dtype=m.dtype).element_size()
+            per = KVCache.layout_bytes_per_block(layout, esz)
+            nb = max(2, budget // per) if per else need
         return int(min(nb, need))
 
     # -------------------------------------------------------- requests --
@@ -622,7 +640,7 @@ class Engine:
             seq = self.waiting[0]
             seq.row = self.free_rows.pop()
             self.rows_hi = max(self.rows_hi, seq.row + 1)
-            if self.cfg.enable_prefix_caching:
+            if self.prefix_caching:
                 self._match_prefix(seq)
             n = min(seq.length - seq.num_cached, budget)
             if not self._ensure_blocks(seq, seq.num_cached + n):
@@ -680,7 +698,7 @@ class Engine:
         ti = 0
         for s, c, d in zip(batch, ctx, done):
             s.num_cached = c
-            if self.cfg.enable_prefix_caching:
+            if self.prefix_caching:
                 self._register_prefix(s, c)
             if d:
                 self.prefilling.remove(s)
@@ -917,7 +935,7 @@ class Engine:
         j = 0
         for s, c, d in zip(batch, ctx, done):
             s.num_cached = c
-            if self.cfg.enable_prefix_caching:
+            if self.prefix_caching:
                 self._register_prefix(s, c)
             if d:
                 self.prefilling.remove(s)
@@ -1142,6 +1160,85 @@ class Engine:
                 self.running.remove(s)
             self._finish(s, reason)
         return StepOutput(s.seq_id, int(tok), reason is not None, reason)
+
+    # ------------------------------------------------------ given tokens --
+    def open_sequence(self) -> Sequence:
+        """A sequence whose tokens the caller gives step by step (``feed``), not sampled."""
+        seq = Sequence(next(self._ids), [], SamplingParams())
+        self.seqs[seq.seq_id] = seq
+        return seq
+
+    def close_sequence(self, seq: Sequence) -> None:
+        """Give back the row, the pages and the state slot of an ``open_sequence``."""
+        self._finish(seq, "closed")
+        self.seqs.pop(seq.seq_id, None)
+
+    def feed(self, entries) -> torch.Tensor | None:
+        """One step over given tokens.  ``entries``: (sequence, its next tokens, offsets among them
+        whose logits are wanted).  All entries run as one batch, from the pages and states earlier
+        steps left: one-token entries as decode rows (the captured graph when there is nothing
+        else), longer ones as prompt portions beside them.  Returns the wanted logits [n, V] in the
+        order of the entries and offsets, or None."""
+        self._wait_meta()
+        entries = [(s, list(toks), list(want)) for s, toks, want in entries]
+        V = self.model.cfg.vocab_size
+        for s, toks, want in entries:
+            if toks and (min(toks) < 0 or max(toks) >= V):
+                raise ValueError(f"token ids must be in [0, {V})")
+            if want and (min(want) < 0 or max(want) >= len(toks)):
+                raise ValueError("wanted offsets must lie among the entry's tokens")
+            if s.num_cached + len(toks) > self.max_model_len:
+                raise ValueError(f"sequence longer than max_model_len {self.max_model_len}")
+        live = [e for e in entries if e[1]]
+        total = sum(len(toks) for _, toks, _ in live)
+        if total > self.meta.max_tokens:
+            raise ValueError(f"step of {total} tokens exceeds max_num_batched_tokens")
+        for s, toks, _ in live:
+            if s.row < 0:  # admitted at its first tokens
+                if not self.free_rows:
+                    raise MemoryError("no free sequence row")
+                s.row = self.free_rows.pop()
+                self.rows_hi = max(self.rows_hi, s.row + 1)
+                s.status = Status.PREFILL
+            if not self._ensure_blocks(s, s.num_cached + len(toks)):
+                raise MemoryError(f"KV cache exhausted: {self.alloc.num_free} pages free")
+        if not live:
+            return None
+        singles = [e for e in live if len(e[1]) == 1]
+        portions = [e for e in live if len(e[1]) > 1]
+        B = len(singles)
+        rows = np.array([s.row for s, _, _ in singles], dtype=np.int32)
+        ctx = np.array([s.num_cached + 1 for s, _, _ in singles], dtype=np.int32)
+        last = np.array([toks[0] for _, toks, _ in singles], dtype=np.int64)
+        p_ctx = [s.num_cached + len(toks) for s, toks, _ in portions]
+        # logits rows come out one per decode row, then the portions' wanted offsets
+        at, n_wanted = {}, sum(len(w) for _, _, w in portions)
+        if B + n_wanted > self.meta.max_logits:
+            raise ValueError("more logits wanted in one step than max_step_logits")
+        for j, (s, _, _) in enumerate(singles):
+            at[s.seq_id] = j
+        o = B
+        for s, _, want in portions:
+            at[s.seq_id] = o
+            o += len(want)
+        bucket = next((b for b in self.buckets if b >= B), None)
+        if not portions and self.graphs.get(bucket) is not None:
+            self.meta.fill_decode(rows, ctx, last, pad_to=bucket)
+            logits = self._launch(KIND_GRAPH, bucket, bucket, bucket, 0, 0, bucket)
+        else:
+            T, nt, nl = self.meta.fill_mixed(rows, ctx, last, [s.row for s, _, _ in portions],
+                                             [len(toks) for _, toks, _ in portions], p_ctx,
+                                             [toks for _, toks, _ in portions], want_logits=[w for _, _, w in portions])
+            part, nparts = plan_partitions(nt, self.model.n_kv, max([*ctx.tolist(), *p_ctx]))
+            logits = self._launch(KIND_EAGER, T, nt, nl, part, nparts, 0)
+        for s, toks, _ in live:
+            s.prompt.extend(toks)
+            s.num_cached += len(toks)
+        self.stats["fed_tokens"] += total
+        idx = [at[s.seq_id] + (j if len(toks) > 1 else 0) for s, toks, want in live for j in range(len(want))]
+        if not idx:
+            return None
+        return logits[torch.tensor(idx, device=logits.device)]
 
     # --------------------------------------------------------- execution --
     def _launch(self, kind: int, T: int, nt: int, nl: int, part: int, nparts: int, bucket: int,

@@ -25,6 +25,7 @@ import collections
 import math
 import os
 import time
+from dataclasses import dataclass
 
 import numpy as np
 import torch
@@ -52,9 +53,50 @@ def _lazy_default(device) -> bool:
     return bool(torch.ops.mlop.vmm_supported(torch.cuda.current_device() if idx is None else idx))
 
 
+@dataclass(frozen=True)
+class KVLayer:
+    """Row sizes of one layer's pages, for models whose layers differ: k [NB, n_kv, 16, k_dim] and
+    v [NB, n_kv, 16, v_dim].  Sizes are whole 128-B lines (``pad_dim``)."""
+    n_kv: int
+    k_dim: int
+    v_dim: int
+
+
+def pad_dim(n: int) -> int:
+    """Head size as stored: a multiple of 64 elements (attention_hd.hip's LDS blocks)."""
+    return -(-n // 64) * 64
+
+
+class StateCache:
+    """Recurrent state of the sequences in flight: one fp32 slot per sequence row and recurrent
+    layer, ``states[i]`` [slots, *shapes[i]].  Constant in the context length.  A slot is not cleared
+    when it changes hands: a sequence's first token starts from the zero state (gla.hip)."""
+
+    def __init__(self, shapes, slots: int, device):
+        self.states = [torch.zeros(slots, *sh, dtype=torch.float32, device=device) for sh in shapes]
+
+    @staticmethod
+    def bytes_per_slot(shapes) -> int:
+        return sum(4 * math.prod(sh) for sh in shapes)
+
+    @property
+    def nbytes(self) -> int:
+        return sum(t.numel() * 4 for t in self.states)
+
+
 class KVCache:
+    """``layout`` (list of KVLayer, instead of num_layers / num_kv_heads / head_dim): layers of
+    different row sizes, eagerly backed, one tensor each.  ``state_shapes`` / ``state_slots``: the
+    recurrent layers' states beside the pages (``states``)."""
+
     def __init__(self, num_layers: int, num_blocks: int, num_kv_heads: int, head_dim: int,
-                 device, dtype=torch.bfloat16, lazy: bool | None = None, initial_blocks: int | None = None):
+                 device, dtype=torch.bfloat16, lazy: bool | None = None, initial_blocks: int | None = None,
+                 layout=None, state_shapes=(), state_slots: int = 0):
+        self.state_cache = StateCache(state_shapes, state_slots, device)
+        self.states = self.state_cache.states
+        self.layout = list(layout) if layout is not None else None
+        if self.layout is not None:
+            num_layers, lazy = len(self.layout), False
         self.num_layers, self.num_blocks = num_layers, num_blocks
         self.num_kv_heads, self.head_dim = num_kv_heads, head_dim
         self.device, self.dtype = torch.device(device), dtype
@@ -65,6 +107,14 @@ class KVCache:
         if self.lazy:
             self._init_lazy(initial_blocks)
             self.timing_ms = {"kv_malloc_ms": int(1e3 * (time.perf_counter() - t0)), "kv_zero_ms": 0}
+        elif self.layout is not None:
+            self.k = [torch.zeros(num_blocks, la.n_kv, BLOCK_SIZE, la.k_dim, device=device, dtype=dtype)
+                      for la in self.layout]
+            self.v = [torch.zeros(num_blocks, la.n_kv, BLOCK_SIZE, la.v_dim, device=device, dtype=dtype)
+                      for la in self.layout]
+            _sync(device)
+            self.timing_ms = {"kv_malloc_ms": int(1e3 * (time.perf_counter() - t0)), "kv_zero_ms": 0}
+            return
         else:
             self.k_all = torch.empty(num_layers, num_blocks, num_kv_heads, BLOCK_SIZE, head_dim,
                                      device=device, dtype=dtype)
@@ -145,11 +195,17 @@ class KVCache:
         return min(self.num_blocks, int(torch.ops.mlop.vmm_chunks_ready(self._flat)) * self.chunk_blocks)
 
     @staticmethod
+    def layout_bytes_per_block(layout, dtype_bytes=2) -> int:
+        return sum(la.n_kv * BLOCK_SIZE * (la.k_dim + la.v_dim) for la in layout) * dtype_bytes
+
+    @staticmethod
     def bytes_per_block(num_layers, num_kv_heads, head_dim, dtype_bytes=2) -> int:
         return 2 * num_layers * num_kv_heads * BLOCK_SIZE * head_dim * dtype_bytes
 
     @property
     def nbytes(self) -> int:
+        if self.layout is not None:
+            return sum(t.numel() * t.element_size() for t in (*self.k, *self.v))
         return 2 * self.num_layers * self.num_blocks * self.num_kv_heads * BLOCK_SIZE * self.head_dim * \
             self.k_all.element_size()
 
