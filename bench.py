@@ -124,6 +124,11 @@ def parse(argv=None):
     ap.add_argument("--ep-model", default="mixtral-8x7b")
     ap.add_argument("--ep-batch", type=int, default=256, help="concurrent requests PER RANK in the EP phase")
     ap.add_argument("--phase-child", choices=("tp", "ep"), default=None, help=argparse.SUPPRESS)
+    ap.add_argument("--hybrid", action="store_true",
+                    help="instead of the headline: prefill / decode throughput of the hybrid design beside a Llama "
+                         "of equal layer sizes, one JSON line each (mlopamd/runtime/bench_hybrid.py)")
+    ap.add_argument("--hybrid-kernels", action="store_true", help="with --hybrid: each workload's kernel times")
+    ap.add_argument("--hybrid-only", default="", help="with --hybrid: models whose size and name contain this")
     ap.add_argument("--cr-ready-samples", type=int, default=3,
                     help="CR -> ready measurements with the predictor as a FRESH OS process (operator -> "
                          "ProcessLauncher -> /v2/health/ready), taken before the serving run on rank 0's GPU; "
@@ -248,6 +253,11 @@ def main(argv=None):
     a = parse(argv)
     if a.http:
         return http_main(a)
+    if a.hybrid:
+        from mlopamd.runtime import bench_hybrid
+
+        bench_hybrid.main(kernels=a.hybrid_kernels, only=a.hybrid_only)
+        return
     if a.phase_child:
         return _phase_child_main(a)
     from mlopamd.parallel.comm import env_rank_info, init_distributed

@@ -7,7 +7,7 @@ linear attention) and possibly a squared-relu feed-forward, on hyper-connection 
       attention: qk_norm_rope (q / k norm, rotary, value mixing, paged stores) -> attention_hd (sink,
                  output gate)
       gla:       gla (decay, recurrence, head norm, output gate)
-  ->  O GEMM  ->  hyper_step  ->  up GEMM, relu^2  ->  down GEMM  ->  hyper_step ...
+  ->  O GEMM  ->  hyper_step  ->  up GEMM (relu^2 epilogue)  ->  down GEMM  ->  hyper_step ...
 
 ``hyper_step`` is this design's add + norm: it mixes the fp32 streams, adds the sublayer's output
 and leaves the next sublayer's normed input, in one pass.  Attention layers keep keys and values in
@@ -26,7 +26,7 @@ from ..runtime.kv_cache import KVLayer, pad_dim
 from .config import AttentionSpec, HybridConfig
 from .layers import fuse_rows, linear, rope_table
 
-GLA_CHUNK = 64  # tokens of a recurrent layer's parallel prompt chunk
+GLA_CHUNK = 64  # tokens of a recurrent layer's parallel prompt chunk (twice that in large steps)
 
 
 class _Source:
@@ -102,7 +102,7 @@ class KosesunModel:
                 L.update(up=src(p + "mlp.up", la.ff, W), down=src(p + "mlp.down", W, la.ff))
                 subs.append((self._mlp, i, self._streams(src, p + "hc2.", S), self._norm(src, p + "norm2", W)))
         self.final_norm = self._norm(src, "final.norm", W)
-        self.head = src("head", cfg.vocab_size, W)
+        self.head = fuse_rows([src("head", cfg.vocab_size, W)])  # (padding rows: the logits rows stay 16-B aligned)
         self.ones = torch.ones(S, device=self.device, dtype=f32)
         self.subs = subs
         self.n_q = self.n_kv
@@ -152,7 +152,7 @@ class KosesunModel:
 
     def _mlp(self, i, x, meta, kv, ctx):
         L = self.layers[i]
-        return linear(ops.relu2(linear(x, L["up"])), L["down"])
+        return linear(ops.gemm(x, L["up"], epi=ops.EPI_RELU2), L["down"])
 
     # ------------------------------------------------------------ forward --
     def forward(self, ids: torch.Tensor, meta, kv) -> torch.Tensor:
@@ -170,7 +170,7 @@ class KosesunModel:
 
     def logits_local(self, hidden: torch.Tensor) -> torch.Tensor:
         """[n, W] -> soft-capped logits [n, vocab] in fp32."""
-        return ops.softcap(linear(hidden, self.head), self.cfg.logit_softcap)
+        return ops.softcap(linear(hidden, self.head), self.cfg.logit_softcap)[:, :self.cfg.vocab_size]
 
     logits = logits_local
 

@@ -179,19 +179,22 @@ def paged_attention(q, k_cache, v_cache, meta, out: torch.Tensor | None = None):
     return out
 
 
-EPI_NONE, EPI_SILU_MUL = 0, 1
+EPI_NONE, EPI_SILU_MUL, EPI_RELU2 = 0, 1, 6
 
 
 def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi: int = EPI_NONE):
     """y = epi(x @ w^T), w [N, K] bf16.  EPI_SILU_MUL expects gate/up rows
-    interleaved in groups of 16 (``interleave_gate_up``) and returns N/2 columns."""
+    interleaved in groups of 16 (``interleave_gate_up``) and returns N/2 columns; EPI_RELU2 is
+    max(y, 0)^2."""
     N = w.shape[0]
-    out_n = N if epi == EPI_NONE else N // 2
+    out_n = N // 2 if epi == EPI_SILU_MUL else N
     if not x.is_cuda:
         y = torch.nn.functional.linear(x, w) if x.dtype != torch.bfloat16 else \
             torch.nn.functional.linear(x.float(), w.float()).to(x.dtype)
         if epi == EPI_SILU_MUL:
             y = ref.silu_mul(deinterleave_cols(y))
+        elif epi == EPI_RELU2:
+            y = ref.relu2(y)
         if out is not None:
             out.copy_(y.view_as(out))
             return out
@@ -203,8 +206,8 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
         x2 = x2.contiguous()
     M, K = x2.shape
     o2 = torch.empty(M, out_n, dtype=x.dtype, device=x.device) if out is None else out.view(M, out_n)
-    if x.dtype == torch.float32 and epi == EPI_NONE:  # true fp32 (library product; no reduced-precision mode)
-        torch.matmul(x2, w.t(), out=o2)
+    if x.dtype == torch.float32 and epi != EPI_SILU_MUL:  # true fp32 (library product; no reduced-precision mode)
+        _gemm_hipblaslt(x2, w, o2, epi)
         return o2.view(*lead, out_n) if out is None else out
     _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi)
     return o2.view(*lead, out_n) if out is None else out
@@ -221,8 +224,10 @@ def _gemm_mlop(x2, w, o2, epi):
 def _gemm_hipblaslt(x2, w, o2, epi):
     """Plain library GEMM (hipBLASLt via torch.matmul); the SiLU-mul epilogue
     then runs as the separate interleaved silu_mul kernel."""
-    if epi == EPI_NONE:
+    if epi != EPI_SILU_MUL:
         torch.matmul(x2, w.t(), out=o2)
+        if epi == EPI_RELU2:
+            torch.ops.mlop.relu2(o2)
     else:
         torch.ops.mlop.silu_mul(o2, torch.matmul(x2, w.t()), 1)
 
@@ -321,7 +326,7 @@ def _gemm_backend_choice(M, N, K, epi, x2, w, o2) -> str:
     """Per-shape choice between the hand-written MFMA kernel and hipBLASLt: the configured
     backend, or (``auto``) measured once per (M bucket, N, K, epilogue) on first eager use
     (never during graph capture).  ``gemm_choices()`` reports the table."""
-    if N % 8 or K % 64 or (epi != EPI_NONE and N % 32):
+    if N % 8 or K % 64 or (epi == EPI_SILU_MUL and N % 32):
         return "hipblaslt"  # shapes outside the MFMA kernel's tiling contract (e.g. tiny routers)
     if GEMM_BACKEND != "auto":
         return GEMM_BACKEND

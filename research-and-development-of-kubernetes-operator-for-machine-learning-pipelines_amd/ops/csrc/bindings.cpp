@@ -274,9 +274,9 @@ void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi) {
   TORCH_CHECK(w.dim() == 2 && w.size(1) == K, "w must be [N, K]");
   TORCH_CHECK(K % 64 == 0, "K must be a multiple of 64");
   TORCH_CHECK(N % 8 == 0 && a.stride(0) % 8 == 0 && out.stride(0) % 8 == 0, "16-B aligned rows");
-  TORCH_CHECK(epi == 0 || epi == 1, "epi");
-  TORCH_CHECK(epi == 0 || N % 32 == 0, "silu_mul epilogue needs N % 32 == 0");
-  TORCH_CHECK(out.size(0) == M && out.size(1) == (epi == 0 ? N : N / 2), "out shape");
+  TORCH_CHECK(epi == 0 || epi == 1 || epi == mlop::kEpiRelu2, "epi");
+  TORCH_CHECK(epi != 1 || N % 32 == 0, "silu_mul epilogue needs N % 32 == 0");
+  TORCH_CHECK(out.size(0) == M && out.size(1) == (epi == 1 ? N / 2 : N), "out shape");
   TORCH_CHECK(reinterpret_cast<uintptr_t>(a.data_ptr()) % 16 == 0 &&
                   reinterpret_cast<uintptr_t>(out.data_ptr()) % 16 == 0, "16-B aligned data");
   float* wsp = nullptr;
@@ -690,8 +690,13 @@ void argmax(Tensor out, Tensor logits) {
   }
   check_logits(logits);
   c10::DeviceGuard g(logits.device());
-  mlop::launch_argmax(out.data_ptr<int64_t>(), logits.data_ptr<float>(), (int)logits.size(0),
-                      (int)logits.size(1), logits.stride(0), cur_stream());
+  const int n = (int)logits.size(0), V = (int)logits.size(1);
+  const bool vec = logits.stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(logits.data_ptr()) % 16 == 0;
+  const int S = vec ? mlop::argmax_splits_f32(n, V) : 1;
+  at::Tensor ws;
+  if (S > 1) ws = at::empty({(int64_t)n * S}, logits.options().dtype(at::kLong));
+  mlop::launch_argmax(out.data_ptr<int64_t>(), logits.data_ptr<float>(), n, V, logits.stride(0),
+                      S > 1 ? ws.data_ptr() : nullptr, cur_stream());
 }
 
 void sample(Tensor out, Tensor logits, Tensor temps, Tensor top_ks, Tensor top_ps, Tensor uniform, bool full) {

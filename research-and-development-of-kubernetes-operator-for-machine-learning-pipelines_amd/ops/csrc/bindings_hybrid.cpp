@@ -279,8 +279,8 @@ void gla(Tensor out, Tensor state, Tensor proj, int64_t H, int64_t dk, int64_t d
   a.inv_tau = (float)(1.0 / tau);
   a.q_scale = (float)(1.0 / std::sqrt((double)dk));
   a.eps = (float)eps;
-  const size_t lds = (size_t)(a.rank + 3 * dk + dv + 1024) * 4;
-  TORCH_CHECK(lds <= 60 * 1024 && (size_t)8 * a.rank * 4 <= 60 * 1024, "gla: sizes past the kernels' LDS");
+  const size_t lds = (size_t)(a.rank + 3 * dk + dv + 4096) * 4;
+  TORCH_CHECK(lds <= 60 * 1024, "gla: sizes past the kernels' LDS");
   c10::DeviceGuard g(proj.device());
   mlop::launch_gla_rows(a, f32, i32_of(rows, "rows"), (int)rows.numel(), cur());
   const int n_items = (int)item_seq.numel(), n_crows = (int)crow_seq.numel();
@@ -291,12 +291,11 @@ void gla(Tensor out, Tensor state, Tensor proj, int64_t H, int64_t dk, int64_t d
     return;
   }
   const auto f = proj.options().dtype(at::kFloat);
-  Tensor logd = at::empty({T, H * dk}, f), o32 = at::empty({T, H * dv}, f);
-  Tensor cstate = at::empty({n_items, H, dk, dv}, f), cdecay = at::empty({n_items, H, dk}, f);
-  mlop::launch_gla_chunks(a, f32, logd.data_ptr<float>(), o32.data_ptr<float>(), cstate.data_ptr<float>(),
-                          cdecay.data_ptr<float>(), (int)T, i32_of(item_seq, "item_seq"), i32_of(item_t0, "item_t0"),
-                          n_items, i32_of(crow_seq, "crow_seq"), i32_of(crow_item0, "crow_item0"), n_crows, (int)chunk,
-                          cur());
+  Tensor cstate = at::empty({n_items, H, dk, dv}, f), cdecay = at::empty({n_items, H, dk}, f), o32;
+  if (mlop::gla_chunks_need_o32((int)dv)) o32 = at::empty({T, H * dv}, f);
+  mlop::launch_gla_chunks(a, f32, o32.defined() ? o32.data_ptr<float>() : nullptr, cstate.data_ptr<float>(),
+                          cdecay.data_ptr<float>(), i32_of(item_seq, "item_seq"), i32_of(item_t0, "item_t0"), n_items,
+                          i32_of(crow_seq, "crow_seq"), i32_of(crow_item0, "crow_item0"), n_crows, (int)chunk, cur());
 }
 
 }  // namespace

@@ -125,6 +125,11 @@ __device__ __forceinline__ float silu_bf(float g) {
   return bf2f(f2bf(gb * __builtin_amdgcn_rcpf(1.f + __expf(-gb))));
 }
 
+__device__ __forceinline__ float relu2_f(float x) {
+  const float r = fmaxf(x, 0.f);
+  return r * r;
+}
+
 __host__ __device__ constexpr int cdiv(int a, int b) { return (a + b - 1) / b; }
 
 }  // namespace mlop

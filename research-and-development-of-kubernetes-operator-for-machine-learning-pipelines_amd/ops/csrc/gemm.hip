@@ -27,7 +27,7 @@
 // (launch-boundary reduce, §5 "Projection GEMM at M = 256" item 2).
 //
 // Epilogues (fp32 LDS copy of the tile, 16-B coalesced stores):
-//   EPI_NONE      C = bf16(acc)
+//   EPI_NONE      C = bf16(acc), or bf16(max(acc, 0)^2) (RopeEpi::relu2)
 //   EPI_SILU_MUL  B rows gate/up interleaved in groups of 16, C[:, j] = silu(g_j) * u_j (N/2 cols)
 //   EPI_ROPE      QKV projection: RoPE on q/k heads + q_out / paged K,V cache stores from the
 //                 staged tile (RopeEpi, launch.h); needs whole 128-wide heads per staged chunk
@@ -375,7 +375,8 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
         const float* s = sC + r * LDC + c;
         u32x4 o;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) o[j] = pack2(s[2 * j], s[2 * j + 1]);
+        for (int j = 0; j < 4; ++j)
+          o[j] = re.relu2 ? pack2(relu2_f(s[2 * j]), relu2_f(s[2 * j + 1])) : pack2(s[2 * j], s[2 * j + 1]);
         *reinterpret_cast<u32x4*>(C + (size_t)(m0 + r) * ldc + n0 + c0 + c) = o;
       }
     } else {
@@ -405,7 +406,7 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
 template <int EPI>
 __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict__ C, int ldc,
                                                            const float* __restrict__ ws, int M,
-                                                           int N, int splits) {
+                                                           int N, int splits, int relu2 = 0) {
   const int outw = EPI == EPI_NONE ? N : N / 2;
   const int vpr = outw / 8;
   const long total = (long)M * vpr;
@@ -430,7 +431,7 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if (EPI == EPI_NONE)
-        o[j] = pack2(a[2 * j], a[2 * j + 1]);
+        o[j] = relu2 ? pack2(relu2_f(a[2 * j]), relu2_f(a[2 * j + 1])) : pack2(a[2 * j], a[2 * j + 1]);
       else
         o[j] = pack2(silu_bf(a[2 * j]) * bf2f(f2bf(b[2 * j])),
                      silu_bf(a[2 * j + 1]) * bf2f(f2bf(b[2 * j + 1])));
@@ -1105,7 +1106,8 @@ __global__ void __launch_bounds__(512, 1) gemm_pp_kernel(
         const int row = i * 16 + 4 * (lane >> 4) + r;
         if constexpr (EPI == EPI_NONE) {
 #pragma unroll
-          for (int j = 0; j < 4; ++j) sC[row * LD + j * 16 + (lane & 15)] = f2bf(acc[i][j][r]);
+          for (int j = 0; j < 4; ++j)
+            sC[row * LD + j * 16 + (lane & 15)] = f2bf(re.relu2 ? relu2_f(acc[i][j][r]) : acc[i][j][r]);
         } else {
 #pragma unroll
           for (int jp = 0; jp < 2; ++jp) {
@@ -1711,6 +1713,7 @@ bool launch_mid_rs(const void* A, int lda, const void* B, void* out, int ldo, in
 }
 
 long gemm_workspace_floats(int M, int N, int K, int epi) {
+  if (epi == kEpiRelu2) epi = EPI_NONE;
   if (gemv_takes(M, N, K, epi)) return 0;
   const Plan p = plan(M, N, K, false, 0, 0);
   return p.splits > 1 ? (long)p.splits * M * N : 0;
@@ -1719,15 +1722,18 @@ long gemm_workspace_floats(int M, int N, int K, int epi) {
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
                  long ws_floats, int M, int N, int K, int epi, hipStream_t st) {
   if (M == 0) return;
+  RopeEpi re{};
+  re.relu2 = epi == kEpiRelu2;
+  if (re.relu2) epi = EPI_NONE;
   if (gemv_takes(M, N, K, epi) && lda % 8 == 0 && ldb % 8 == 0) {
-    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, epi, st);
+    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, re.relu2 ? kEpiRelu2 : epi, st);
     return;
   }
   Plan p = plan(M, N, K, false, 0, 0);
   if (p.splits > 1 && (long)p.splits * M * N > ws_floats) { p.splits = 1; p.k_chunk = K; }
   if (epi == EPI_NONE)
     launch_plan<EPI_NONE, false>(p, (const uint16_t*)A, lda, (const uint16_t*)B, ldb, (uint16_t*)C,
-                                 ldc, ws, M, N, K, nullptr, 0, st);
+                                 ldc, ws, M, N, K, nullptr, 0, st, re);
   else
     launch_plan<EPI_SILU_MUL, false>(p, (const uint16_t*)A, lda, (const uint16_t*)B, ldb,
                                      (uint16_t*)C, ldc, ws, M, N, K, nullptr, 0, st);
@@ -1736,7 +1742,7 @@ void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ld
     const long total = (long)M * (outw / 8);
     const int g = (int)std::min<long>((total + 255) / 256, 4096);
     if (epi == EPI_NONE)
-      splitk_reduce_kernel<EPI_NONE><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits);
+      splitk_reduce_kernel<EPI_NONE><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, re.relu2);
     else
       splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits);
   }

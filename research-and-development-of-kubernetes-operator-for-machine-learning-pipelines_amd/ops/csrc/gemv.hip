@@ -300,7 +300,8 @@ __global__ void __launch_bounds__(256) gemv_kernel(const uint16_t* __restrict__ 
     for (int m = 0; m < M; ++m)
 #pragma unroll
       for (int r = 0; r < R; ++r)
-        if (lane == m * R + r && m < mc) C[(size_t)m * ldc + set * R + r] = f2bf(acc[r][m]);
+        if (lane == m * R + r && m < mc)
+          C[(size_t)m * ldc + set * R + r] = f2bf(re.relu2 ? relu2_f(acc[r][m]) : acc[r][m]);
   }
 }
 
@@ -379,7 +380,8 @@ void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ld
   auto* a = (const uint16_t*)A;
   auto* b = (const uint16_t*)B;
   auto* c = (uint16_t*)C;
-  const RopeEpi none{};
+  RopeEpi none{};
+  none.relu2 = epi == kEpiRelu2;
   if (epi == EPI_SILU_MUL) run_gemv<EPI_SILU_MUL>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
   else run_gemv<EPI_NONE>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
 }

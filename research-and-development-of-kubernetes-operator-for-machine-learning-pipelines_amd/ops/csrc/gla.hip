@@ -50,8 +50,8 @@ __device__ __forceinline__ float decay_logit(const GlaArgs& a, int n, const floa
 
 // Workgroup = (row, head).  Threads own VEC-column strips: strip s = tid % strips, key rows
 // rg, rg + RG, ... with rg = tid / strips.
-template <typename E, int VEC>
-__global__ void __launch_bounds__(256) gla_rows_kernel(GlaArgs a, const int* __restrict__ rows) {
+template <typename E, int VEC, int BT>
+__global__ void __launch_bounds__(BT) gla_rows_kernel(GlaArgs a, const int* __restrict__ rows) {
   extern __shared__ float sm[];
   __shared__ float scratch[16];
   const int s = rows[blockIdx.x], h = blockIdx.y, tid = threadIdx.x;
@@ -61,23 +61,23 @@ __global__ void __launch_bounds__(256) gla_rows_kernel(GlaArgs a, const int* __r
   float* q = dec + dk;             // [dk]
   float* k = q + dk;               // [dk]
   float* o = k + dk;               // [dv]
-  float* red = o + dv;             // [256 * VEC]
+  float* red = o + dv;             // [BT * VEC]
   const int ql = a.q_len[s], ctx = a.ctx_len[s], qs = a.q_start[s];
   E* outp = reinterpret_cast<E*>(a.out);
   if (ctx < ql || s >= a.n_slots) {  // graph padding: attends to nothing, holds no state
     for (int t = 0; t < ql; ++t)
-      for (int c = tid; c < dv; c += 256) st1(outp + ((size_t)(qs + t) * a.H + h) * dv + c, 0.f);
+      for (int c = tid; c < dv; c += BT) st1(outp + ((size_t)(qs + t) * a.H + h) * dv + c, 0.f);
     return;
   }
   float* S = a.state + ((size_t)s * a.H + h) * dk * dv;
-  const int nstrip = dv / VEC, per = min(nstrip, 256), RG = 256 / per;
+  const int nstrip = dv / VEC, per = min(nstrip, BT), RG = BT / per;
   const int HK = a.H * dk, HV = a.H * dv;
   for (int t = 0; t < ql; ++t) {
     const E* row = reinterpret_cast<const E*>(a.proj) + (size_t)(qs + t) * a.ldp;
     const bool fresh = ctx - ql + t == 0;
-    for (int i = tid; i < a.rank; i += 256) a1[i] = ld1(row + 2 * HK + 2 * HV + i);
+    for (int i = tid; i < a.rank; i += BT) a1[i] = ld1(row + 2 * HK + 2 * HV + i);
     __syncthreads();
-    for (int d = tid; d < dk; d += 256) {
+    for (int d = tid; d < dk; d += BT) {
       dec[d] = expf(log_sigmoid(decay_logit<E>(a, h * dk + d, a1)) * a.inv_tau);
       q[d] = ld1(row + h * dk + d) * a.q_scale;
       k[d] = ld1(row + HK + h * dk + d);
@@ -94,7 +94,7 @@ __global__ void __launch_bounds__(256) gla_rows_kernel(GlaArgs a, const int* __r
 #pragma unroll
         for (int e = 0; e < VEC; ++e) v[e] = ld1(vp + e);
         float* col = S + strip * VEC;
-#pragma unroll 8
+#pragma unroll BT >= 1024 ? 4 : 8
         for (int d = rg; d < dk; d += RG) {
           float x[VEC];
           if (fresh) {
@@ -115,7 +115,7 @@ __global__ void __launch_bounds__(256) gla_rows_kernel(GlaArgs a, const int* __r
 #pragma unroll
       for (int e = 0; e < VEC; ++e) red[tid * VEC + e] = acc[e];
       __syncthreads();
-      for (int c = tid; c < per * VEC; c += 256) {
+      for (int c = tid; c < per * VEC; c += BT) {
         if (s0 * VEC + c < dv) {
           float x = 0.f;
           for (int g = 0; g < RG; ++g) x += red[g * per * VEC + c];
@@ -125,165 +125,222 @@ __global__ void __launch_bounds__(256) gla_rows_kernel(GlaArgs a, const int* __r
       __syncthreads();
     }
     float ss = 0.f;
-    for (int c = tid; c < dv; c += 256) ss = fmaf(o[c], o[c], ss);
+    for (int c = tid; c < dv; c += BT) ss = fmaf(o[c], o[c], ss);
     ss = block_sum(ss, scratch);
     const float inv = 1.f / sqrtf(ss / (float)dv + a.eps);
     const E* gp = row + 2 * HK + HV + h * dv;
-    for (int c = tid; c < dv; c += 256)
+    for (int c = tid; c < dv; c += BT)
       st1(outp + ((size_t)(qs + t) * a.H + h) * dv + c, o[c] * inv * a.norm_w[c] * silu_f(ld1(gp + c)));
   }
 }
 
-// logd[t, n] = log_sigmoid(z) / tau for 8 tokens per workgroup (A2 rows reused over them)
-template <typename E>
-__global__ void __launch_bounds__(256) gla_decay_kernel(GlaArgs a, float* __restrict__ logd, int T) {
-  extern __shared__ float sm[];  // [8][rank]
-  const int t0 = blockIdx.x * 8, n = min(8, T - t0), HK = a.H * a.dk, off = 2 * HK + 2 * a.H * a.dv;
-  for (int i = threadIdx.x; i < n * a.rank; i += 256)
-    sm[i] = ld1(reinterpret_cast<const E*>(a.proj) + (size_t)(t0 + i / a.rank) * a.ldp + off + i % a.rank);
-  __syncthreads();
-  for (int c = blockIdx.y * 256 + threadIdx.x; c < HK; c += gridDim.y * 256) {
-    const E* w = reinterpret_cast<const E*>(a.a2) + (size_t)c * a.rank;
-    const float b = a.a2_b[c];
-    float z[8];
-#pragma unroll
-    for (int j = 0; j < 8; ++j) z[j] = b;
-    for (int i = 0; i < a.rank; ++i) {
-      const float wi = ld1(w + i);
-#pragma unroll
-      for (int j = 0; j < 8; ++j)
-        if (j < n) z[j] = fmaf(wi, sm[j * a.rank + i], z[j]);
-    }
-#pragma unroll
-    for (int j = 0; j < 8; ++j)
-      if (j < n) logd[(size_t)(t0 + j) * HK + c] = log_sigmoid(z[j]) * a.inv_tau;
-  }
+// One chunk of one head for a group of 128 NCT value columns; 8 waves.
+//   OUT = false: the chunk's own contribution from a zero state -> cstate, total decay -> cdecay
+//   OUT = true:  outputs from the chunk's starting state in cstate: normed and gated straight to `out`
+//                when the group holds the whole head (dv <= 128 NCT), else raw to o32
+// Elementwise part: a wave takes 16 key channels at a time, lane = (channel l & 15, tokens
+// 4 (l >> 4) .. + 3) -- the accumulator layout of z = a1 A2^T, which the MFMA computes in place.  The
+// decays live in the log2 domain.  Products: wave w owns 16 NCT value columns, the state
+// [16 NKT, 16 NCT] in its accumulators.
+constexpr int kGlaWaves = 8;
+
+__device__ __forceinline__ float exp2_g(float x) { return __builtin_amdgcn_exp2f(x); }
+// log2(sigmoid(z)): log1p by the quotient form, exact where 1 + e rounds
+__device__ __forceinline__ float log2_sigmoid(float z) {
+  const float e = exp2_g(-fabsf(z) * 1.44269504f), u = 1.f + e, d = u - 1.f;
+  const float l = d == 0.f ? e * 1.44269504f : __builtin_amdgcn_logf(u) * (e / d);
+  return fminf(z, 0.f) * 1.44269504f - l;
 }
 
-// One chunk of one head for a group of 16 NW value columns.  Thread d < dk owns key channel d in the
-// elementwise part (its running decay over the block's 16 tokens); wave w owns 16 value columns in
-// the products, the state [16 NKT, 16] in its accumulators.
-//   OUT = false: the chunk's own contribution from a zero state -> cstate, total decay -> cdecay
-//   OUT = true:  outputs from the chunk's starting state in cstate
-template <typename E, int NKT, bool OUT>
-__global__ void __launch_bounds__(512) gla_chunk_kernel(GlaArgs a, float* __restrict__ o32,
-                                                        float* __restrict__ cstate, float* __restrict__ cdecay,
-                                                        const float* __restrict__ logd,
-                                                        const int* __restrict__ item_seq,
-                                                        const int* __restrict__ item_t0, int chunk) {
-  constexpr int DKP = 16 * NKT, LD = DKP + 4, LT = 20;
+// waves per SIMD the chunk kernel is built for: 4 = two workgroups per CU (128 VGPRs), 2 = one
+constexpr int chunk_waves(int nkt, int nct, bool out) {
+  return (out ? nct == 1 && nkt <= 8 : nkt * nct <= 16 && nkt <= 12) ? 4 : 2;
+}
+
+template <typename E, int NKT, int NCT, bool OUT>
+__global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gla_chunk_kernel(
+    GlaArgs a, float* __restrict__ o32, float* __restrict__ cstate, float* __restrict__ cdecay,
+    const int* __restrict__ item_seq, const int* __restrict__ item_t0, int chunk) {
+  constexpr int NW = kGlaWaves, DKP = 16 * NKT, LD = DKP + 4, LT = 20, NP = (NKT + NW - 1) / NW;
+  constexpr float kFast2 = kFastDecay * 1.44269504f;
+  // operands fetched one block ahead where the registers allow it at two workgroups per CU
+  constexpr bool AHEAD = chunk_waves(NKT, NCT, OUT) == 2 || NKT * NCT <= (OUT ? 6 : 12);
   extern __shared__ __attribute__((aligned(16))) float sm[];
   float* KT = sm;                     // [DKP][LT]: k_j e^{b_16 - b_j}, token fastest
   float* En = KT + DKP * LT;          // [DKP]: e^{b_16}
-  float* Qs = En + DKP;               // [16][LD]: q e^b
+  float* Qs = En + DKP;               // [16][LD]: q e^b            (OUT only from here on)
   float* Ks = Qs + 16 * LD;           // [16][LD]: k e^-b
   float* part = Ks + 16 * LD;         // [NW][256]
-  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, NW = blockDim.x >> 6;
+  float* red = part + NW * 256;       // [NW][16]
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int item = blockIdx.x, h = blockIdx.y;
   const int s = item_seq[item], t0 = item_t0[item];
   const int n = min(chunk, a.q_len[s] - t0), tok0 = a.q_start[s] + t0;
-  const int dk = a.dk, dv = a.dv, HK = a.H * dk, HV = a.H * dv;
+  const int dk = a.dk, dv = a.dv, HK = a.H * dk, HV = a.H * dv, rank = a.rank;
   const int l15 = lane & 15, g4 = lane >> 4;
-  const int col = (blockIdx.z * NW + wid) * 16 + l15;
-  const bool wave_cols = (blockIdx.z * NW + wid) * 16 < dv, col_ok = col < dv;
-  const bool own = tid < DKP, own_ok = tid < dk;
+  const int col0 = ((int)blockIdx.z * NW + wid) * 16 * NCT;  // first column of this wave
+  const bool wave_cols = col0 < dv;
+  const bool fused = OUT && gridDim.z == 1;
   const E* proj = reinterpret_cast<const E*>(a.proj) + (size_t)tok0 * a.ldp;
+  const E* pq = proj + h * dk;
+  const E* pk = proj + HK + h * dk;
+  const E* pv = proj + 2 * HK + h * dv;
+  const E* pg = proj + 2 * HK + HV + h * dv;
+  const E* pa = proj + 2 * HK + 2 * HV;
   float* cst = cstate + ((size_t)item * a.H + h) * dk * dv;
 
-  f32x4 S[NKT];
+  f32x4 S[NKT][NCT];
 #pragma unroll
-  for (int kt = 0; kt < NKT; ++kt) {
-    S[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (OUT && col_ok) {
+  for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = 16 * kt + 4 * g4 + i;
-        if (d < dk) S[kt][i] = cst[(size_t)d * dv + col];
+    for (int c = 0; c < NCT; ++c) {
+      S[kt][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+      const int col = col0 + 16 * c + l15;
+      if (OUT && col < dv) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int d = 16 * kt + 4 * g4 + i;
+          if (d < dk) S[kt][c][i] = cst[(size_t)d * dv + col];
+        }
       }
     }
-  }
-  float total = 0.f;
+  float total[NP];
+#pragma unroll
+  for (int p = 0; p < NP; ++p) total[p] = 0.f;
+
+  float kk[NP][4], qq[NP][4], vv[NCT][4], x1[4];
+  auto fetch = [&](int t) {
+    const int nt = n - t;
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      const int d = (p * NW + wid) * 16 + l15;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const bool ok = d < dk && 4 * g4 + i < nt;
+        const size_t o = (size_t)(t + 4 * g4 + i) * a.ldp + d;
+        kk[p][i] = ok ? ld1(pk + o) : 0.f;
+        if (OUT) qq[p][i] = ok ? ld1(pq + o) * a.q_scale : 0.f;
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < NCT; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int col = col0 + 16 * c + l15;
+        const bool ok = col < dv && 4 * g4 + i < nt;
+        const size_t o = (size_t)(t + 4 * g4 + i) * a.ldp + col;
+        vv[c][i] = ok ? ld1(pv + o) : 0.f;
+      }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) x1[i] = (l15 < nt && 4 * g4 + i < rank) ? ld1(pa + (size_t)(t + l15) * a.ldp + 4 * g4 + i) : 0.f;
+  };
+  if (AHEAD) fetch(0);
   for (int t = 0; t < n; t += 16) {
     const int nt = min(16, n - t);
-    float b[16], kk[16], qq[16];
+    if (!AHEAD) fetch(t);
+    // log2 decays of this wave's channels, running sums over the block's tokens
+    float b[NP][4], bn[NP];
+    bool slow = false;
 #pragma unroll
-    for (int j = 0; j < 16; ++j) {
-      const bool ok = own_ok && j < nt;
-      b[j] = ok ? logd[(size_t)(tok0 + t + j) * HK + h * dk + tid] : 0.f;
-      kk[j] = ok ? ld1(proj + (size_t)(t + j) * a.ldp + HK + h * dk + tid) : 0.f;
-      if (OUT) qq[j] = ok ? ld1(proj + (size_t)(t + j) * a.ldp + h * dk + tid) * a.q_scale : 0.f;
+    for (int p = 0; p < NP; ++p) {
+      const int d = (p * NW + wid) * 16 + l15;
+      const bool ok = d < dk;
+      const int nrow = h * dk + (ok ? d : 0);
+      const float bias = a.a2_b[nrow];
+      f32x4 z = {bias, bias, bias, bias};
+      const E* w = reinterpret_cast<const E*>(a.a2) + (size_t)nrow * rank;
+      for (int r0 = 0; r0 < rank; r0 += 16) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int r = r0 + 4 * g4 + i;
+          float x = x1[i];
+          if (r0) x = (l15 < nt && r < rank) ? ld1(pa + (size_t)(t + l15) * a.ldp + r) : 0.f;
+          z = mfma4(x, r < rank ? ld1(w + r) : 0.f, z);
+        }
+      }
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        if (ok && 4 * g4 + i < nt) sum += log2_sigmoid(z[i]) * a.inv_tau;
+        b[p][i] = sum;
+      }
+      float before = 0.f, all = 0.f;
+#pragma unroll
+      for (int g = 0; g < 4; ++g) {
+        const float x = __shfl(sum, l15 + 16 * g);
+        if (g < g4) before += x;
+        all += x;
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) b[p][i] += before;
+      bn[p] = all;
+      total[p] += all;
+      slow |= all < kFast2;
     }
-    float vv[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int j = 4 * g4 + i;
-      vv[i] = (col_ok && j < nt) ? ld1(proj + (size_t)(t + j) * a.ldp + 2 * HK + h * dv + col) : 0.f;
-    }
-#pragma unroll
-    for (int j = 1; j < 16; ++j) b[j] += b[j - 1];
-    const float bn = b[15];
-    total += bn;
     bool fast = true;
-    if (OUT) fast = !__syncthreads_or(own && bn < kFastDecay);  // also: the last block's LDS reads are done
+    if (OUT) fast = !__syncthreads_or(slow);  // also: the last block's LDS reads are done
     else __syncthreads();
     auto put_kt = [&]() {
 #pragma unroll
-      for (int j = 0; j < 16; j += 4)
-        *reinterpret_cast<f32x4*>(KT + tid * LT + j) =
-            f32x4{kk[j] * expf(bn - b[j]), kk[j + 1] * expf(bn - b[j + 1]), kk[j + 2] * expf(bn - b[j + 2]),
-                  kk[j + 3] * expf(bn - b[j + 3])};
+      for (int p = 0; p < NP; ++p) {
+        const int d = (p * NW + wid) * 16 + l15;
+        if (d < DKP)
+          *reinterpret_cast<f32x4*>(KT + d * LT + 4 * g4) =
+              f32x4{kk[p][0] * exp2_g(bn[p] - b[p][0]), kk[p][1] * exp2_g(bn[p] - b[p][1]),
+                    kk[p][2] * exp2_g(bn[p] - b[p][2]), kk[p][3] * exp2_g(bn[p] - b[p][3])};
+      }
     };
-    if (own) {
-      En[tid] = expf(bn);
-      if (OUT) {
-        if (fast) {
 #pragma unroll
-          for (int j = 0; j < 16; ++j) {
-            const float e = expf(b[j]);
-            Qs[j * LD + tid] = qq[j] * e;
-            Ks[j * LD + tid] = kk[j] / e;
-          }
-        } else {
+    for (int p = 0; p < NP; ++p) {
+      const int d = (p * NW + wid) * 16 + l15;
+      if (d < DKP) {
+        if (g4 == 0) En[d] = exp2_g(bn[p]);
+        if (OUT) {
 #pragma unroll
-          for (int j = 0; j < 16; ++j) {
-            Qs[j * LD + tid] = qq[j];
-            Ks[j * LD + tid] = kk[j];
-            KT[j * LD + tid] = b[j];  // (DKP * LT >= 16 * LD)
+          for (int i = 0; i < 4; ++i) {
+            const int j = 4 * g4 + i;
+            Qs[j * LD + d] = fast ? qq[p][i] * exp2_g(b[p][i]) : qq[p][i];
+            Ks[j * LD + d] = fast ? kk[p][i] * exp2_g(-b[p][i]) : kk[p][i];
+            if (!fast) KT[j * LD + d] = b[p][i];  // (DKP * LT >= 16 * LD)
           }
         }
       }
-      if (!OUT || fast) put_kt();
     }
+    if (!OUT || fast) put_kt();
     __syncthreads();
     f32x4 A = {0.f, 0.f, 0.f, 0.f};  // scores^T: row j = 4 g4 + i, column = token l15
     if (OUT) {
-      int nsum = NW;
+      int nsum = min(NW, NKT);
       if (fast) {
-        f32x4 p = {0.f, 0.f, 0.f, 0.f};
+        f32x4 sc = {0.f, 0.f, 0.f, 0.f};
         for (int kt = wid; kt < NKT; kt += NW) {
           const f32x4 x = *reinterpret_cast<const f32x4*>(Ks + l15 * LD + 16 * kt + 4 * g4);
           const f32x4 y = *reinterpret_cast<const f32x4*>(Qs + l15 * LD + 16 * kt + 4 * g4);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) p = mfma4(x[i], y[i], p);
+          for (int i = 0; i < 4; ++i) sc = mfma4(x[i], y[i], sc);
         }
+        if (wid < NKT) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) part[wid * 256 + (4 * g4 + i) * 16 + l15] = p[i];
+          for (int i = 0; i < 4; ++i) part[wid * 256 + (4 * g4 + i) * 16 + l15] = sc[i];
+        }
       } else {
-        nsum = 1;
-        if (tid < 256) {
-          const int j = tid >> 4, tt = tid & 15;
-          float x = 0.f;
-          if (j <= tt)
-            for (int d = 0; d < dk; ++d)
-              x = fmaf(Qs[tt * LD + d] * Ks[j * LD + d], expf(KT[tt * LD + d] - KT[j * LD + d]), x);
-          part[tid] = x;
-        }
+        nsum = 2;
+        const int half = tid >> 8, j = (tid >> 4) & 15, tt = tid & 15;
+        float x = 0.f;
+        if (j <= tt)
+          for (int d = half; d < dk; d += 2)
+            x = fmaf(Qs[tt * LD + d] * Ks[j * LD + d], exp2_g(KT[tt * LD + d] - KT[j * LD + d]), x);
+        part[tid] = x;
         __syncthreads();
-        if (own) {
 #pragma unroll
-          for (int j = 0; j < 16; ++j) Qs[j * LD + tid] = qq[j] * expf(b[j]);
-          put_kt();
+        for (int p = 0; p < NP; ++p) {
+          const int d = (p * NW + wid) * 16 + l15;
+          if (d < DKP) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) Qs[(4 * g4 + i) * LD + d] = qq[p][i] * exp2_g(b[p][i]);
+          }
         }
+        put_kt();
       }
       __syncthreads();
       for (int w = 0; w < nsum; ++w)
@@ -293,46 +350,108 @@ __global__ void __launch_bounds__(512) gla_chunk_kernel(GlaArgs a, float* __rest
       for (int i = 0; i < 4; ++i)
         if (4 * g4 + i > l15) A[i] = 0.f;
     }
-    if (wave_cols) {
-      if (OUT) {
-        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    float cv[NCT][4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o = mfma4(A[i], vv[i], o);
+    for (int c = 0; c < NCT; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) cv[c][i] = vv[c][i];
+    if (AHEAD && t + 16 < n) fetch(t + 16);  // under the products
+    f32x4 o[NCT];
+    if (OUT) {
+#pragma unroll
+      for (int c = 0; c < NCT; ++c) {
+        o[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[c] = mfma4(A[i], cv[c][i], o[c]);
+      }
+      if (wave_cols) {
 #pragma unroll
         for (int kt = 0; kt < NKT; ++kt) {
           const f32x4 y = *reinterpret_cast<const f32x4*>(Qs + l15 * LD + 16 * kt + 4 * g4);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) o = mfma4(y[i], S[kt][i], o);
-        }
-        if (col_ok) {
+          for (int c = 0; c < NCT; ++c)
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (4 * g4 + i < nt) o32[(size_t)(tok0 + t + 4 * g4 + i) * HV + h * dv + col] = o[i];
+            for (int i = 0; i < 4; ++i) o[c] = mfma4(y[i], S[kt][c][i], o[c]);
         }
       }
-      if (!OUT || t + 16 < n) {
+    }
+    if (wave_cols && (!OUT || t + 16 < n)) {
 #pragma unroll
-        for (int kt = 0; kt < NKT; ++kt) {
-          const f32x4 e = *reinterpret_cast<const f32x4*>(En + 16 * kt + 4 * g4);
-          const f32x4 x = *reinterpret_cast<const f32x4*>(KT + (16 * kt + l15) * LT + 4 * g4);
-          S[kt] *= e;
+      for (int kt = 0; kt < NKT; ++kt) {
+        const f32x4 e = *reinterpret_cast<const f32x4*>(En + 16 * kt + 4 * g4);
+        const f32x4 x = *reinterpret_cast<const f32x4*>(KT + (16 * kt + l15) * LT + 4 * g4);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) S[kt] = mfma4(x[i], vv[i], S[kt]);
+        for (int c = 0; c < NCT; ++c) {
+          S[kt][c] *= e;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) S[kt][c] = mfma4(x[i], cv[c][i], S[kt][c]);
         }
       }
+    }
+    if (fused) {  // o row 4 g4 + i = token, over the head's columns: rms, weight, gate
+      float gg[NCT][4];
+#pragma unroll
+      for (int c = 0; c < NCT; ++c)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int col = col0 + 16 * c + l15;
+          gg[c][i] = (col < dv && 4 * g4 + i < nt) ? ld1(pg + (size_t)(t + 4 * g4 + i) * a.ldp + col) : 0.f;
+        }
+      float ss[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        ss[i] = 0.f;
+#pragma unroll
+        for (int c = 0; c < NCT; ++c) ss[i] = fmaf(o[c][i], o[c][i], ss[i]);  // columns past dv are zero
+        ss[i] += detail::dpp<0xB1>(ss[i]);
+        ss[i] += detail::dpp<0x4E>(ss[i]);
+        ss[i] += detail::dpp<0x141>(ss[i]);
+        ss[i] += detail::dpp<0x140>(ss[i]);
+      }
+      if (l15 == 0) *reinterpret_cast<f32x4*>(red + wid * 16 + 4 * g4) = f32x4{ss[0], ss[1], ss[2], ss[3]};
+      __syncthreads();
+      f32x4 tot = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int w = 0; w < NW; ++w) tot += *reinterpret_cast<const f32x4*>(red + w * 16 + 4 * g4);
+      E* op = reinterpret_cast<E*>(a.out) + (size_t)(tok0 + t) * HV + h * dv;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int j = 4 * g4 + i;
+        const float inv = 1.f / sqrtf(tot[i] / (float)dv + a.eps);
+#pragma unroll
+        for (int c = 0; c < NCT; ++c) {
+          const int col = col0 + 16 * c + l15;
+          if (col < dv && j < nt) {
+            const float g = gg[c][i];
+            st1(op + (size_t)j * HV + col, o[c][i] * inv * a.norm_w[col] * (g / (1.f + exp2_g(-g * 1.44269504f))));
+          }
+        }
+      }
+    } else if (OUT) {
+#pragma unroll
+      for (int c = 0; c < NCT; ++c)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int j = 4 * g4 + i, col = col0 + 16 * c + l15;
+          if (col < dv && j < nt) o32[(size_t)(tok0 + t + j) * HV + h * dv + col] = o[c][i];
+        }
     }
   }
   if (!OUT) {
-    if (col_ok) {
 #pragma unroll
-      for (int kt = 0; kt < NKT; ++kt)
+    for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+      for (int c = 0; c < NCT; ++c)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const int d = 16 * kt + 4 * g4 + i;
-          if (d < dk) cst[(size_t)d * dv + col] = S[kt][i];
+          const int d = 16 * kt + 4 * g4 + i, col = col0 + 16 * c + l15;
+          if (d < dk && col < dv) cst[(size_t)d * dv + col] = S[kt][c][i];
         }
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      const int d = (p * NW + wid) * 16 + l15;
+      if (d < dk && g4 == 0 && blockIdx.z == 0) cdecay[((size_t)item * a.H + h) * dk + d] = exp2_g(total[p]);
     }
-    if (own_ok && blockIdx.z == 0) cdecay[((size_t)item * a.H + h) * dk + tid] = expf(total);
   }
 }
 
@@ -379,12 +498,19 @@ __global__ void __launch_bounds__(256) gla_gate_kernel(GlaArgs a, const float* _
   for (int c = lane; c < a.dv; c += 64) st1(out + c, o[c] * inv * a.norm_w[c] * silu_f(ld1(g + c)));
 }
 
+template <typename E, int BT>
+static void run_rows_t(const GlaArgs& a, const int* rows, int n_rows, hipStream_t st) {
+  const bool v4 = a.dv % 4 == 0;
+  const size_t lds = (size_t)(a.rank + 3 * a.dk + a.dv + BT * (v4 ? 4 : 1)) * 4;
+  if (v4) gla_rows_kernel<E, 4, BT><<<dim3(n_rows, a.H), BT, lds, st>>>(a, rows);
+  else gla_rows_kernel<E, 1, BT><<<dim3(n_rows, a.H), BT, lds, st>>>(a, rows);
+}
+
 template <typename E>
 static void run_rows(const GlaArgs& a, const int* rows, int n_rows, hipStream_t st) {
-  const bool v4 = a.dv % 4 == 0;
-  const size_t lds = (size_t)(a.rank + 3 * a.dk + a.dv + 256 * (v4 ? 4 : 1)) * 4;
-  if (v4) gla_rows_kernel<E, 4><<<dim3(n_rows, a.H), 256, lds, st>>>(a, rows);
-  else gla_rows_kernel<E, 1><<<dim3(n_rows, a.H), 256, lds, st>>>(a, rows);
+  // few (row, head) pairs: a whole CU's threads on each, so that its state is in flight at once
+  if (n_rows * a.H <= 512 && (long)a.dk * a.dv >= 8192) run_rows_t<E, 1024>(a, rows, n_rows, st);
+  else run_rows_t<E, 256>(a, rows, n_rows, st);
 }
 
 void launch_gla_rows(const GlaArgs& a, bool f32, const int* rows, int n_rows, hipStream_t st) {
@@ -393,40 +519,45 @@ void launch_gla_rows(const GlaArgs& a, bool f32, const int* rows, int n_rows, hi
   else run_rows<uint16_t>(a, rows, n_rows, st);
 }
 
-template <typename E, int NKT>
-static void run_chunks(const GlaArgs& a, float* logd, float* o32, float* cstate, float* cdecay, int T,
-                       const int* item_seq, const int* item_t0, int n_items, const int* crow_seq,
-                       const int* crow_item0, int n_crows, int chunk, hipStream_t st) {
-  const int HK = a.H * a.dk;
-  gla_decay_kernel<E><<<dim3(cdiv(T, 8), std::min(8, cdiv(HK, 256))), 256, (size_t)8 * a.rank * 4, st>>>(a, logd, T);
-  const int NW = a.dv <= 64 ? 4 : 8;
-  const dim3 grid(n_items, a.H, cdiv(a.dv, 16 * NW));
+template <typename E, int NKT, int NCT>
+static void run_chunks(const GlaArgs& a, float* o32, float* cstate, float* cdecay, const int* item_seq,
+                       const int* item_t0, int n_items, const int* crow_seq, const int* crow_item0, int n_crows,
+                       int chunk, hipStream_t st) {
+  const dim3 grid(n_items, a.H, cdiv(a.dv, 16 * kGlaWaves * NCT));
   constexpr int DKP = 16 * NKT, LD = DKP + 4;
-  const size_t lds1 = (size_t)(DKP * 20 + DKP) * 4, lds2 = lds1 + (size_t)(2 * 16 * LD + NW * 256) * 4;
-  auto k1 = gla_chunk_kernel<E, NKT, false>;
-  auto k2 = gla_chunk_kernel<E, NKT, true>;
+  constexpr size_t lds1 = (size_t)(DKP * 20 + DKP) * 4;
+  constexpr size_t lds2 = lds1 + (size_t)(2 * 16 * LD + kGlaWaves * (256 + 16)) * 4;
+  auto k1 = gla_chunk_kernel<E, NKT, NCT, false>;
+  auto k2 = gla_chunk_kernel<E, NKT, NCT, true>;
   static bool attr = false;
-  if (!attr) {
-    (void)hipFuncSetAttribute((const void*)k2, hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 1024);
+  if (!attr && lds2 > 65536) {
+    (void)hipFuncSetAttribute((const void*)k2, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds2);
     attr = true;
   }
-  k1<<<grid, NW * 64, lds1, st>>>(a, nullptr, cstate, cdecay, logd, item_seq, item_t0, chunk);
+  k1<<<grid, 64 * kGlaWaves, lds1, st>>>(a, nullptr, cstate, cdecay, item_seq, item_t0, chunk);
   gla_scan_kernel<<<dim3(n_crows, a.H, cdiv(a.dk * a.dv, 256)), 256, 0, st>>>(a, cstate, cdecay, crow_seq, crow_item0,
                                                                               chunk);
-  k2<<<grid, NW * 64, lds2, st>>>(a, o32, cstate, cdecay, logd, item_seq, item_t0, chunk);
-  gla_gate_kernel<E><<<dim3(n_items, cdiv(chunk * a.H, 4)), 256, 0, st>>>(a, o32, item_seq, item_t0, chunk);
+  k2<<<grid, 64 * kGlaWaves, lds2, st>>>(a, o32, cstate, cdecay, item_seq, item_t0, chunk);
+  if (grid.z > 1)
+    gla_gate_kernel<E><<<dim3(n_items, cdiv(chunk * a.H, 4)), 256, 0, st>>>(a, o32, item_seq, item_t0, chunk);
 }
 
-void launch_gla_chunks(const GlaArgs& a, bool f32, float* logd, float* o32, float* cstate, float* cdecay, int T,
-                       const int* item_seq, const int* item_t0, int n_items, const int* crow_seq,
-                       const int* crow_item0, int n_crows, int chunk, hipStream_t st) {
+bool gla_chunks_need_o32(int dv) { return dv > 2 * 16 * kGlaWaves; }
+
+void launch_gla_chunks(const GlaArgs& a, bool f32, float* o32, float* cstate, float* cdecay, const int* item_seq,
+                       const int* item_t0, int n_items, const int* crow_seq, const int* crow_item0, int n_crows,
+                       int chunk, hipStream_t st) {
   if (n_items == 0) return;
-#define MLOP_GLA(N)                                                                                             \
-  do {                                                                                                          \
-    if (f32) run_chunks<float, N>(a, logd, o32, cstate, cdecay, T, item_seq, item_t0, n_items, crow_seq,        \
-                                  crow_item0, n_crows, chunk, st);                                              \
-    else run_chunks<uint16_t, N>(a, logd, o32, cstate, cdecay, T, item_seq, item_t0, n_items, crow_seq,         \
-                                 crow_item0, n_crows, chunk, st);                                               \
+#define MLOP_GLA_C(N, C)                                                                                          \
+  do {                                                                                                            \
+    if (f32) run_chunks<float, N, C>(a, o32, cstate, cdecay, item_seq, item_t0, n_items, crow_seq, crow_item0,    \
+                                     n_crows, chunk, st);                                                         \
+    else run_chunks<uint16_t, N, C>(a, o32, cstate, cdecay, item_seq, item_t0, n_items, crow_seq, crow_item0,     \
+                                    n_crows, chunk, st);                                                          \
+  } while (0)
+#define MLOP_GLA(N)                                                        \
+  do {                                                                     \
+    if (a.dv <= 16 * kGlaWaves) MLOP_GLA_C(N, 1); else MLOP_GLA_C(N, 2);   \
   } while (0)
   const int nkt = cdiv(a.dk, 16);
   if (nkt <= 1) MLOP_GLA(1);
@@ -437,6 +568,7 @@ void launch_gla_chunks(const GlaArgs& a, bool f32, float* logd, float* o32, floa
   else if (nkt <= 12) MLOP_GLA(12);
   else MLOP_GLA(16);
 #undef MLOP_GLA
+#undef MLOP_GLA_C
 }
 
 }  // namespace mlop

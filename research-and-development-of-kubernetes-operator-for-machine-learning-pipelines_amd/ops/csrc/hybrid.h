@@ -90,11 +90,12 @@ struct GlaArgs {
 };
 // every token of each listed row in turn (one-token rows; any sizes)
 void launch_gla_rows(const GlaArgs& a, bool f32, const int* rows, int n_rows, hipStream_t st);
-// chunks of `chunk` tokens in parallel: logd [T, H * dk], o32 [T, H, dv], cstate [items, H, dk, dv],
-// cdecay [items, H, dk] are scratch; crow_* list the sequences and their items
-void launch_gla_chunks(const GlaArgs& a, bool f32, float* logd, float* o32, float* cstate, float* cdecay, int T,
-                       const int* item_seq, const int* item_t0, int n_items, const int* crow_seq,
-                       const int* crow_item0, int n_crows, int chunk, hipStream_t st);
+// chunks of `chunk` tokens in parallel; o32 [T, H, dv] (only if gla_chunks_need_o32), cstate
+// [items, H, dk, dv], cdecay [items, H, dk] are scratch; crow_* list the sequences and their items
+void launch_gla_chunks(const GlaArgs& a, bool f32, float* o32, float* cstate, float* cdecay, const int* item_seq,
+                       const int* item_t0, int n_items, const int* crow_seq, const int* crow_item0, int n_crows,
+                       int chunk, hipStream_t st);
+bool gla_chunks_need_o32(int dv);
 constexpr int kGlaMaxDk = 256;    // key size of the chunked kernel
 
 // ---- elementwise (hyper.hip)

@@ -72,7 +72,10 @@ struct RopeEpi {
   // mid norm chain (gemm.hip mid_chain_finish): 1 = the finishing split reads the partials with
   // plain loads behind one agent acquire, 0 = with sc1 loads only (gemm_mid_chain op 2 / 1)
   int mid_acq = 0;
+  // plain epilogue only: C = bf16(max(acc, 0)^2) instead of bf16(acc) (EPI_RELU2 of launch_gemm)
+  int relu2 = 0;
 };
+constexpr int kEpiRelu2 = 6;  // launch_gemm: plain product with the squared-relu epilogue
 // RoPE + paged-cache stores from the QKV projection's fp32 split-K slabs ws[splits][T][N] (the
 // split-K reduce fused in: small-M launch_gemm_rope)
 void launch_rope_cache_slabs(const RopeEpi& re, const float* ws, int splits, int T, int N, hipStream_t st);
@@ -196,9 +199,10 @@ void launch_moe_dispatch_small(float* topw, int* topi, void* xp, int* offsets, i
 // combine + residual add + RMSNorm in one launch; false = hidden size not instantiated
 bool launch_moe_combine_add_rmsnorm(void* out, void* residual, const void* y, const int* inv, const float* topw,
                                     const void* w, float eps, int T, int k, int H, hipStream_t st);
-void launch_argmax(long* out, const float* logits, int n, int V, long ld, hipStream_t st);
-// bf16 greedy argmax; ws (>= argmax_splits(n, V) * n int64, or null) splits small batches' rows
+// greedy argmax; ws (>= argmax_splits(n, V) * n int64, or null) splits small batches' rows
+void launch_argmax(long* out, const float* logits, int n, int V, long ld, void* ws, hipStream_t st);
 int argmax_splits(int n, int V);
+int argmax_splits_f32(int n, int V);  // (rows 16-B aligned)
 void launch_argmax_bf16(long* out, const void* logits, int n, int V, long ld, void* ws, hipStream_t st);
 // temperature / top-k / top-p draw; small batches pre-select per-slice top-K candidates into ws
 // (sample_workspace_bytes(n, V) bytes, 0 = not needed)

@@ -11,6 +11,7 @@
 #include <algorithm>
 
 #include "common.h"
+#include "elem.h"
 #include "launch.h"
 
 namespace mlop {
@@ -115,27 +116,25 @@ __device__ __forceinline__ unsigned long long amax_key(float v, int i) {
   return ((unsigned long long)fkey(v) << 32) | (unsigned long long)(0xffffffffu - (uint32_t)i);
 }
 
-__global__ void __launch_bounds__(kSampleThreads) argmax_bf16_split_kernel(
-    unsigned long long* __restrict__ keys, const uint16_t* __restrict__ logits, int V, long ld, int S) {
+template <typename E>  // uint16_t (bf16) or float logits
+__global__ void __launch_bounds__(kSampleThreads) argmax_split_kernel(
+    unsigned long long* __restrict__ keys, const E* __restrict__ logits, int V, long ld, int S) {
   __shared__ float sv[kSampleThreads / 64];
   __shared__ int si[kSampleThreads / 64];
   const int s = blockIdx.x, row_id = blockIdx.y;
-  const uint16_t* row = logits + row_id * ld;
+  const E* row = logits + row_id * ld;
   const int nv8 = V >> 3, per = (nv8 + S - 1) / S;
   const int j0 = s * per, j1 = min(nv8, j0 + per);
   float v = -INFINITY;
   int idx = 0x7fffffff;
-  const u32x4* r8 = reinterpret_cast<const u32x4*>(row);
   for (int j = j0 + threadIdx.x; j < j1; j += blockDim.x) {
-    const u32x4 x = r8[j];
+    float x[8];
+    ldn<8>(row + 8 * (long)j, x);
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      amax_merge(v, idx, lo_bf(x[k]), 8 * j + 2 * k);
-      amax_merge(v, idx, hi_bf(x[k]), 8 * j + 2 * k + 1);
-    }
+    for (int k = 0; k < 8; ++k) amax_merge(v, idx, x[k], 8 * j + k);
   }
   if (s == S - 1)
-    for (int j = (nv8 << 3) + threadIdx.x; j < V; j += blockDim.x) amax_merge(v, idx, bf2f(row[j]), j);
+    for (int j = (nv8 << 3) + threadIdx.x; j < V; j += blockDim.x) amax_merge(v, idx, ld1(row + j), j);
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) {
     float ov = __shfl_xor(v, o, 64);
@@ -562,8 +561,15 @@ int sample_splits(int n, int V) {
   return S <= 1 ? 1 : S;
 }
 
-void launch_argmax(long* out, const float* logits, int n, int V, long ld, hipStream_t st) {
+void launch_argmax(long* out, const float* logits, int n, int V, long ld, void* ws, hipStream_t st) {
   if (n == 0) return;
+  if (ws) {
+    const int S = argmax_splits_f32(n, V);
+    auto* keys = (unsigned long long*)ws;
+    argmax_split_kernel<<<dim3(S, n), kSampleThreads, 0, st>>>(keys, logits, V, ld, S);
+    argmax_keys_kernel<<<n, 64, 0, st>>>(out, keys, S);
+    return;
+  }
   argmax_kernel<<<n, kSampleThreads, 0, st>>>(out, logits, V, ld);
 }
 
@@ -573,6 +579,8 @@ int argmax_splits(int n, int V) {
   const int by_size = V / (8 * kSampleThreads * 2);
   return std::max(1, std::min({64, by_size, (256 + n - 1) / n}));
 }
+// fp32 rows are twice the bytes and have no vectorised one-workgroup form: four splits at any n
+int argmax_splits_f32(int n, int V) { return std::max(argmax_splits(n, V), V >= 8192 ? 4 : 1); }
 
 void launch_argmax_bf16(long* out, const void* logits, int n, int V, long ld, void* ws, hipStream_t st) {
   if (n == 0) return;
@@ -582,7 +590,7 @@ void launch_argmax_bf16(long* out, const void* logits, int n, int V, long ld, vo
     return;
   }
   auto* keys = (unsigned long long*)ws;
-  argmax_bf16_split_kernel<<<dim3(S, n), kSampleThreads, 0, st>>>(keys, (const uint16_t*)logits, V, ld, S);
+  argmax_split_kernel<<<dim3(S, n), kSampleThreads, 0, st>>>(keys, (const uint16_t*)logits, V, ld, S);
   argmax_keys_kernel<<<n, 64, 0, st>>>(out, keys, S);
 }
 

@@ -127,7 +127,7 @@ class MetaBuffers:
         sizes = [("positions", max_tokens), ("slots", max_tokens), ("tile_seq", self.max_tiles),
                  ("tile_q0", self.max_tiles), ("ptile_seq", self.max_tiles), ("ptile_q0", self.max_tiles),
                  ("q_start", max_seqs), ("q_len", max_seqs), ("ctx_len", max_seqs)]
-        self.chunk = chunk
+        self.chunk = self.step_chunk = chunk
         self.n_items = self.n_crows = 0  # recurrent chunk items / rows of the last fill
         if chunk:
             ni = max_tokens // chunk + min(max_seqs, max_tokens // 2) + 1
@@ -221,7 +221,7 @@ class MetaBuffers:
             return {}
         n, r = self.n_items, self.n_crows
         return {"citem_seq": self.view_d("citem_seq", n), "citem_t0": self.view_d("citem_t0", n),
-                "crow_seq": self.view_d("crow_seq", r), "crow_item0": self.view_d("crow_item0", r), "chunk": self.chunk}
+                "crow_seq": self.view_d("crow_seq", r), "crow_item0": self.view_d("crow_item0", r), "chunk": self.step_chunk}
 
     def fill(self, rows, q_lens, ctx_lens, token_ids_per_seq, want_logits=None):
         """Fill host arrays for a ragged batch.
@@ -250,6 +250,9 @@ class MetaBuffers:
         pts_h, ptq_h = self.view_h("ptile_seq"), self.view_h("ptile_q0")
         npt, pqt = 0, self.pqt
         ni = nr = 0
+        if self.chunk:
+            # enough chunks to fill the chip either way: longer ones halve the chunk states' traffic
+            self.step_chunk = self.chunk * (2 if sum(int(q) for q in q_lens) >= 64 * self.chunk else 1)
         max_flash_q = 0
         qs_h, ql_h, cl_h = self.view_h("q_start"), self.view_h("q_len"), self.view_h("ctx_len")
         qt = self.qt
@@ -273,10 +276,10 @@ class MetaBuffers:
                 tq_h[nt:nt + ntile] = np.arange(ntile, dtype=np.int32) * qt
                 nt += ntile
             if self.chunk and ql > 1:
-                n = -(-ql // self.chunk)
+                n = -(-ql // self.step_chunk)
                 self.view_h("crow_seq")[nr], self.view_h("crow_item0")[nr] = row, ni
                 self.view_h("citem_seq")[ni:ni + n] = row
-                self.view_h("citem_t0")[ni:ni + n] = np.arange(n, dtype=np.int32) * self.chunk
+                self.view_h("citem_t0")[ni:ni + n] = np.arange(n, dtype=np.int32) * self.step_chunk
                 ni, nr = ni + n, nr + 1
             w = True if want_logits is None else want_logits[i]
             if isinstance(w, (list, tuple)):

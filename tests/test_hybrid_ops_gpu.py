@@ -153,6 +153,28 @@ def test_attention_hd_one_key_stands_out(gpu, dtype, H, G, D, V):
     assert _attention_case(gpu, dtype, H, G, D, V, [1, 1, 1], [300, 257, 16], spike=True, min_part=64) < TOL[dtype]
 
 
+@pytest.mark.parametrize("M,N,K", [(1, 96, 64), (3, 1024, 512), (16, 320, 320), (40, 512, 2048), (100, 96, 192),
+                                   (300, 384, 320), (700, 2048, 512), (2049, 2304, 384), (33, 40, 72), (4100, 2560, 1024)])
+def test_gemm_relu2_epilogue(gpu, M, N, K):
+    """Every row regime of the GEMM planner (GEMV, split-K, ring tiles, ping-pong, four-wave, library)."""
+    x, w = rnd(M, K, seed=1, dtype=torch.bfloat16), rnd(N, K, seed=2, dtype=torch.bfloat16, gain=K ** -0.5)
+    y = ops.gemm(x.to(gpu), w.to(gpu), epi=ops.EPI_RELU2)
+    assert rel_err(y, orc.relu2(x.double() @ w.double().T)) < 1.5e-2
+    plain = ops.gemm(x.to(gpu), w.to(gpu))
+    assert rel_err(plain, x.double() @ w.double().T) < 1e-2
+    z = ops.gemm(x.float().to(gpu), w.float().to(gpu), epi=ops.EPI_RELU2)
+    assert rel_err(z, orc.relu2(x.double() @ w.double().T)) < 1e-5
+
+
+@pytest.mark.parametrize("n,V", [(1, 128256), (3, 150), (200, 9000), (2, 131)])
+def test_argmax_fp32_rows(gpu, n, V):
+    x = rnd(n, (V + 3) // 4 * 4, seed=4)[:, :V]
+    x[:, V // 2] = x[:, 3 * V // 4] = 9.0  # a tie: the lower index
+    d = torch.zeros(n, (V + 3) // 4 * 4, device=gpu)
+    d[:, :V] = x.to(gpu)
+    assert ops.argmax(d[:, :V]).tolist() == [V // 2] * n
+
+
 def _gla_inputs(step, H, dk, dv, rank, dtype, bias, seed=0):
     nproj = (2 * H * dk + 2 * H * dv + rank + 15) // 16 * 16
     a2, b = rnd(H * dk, rank, seed=seed + 2, dtype=dtype, gain=1.5 / rank ** 0.5), bias + rnd(H * dk, seed=seed + 3)
