@@ -144,11 +144,18 @@ __global__ void __launch_bounds__(BT) gla_rows_kernel(GlaArgs a, const int* __re
 // [16 NKT, 16 NCT] in its accumulators.
 constexpr int kGlaWaves = 8;
 
+// workgroup barrier for LDS hand-offs only: outstanding global loads (the next block's operands) and
+// stores stay in flight across it, which __syncthreads would wait for
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  raw_barrier();
+}
+
 __device__ __forceinline__ float exp2_g(float x) { return __builtin_amdgcn_exp2f(x); }
 // log2(sigmoid(z)): log1p by the quotient form, exact where 1 + e rounds
 __device__ __forceinline__ float log2_sigmoid(float z) {
   const float e = exp2_g(-fabsf(z) * 1.44269504f), u = 1.f + e, d = u - 1.f;
-  const float l = d == 0.f ? e * 1.44269504f : __builtin_amdgcn_logf(u) * (e / d);
+  const float l = d == 0.f ? e * 1.44269504f : __builtin_amdgcn_logf(u) * (e * __builtin_amdgcn_rcpf(d));
   return fminf(z, 0.f) * 1.44269504f - l;
 }
 
@@ -172,6 +179,7 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
   float* Ks = Qs + 16 * LD;           // [16][LD]: k e^-b
   float* part = Ks + 16 * LD;         // [NW][256]
   float* red = part + NW * 256;       // [NW][16]
+  float* flags = red + NW * 16;       // [2][NW]
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int item = blockIdx.x, h = blockIdx.y;
   const int s = item_seq[item], t0 = item_t0[item];
@@ -204,6 +212,10 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
         }
       }
     }
+  float nw[NCT];
+#pragma unroll
+  for (int c = 0; c < NCT; ++c) nw[c] = (fused && col0 + 16 * c + l15 < dv) ? a.norm_w[col0 + 16 * c + l15] : 0.f;
+  const float inv_dv = 1.f / (float)dv;
   float total[NP];
 #pragma unroll
   for (int p = 0; p < NP; ++p) total[p] = 0.f;
@@ -278,8 +290,18 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
       slow |= all < kFast2;
     }
     bool fast = true;
-    if (OUT) fast = !__syncthreads_or(slow);  // also: the last block's LDS reads are done
-    else __syncthreads();
+    if (OUT) {
+      float* fl = flags + (t & 16 ? NW : 0);
+      const bool any = __ballot(slow) != 0;
+      if (lane == 0) fl[wid] = any ? 1.f : 0.f;
+      lds_barrier();  // also: the last block's LDS reads are done
+      float f = 0.f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) f += fl[w];
+      fast = f == 0.f;
+    } else {
+      lds_barrier();
+    }
     auto put_kt = [&]() {
 #pragma unroll
       for (int p = 0; p < NP; ++p) {
@@ -307,7 +329,15 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
       }
     }
     if (!OUT || fast) put_kt();
-    __syncthreads();
+    lds_barrier();
+    float gg[NCT][4];  // gates of this block's outputs
+#pragma unroll
+    for (int c = 0; c < NCT; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int col = col0 + 16 * c + l15;
+        gg[c][i] = (fused && col < dv && 4 * g4 + i < nt) ? ld1(pg + (size_t)(t + 4 * g4 + i) * a.ldp + col) : 0.f;
+      }
     f32x4 A = {0.f, 0.f, 0.f, 0.f};  // scores^T: row j = 4 g4 + i, column = token l15
     if (OUT) {
       int nsum = min(NW, NKT);
@@ -331,7 +361,7 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
           for (int d = half; d < dk; d += 2)
             x = fmaf(Qs[tt * LD + d] * Ks[j * LD + d], exp2_g(KT[tt * LD + d] - KT[j * LD + d]), x);
         part[tid] = x;
-        __syncthreads();
+        lds_barrier();
 #pragma unroll
         for (int p = 0; p < NP; ++p) {
           const int d = (p * NW + wid) * 16 + l15;
@@ -342,7 +372,7 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
         }
         put_kt();
       }
-      __syncthreads();
+      lds_barrier();
       for (int w = 0; w < nsum; ++w)
 #pragma unroll
         for (int i = 0; i < 4; ++i) A[i] += part[w * 256 + (4 * g4 + i) * 16 + l15];
@@ -389,14 +419,6 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
       }
     }
     if (fused) {  // o row 4 g4 + i = token, over the head's columns: rms, weight, gate
-      float gg[NCT][4];
-#pragma unroll
-      for (int c = 0; c < NCT; ++c)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int col = col0 + 16 * c + l15;
-          gg[c][i] = (col < dv && 4 * g4 + i < nt) ? ld1(pg + (size_t)(t + 4 * g4 + i) * a.ldp + col) : 0.f;
-        }
       float ss[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -409,7 +431,7 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
         ss[i] += detail::dpp<0x140>(ss[i]);
       }
       if (l15 == 0) *reinterpret_cast<f32x4*>(red + wid * 16 + 4 * g4) = f32x4{ss[0], ss[1], ss[2], ss[3]};
-      __syncthreads();
+      lds_barrier();
       f32x4 tot = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int w = 0; w < NW; ++w) tot += *reinterpret_cast<const f32x4*>(red + w * 16 + 4 * g4);
@@ -417,13 +439,13 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int j = 4 * g4 + i;
-        const float inv = 1.f / sqrtf(tot[i] / (float)dv + a.eps);
+        const float inv = rsqrtf(tot[i] * inv_dv + a.eps);
 #pragma unroll
         for (int c = 0; c < NCT; ++c) {
           const int col = col0 + 16 * c + l15;
           if (col < dv && j < nt) {
             const float g = gg[c][i];
-            st1(op + (size_t)j * HV + col, o[c][i] * inv * a.norm_w[col] * (g / (1.f + exp2_g(-g * 1.44269504f))));
+            st1(op + (size_t)j * HV + col, o[c][i] * inv * nw[c] * (g * __builtin_amdgcn_rcpf(1.f + exp2_g(-g * 1.44269504f))));
           }
         }
       }
@@ -509,7 +531,7 @@ static void run_rows_t(const GlaArgs& a, const int* rows, int n_rows, hipStream_
 template <typename E>
 static void run_rows(const GlaArgs& a, const int* rows, int n_rows, hipStream_t st) {
   // few (row, head) pairs: a whole CU's threads on each, so that its state is in flight at once
-  if (n_rows * a.H <= 512 && (long)a.dk * a.dv >= 8192) run_rows_t<E, 1024>(a, rows, n_rows, st);
+  if (n_rows * a.H <= 256 && (long)a.dk * a.dv >= 8192) run_rows_t<E, 1024>(a, rows, n_rows, st);
   else run_rows_t<E, 256>(a, rows, n_rows, st);
 }
 
@@ -526,7 +548,7 @@ static void run_chunks(const GlaArgs& a, float* o32, float* cstate, float* cdeca
   const dim3 grid(n_items, a.H, cdiv(a.dv, 16 * kGlaWaves * NCT));
   constexpr int DKP = 16 * NKT, LD = DKP + 4;
   constexpr size_t lds1 = (size_t)(DKP * 20 + DKP) * 4;
-  constexpr size_t lds2 = lds1 + (size_t)(2 * 16 * LD + kGlaWaves * (256 + 16)) * 4;
+  constexpr size_t lds2 = lds1 + (size_t)(2 * 16 * LD + kGlaWaves * (256 + 16 + 2)) * 4;
   auto k1 = gla_chunk_kernel<E, NKT, NCT, false>;
   auto k2 = gla_chunk_kernel<E, NKT, NCT, true>;
   static bool attr = false;
