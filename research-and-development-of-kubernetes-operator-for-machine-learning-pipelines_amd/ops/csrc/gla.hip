@@ -161,7 +161,7 @@ __device__ __forceinline__ float log2_sigmoid(float z) {
 
 // waves per SIMD the chunk kernel is built for: 4 = two workgroups per CU (128 VGPRs), 2 = one
 constexpr int chunk_waves(int nkt, int nct, bool out) {
-  return (out ? nct == 1 && nkt <= 8 : nkt * nct <= 16 && nkt <= 12) ? 4 : 2;
+  return (nct == 1 ? nkt <= 8 : !out && nkt <= 4) ? 4 : 2;
 }
 
 template <typename E, int NKT, int NCT, bool OUT>
@@ -171,7 +171,7 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
   constexpr int NW = kGlaWaves, DKP = 16 * NKT, LD = DKP + 4, LT = 20, NP = (NKT + NW - 1) / NW;
   constexpr float kFast2 = kFastDecay * 1.44269504f;
   // operands fetched one block ahead where the registers allow it at two workgroups per CU
-  constexpr bool AHEAD = chunk_waves(NKT, NCT, OUT) == 2 || NKT * NCT <= (OUT ? 6 : 12);
+  constexpr bool AHEAD = NKT * NCT <= (chunk_waves(NKT, NCT, OUT) == 2 ? 16 : OUT ? 2 : 8);
   extern __shared__ __attribute__((aligned(16))) float sm[];
   float* KT = sm;                     // [DKP][LT]: k_j e^{b_16 - b_j}, token fastest
   float* En = KT + DKP * LT;          // [DKP]: e^{b_16}
@@ -190,10 +190,6 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
   const bool wave_cols = col0 < dv;
   const bool fused = OUT && gridDim.z == 1;
   const E* proj = reinterpret_cast<const E*>(a.proj) + (size_t)tok0 * a.ldp;
-  const E* pq = proj + h * dk;
-  const E* pk = proj + HK + h * dk;
-  const E* pv = proj + 2 * HK + h * dv;
-  const E* pg = proj + 2 * HK + HV + h * dv;
   const E* pa = proj + 2 * HK + 2 * HV;
   float* cst = cstate + ((size_t)item * a.H + h) * dk * dv;
 
@@ -220,36 +216,71 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
 #pragma unroll
   for (int p = 0; p < NP; ++p) total[p] = 0.f;
 
-  float kk[NP][4], qq[NP][4], vv[NCT][4], x1[4];
+  // A block's operands as stored: loads at clamped addresses, unconditional and not converted here, so
+  // that all of them are in flight together; `take` converts and zeroes what is out of range.
+  E rk[NP][4], rq[NP][4], rv[NCT][4], rg[NCT][4], rx[4];
   auto fetch = [&](int t) {
-    const int nt = n - t;
+    const E* rows[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) rows[i] = proj + (size_t)min(t + 4 * g4 + i, n - 1) * a.ldp;
+    const E* xrow = proj + (size_t)min(t + l15, n - 1) * a.ldp + 2 * HK + 2 * HV;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) rx[i] = xrow[min(4 * g4 + i, rank - 1)];
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
-      const int d = (p * NW + wid) * 16 + l15;
+      const int d = h * dk + min((p * NW + wid) * 16 + l15, dk - 1);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const bool ok = d < dk && 4 * g4 + i < nt;
-        const size_t o = (size_t)(t + 4 * g4 + i) * a.ldp + d;
-        kk[p][i] = ok ? ld1(pk + o) : 0.f;
-        if (OUT) qq[p][i] = ok ? ld1(pq + o) * a.q_scale : 0.f;
+        rk[p][i] = rows[i][HK + d];
+        if (OUT) rq[p][i] = rows[i][d];
       }
     }
 #pragma unroll
-    for (int c = 0; c < NCT; ++c)
+    for (int c = 0; c < NCT; ++c) {
+      const int v = 2 * HK + h * dv + min(col0 + 16 * c + l15, dv - 1);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int col = col0 + 16 * c + l15;
-        const bool ok = col < dv && 4 * g4 + i < nt;
-        const size_t o = (size_t)(t + 4 * g4 + i) * a.ldp + col;
-        vv[c][i] = ok ? ld1(pv + o) : 0.f;
+        rv[c][i] = rows[i][v];
+        if (OUT) rg[c][i] = rows[i][HV + v];
+      }
+    }
+  };
+  float kk[NP][4], qq[NP][4], cv[NCT][4], gg[NCT][4], x1[4];
+  auto take = [&](int nt) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const bool in = 4 * g4 + i < nt;
+      x1[i] = (l15 < nt && 4 * g4 + i < rank) ? ld1(&rx[i]) : 0.f;
+#pragma unroll
+      for (int p = 0; p < NP; ++p) {
+        const bool ok = in && (p * NW + wid) * 16 + l15 < dk;
+        kk[p][i] = ok ? ld1(&rk[p][i]) : 0.f;
+        if (OUT) qq[p][i] = ok ? ld1(&rq[p][i]) * a.q_scale : 0.f;
       }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) x1[i] = (l15 < nt && 4 * g4 + i < rank) ? ld1(pa + (size_t)(t + l15) * a.ldp + 4 * g4 + i) : 0.f;
+      for (int c = 0; c < NCT; ++c) {
+        cv[c][i] = (in && col0 + 16 * c + l15 < dv) ? ld1(&rv[c][i]) : 0.f;
+        if (OUT) gg[c][i] = ld1(&rg[c][i]);
+      }
+    }
   };
+  // this wave's rows of A2 (its first 16 columns) and biases, kept over the chunk: a load inside the
+  // loop would wait behind the previous block's stores
+  float w1[NP][4], bias[NP];
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int d = (p * NW + wid) * 16 + l15, nrow = h * dk + (d < dk ? d : 0);
+    bias[p] = a.a2_b[nrow];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      w1[p][i] = 4 * g4 + i < rank ? ld1(reinterpret_cast<const E*>(a.a2) + (size_t)nrow * rank + 4 * g4 + i) : 0.f;
+  }
   if (AHEAD) fetch(0);
   for (int t = 0; t < n; t += 16) {
     const int nt = min(16, n - t);
     if (!AHEAD) fetch(t);
+    take(nt);
+    if (AHEAD && t + 16 < n) fetch(t + 16);
     // log2 decays of this wave's channels, running sums over the block's tokens
     float b[NP][4], bn[NP];
     bool slow = false;
@@ -257,16 +288,15 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
     for (int p = 0; p < NP; ++p) {
       const int d = (p * NW + wid) * 16 + l15;
       const bool ok = d < dk;
-      const int nrow = h * dk + (ok ? d : 0);
-      const float bias = a.a2_b[nrow];
-      f32x4 z = {bias, bias, bias, bias};
-      const E* w = reinterpret_cast<const E*>(a.a2) + (size_t)nrow * rank;
-      for (int r0 = 0; r0 < rank; r0 += 16) {
+      f32x4 z = {bias[p], bias[p], bias[p], bias[p]};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) z = mfma4(x1[i], w1[p][i], z);
+      const E* w = reinterpret_cast<const E*>(a.a2) + (size_t)(h * dk + (ok ? d : 0)) * rank;
+      for (int r0 = 16; r0 < rank; r0 += 16) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int r = r0 + 4 * g4 + i;
-          float x = x1[i];
-          if (r0) x = (l15 < nt && r < rank) ? ld1(pa + (size_t)(t + l15) * a.ldp + r) : 0.f;
+          const float x = (l15 < nt && r < rank) ? ld1(pa + (size_t)(t + l15) * a.ldp + r) : 0.f;
           z = mfma4(x, r < rank ? ld1(w + r) : 0.f, z);
         }
       }
@@ -330,14 +360,6 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
     }
     if (!OUT || fast) put_kt();
     lds_barrier();
-    float gg[NCT][4];  // gates of this block's outputs
-#pragma unroll
-    for (int c = 0; c < NCT; ++c)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int col = col0 + 16 * c + l15;
-        gg[c][i] = (fused && col < dv && 4 * g4 + i < nt) ? ld1(pg + (size_t)(t + 4 * g4 + i) * a.ldp + col) : 0.f;
-      }
     f32x4 A = {0.f, 0.f, 0.f, 0.f};  // scores^T: row j = 4 g4 + i, column = token l15
     if (OUT) {
       int nsum = min(NW, NKT);
@@ -380,12 +402,6 @@ __global__ void __launch_bounds__(64 * kGlaWaves, chunk_waves(NKT, NCT, OUT)) gl
       for (int i = 0; i < 4; ++i)
         if (4 * g4 + i > l15) A[i] = 0.f;
     }
-    float cv[NCT][4];
-#pragma unroll
-    for (int c = 0; c < NCT; ++c)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) cv[c][i] = vv[c][i];
-    if (AHEAD && t + 16 < n) fetch(t + 16);  // under the products
     f32x4 o[NCT];
     if (OUT) {
 #pragma unroll

@@ -117,6 +117,7 @@ __global__ void __launch_bounds__(256) qk_norm_reg_kernel(QkNormArgs a, int TB) 
   }
   const float lam = a.v_first ? *a.lam : 0.f;
   const bool v8 = a.V % 8 == 0 && a.ldf % 8 == 0 && (reinterpret_cast<uintptr_t>(a.v_first) & 15) == 0;
+  const bool r8 = a.R % 8 == 0;  // whole vectors turn, or none of their pairs does
   const int pad = a.KP - a.D;
   const int t_end = min(a.T, ((int)blockIdx.x + 1) * TB);
   for (int t = blockIdx.x * TB; t < t_end; ++t) {
@@ -159,6 +160,20 @@ __global__ void __launch_bounds__(256) qk_norm_reg_kernel(QkNormArgs a, int TB) 
     auto turn = [&](float (&o)[8], const float (&w)[8], float inv, int d) {
 #pragma unroll
       for (int e = 0; e < 8; ++e) o[e] *= inv * w[e];
+      if (r8) {
+        if (d < a.R) {
+          float c[4], s[4];
+          ldn<4>(cs + (d >> 1), c);
+          ldn<4>(cs + half + (d >> 1), s);
+#pragma unroll
+          for (int e = 0; e < 8; e += 2) {
+            const float x = o[e], y = o[e + 1];
+            o[e] = x * c[e >> 1] - y * s[e >> 1];
+            o[e + 1] = y * c[e >> 1] + x * s[e >> 1];
+          }
+        }
+        return;
+      }
 #pragma unroll
       for (int e = 0; e < 8; e += 2) {
         if (d + e < a.R) {

@@ -117,3 +117,57 @@ def save_checkpoint(path, cfg, weights):
     (path / "config.json").write_text(json.dumps(cfg))
     save_file({k: v.contiguous() for k, v in weights.items()}, str(path / "model.safetensors"))
     return path
+
+
+def make_engine(path, device, dtype, max_tokens=1024, seqs=4, graphs=True, **kw):
+    from mlopamd.models.loader import load_pretrained
+    from mlopamd.runtime.engine import Engine, EngineConfig
+
+    model = load_pretrained(path, device=device, dtype=dtype)
+    kw = {"max_num_seqs": seqs, "max_num_batched_tokens": max_tokens, "max_model_len": max_tokens,
+          "num_kv_blocks": blocks_needed(max_tokens) + 1, "graph_buckets": (1, 2, 4), "max_step_logits": max_tokens + 8,
+          "use_graphs": graphs, **kw}
+    return Engine(model, EngineConfig(**kw))
+
+
+def feed_schedule(eng, prompts, schedule):
+    """``schedule``: steps of [(request, tokens)]; every position's logits, per request.  A request is
+    closed when its tokens are through."""
+    seqs, at, out = {}, {}, {r: [] for r, _ in enumerate(prompts)}
+    for step in schedule:
+        entries = []
+        for r, n in step:
+            if r not in seqs:
+                seqs[r], at[r] = eng.open_sequence(), 0
+            entries.append((seqs[r], prompts[r][at[r]:at[r] + n], list(range(n))))
+            at[r] += n
+        logits, o = eng.feed(entries).float().cpu(), 0
+        for r, n in step:
+            out[r].append(logits[o:o + n])
+            o += n
+            if at[r] == len(prompts[r]):
+                eng.close_sequence(seqs.pop(r))
+    return [torch.cat(out[r]) for r in range(len(prompts))]
+
+
+def portions(n, sizes):
+    """Cut n tokens into the repeated ``sizes``."""
+    out, i = [], 0
+    while n:
+        k = min(n, sizes[i % len(sizes)])
+        out.append(k)
+        n, i = n - k, i + 1
+    return out
+
+
+def random_prompts(lens, vocab, seed=0):
+    g = torch.Generator().manual_seed(seed)
+    return [torch.randint(0, vocab, (n,), generator=g).tolist() for n in lens]
+
+
+def logits_err(got, want):
+    """Worst position: rms over the vocabulary of the mean-free difference, over the logits' spread."""
+    got, want = got.double().cpu(), want.double().cpu()
+    d = got - want
+    d = d - d.mean(-1, keepdim=True)
+    return float(d.pow(2).mean(-1).sqrt().max() / want.std())

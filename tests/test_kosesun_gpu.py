@@ -1,0 +1,52 @@
+"""Kosesun end to end on the GPU (kernels, paged cache, state slots, graphs) in both element types
+against the plain oracle; the scenarios of the CPU tests, on the product's compute path."""
+import pytest
+import torch
+
+import kosesun_cases as cases
+
+pytestmark = pytest.mark.gpu
+# worst position's rms error over the logits' spread; bf16 rounds every projection and sublayer output
+TOL = {torch.float32: 3e-4, torch.bfloat16: 8e-2}
+DTYPES = [torch.float32, torch.bfloat16]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", list(cases.CONFIGS))
+def test_whole_and_portions(gpu, tmp_path, name, dtype):
+    cases.whole_and_portions(tmp_path, gpu, dtype, name, TOL[dtype])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_batches(gpu, tmp_path, dtype):
+    cases.batches(tmp_path, gpu, dtype, TOL[dtype])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_decoding(gpu, tmp_path, dtype):
+    cases.long_decoding(tmp_path, gpu, dtype, TOL[dtype])
+
+
+@pytest.mark.parametrize("tight", [False, True])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_greedy_generation(gpu, tmp_path, dtype, tight):
+    eng = cases.greedy_generation(tmp_path, gpu, dtype, 1e-3 if dtype == torch.float32 else 0.3, tight=tight)
+    assert eng.stats["graph_steps"] > 0
+
+
+def test_preset_layer_shapes(gpu):
+    """Two layers at full preset width through graphs, mixed steps and sampling."""
+    from mlopamd.models import build_model
+    from mlopamd.models.config import get_config
+    from mlopamd.runtime.engine import Engine, EngineConfig
+    from mlopamd.runtime.sampler import SamplingParams
+
+    m = build_model(get_config("kosesun-8b", num_layers=2), device=gpu)
+    eng = Engine(m, EngineConfig(max_num_seqs=8, max_num_batched_tokens=2048, max_model_len=4096, num_kv_blocks=1024,
+                                 graph_buckets=(1, 8)))
+    prompts = [torch.randint(0, 128000, (n,)).tolist() for n in (3000, 200, 1, 77)]
+    outs = eng.generate(prompts, SamplingParams(max_tokens=8, ignore_eos=True))
+    again = eng.generate(prompts[1:2], SamplingParams(max_tokens=8, ignore_eos=True))
+    assert all(len(o) == 8 for o in outs) and again[0][0] == outs[1][0]
+    outs = eng.generate(prompts[:2], SamplingParams(max_tokens=8, temperature=0.7, top_p=0.9, ignore_eos=True))
+    assert all(0 <= t < 128256 for o in outs for t in o)
