@@ -6,8 +6,9 @@ import torch
 import kosesun_cases as cases
 
 pytestmark = pytest.mark.gpu
-# worst position's rms error over the logits' spread; bf16 rounds every projection and sublayer output
-TOL = {torch.float32: 3e-4, torch.bfloat16: 8e-2}
+# rms error over the logits' spread (hybrid_util.logits_err); bf16 rounds every projection and sublayer
+# output, and these models' squared relus and sharp attention amplify it
+TOL = {torch.float32: 3e-4, torch.bfloat16: 0.16}
 DTYPES = [torch.float32, torch.bfloat16]
 
 

@@ -31,6 +31,8 @@ def test_vmm_arena_under_sanitizers(variant):
     env["UBSAN_OPTIONS"] = "halt_on_error=1:print_stacktrace=1"
     r = subprocess.run([exe], env=env, capture_output=True, text=True, timeout=150)
     log = r.stdout + r.stderr
+    if r.returncode == 77 and variant != "plain":
+        pytest.skip(f"the HIP runtime does not come up under this sanitizer on this host: {r.stdout.strip()}")
     assert r.returncode == 0 and "vmm_stress ok" in r.stdout, log[-4000:]
     for marker in ("WARNING: ThreadSanitizer", "ERROR: AddressSanitizer", "ERROR: LeakSanitizer",
                    "runtime error:"):
