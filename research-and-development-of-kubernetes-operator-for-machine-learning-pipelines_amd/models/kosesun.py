@@ -80,8 +80,8 @@ class KosesunModel:
                 if m.v_mix and first_mix is None:
                     first_mix = m
                 elif m.v_mix:
-                    if (m.kv_heads, m.vdim) != (first_mix.kv_heads, first_mix.vdim):
-                        raise ValueError(f"layer {i}: value mixing needs the first mixing layer's value sizes")
+                    if m.kv_heads * m.vdim != first_mix.kv_heads * first_mix.vdim:
+                        raise ValueError(f"layer {i}: value mixing needs the first mixing layer's value size")
                     L["lam"] = src(p + "mix.vmix", dtype=f32, mean=0.5, std=0.0).reshape(1)
                 self.cache_layout.append(KVLayer(m.kv_heads, pad_dim(m.dim), pad_dim(m.vdim)))
                 self._rope_spec.add((m.rot_base, m.rot_dims))
@@ -105,6 +105,10 @@ class KosesunModel:
         self.head = fuse_rows([src("head", cfg.vocab_size, W)])  # (padding rows: the logits rows stay 16-B aligned)
         self.ones = torch.ones(S, device=self.device, dtype=f32)
         self.subs = subs
+        # decode graphs only where every product is a kernel of this package: a library product may
+        # record memory-set nodes, which have replayed wrongly
+        ws = [self.head] + [L[k] for L in self.layers for k in ("proj", "o", "up", "down") if k in L]
+        self.graph_safe = dtype == torch.bfloat16 and all(ops.gemm_is_native(*w.shape) for w in ws)
         self.n_q = self.n_kv
         # step metadata: one decode tile per one-token row, 128-token prompt tiles for every longer
         # portion (both independent of a layer's head counts), chunks for the recurrent layers

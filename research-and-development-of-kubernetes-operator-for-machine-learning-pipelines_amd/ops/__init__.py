@@ -322,6 +322,11 @@ def _gemm_backend(M, N, K, epi, x2, w, o2) -> str:
     return c
 
 
+def gemm_is_native(N: int, K: int) -> bool:
+    """Whether a plain product with a [N, K] bf16 weight runs on the package's own kernels."""
+    return GEMM_BACKEND == "mlop" and N % 8 == 0 and K % 64 == 0
+
+
 def _gemm_backend_choice(M, N, K, epi, x2, w, o2) -> str:
     """Per-shape choice between the hand-written MFMA kernel and hipBLASLt: the configured
     backend, or (``auto``) measured once per (M bucket, N, K, epilogue) on first eager use

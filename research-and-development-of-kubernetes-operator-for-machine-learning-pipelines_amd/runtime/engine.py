@@ -381,7 +381,7 @@ class Engine:
 
         # TP decode graphs capture the row-parallel all-reduces (K15 one-shot kernel, or RCCL
         # inside capture); the vocab gather runs after the replay (``_gather``).
-        if cfg.use_graphs and self.device.type == "cuda":
+        if cfg.use_graphs and self.device.type == "cuda" and getattr(model, "graph_safe", True):
             self.capture_graphs()
         self.kv.start_background_fill()  # after capture: the rest of a lazy KV arena
         self.stats["kv_ready_blocks_at_start"] = self.alloc.available

@@ -13,6 +13,9 @@ CONFIGS = {
     "no_first_mix": dict(layers="aaaga", no_mix=(0, 2), heads=4, kv_heads=4, dim=16, vdim=16, rot=16, streams=5),
     "attention_only": dict(layers="aa", streams=1, heads=7, kv_heads=1, dim=34, vdim=50, rot=6, width=64, ff=64, vocab=128),
     "gla_only": dict(layers="gg", streams=4, gla_heads=1, gla_dim=64, gla_vdim=64, tau=30.0, width=128, cap=40.0),
+    # every product on the package's own kernels: decode runs from captured graphs
+    "native": dict(layers="agag", width=128, ff=192, heads=6, vdim=32, dim=40, rot=24, gla_heads=4, gla_dim=24, gla_vdim=16,
+                   vocab=150, streams=4),
     "wide_groups": dict(layers="ag", heads=40, kv_heads=2, dim=32, vdim=64, rot=32, streams=3, gla_heads=5, gla_dim=16,
                         gla_vdim=136),
 }
@@ -90,7 +93,7 @@ def greedy_generation(tmp_path, device, dtype, margin, tight=False):
     the oracle's two best logits lie within ``margin`` of its spread either may be picked."""
     from mlopamd.runtime.sampler import SamplingParams
 
-    cfg, w, path = setup(tmp_path, "mixed", seed=7)
+    cfg, w, path = setup(tmp_path, "native", seed=7)
     oracle = Oracle(cfg, w)
     eng = make_engine(path, device, dtype, max_tokens=256, seqs=3, max_num_batched_tokens=48, mixed_min_chunk=8,
                       max_model_len=256, num_kv_blocks=8 if tight else 40)
