@@ -85,159 +85,137 @@ __global__ void __launch_bounds__(256) qk_norm_kernel(QkNormArgs a) {
   }
 }
 
-// Register form (head size a multiple of 8): a thread keeps its NQ q vectors and NK k vectors of 8
-// elements from the sums of squares to the stores, with their norm weights, for TB tokens in turn
-// (one norm-weight read per workgroup; the next token's row is fetched under this one's stores).
-template <typename E, int NQ, int NK>
-__global__ void __launch_bounds__(256) qk_norm_reg_kernel(QkNormArgs a, int TB) {
-  __shared__ float scratch[2][4];
-  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+// Vector form (head sizes multiples of 8): the token's [q | k | v] vectors of 8 elements are dealt to
+// the threads of one workgroup (NI each, one at the usual sizes), which keep them, and their norm
+// weights, in registers from the sums of squares to the stores, for TB tokens in turn.
+template <typename E, int NI>
+__global__ void __launch_bounds__(1024) qk_norm_vec_kernel(QkNormArgs a, int TB) {
+  __shared__ float scratch[2][2][16];
+  const int tid = threadIdx.x, BT = blockDim.x, lane = tid & 63, wid = tid >> 6, NWv = BT >> 6;
   const int nq = a.H * a.D, nk = a.G * a.D, nv = a.G * a.V, half = a.R / 2;
-  int qc[NQ], qd[NQ], qdst[NQ], kc_[NK], kd[NK], kdst[NK];
-  float qw[NQ][8], kw[NK][8];
+  enum { NONE, Q, K, V };
+  int kind[NI], d[NI], dst[NI];
+  float w[NI][8];
 #pragma unroll
-  for (int i = 0; i < NQ; ++i) {
-    const int c = (tid + 256 * i) * 8, h = c / a.D;
-    qc[i] = c < nq ? c : -1;
-    qd[i] = c - h * a.D;
-    qdst[i] = h * a.KP + qd[i];
+  for (int i = 0; i < NI; ++i) {
+    const int c = (tid + BT * i) * 8;
+    kind[i] = c < nq ? Q : c < nq + nk ? K : c < nq + nk + nv ? V : NONE;
+    const int cc = kind[i] == Q ? c : kind[i] == K ? c - nq : c - nq - nk;
+    const int sz = kind[i] == V ? a.V : a.D, h = cc / sz;
+    d[i] = kind[i] == V ? a.R : cc - h * sz;  // (values never turn)
+    dst[i] = (kind[i] == Q ? h * a.KP : h * a.BS * (kind[i] == V ? a.VP : a.KP)) + cc - h * sz;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) qw[i][e] = 1.f;
-    if (a.q_w && c < nq) ldn<8>(a.q_w + c, qw[i]);
-  }
-#pragma unroll
-  for (int i = 0; i < NK; ++i) {
-    const int c = (tid + 256 * i) * 8, g = c / a.D;
-    kc_[i] = c < nk ? c : -1;
-    kd[i] = c - g * a.D;
-    kdst[i] = g * a.BS * a.KP + kd[i];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) kw[i][e] = 1.f;
-    if (a.k_w && c < nk) ldn<8>(a.k_w + c, kw[i]);
+    for (int e = 0; e < 8; ++e) w[i][e] = 1.f;
+    if (a.q_w && kind[i] == Q) ldn<8>(a.q_w + cc, w[i]);
+    if (a.k_w && kind[i] == K) ldn<8>(a.k_w + cc, w[i]);
   }
   const float lam = a.v_first ? *a.lam : 0.f;
-  const bool v8 = a.V % 8 == 0 && a.ldf % 8 == 0 && (reinterpret_cast<uintptr_t>(a.v_first) & 15) == 0;
-  const bool r8 = a.R % 8 == 0;  // whole vectors turn, or none of their pairs does
+  const bool r8 = a.R > 0 && a.R % 8 == 0;  // whole vectors turn, or none of their pairs does
   const int pad = a.KP - a.D;
   const int t_end = min(a.T, ((int)blockIdx.x + 1) * TB);
   for (int t = blockIdx.x * TB; t < t_end; ++t) {
     const E* row = reinterpret_cast<const E*>(a.proj) + (size_t)t * a.ldp;
-    float q[NQ][8], k[NK][8], sq = 0.f, sk = 0.f;
+    float x[NI][8];
 #pragma unroll
-    for (int i = 0; i < NQ; ++i) {
-#pragma unroll
-      for (int e = 0; e < 8; ++e) q[i][e] = 0.f;
-      if (qc[i] >= 0) ldn<8>(row + qc[i], q[i]);
-    }
-#pragma unroll
-    for (int i = 0; i < NK; ++i) {
-#pragma unroll
-      for (int e = 0; e < 8; ++e) k[i][e] = 0.f;
-      if (kc_[i] >= 0) ldn<8>(row + nq + kc_[i], k[i]);
+    for (int i = 0; i < NI; ++i) {
+ldn<8>(row + (kind[i] == NONE ? 0 : (tid + BT * i) * 8), x[i]);
     }
     const float* cs = a.cos_sin + (size_t)a.pos[t] * a.R;
     const int slot = a.slots[t];
-    float iq = 1.f, ik = 1.f;
+    // cos / sin and the values to mix in are fetched beside the row, unconditionally (clamped)
+    float cc[NI][4], sc4[NI][4], f[NI][8];
+    if (r8) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int o = d[i] < a.R ? d[i] >> 1 : 0;
+        ldn<4>(cs + o, cc[i]);
+        ldn<4>(cs + half + o, sc4[i]);
+      }
+    }
+    if (a.v_first) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+        ldn<8>(reinterpret_cast<const E*>(a.v_first) + (size_t)t * a.ldf + (kind[i] == V ? (tid + BT * i) * 8 - nq - nk : 0),
+               f[i]);
+    }
+    float inv[2] = {1.f, 1.f};
     if (a.q_w) {
+      float sq = 0.f, sk = 0.f;
 #pragma unroll
-      for (int i = 0; i < NQ; ++i)
+      for (int i = 0; i < NI; ++i) {
+        float s = 0.f;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) sq = fmaf(q[i][e], q[i][e], sq);
-#pragma unroll
-      for (int i = 0; i < NK; ++i)
-#pragma unroll
-        for (int e = 0; e < 8; ++e) sk = fmaf(k[i][e], k[i][e], sk);
+        for (int e = 0; e < 8; ++e) s = fmaf(x[i][e], x[i][e], s);
+        sq += kind[i] == Q ? s : 0.f;
+        sk += kind[i] == K ? s : 0.f;
+      }
       sq = wave_sum(sq);
       sk = wave_sum(sk);
-      if (lane == 0) scratch[0][wid] = sq, scratch[1][wid] = sk;
-      __syncthreads();
-      sq = scratch[0][0] + scratch[0][1] + scratch[0][2] + scratch[0][3];
-      sk = scratch[1][0] + scratch[1][1] + scratch[1][2] + scratch[1][3];
-      __syncthreads();
-      iq = 1.f / sqrtf(sq / (float)nq + a.eps);
-      ik = 1.f / sqrtf(sk / (float)nk + a.eps);
+      // double-buffered over the tokens: one barrier each, for LDS only (stores stay in flight)
+      float (*sc)[16] = scratch[t & 1];
+      if (lane == 0) sc[0][wid] = sq, sc[1][wid] = sk;
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      raw_barrier();
+      sq = sk = 0.f;
+      for (int k = 0; k < NWv; ++k) sq += sc[0][k], sk += sc[1][k];
+      inv[0] = 1.f / sqrtf(sq / (float)nq + a.eps);
+      inv[1] = 1.f / sqrtf(sk / (float)nk + a.eps);
     }
-    auto turn = [&](float (&o)[8], const float (&w)[8], float inv, int d) {
+    const int blk = slot >= 0 ? slot / a.BS : 0, off = slot - blk * a.BS;
+    E* qo = reinterpret_cast<E*>(a.q_out) + (size_t)t * a.H * a.KP;
+    E* ko = reinterpret_cast<E*>(a.k_cache) + ((size_t)blk * a.G * a.BS + off) * a.KP;
+    E* vo = reinterpret_cast<E*>(a.v_cache) + ((size_t)blk * a.G * a.BS + off) * a.VP;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] *= inv * w[e];
-      if (r8) {
-        if (d < a.R) {
-          float c[4], s[4];
-          ldn<4>(cs + (d >> 1), c);
-          ldn<4>(cs + half + (d >> 1), s);
+    for (int i = 0; i < NI; ++i) {
+      if (kind[i] == NONE || (kind[i] != Q && slot < 0)) continue;
+      if (kind[i] == V) {
+        if (a.v_first) {
 #pragma unroll
-          for (int e = 0; e < 8; e += 2) {
-            const float x = o[e], y = o[e + 1];
-            o[e] = x * c[e >> 1] - y * s[e >> 1];
-            o[e + 1] = y * c[e >> 1] + x * s[e >> 1];
+          for (int e = 0; e < 8; ++e) x[i][e] = (1.f - lam) * x[i][e] + lam * f[i][e];
+        }
+        stn<8>(vo + dst[i], x[i]);
+        continue;
+      }
+      const float n = kind[i] == Q ? inv[0] : inv[1];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[i][e] *= n * w[i][e];
+      if (d[i] < a.R) {
+        float c[4], s[4];
+        if (r8) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) c[e] = cc[i][e], s[e] = sc4[i][e];
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const bool in = d[i] + 2 * e < a.R;
+            c[e] = in ? cs[(d[i] >> 1) + e] : 1.f;
+            s[e] = in ? cs[half + (d[i] >> 1) + e] : 0.f;
           }
         }
-        return;
-      }
 #pragma unroll
-      for (int e = 0; e < 8; e += 2) {
-        if (d + e < a.R) {
-          const float c = cs[(d + e) >> 1], s = cs[half + ((d + e) >> 1)];
-          const float x = o[e], y = o[e + 1];
-          o[e] = x * c - y * s;
-          o[e + 1] = y * c + x * s;
+        for (int e = 0; e < 8; e += 2) {
+          const float u = x[i][e], y = x[i][e + 1];
+          x[i][e] = u * c[e >> 1] - y * s[e >> 1];
+          x[i][e + 1] = y * c[e >> 1] + u * s[e >> 1];
         }
       }
-    };
-    E* qo = reinterpret_cast<E*>(a.q_out) + (size_t)t * a.H * a.KP;
-#pragma unroll
-    for (int i = 0; i < NQ; ++i)
-      if (qc[i] >= 0) {
-        turn(q[i], qw[i], iq, qd[i]);
-        stn<8>(qo + qdst[i], q[i]);
-      }
-    if (pad)
-      for (int c = tid; c < a.H * pad; c += 256) st1(qo + (size_t)(c / pad) * a.KP + a.D + c % pad, 0.f);
-    if (slot < 0) continue;
-    const int blk = slot / a.BS, off = slot - blk * a.BS;
-    E* ko = reinterpret_cast<E*>(a.k_cache) + ((size_t)blk * a.G * a.BS + off) * a.KP;
-#pragma unroll
-    for (int i = 0; i < NK; ++i)
-      if (kc_[i] >= 0) {
-        turn(k[i], kw[i], ik, kd[i]);
-        stn<8>(ko + kdst[i], k[i]);
-      }
-    E* vo = reinterpret_cast<E*>(a.v_cache) + ((size_t)blk * a.G * a.BS + off) * a.VP;
-    const E* v0 = row + nq + nk;
-    const E* vf = reinterpret_cast<const E*>(a.v_first) + (a.v_first ? (size_t)t * a.ldf : 0);
-    if (v8) {
-      for (int c = tid * 8; c < nv; c += 2048) {
-        const int g = c / a.V, d = c - g * a.V;
-        float v[8];
-        ldn<8>(v0 + c, v);
-        if (a.v_first) {
-          float f[8];
-          ldn<8>(vf + c, f);
-#pragma unroll
-          for (int e = 0; e < 8; ++e) v[e] = (1.f - lam) * v[e] + lam * f[e];
-        }
-        stn<8>(vo + (size_t)g * a.BS * a.VP + d, v);
-      }
-    } else {
-      for (int c = tid; c < nv; c += 256) {
-        const int g = c / a.V, d = c - g * a.V;
-        float v = ld1(v0 + c);
-        if (a.v_first) v = (1.f - lam) * v + lam * ld1(vf + c);
-        st1(vo + (size_t)g * a.BS * a.VP + d, v);
-      }
+      stn<8>((kind[i] == Q ? qo : ko) + dst[i], x[i]);
     }
+    if (pad)
+      for (int c = tid; c < a.H * pad; c += BT) st1(qo + (size_t)(c / pad) * a.KP + a.D + c % pad, 0.f);
   }
 }
 
 template <typename E>
 static void run_qk(const QkNormArgs& a, hipStream_t st) {
-  const int nq = cdiv(a.H * a.D, 2048), nk = cdiv(a.G * a.D, 2048);
-  if (a.D % 8 == 0 && a.ldp % 8 == 0 && nq <= 4 && nk <= 2) {
-    const int TB = a.T >= 4096 ? 4 : 1, grid = cdiv(a.T, TB);
-    if (nk == 2) qk_norm_reg_kernel<E, 4, 2><<<grid, 256, 0, st>>>(a, TB);
-    else if (nq <= 1) qk_norm_reg_kernel<E, 1, 1><<<grid, 256, 0, st>>>(a, TB);
-    else if (nq <= 2) qk_norm_reg_kernel<E, 2, 1><<<grid, 256, 0, st>>>(a, TB);
-    else qk_norm_reg_kernel<E, 4, 1><<<grid, 256, 0, st>>>(a, TB);
+  const int items = cdiv(a.H * a.D + a.G * (a.D + a.V), 8);
+  const bool vf = !a.v_first || (a.ldf % 8 == 0 && (reinterpret_cast<uintptr_t>(a.v_first) & 15) == 0);
+  if (a.D % 8 == 0 && a.V % 8 == 0 && a.ldp % 8 == 0 && vf && items <= 4096) {
+    const int ni = items <= 1024 ? 1 : items <= 2048 ? 2 : 4;
+    const int block = cdiv(cdiv(items, ni), 64) * 64, TB = a.T >= 8192 ? 8 : a.T >= 2048 ? 4 : 1, grid = cdiv(a.T, TB);
+    if (ni == 1) qk_norm_vec_kernel<E, 1><<<grid, block, 0, st>>>(a, TB);
+    else if (ni == 2) qk_norm_vec_kernel<E, 2><<<grid, block, 0, st>>>(a, TB);
+    else qk_norm_vec_kernel<E, 4><<<grid, block, 0, st>>>(a, TB);
   } else if (a.D % 8 == 0 && a.ldp % 8 == 0) {
     qk_norm_kernel<E, 8><<<a.T, 256, 0, st>>>(a);
   } else {

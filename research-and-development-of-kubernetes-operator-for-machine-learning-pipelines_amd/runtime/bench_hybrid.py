@@ -77,7 +77,8 @@ def _prefill(eng, n, length, kernels) -> dict:
 
 def _decode(eng, n, ctx, steps, kernels) -> dict:
     V = eng.model.cfg.vocab_size
-    params = SamplingParams(max_tokens=steps + 24, ignore_eos=True)
+    # (the first sequences decode while the last prompts are read)
+    params = SamplingParams(max_tokens=steps + 32 + n * ctx // 4096, ignore_eos=True)
     for p in _prompts(n, ctx, V, 7):
         eng.add_request(p, params)
     while eng.waiting or eng.prefilling:
@@ -90,6 +91,7 @@ def _decode(eng, n, ctx, steps, kernels) -> dict:
         eng.step()
     torch.cuda.synchronize()
     dt = time.perf_counter() - t0
+    assert len(eng.running) == n, "a sequence ended inside the timed steps"
     out = {"workload": f"decode {n} @ {ctx}", "tok_per_s": round(n * steps / dt), "ms": round(1e3 * dt / steps, 4)}
     if kernels:
         out["kernels"] = _kernels(lambda: [eng.step() for _ in range(8)])
@@ -107,7 +109,7 @@ def main(device=None, steps: int = 64, kernels: bool = False, only: str = "") ->
                 continue
             eng = Engine(build_model(cfg, device=device),
                          EngineConfig(max_num_seqs=256, max_num_batched_tokens=8192, max_model_len=8320,
-                                      num_kv_blocks=256 * 76, graph_buckets=(1, 32, 256), enable_prefix_caching=False))
+                                      num_kv_blocks=256 * 80, graph_buckets=(1, 32, 256), enable_prefix_caching=False))
             runs = [lambda w=w: _prefill(eng, *w, kernels) for w in PREFILL] + \
                    [lambda w=w: _decode(eng, *w, steps, kernels) for w in DECODE]
             for run in runs:

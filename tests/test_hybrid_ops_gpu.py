@@ -234,3 +234,27 @@ def test_gla_graph_padding_rows(gpu):
     out = ops.gla(x.to(gpu), H, dk, dv, a2.to(gpu), b.to(gpu), nw.to(gpu), 2.0, 1e-4, d_state, meta)
     assert float(out[1:].abs().max()) == 0 and float(out[0].abs().max()) > 0
     assert torch.equal(d_state[[0, 2, 3]].cpu(), state[[0, 2, 3]])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_gla_large_step(gpu, dtype):
+    """A step large enough for the longer chunks (the state passes through dozens of them)."""
+    H, dk, dv, rank, tau, eps = 1, 20, 36, 9, 40.0, 1e-4
+    q_lens, ctx = [1, 4000, 99, 130], [30, 4100, 99, 131]
+    step = Step(q_lens, ctx, gpu, chunk=64)
+    assert step.meta.chunk == 128
+    x, a2, b, nw = _gla_inputs(step, H, dk, dv, rank, dtype, 2.0, seed=40)
+    state = rnd(len(q_lens) + 2, H, dk, dv, seed=9)
+    d_state = state.to(gpu)
+    out = ops.gla(x.to(gpu), H, dk, dv, a2.to(gpu), b.to(gpu), nw.to(gpu), tau, eps, d_state, step.meta)
+    for n, c, s, row in zip(step.q_lens, step.ctx, step.starts(), step.rows.tolist()):
+        o, S = _gla_oracle(x[s:s + n], H, dk, dv, rank, a2, b, nw, tau, eps, None if c == n else state[row].double())
+        assert rel_err(out[s:s + n], o) < TOL[dtype], (n, c)
+        assert rel_err(d_state[row], S) < 5e-5, (n, c)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_attention_hd_long_context(gpu, dtype):
+    """Hundreds of pages: prompts over many tiles, decode over many partitions, far keys that stand out."""
+    assert _attention_case(gpu, dtype, 2, 1, 64, 48, [1, 700, 1], [1500, 1200, 1025], spike=True, min_part=128) < TOL[dtype]
+    assert _attention_case(gpu, dtype, 2, 2, 96, 64, [1, 300], [900, 1000]) < TOL[dtype]
