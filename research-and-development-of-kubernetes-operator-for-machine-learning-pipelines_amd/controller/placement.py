@@ -75,7 +75,7 @@ def _plan(arch, max_model_len, max_num_seqs, hbm_gb, gpus_per_node, utilization,
         kv_split = min(tp, cfg.num_kv_heads)  # kv heads replicate beyond Hkv
         kv_per_gpu = kv_target / kv_split
         free = usable * GB - reserve_gb * GB - w
-        cap = int(max(0.0, free) * kv_split / kv_tok)
+        cap = int(max(0.0, free) * kv_split / max(1, kv_tok))  # (0: no layer keeps pages)
         fits = free >= kv_per_gpu
         return Placement(cfg.name, tp, ep, shards, round(w / GB, 2), round(max(0.0, free) / GB, 2), cap,
                          hbm_gb, fits, "" if fits else

@@ -1,10 +1,10 @@
-"""Model zoo: Llama-3 (8B / 70B), Mixtral-8x7B (MoE) and Kosesun (hybrid), random-init bf16.
+"""Model zoo: Llama-3 (8B / 70B), Mixtral-8x7B (MoE), Kosesun and Regesun (hybrids), random-init bf16.
 
 The configs import without torch (the operator image's placement planner reads them);
 ``build_model`` pulls in torch and the model code on first use."""
 from __future__ import annotations
 
-from .config import HybridConfig, ModelConfig, get_config, PRESETS  # noqa: F401
+from .config import HybridConfig, KosesunConfig, ModelConfig, RegesunConfig, get_config, PRESETS  # noqa: F401
 
 
 def build_model(name_or_cfg, device="cuda", dtype=None, pstate=None, seed: int = 0, weights=None):
@@ -13,7 +13,11 @@ def build_model(name_or_cfg, device="cuda", dtype=None, pstate=None, seed: int =
 
     dtype = torch.bfloat16 if dtype is None else dtype
     cfg = name_or_cfg if isinstance(name_or_cfg, ModelConfig) else get_config(name_or_cfg)
-    if isinstance(cfg, HybridConfig):
+    if isinstance(cfg, RegesunConfig):
+        from .regesun import RegesunModel
+
+        return RegesunModel(cfg, device=device, dtype=dtype, pstate=pstate, seed=seed, weights=weights)
+    if isinstance(cfg, KosesunConfig):
         from .kosesun import KosesunModel
 
         return KosesunModel(cfg, device=device, dtype=dtype, pstate=pstate, seed=seed, weights=weights)

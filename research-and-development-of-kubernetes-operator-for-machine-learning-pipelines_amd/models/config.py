@@ -115,21 +115,93 @@ class GLASpec:
         hk, hv = self.heads * self.dim, self.heads * self.vdim
         return width * (2 * hk + 3 * hv + self.rank) + hk * self.rank + 2 * hk * self.vdim
 
+    def state_elems(self) -> int:
+        return self.heads * self.dim * self.vdim
+
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Softmax-attention mixer over cached latents, without positions."""
+    heads: int
+    dim: int                 # query / key head size
+    vdim: int                # value head size
+    rank: int                # latent size (all that is cached)
+    scale: float             # score scale
+    window: int = 0          # a token sees itself and the window - 1 tokens before it (0: all)
+
+    def params(self, width: int) -> int:
+        hq, hv = self.heads * self.dim, self.heads * self.vdim
+        return width * (hq + self.rank + 2 * hv) + self.rank * (hq + hv + 1) + self.heads
+
+    def macs(self, width: int) -> int:
+        hq, hv = self.heads * self.dim, self.heads * self.vdim
+        return width * (hq + self.rank + 2 * hv) + self.rank * (hq + hv)
+
+
+@dataclass(frozen=True)
+class SSDSpec:
+    """Selective-state-space mixer (Mamba-2): a [state, vdim] state per head with one decay per head,
+    behind a short convolution."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int              # B and C are shared by heads / groups heads
+    taps: int                # of the convolution
+    norm_groups: int         # equal parts of the output norm
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        """Convolved channels: x, B and C."""
+        return self.inner + 2 * self.groups * self.state
+
+    def params(self, width: int) -> int:
+        return (width * (2 * self.inner + 2 * self.groups * self.state + self.heads) + width * self.inner +
+                self.channels * (self.taps + 1) + 3 * self.heads + self.inner)
+
+    def macs(self, width: int) -> int:
+        return (width * (3 * self.inner + 2 * self.groups * self.state + self.heads) + self.channels * self.taps +
+                2 * self.inner * self.state)
+
+    def state_elems(self) -> int:
+        return self.inner * self.state + (self.taps - 1) * self.channels
+
+
+@dataclass(frozen=True)
+class DeltaSpec:
+    """Generalized-delta-rule mixer: a [dim, dim] state per head with a decay and a removal rate per key
+    channel."""
+    heads: int
+    dim: int
+    rank: int                # inner size of the decay projection
+
+    def params(self, width: int) -> int:
+        n = self.heads * self.dim
+        return width * (6 * n + self.rank) + n * (self.rank + 3)
+
+    def macs(self, width: int) -> int:
+        n = self.heads * self.dim
+        return width * (6 * n + self.rank) + n * self.rank + 3 * n * self.dim
+
+    def state_elems(self) -> int:
+        return self.heads * self.dim * self.dim
+
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: AttentionSpec | GLASpec
-    ff: int = 0              # squared-relu feed-forward width (0: none)
+    mixer: AttentionSpec | GLASpec | LatentAttentionSpec | SSDSpec | DeltaSpec
+    ff: int = 0              # feed-forward width (0: none)
+    limit: float = 0.0       # clamp of a gated feed-forward (designs that have one)
 
 
 @dataclass(frozen=True)
 class HybridConfig(ModelConfig):
-    """A decoder whose layers are listed one by one (``layers``), on hyper-connection streams
-    (Kosesun).  The uniform fields of ``ModelConfig`` hold the largest layer's sizes."""
+    """A decoder whose layers are listed one by one (``layers``).  The uniform fields of ``ModelConfig``
+    hold the largest layer's sizes."""
     layers: tuple = ()
-    streams: int = 1
-    embed_scale: float = 1.0
-    logit_softcap: float = 0.0
 
     def __post_init__(self):
         # replace(num_layers=n) keeps the first n layers
@@ -137,11 +209,32 @@ class HybridConfig(ModelConfig):
 
     @property
     def attention(self) -> tuple:
-        return tuple(la.mixer for la in self.layers if isinstance(la.mixer, AttentionSpec))
+        """Mixers that keep pages."""
+        return tuple(la.mixer for la in self.layers if isinstance(la.mixer, (AttentionSpec, LatentAttentionSpec)))
 
     @property
     def recurrent(self) -> tuple:
-        return tuple(la.mixer for la in self.layers if isinstance(la.mixer, GLASpec))
+        """Mixers that keep a state."""
+        return tuple(la.mixer for la in self.layers if isinstance(la.mixer, (GLASpec, SSDSpec, DeltaSpec)))
+
+    def active_params(self) -> int:
+        return self.num_params()
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        return sum(m.rank if isinstance(m, LatentAttentionSpec) else m.kv_heads * (m.dim + m.vdim)
+                   for m in self.attention) * dtype_bytes
+
+    def state_bytes_per_seq(self) -> int:
+        return 4 * sum(m.state_elems() for m in self.recurrent)
+
+
+@dataclass(frozen=True)
+class KosesunConfig(HybridConfig):
+    """Kosesun: attention and gated linear attention on hyper-connection streams, squared-relu
+    feed-forward."""
+    streams: int = 1
+    embed_scale: float = 1.0
+    logit_softcap: float = 0.0
 
     def num_params(self) -> int:
         W, S, n = self.hidden_size, self.streams, 2 * self.vocab_size * self.hidden_size + self.hidden_size
@@ -150,30 +243,49 @@ class HybridConfig(ModelConfig):
             n += la.mixer.params(W) + 2 * W * la.ff + sub * (W + S * (S + 2))
         return n
 
-    def active_params(self) -> int:
-        return self.num_params()
-
     def flops_per_token(self) -> int:
         W = self.hidden_size
         return 2 * (self.vocab_size * W + sum(la.mixer.macs(W) + 2 * W * la.ff for la in self.layers))
 
-    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
-        return sum(m.kv_heads * (m.dim + m.vdim) for m in self.attention) * dtype_bytes
 
-    def state_bytes_per_seq(self) -> int:
-        return sum(m.heads * m.dim * m.vdim for m in self.recurrent) * 4
+@dataclass(frozen=True)
+class RegesunConfig(HybridConfig):
+    """Regesun: windowed latent attention, selective state space and generalized delta rule, a norm
+    before and behind every sublayer with a layer scale, learned positions (``max_position`` of them),
+    clamped gated feed-forward."""
+
+    def num_params(self) -> int:
+        W = self.hidden_size
+        n = (2 * self.vocab_size + self.max_position + 1) * W
+        for la in self.layers:
+            n += la.mixer.params(W) + 3 * W * la.ff + 3 * W * (1 + bool(la.ff))
+        return n
+
+    def flops_per_token(self) -> int:
+        W = self.hidden_size
+        return 2 * (self.vocab_size * W + sum(la.mixer.macs(W) + 3 * W * la.ff for la in self.layers))
 
 
-def hybrid_config(name: str, vocab: int, width: int, layers, streams: int, embed_scale: float, logit_softcap: float,
-                  eps: float = 1e-5, **kw) -> HybridConfig:
+def _hybrid(cls, name: str, vocab: int, width: int, layers, eps: float, **kw):
+    """``cls`` over listed layers, the uniform fields from the largest attention layer."""
     layers = tuple(layers)
-    att = [la.mixer for la in layers if isinstance(la.mixer, AttentionSpec)]
-    return HybridConfig(
+    att = [la.mixer for la in layers if isinstance(la.mixer, (AttentionSpec, LatentAttentionSpec))]
+    return cls(
         name=name, vocab_size=vocab, hidden_size=width, intermediate_size=max((la.ff for la in layers), default=0),
         num_layers=len(layers), num_heads=max((m.heads for m in att), default=1),
-        num_kv_heads=max((m.kv_heads for m in att), default=1), head_dim=max((m.dim for m in att), default=64),
-        rms_eps=eps, layers=layers, streams=streams, embed_scale=embed_scale, logit_softcap=logit_softcap,
+        num_kv_heads=max((getattr(m, "kv_heads", 1) for m in att), default=1),
+        head_dim=max((m.dim for m in att), default=64), rms_eps=eps, layers=layers,
         **{"max_position": 131072, "eos_token_id": -1, **kw})
+
+
+def kosesun_config(name: str, vocab: int, width: int, layers, streams: int, embed_scale: float, logit_softcap: float,
+                   eps: float = 1e-5, **kw) -> KosesunConfig:
+    return _hybrid(KosesunConfig, name, vocab, width, layers, eps, streams=streams, embed_scale=embed_scale,
+                   logit_softcap=logit_softcap, **kw)
+
+
+def regesun_config(name: str, vocab: int, width: int, layers, max_position: int, eps: float = 1e-5, **kw) -> RegesunConfig:
+    return _hybrid(RegesunConfig, name, vocab, width, layers, eps, max_position=max_position, **kw)
 
 
 LLAMA3_8B = ModelConfig(
@@ -211,12 +323,12 @@ TINY_LLAMA_8H = replace(TINY_LLAMA, name="tiny-llama-8h", num_heads=8)
 TINY_MIXTRAL_8E = replace(TINY_MIXTRAL, name="tiny-mixtral-8e", num_experts=8)
 
 def _kosesun(name: str, width: int, ff: int, n_layers: int, vocab: int, heads: int, kv_heads: int, dim: int, vdim: int,
-             gla: GLASpec, **kw) -> HybridConfig:
+             gla: GLASpec, **kw) -> KosesunConfig:
     """One recurrent layer in three, attention elsewhere, four streams."""
     att = AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=dim ** -0.5, rot_base=500000.0,
                         rot_dims=dim // 2, v_mix=True)
     layers = [LayerSpec(gla if i % 3 == 1 else att, ff) for i in range(n_layers)]
-    return hybrid_config(name, vocab, width, layers, streams=4, embed_scale=width ** 0.5, logit_softcap=30.0, **kw)
+    return kosesun_config(name, vocab, width, layers, streams=4, embed_scale=width ** 0.5, logit_softcap=30.0, **kw)
 
 
 # layers of the size of the Llama-3 presets' (same width, query / key / value sizes, feed-forward
@@ -228,9 +340,31 @@ KOSESUN_1B = _kosesun("kosesun-1b", width=2048, ff=8192, n_layers=18, vocab=1282
 TINY_KOSESUN = _kosesun("tiny-kosesun", width=256, ff=384, n_layers=4, vocab=512, heads=6, kv_heads=2, dim=32, vdim=48,
                         gla=GLASpec(heads=3, dim=24, vdim=40, tau=8.0, rank=12), max_position=2048)
 
+
+def _regesun(name: str, width: int, ff: int, n_layers: int, vocab: int, ssd: SSDSpec, latent: LatentAttentionSpec,
+             delta: DeltaSpec, limit: float, max_position: int) -> RegesunConfig:
+    """State space, windowed latent attention and delta rule in turn, a feed-forward in every layer."""
+    mixers = (ssd, latent, delta)
+    return regesun_config(name, vocab, width, [LayerSpec(mixers[i % 3], ff, limit) for i in range(n_layers)], max_position)
+
+
+# layers of the size of the Kosesun presets' (same width, feed-forward parameters, vocabulary)
+REGESUN_8B = _regesun("regesun-8b", width=4096, ff=14336, n_layers=32, vocab=128256,
+                      ssd=SSDSpec(heads=64, vdim=128, state=128, groups=8, taps=4, norm_groups=8),
+                      latent=LatentAttentionSpec(heads=32, dim=128, vdim=128, rank=512, scale=128 ** -0.5, window=4096),
+                      delta=DeltaSpec(heads=32, dim=128, rank=64), limit=7.0, max_position=32768)
+REGESUN_1B = _regesun("regesun-1b", width=2048, ff=5376, n_layers=18, vocab=128256,
+                      ssd=SSDSpec(heads=64, vdim=64, state=128, groups=1, taps=4, norm_groups=1),
+                      latent=LatentAttentionSpec(heads=16, dim=128, vdim=64, rank=256, scale=128 ** -0.5, window=1024),
+                      delta=DeltaSpec(heads=32, dim=64, rank=32), limit=7.0, max_position=32768)
+TINY_REGESUN = _regesun("tiny-regesun", width=256, ff=320, n_layers=4, vocab=512,
+                        ssd=SSDSpec(heads=4, vdim=40, state=24, groups=2, taps=3, norm_groups=2),
+                        latent=LatentAttentionSpec(heads=5, dim=24, vdim=32, rank=72, scale=0.2, window=40),
+                        delta=DeltaSpec(heads=3, dim=56, rank=12), limit=2.0, max_position=2048)
+
 PRESETS = {c.name: c for c in (LLAMA3_8B, LLAMA3_70B, LLAMA31_8B, LLAMA31_70B, MIXTRAL_8X7B, TINY_LLAMA,
                                 TINY_MIXTRAL, TINY_LLAMA_8H, TINY_MIXTRAL_8E, KOSESUN_8B, KOSESUN_1B,
-                                TINY_KOSESUN)}
+                                TINY_KOSESUN, REGESUN_8B, REGESUN_1B, TINY_REGESUN)}
 # accepted aliases (MLflow tags / CR annotations use HF-ish names)
 ALIASES = {
     "meta-llama/Meta-Llama-3-8B": "llama3-8b", "llama-3-8b": "llama3-8b", "Llama-3-8B": "llama3-8b",

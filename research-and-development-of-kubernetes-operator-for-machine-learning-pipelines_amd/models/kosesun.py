@@ -23,33 +23,14 @@ import torch
 from .. import ops
 from ..parallel.comm import ParallelState, single
 from ..runtime.kv_cache import KVLayer, pad_dim
-from .config import AttentionSpec, HybridConfig
-from .layers import fuse_rows, linear, rope_table
+from .config import AttentionSpec, KosesunConfig
+from .layers import ParamSource, fuse_rows, linear, rope_table
 
 GLA_CHUNK = 64  # tokens of a recurrent layer's parallel prompt chunk (twice that in large steps)
 
 
-class _Source:
-    """Tensors by name: a checkpoint's, or random ones of the asked shape."""
-
-    def __init__(self, weights, device, dtype, seed: int):
-        self.w, self.device, self.dtype = weights, device, dtype
-        self.gen = torch.Generator(device=device)
-        self.gen.manual_seed(seed)
-
-    def __call__(self, name: str, *shape, dtype=None, mean: float = 0.0, std: float = 0.02) -> torch.Tensor:
-        dtype = dtype or self.dtype
-        if self.w is None:
-            t = torch.empty(shape, device=self.device, dtype=dtype)
-            return t.normal_(mean, std, generator=self.gen) if std else t.fill_(mean)
-        t = self.w.get(name)
-        if tuple(t.shape) != shape:
-            raise ValueError(f"checkpoint tensor {name!r} has shape {tuple(t.shape)}, expected {shape}")
-        return t.to(self.device, dtype).contiguous()
-
-
 class KosesunModel:
-    def __init__(self, cfg: HybridConfig, device="cuda", dtype=torch.bfloat16, pstate: ParallelState | None = None,
+    def __init__(self, cfg: KosesunConfig, device="cuda", dtype=torch.bfloat16, pstate: ParallelState | None = None,
                  seed: int = 0, weights=None):
         self.cfg = cfg
         self.device = torch.device(device)
@@ -58,7 +39,7 @@ class KosesunModel:
         if self.ps.tp.size > 1 or self.ps.ep.size > 1:
             raise ValueError("Kosesun runs on one GPU (no tensor / expert parallel form)")
         W, S = cfg.hidden_size, cfg.streams
-        src = _Source(weights, self.device, dtype, seed * 1000)
+        src = ParamSource(weights, self.device, dtype, seed * 1000)
         f32 = torch.float32
         self.embed = src("embed", cfg.vocab_size, W)
         self.layers, self.cache_layout, self.state_shapes = [], [], []

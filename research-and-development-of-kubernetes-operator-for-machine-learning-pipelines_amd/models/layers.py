@@ -62,3 +62,22 @@ def fuse_rows(parts, multiple: int = 16, large: int = 256) -> torch.Tensor:
     if pad:
         parts = [*parts, parts[0].new_zeros(pad, parts[0].shape[1])]
     return torch.cat(parts, 0).contiguous()
+
+
+class ParamSource:
+    """Tensors by name while a model is built: a checkpoint's, or random ones of the asked shape."""
+
+    def __init__(self, weights, device, dtype, seed: int):
+        self.w, self.device, self.dtype = weights, device, dtype
+        self.gen = torch.Generator(device=device)
+        self.gen.manual_seed(seed)
+
+    def __call__(self, name: str, *shape, dtype=None, mean: float = 0.0, std: float = 0.02) -> torch.Tensor:
+        dtype = dtype or self.dtype
+        if self.w is None:
+            t = torch.empty(shape, device=self.device, dtype=dtype)
+            return t.normal_(mean, std, generator=self.gen) if std else t.fill_(mean)
+        t = self.w.get(name)
+        if tuple(t.shape) != shape:
+            raise ValueError(f"checkpoint tensor {name!r} has shape {tuple(t.shape)}, expected {shape}")
+        return t.to(self.device, dtype).contiguous()

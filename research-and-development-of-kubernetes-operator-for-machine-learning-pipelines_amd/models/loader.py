@@ -18,8 +18,8 @@ Layout mapping (HF name -> ours; TP sharding then reuses ``load_shard_from``):
   Mixtral: block_sparse_moe.gate | mlp.gate      -> router
            experts.{e}.w1 / w3 (legacy) or experts.gate_up_proj (fused) -> w13 (interleaved)
            experts.{e}.w2 or experts.down_proj   -> w2
-Kosesun checkpoints (``"architecture": "Kosesun"``; tensors ``l<i>.mix.*`` ...) are read by the model
-itself as it is built (models/kosesun.py).
+Kosesun and Regesun checkpoints (``"architecture"`` in config.json; tensors ``l<i>.mix.*`` ...) are read
+by the model itself as it is built (models/kosesun.py, models/regesun.py).
 Tensors are read lazily, one layer at a time (safetensors memory map), so a 141 GB
 checkpoint never sits in host memory at once.
 """
@@ -32,7 +32,8 @@ from pathlib import Path
 
 import torch
 
-from .config import AttentionSpec, GLASpec, LayerSpec, ModelConfig, PRESETS, hybrid_config
+from .config import (AttentionSpec, DeltaSpec, GLASpec, LatentAttentionSpec, LayerSpec, ModelConfig, PRESETS, SSDSpec,
+                     kosesun_config, regesun_config)
 
 _ARCH_NAMES = {"LlamaForCausalLM": "llama", "MixtralForCausalLM": "mixtral", "MistralForCausalLM": "llama"}
 
@@ -106,7 +107,7 @@ def _only(d: dict, known: set, where: str) -> None:
 
 
 def config_from_kosesun(d: dict, shape_of, name: str | None = None, max_position: int | None = None) -> ModelConfig:
-    """HybridConfig from a Kosesun ``config.json`` dict.  ``shape_of(tensor name)``: sizes that only
+    """KosesunConfig from a Kosesun ``config.json`` dict.  ``shape_of(tensor name)``: sizes that only
     the checkpoint's tensors give (the decay projection's inner size).  Settings this runtime does
     not know are rejected, never dropped."""
     _only(d, {"architecture", "embedding", "layers", "logit_softcap", "norm", "streams", "vocab", "width"}, "config")
@@ -137,8 +138,52 @@ def config_from_kosesun(d: dict, shape_of, name: str | None = None, max_position
                 raise ValueError(f"layer {i}: unsupported feed-forward {mlp['kind']!r}")
         layers.append(LayerSpec(mixer, int(mlp["ff"]) if mlp is not None else 0))
     kw = {} if max_position is None else {"max_position": max_position}
-    return hybrid_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers, int(d["streams"]),
+    return kosesun_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers, int(d["streams"]),
                          float(d["embedding"]["scale"]), float(d["logit_softcap"]), float(d["norm"]["eps"]), **kw)
+
+
+def config_from_regesun(d: dict, shape_of, name: str | None = None) -> ModelConfig:
+    """RegesunConfig from a Regesun ``config.json`` dict.  ``shape_of(tensor name)``: sizes that only the
+    checkpoint's tensors give (the decay projection's inner size).  Settings this runtime does not know
+    are rejected, never dropped."""
+    _only(d, {"architecture", "layers", "max_positions", "norm", "vocab", "width"}, "config")
+    _only(d["norm"], {"eps"}, "norm")
+    layers = []
+    for i, la in enumerate(d["layers"]):
+        _only(la, {"type", "mixer", "mlp"}, f"layer {i}")
+        m, mlp = la["mixer"], la.get("mlp")
+        if la["type"] == "latent_attention":
+            _only(m, {"dim", "heads", "kv_rank", "mask", "scale", "vdim"}, f"layer {i} mixer")
+            mask = m.get("mask") or {"size": 0}
+            _only(mask, {"size"}, f"layer {i} mask")
+            mixer = LatentAttentionSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                        rank=int(m["kv_rank"]), scale=float(m["scale"]), window=int(mask["size"]))
+            if mixer.scale <= 0 or mixer.window < 0:
+                raise ValueError(f"layer {i}: unsupported attention settings {m}")
+        elif la["type"] == "mamba2":
+            _only(m, {"conv", "groups", "heads", "norm_groups", "state", "vdim"}, f"layer {i} mixer")
+            mixer = SSDSpec(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
+                            taps=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+            if mixer.heads % mixer.groups or mixer.inner % mixer.norm_groups or mixer.taps < 1:
+                raise ValueError(f"layer {i}: unsupported state-space sizes {m}")
+        elif la["type"] == "general_delta":
+            _only(m, {"dim", "heads"}, f"layer {i} mixer")
+            mixer = DeltaSpec(heads=int(m["heads"]), dim=int(m["dim"]), rank=int(shape_of(f"l{i}.mix.w1")[0]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {la['type']!r}")
+        if mlp is not None:
+            _only(mlp, {"ff", "kind", "limit"}, f"layer {i} mlp")
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unsupported feed-forward {mlp['kind']!r}")
+            if float(mlp["limit"]) <= 0:
+                raise ValueError(f"layer {i}: the feed-forward's limit must be positive")
+        layers.append(LayerSpec(mixer, int(mlp["ff"]), float(mlp["limit"])) if mlp is not None else LayerSpec(mixer))
+    return regesun_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers, int(d["max_positions"]),
+                          float(d["norm"]["eps"]))
+
+
+# config.json's "architecture" -> its reader
+_HYBRIDS = {"Kosesun": config_from_kosesun, "Regesun": config_from_regesun}
 
 
 class _Tensors:
@@ -229,16 +274,16 @@ class HFWeights:
 def load_pretrained(path: str | os.PathLike, device="cuda", dtype=torch.bfloat16, pstate=None,
                     name: str | None = None, fold_norms: bool = True):
     """Build our model for the checkpoint in ``path`` and copy its (TP-sharded) weights in.  The
-    model class follows from config.json: ``architecture`` (Kosesun) or HF's ``architectures``."""
+    model class follows from config.json: ``architecture`` (Kosesun, Regesun) or HF's ``architectures``."""
     from . import build_model
 
     path = Path(path)
     d = json.loads((path / "config.json").read_text())
     if "architecture" in d:
-        if d["architecture"] != "Kosesun":
-            raise ValueError(f"unsupported checkpoint architecture {d['architecture']!r}")
+        if d["architecture"] not in _HYBRIDS:
+            raise ValueError(f"unsupported checkpoint architecture {d['architecture']!r} (supported: {sorted(_HYBRIDS)})")
         t = _Tensors(path)
-        cfg = config_from_kosesun(d, t.shape, name=name or path.name)
+        cfg = _HYBRIDS[d["architecture"]](d, t.shape, name=name or path.name)
         return build_model(cfg, device=device, dtype=dtype, pstate=pstate, weights=t)
     cfg = config_from_hf(d, name=name or path.name)
     model = build_model(cfg, device=device, dtype=dtype, pstate=pstate)

@@ -182,17 +182,20 @@ def paged_attention(q, k_cache, v_cache, meta, out: torch.Tensor | None = None):
 EPI_NONE, EPI_SILU_MUL, EPI_RELU2 = 0, 1, 6
 
 
-def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi: int = EPI_NONE):
+def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi: int = EPI_NONE,
+         glu: tuple | None = None):
     """y = epi(x @ w^T), w [N, K] bf16.  EPI_SILU_MUL expects gate/up rows
-    interleaved in groups of 16 (``interleave_gate_up``) and returns N/2 columns; EPI_RELU2 is
-    max(y, 0)^2."""
+    interleaved in groups of 16 (``interleave_gate_up``) and returns N/2 columns; with ``glu`` =
+    (alpha, limit) it is the clamped gated unit g sigmoid(alpha g) (u + 1) of g = min(gate, limit),
+    u = clamp(up, -limit, limit) instead.  EPI_RELU2 is max(y, 0)^2."""
     N = w.shape[0]
     out_n = N // 2 if epi == EPI_SILU_MUL else N
     if not x.is_cuda:
         y = torch.nn.functional.linear(x, w) if x.dtype != torch.bfloat16 else \
             torch.nn.functional.linear(x.float(), w.float()).to(x.dtype)
         if epi == EPI_SILU_MUL:
-            y = ref.silu_mul(deinterleave_cols(y))
+            y = deinterleave_cols(y)
+            y = ref.silu_mul(y) if glu is None else ref.clamp_glu(y, *glu)
         elif epi == EPI_RELU2:
             y = ref.relu2(y)
         if out is not None:
@@ -206,28 +209,33 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
         x2 = x2.contiguous()
     M, K = x2.shape
     o2 = torch.empty(M, out_n, dtype=x.dtype, device=x.device) if out is None else out.view(M, out_n)
-    if x.dtype == torch.float32 and epi != EPI_SILU_MUL:  # true fp32 (library product; no reduced-precision mode)
-        _gemm_hipblaslt(x2, w, o2, epi)
+    if x.dtype == torch.float32 and (epi != EPI_SILU_MUL or glu):  # true fp32 (library product; no reduced-precision mode)
+        _gemm_hipblaslt(x2, w, o2, epi, glu)
         return o2.view(*lead, out_n) if out is None else out
-    _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi)
+    _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi, glu)
     return o2.view(*lead, out_n) if out is None else out
 
 
-def _gemm_mlop(x2, w, o2, epi):
+def _gemm_mlop(x2, w, o2, epi, glu=None):
     _sk_reserve(x2.device)
     M, K = x2.shape
     nws = torch.ops.mlop.gemm_workspace(M, w.shape[0], K, epi)
     ws = torch.empty(max(nws, 1), dtype=torch.float32, device=x2.device) if nws else _EMPTY.get(x2.device)
-    torch.ops.mlop.gemm(o2, x2, w, ws, epi)
+    if glu is None:
+        torch.ops.mlop.gemm(o2, x2, w, ws, epi)
+    else:
+        torch.ops.mlop.gemm(o2, x2, w, ws, epi, *glu)
 
 
-def _gemm_hipblaslt(x2, w, o2, epi):
-    """Plain library GEMM (hipBLASLt via torch.matmul); the SiLU-mul epilogue
-    then runs as the separate interleaved silu_mul kernel."""
+def _gemm_hipblaslt(x2, w, o2, epi, glu=None):
+    """Plain library GEMM (hipBLASLt via torch.matmul); the SiLU-mul epilogue (or the clamped gated
+    unit) then runs as a separate kernel on the interleaved columns."""
     if epi != EPI_SILU_MUL:
         torch.matmul(x2, w.t(), out=o2)
         if epi == EPI_RELU2:
             torch.ops.mlop.relu2(o2)
+    elif glu is not None:
+        torch.ops.mlop.clamp_glu(o2, torch.matmul(x2, w.t()), *glu)
     else:
         torch.ops.mlop.silu_mul(o2, torch.matmul(x2, w.t()), 1)
 
@@ -781,7 +789,8 @@ def qk_norm_rope(proj, n_heads: int, dim: int, vdim: int, q_w, k_w, eps: float, 
 
 def attention_hd(q, k_cache, v_cache, meta, dim: int, vdim: int, scale: float, sink=None, gate=None):
     """Ragged causal paged attention of any head sizes: q [T, H, KP] -> [T, H, vdim].  ``sink`` [H] joins
-    each head's softmax denominator; ``gate`` [T, H]: the head's output times sigmoid(gate)."""
+    each head's softmax denominator; ``gate`` [T, H]: the head's output times sigmoid(gate).  (Windows,
+    gates per element and dense keys: ``latent_attention``.)"""
     if not q.is_cuda:
         return ref.attention_hd(q, k_cache, v_cache, meta, dim, vdim, scale, sink, gate)
     _need_gpu()
@@ -802,6 +811,124 @@ def gla(proj, n_heads: int, dim: int, vdim: int, a2, a2_b, norm_w, tau: float, e
     torch.ops.mlop.gla(out, state, proj, n_heads, dim, vdim, a2, a2_b, norm_w, tau, eps, meta.q_start, meta.q_len,
                        meta.ctx_len, meta.tile_seq, meta.citem_seq, meta.citem_t0, meta.crow_seq, meta.crow_item0,
                        meta.chunk)
+    return out
+
+
+def residual_begin(ids, table, scale: float, pos_table, positions, norm_w, eps: float):
+    """fp32 residual x = scale table[id] + pos_table[position] (``pos_table`` None: none) and the first
+    sublayer's input norm_w x / rms(x) in the table's dtype."""
+    if not table.is_cuda:
+        return ref.residual_begin(ids, table, scale, pos_table, positions, norm_w, eps)
+    _need_gpu()
+    x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=table.device)
+    xn = torch.empty(x.shape, dtype=table.dtype, device=table.device)
+    torch.ops.mlop.residual_begin(xn, x, ids, table, scale, pos_table, positions, norm_w, eps)
+    return x, xn
+
+
+def residual_step(x, y, post_w, norm_w, eps: float, store: bool = True):
+    """x <- x + post_w y / rms(y) (``post_w`` None: x + y), in place unless ``store`` is off (nothing reads it
+    again); returns the next sublayer's input norm_w x / rms(x)."""
+    if not y.is_cuda:
+        return ref.residual_step(x, y, post_w, norm_w, eps)
+    _need_gpu()
+    xn = torch.empty_like(y)
+    torch.ops.mlop.residual_step(xn, x, y, post_w, norm_w, eps, store)
+    return xn
+
+
+def gated_norm(y, gate, w, groups: int, eps: float, act: str, gate_first: bool):
+    """y [T, n] in ``groups`` equal parts, each divided by its own root mean square, times w; times
+    act(gate) (``act``: "silu" or "sigmoid") before the norm (``gate_first``) or behind it."""
+    if not y.is_cuda:
+        return ref.gated_norm(y, gate, w, groups, eps, act == "silu", gate_first)
+    _need_gpu()
+    out = torch.empty_like(y)
+    torch.ops.mlop.gated_norm(out, y, gate, w, groups, eps, ("silu", "sigmoid").index(act), gate_first)
+    return out
+
+
+def _step_rows(meta):
+    return (meta.q_start, meta.q_len, meta.ctx_len, meta.tile_seq, meta.citem_seq, meta.citem_t0, meta.crow_seq,
+            meta.crow_item0, meta.chunk)
+
+
+def short_conv(x, w, b, tail, meta):
+    """silu of a causal convolution per channel: x [T, C], w [C, taps] fp32 (last column: the current
+    token), b [C] or None; ``tail`` [slots, taps - 1, C] fp32 holds each sequence's last inputs."""
+    if not x.is_cuda:
+        return ref.short_conv(x, w, b, tail, meta)
+    _need_gpu()
+    out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    torch.ops.mlop.short_conv(out, tail, x, w, b, *_step_rows(meta))
+    return out
+
+
+def ssd(xbc, dt, groups: int, dt_bias, a_neg, d_skip, state, meta):
+    """Selective state space of a ragged step: xbc [T, H V + 2 G N] = [x | B | C], dt [T, H] before bias and
+    softplus -> [T, H V]; ``state`` [slots, H, N, V] fp32 (slot = sequence row) is advanced."""
+    if not xbc.is_cuda:
+        return ref.ssd(xbc, dt, groups, dt_bias, a_neg, d_skip, state, meta)
+    _need_gpu()
+    y = torch.empty(xbc.shape[0], state.shape[1] * state.shape[3], dtype=xbc.dtype, device=xbc.device)
+    torch.ops.mlop.ssd(y, state, xbc, dt, groups, dt_bias, a_neg, d_skip, *_step_rows(meta))
+    return y
+
+
+def delta(proj, w2, w0, a_b, decay_scale: float, unit_eps: float, state, meta):
+    """Generalized delta rule of a ragged step: proj [T, ...] = [r | k | v | a | w1 | ...] -> [T, H dv] before
+    norm and gate; ``state`` [slots, H, dk, dv] fp32 (slot = sequence row) is advanced."""
+    if not proj.is_cuda:
+        return ref.delta(proj, w2, w0, a_b, decay_scale, unit_eps, state, meta)
+    _need_gpu()
+    o = torch.empty(proj.shape[0], state.shape[1] * state.shape[3], dtype=proj.dtype, device=proj.device)
+    torch.ops.mlop.delta(o, state, proj, w2, w0, a_b, decay_scale, unit_eps, *_step_rows(meta))
+    return o
+
+
+def latent_store(latents, w, eps: float, slots, cache):
+    """w l / rms(l) of the step's latents [T, R] into their cache slots ([NB, 1, BS, RP])."""
+    if not latents.is_cuda:
+        return ref.latent_store(latents, w, eps, slots, cache)
+    _need_gpu()
+    torch.ops.mlop.latent_store(cache, latents, w, eps, slots)
+
+
+def latent_attention(q, gate, cache, w_kv, w_qk, w_vo, vdim: int, scale: float, window: int, sink, meta):
+    """Ragged attention over cached latents: q [T, H, KP] -> [T, H vdim].  A head's keys and values are linear
+    in a latent row: ``w_kv`` [H (KP + VP), RP] expands a portion's keys and values; decoded tokens stay in the
+    latent space, with ``w_qk`` [H, RP, KP] (the keys' map, transposed) on the query and ``w_vo`` [H, vdim,
+    RP] (the values' map) on the result.  ``window``: tokens a token sees (0: all); ``sink`` [H] joins each
+    head's denominator; ``gate`` [T, H vdim]: the result times sigmoid(gate)."""
+    T, H, KP = q.shape
+    if not q.is_cuda:
+        return ref.latent_attention(q, gate, cache, w_kv, H, vdim, scale, window, sink, meta)
+    _need_gpu()
+    from ..runtime.attn_meta import plan_partitions
+
+    op, dev = torch.ops.mlop, q.device
+    out = torch.empty(T, H * vdim, dtype=q.dtype, device=dev)
+    step = (meta.q_start, meta.q_len, meta.ctx_len)
+    none = meta.tile_seq[:0]
+    nt, RP = meta.tile_seq.numel(), cache.shape[3]
+    if nt:
+        ql = torch.empty(nt, H, RP, dtype=q.dtype, device=dev)
+        op.head_mm(ql, q, w_qk, meta.tile_seq, meta.tile_q0, meta.q_start, meta.q_len, True, False, None)
+        ol = torch.empty_like(ql)
+        keys = meta.part_tokens * meta.nparts
+        part, nparts = plan_partitions(nt, -(-H // 16), min(keys, window + 31) if window else keys)
+        op.attention_hd(ol, meta.part_o, meta.part_ml, meta.part_sem, ql, cache, cache, meta.block_tables, meta.tile_seq,
+                        meta.tile_q0, none, none, *step, RP, scale, sink, None, part, nparts, window, None, True)
+        op.head_mm(out.view(T, H, vdim), ol, w_vo, meta.tile_seq, meta.tile_q0, meta.q_start, meta.q_len, False, True, gate)
+    if meta.ptile_seq.numel():
+        rows = torch.empty(meta.x_rows + 32, RP, dtype=q.dtype, device=dev)
+        op.latent_gather(rows, cache, meta.block_tables, meta.xbase, meta.q_len, meta.ctx_len, meta.crow_seq, meta.x_rows,
+                         meta.x_max, meta.x_window)
+        kv = gemm(rows, w_kv)
+        VP = kv.shape[1] // H - KP
+        k, v = kv[:, :H * KP].unflatten(1, (H, KP)), kv[:, H * KP:].unflatten(1, (H, VP))
+        op.attention_hd(out.view(T, H, vdim), meta.part_o, meta.part_ml, meta.part_sem, q, k, v, meta.block_tables, none,
+                        none, meta.ptile_seq, meta.ptile_q0, *step, KP, scale, sink, gate, 32, 1, window, meta.xbase, False)
     return out
 
 

@@ -11,7 +11,10 @@
 //     decode tile is one token with up to 16 heads of a kv head as MFMA rows (more heads take
 //     further workgroups), a prompt tile is 128 tokens of ONE head;
 //   * sink: a number per head that joins the softmax's denominator once, with no key and no value;
-//   * gate: head h's output times sigmoid(gate[t, h]), in the epilogue.
+//   * gate: head h's output times sigmoid(gate[t, h]), or an element's with its own gate, in the epilogue;
+//   * window: a token sees itself and the window - 1 tokens before it; pages in front are not read;
+//   * a prompt's keys and values may also come from dense rows (latent attention's expanded keys), and
+//     decode's keys and values may be the same rows (its latents).
 // The sizes above 256 and fp32 operands take attn_any_kernel (one wave per query and head).
 //
 // REQUIREMENT: the cache is zero-initialised at allocation (as attention.hip's) and the pad
@@ -43,9 +46,22 @@ __device__ __forceinline__ uint32_t pk_bf16(float lo, float hi) {
   return r;
 }
 __device__ __forceinline__ float gate_of(const AttnHdArgs& a, int tok, int head) {
-  if (!a.gate) return 1.f;
+  if (!a.gate || a.gate_elem) return 1.f;
   const float g = bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)tok * a.gate_stride + head]);
   return 1.f / (1.f + __expf(-g));
+}
+
+// an element's own gate
+__device__ __forceinline__ float gate_at(const AttnHdArgs& a, int tok, int head, int c) {
+  const float g = bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)tok * a.gate_stride + head * a.V + c]);
+  return 1.f / (1.f + __expf(-g));
+}
+template <int N>
+__device__ __forceinline__ void gate_elems(const AttnHdArgs& a, int tok, int head, int c, float (&v)[N]) {
+  if (!a.gate || !a.gate_elem) return;
+#pragma unroll
+  for (int j = 0; j < N; ++j)
+    if (c + j < a.V) v[j] *= gate_at(a, tok, head, c + j);
 }
 
 // 8 consecutive outputs of a head, dims c .. c + 7 (only those below V)
@@ -88,13 +104,16 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
   const int* bt = a.bt + (size_t)s * a.bt_stride;
   const bool live = qi < ql;
   const int kv_end = live ? max(0, ctx - ql + qi + 1) : 0;
-  const int p_begin = part * part_tokens;
+  const int orow = a.by_tile ? tile : tok;  // row of q and out
+  // keys [k_lo, kv_end) in partitions counted from k_lo's page pair
+  const int k_lo = a.window > 0 ? max(0, kv_end - a.window) : 0, k_base = k_lo & ~31;
+  const int p_begin = k_base + part * part_tokens;
   const int p_end = min(kv_end, p_begin + part_tokens);
   if (p_begin >= p_end && nparts > 1) {
     // no partition of an empty row (graph padding) draws the last ticket: partition 0 zeroes it
     if (part == 0 && kv_end <= 0 && live) {
       for (int e = threadIdx.x; e < nh * a.V; e += 256)
-        out[((size_t)tok * a.H + head0 + e / a.V) * a.V + e % a.V] = 0;
+        out[((size_t)orow * a.H + head0 + e / a.V) * a.V + e % a.V] = 0;
     }
     return;
   }
@@ -103,7 +122,7 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
   const bool row_ok = live && r < nh;
   bf16x8 qf[NK];
   {
-    const uint16_t* qrow = reinterpret_cast<const uint16_t*>(a.q) + ((size_t)tok * a.H + head0 + (row_ok ? r : 0)) * KP;
+    const uint16_t* qrow = reinterpret_cast<const uint16_t*>(a.q) + (size_t)orow * a.q_row + (head0 + (row_ok ? r : 0)) * a.q_head;
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
       const bf16x8 v = live ? *reinterpret_cast<const bf16x8*>(qrow + kk * 32 + g4 * 8) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
@@ -164,8 +183,8 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
     float pa[4], pb[4], mx = kLow;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      pa[i] = tokA + i < p_end ? sa[i] * a.scale_log2 : -INFINITY;
-      pb[i] = tokB + i < p_end ? sb[i] * a.scale_log2 : -INFINITY;
+      pa[i] = tokA + i < p_end && tokA + i >= k_lo ? sa[i] * a.scale_log2 : -INFINITY;
+      pb[i] = tokB + i < p_end && tokB + i >= k_lo ? sb[i] * a.scale_log2 : -INFINITY;
       mx = fmaxf(mx, fmaxf(pa[i], pb[i]));
     }
     mx = max_x16_x32(mx);
@@ -235,7 +254,8 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
       const float inv = L > 0.f ? gate_of(a, tok, head0 + rr) / L : 0.f;
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[j] *= inv;
-      store8(out + ((size_t)tok * a.H + head0 + rr) * a.V, c, a.V, acc);
+      gate_elems(a, tok, head0 + rr, c, acc);
+      store8(out + ((size_t)orow * a.H + head0 + rr) * a.V, c, a.V, acc);
     } else {
       // partial (O, m, l) of this key range, stored through to the memory side (sc1) so that the
       // ticket below needs no release fence
@@ -261,7 +281,7 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
   // the partition that draws the last ticket combines all of them and re-arms the counter
   // (attention.hip's hand-off: sc1 stores, vmcnt(0) in every wave, barrier, relaxed ticket,
   // agent acquire on the consumer's side)
-  const int nvalid = min(nparts, (kv_end + part_tokens - 1) / part_tokens);
+  const int nvalid = min(nparts, (kv_end - k_base + part_tokens - 1) / part_tokens);
   int* cnt = sem + (size_t)tile * ny + blockIdx.y;
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   __syncthreads();
@@ -296,7 +316,8 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
     const float inv = L > 0.f ? gate_of(a, tok, head0 + rr) / L : 0.f;
 #pragma unroll
     for (int j = 0; j < 8; ++j) acc[j] *= inv;
-    store8(out + ((size_t)tok * a.H + head0 + rr) * a.V, c, a.V, acc);
+    gate_elems(a, tok, head0 + rr, c, acc);
+    store8(out + ((size_t)orow * a.H + head0 + rr) * a.V, c, a.V, acc);
   }
 }
 
@@ -323,18 +344,22 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
   const int last_q = min(q0 + kHdTile, ql) - 1;
   const int kv_end = ctx - ql + last_q + 1;
   const int n_pairs = (kv_end + 31) >> 5;
+  const int pp0 = a.window > 0 ? max(0, ctx - ql + q0 - a.window + 1) >> 5 : 0;  // first pair a query sees
   const int n_pages = (kv_end + kPg - 1) / kPg;
   const int col = lane & 31, h = lane >> 5;
   const int qi = q0 + 32 * wid + col;
   const bool q_ok = qi < ql;
   const int pos_r = q_ok ? ctx - ql + qi : -1;
+  const int low_r = a.window > 0 ? pos_r - a.window + 1 : 0;  // first key of this row
   // positions of this wave's rows: pairs past the last are masked whole, pairs up to the first need no mask
   const bool wave_live = q0 + 32 * wid < ql;
   const int wave_min = ctx - ql + q0 + 32 * wid, wave_max = min(wave_min + 31, kv_end - 1);
+  // first key any row of the wave sees, first key all of them see
+  const int wave_low = a.window > 0 ? wave_min - a.window + 1 : 0, wave_in = a.window > 0 ? wave_max - a.window + 1 : 0;
 
   bf16x8 qf[NQ];
   {
-    const uint16_t* qrow = reinterpret_cast<const uint16_t*>(a.q) + ((size_t)(qs + (q_ok ? qi : 0)) * a.H + head) * KP + 8 * h;
+    const uint16_t* qrow = reinterpret_cast<const uint16_t*>(a.q) + (size_t)(qs + (q_ok ? qi : 0)) * a.q_row + head * a.q_head + 8 * h;
 #pragma unroll
     for (int t = 0; t < NQ; ++t) {
       const bf16x8 v = *reinterpret_cast<const bf16x8*>(qrow + 16 * t);
@@ -349,19 +374,19 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
   float m = kLow, l = 0.f;
 
   const int* bt = a.bt + (size_t)s * a.bt_stride;
-  const size_t k_page = (size_t)a.G * kPg * KP, v_page = (size_t)a.G * kPg * VP;
+  const int xb = a.xbase ? a.xbase[s] : 0;
   // LDS-DMA: wave w brings rows 8w .. 8w + 7 of every block (page A: waves 0, 1; page B: 2, 3)
   const int row32 = 8 * wid + (lane >> 3), row = row32 & 15;
-  const size_t k_off = (size_t)kvh * kPg * KP + row * KP + (((lane & 7) ^ ((row32 >> 1) & 7)) << 3);
-  const size_t v_off = (size_t)kvh * kPg * VP + row * VP + (((lane & 7) ^ vsw(row)) << 3);
-  auto page_of = [&](int pair) {
+  const size_t k_off = kvh * a.k_head + row * a.k_row + (((lane & 7) ^ ((row32 >> 1) & 7)) << 3);
+  const size_t v_off = kvh * a.v_head + row * a.v_row + (((lane & 7) ^ vsw(row)) << 3);
+  auto page_of = [&](int pair) {  // first row of this wave's page
     const int i = min(2 * pair + (wid >> 1), n_pages - 1);
-    return min(max(bt[i], 0), a.num_blocks - 1);
+    return a.xbase ? xb + i * kPg : min(max(bt[i], 0), a.num_blocks - 1) * kPg;
   };
   auto issue = [&](int buf, int pg) {
     uint16_t* base = smem + buf * (STAGE / 2) + wid * 512;
-    const uint16_t* ks = kc + pg * k_page + k_off;
-    const uint16_t* vs = vc + pg * v_page + v_off;
+    const uint16_t* ks = kc + pg * a.k_pitch + k_off;
+    const uint16_t* vs = vc + pg * a.v_pitch + v_off;
 #pragma unroll
     for (int b = 0; b < NKB; ++b)
       __builtin_amdgcn_global_load_lds((const void*)(ks + b * 64), (lds_void_t*)(base + b * 2048), 16, 0, 0);
@@ -413,12 +438,12 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
     return sc;
   };
   auto softmax = [&](f32x16 sc, int pp, bf16x8 (&pf)[2]) {
-    if (pp * 32 + 31 > wave_min) {
-      asm volatile("");  // keep the branch: the mask is needed on the diagonal only
+    if (pp * 32 + 31 > wave_min || pp * 32 < wave_in) {
+      asm volatile("");  // keep the branch: the mask is needed on the diagonal and at the window's edge only
 #pragma unroll
       for (int e = 0; e < 16; ++e) {
         const int tk = pp * 32 + (e & 3) + 8 * (e >> 2) + 4 * h;
-        sc[e] = tk <= pos_r ? sc[e] : -INFINITY;
+        sc[e] = tk <= pos_r && tk >= low_r ? sc[e] : -INFINITY;
       }
     }
     float mx = fmaxf(fmaxf(sc[0], sc[1]), sc[2]);
@@ -489,11 +514,11 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
     }
   };
 
-  issue(0, page_of(0));
-  if (n_pairs > 1) issue(1, page_of(1));
-  int nxt = page_of(2);
+  issue(0, page_of(pp0));
+  if (n_pairs - pp0 > 1) issue(1, page_of(pp0 + 1));
+  int nxt = page_of(pp0 + 2);
   int buf = 0;
-  for (int pp = 0; pp < n_pairs; ++pp) {
+  for (int pp = pp0; pp < n_pairs; ++pp) {
     if (pp + 1 < n_pairs) wait_vmcnt<OPS>(); else wait_vmcnt<0>();
     raw_barrier();  // pair pp visible to every wave; the slot consumed one step ago is free
     if (pp + 2 < n_pairs) {
@@ -501,7 +526,7 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
       issue(to, nxt);
       nxt = page_of(pp + 3);
     }
-    if (wave_live && pp * 32 <= wave_max) {
+    if (wave_live && pp * 32 <= wave_max && pp * 32 + 31 >= wave_low) {
       bf16x8 pf[2];
       const uint32_t so = buf * STAGE;
       softmax(qk(so), pp, pf);
@@ -530,7 +555,8 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
       const int c = 32 * d + 8 * b + 4 * h;
-      const float v[4] = {o[d][4 * b] * inv, o[d][4 * b + 1] * inv, o[d][4 * b + 2] * inv, o[d][4 * b + 3] * inv};
+      float v[4] = {o[d][4 * b] * inv, o[d][4 * b + 1] * inv, o[d][4 * b + 2] * inv, o[d][4 * b + 3] * inv};
+      gate_elems(a, qs + qi, head, c, v);
       if (v4) {
         if (c < a.V) stn<4>(orow + c, v);
       } else {
@@ -554,10 +580,11 @@ __global__ void __launch_bounds__(256) attn_any_kernel(AttnHdArgs a, const int* 
   const int qi = tile_q0[tile] + sub;
   const int ql = a.q_len[s], ctx = a.ctx_len[s];
   if (sub >= tile_tokens || qi >= ql) return;  // whole waves; no barrier below
-  const int tok = a.q_start[s] + qi, n_keys = max(0, ctx - ql + qi + 1);
+  const int tok = a.q_start[s] + qi, n_keys = max(0, ctx - ql + qi + 1), orow = a.by_tile ? tile : tok;
+  const int k_lo = a.window > 0 ? max(0, n_keys - a.window) : 0;
   const E* kc = reinterpret_cast<const E*>(a.k_cache);
   const E* vc = reinterpret_cast<const E*>(a.v_cache);
-  const E* q = reinterpret_cast<const E*>(a.q) + ((size_t)tok * a.H + head) * a.KP;
+  const E* q = reinterpret_cast<const E*>(a.q) + (size_t)orow * a.q_row + head * a.q_head;
   float* qs = sm_q + wid * a.D;
   for (int d = lane; d < a.D; d += 64) qs[d] = ld1(q + d);
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
@@ -567,11 +594,10 @@ __global__ void __launch_bounds__(256) attn_any_kernel(AttnHdArgs a, const int* 
 #pragma unroll
   for (int i = 0; i < kHdMaxV / 64; ++i) acc[i] = 0.f;
   float m = kLow, l = 0.f;
-  for (int k0 = 0; k0 < n_keys; k0 += 64) {
+  for (int k0 = k_lo; k0 < n_keys; k0 += 64) {
     const int key = min(k0 + lane, n_keys - 1), n = min(64, n_keys - k0);
-    const int pg = min(max(bt[key / kPg], 0), a.num_blocks - 1);
-    const size_t line = ((size_t)pg * a.G + kvh) * kPg + key % kPg;
-    const E* kr = kc + line * a.KP;
+    const int line = a.xbase ? a.xbase[s] + key : min(max(bt[key / kPg], 0), a.num_blocks - 1) * kPg + key % kPg;
+    const E* kr = kc + line / kPg * (kPg * a.k_pitch) + line % kPg * a.k_row + kvh * a.k_head;
     float dot = 0.f;
     for (int d = 0; d < a.D; ++d) dot = fmaf(qs[d], ld1(kr + d), dot);
     const float sc = lane < n ? dot * a.scale_log2 : -INFINITY;
@@ -583,8 +609,8 @@ __global__ void __launch_bounds__(256) attn_any_kernel(AttnHdArgs a, const int* 
     for (int i = 0; i < kHdMaxV / 64; ++i) acc[i] *= alpha;
     for (int j = 0; j < n; ++j) {
       const float pj = __shfl(p, j);
-      const size_t lj = (size_t)__shfl((int)line, j);
-      const E* vr = vc + lj * a.VP;
+      const int lj = __shfl(line, j);
+      const E* vr = vc + lj / kPg * (kPg * a.v_pitch) + lj % kPg * a.v_row + kvh * a.v_head;
 #pragma unroll
       for (int i = 0; i < kHdMaxV / 64; ++i)
         if (i * 64 + lane < a.V) acc[i] = fmaf(pj, ld1(vr + i * 64 + lane), acc[i]);
@@ -597,11 +623,14 @@ __global__ void __launch_bounds__(256) attn_any_kernel(AttnHdArgs a, const int* 
     l = l * f + exp2f(s2 - M);
   }
   float inv = l > 0.f ? f / l : 0.f;
-  if (a.gate) inv /= 1.f + expf(-ld1(reinterpret_cast<const E*>(a.gate) + (size_t)tok * a.gate_stride + head));
-  E* orow = reinterpret_cast<E*>(a.out) + ((size_t)tok * a.H + head) * a.V;
+  const E* gate = reinterpret_cast<const E*>(a.gate) + (size_t)tok * a.gate_stride;
+  if (a.gate && !a.gate_elem) inv /= 1.f + expf(-ld1(gate + head));
+  E* dst = reinterpret_cast<E*>(a.out) + ((size_t)orow * a.H + head) * a.V;
 #pragma unroll
-  for (int i = 0; i < kHdMaxV / 64; ++i)
-    if (i * 64 + lane < a.V) st1(orow + i * 64 + lane, acc[i] * inv);
+  for (int i = 0; i < kHdMaxV / 64; ++i) {
+    const int c = i * 64 + lane;
+    if (c < a.V) st1(dst + c, a.gate && a.gate_elem ? acc[i] * inv / (1.f + expf(-ld1(gate + head * a.V + c))) : acc[i] * inv);
+  }
 }
 
 template <typename E>
@@ -630,10 +659,20 @@ void launch_paged_hd(const AttnHdArgs& a, bool f32, float* part_o, float* part_m
                      const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st) {
   if (num_tiles == 0) return;
   if (f32) return run_any<float>(a, tile_seq, tile_q0, num_tiles, 1, st);
-  if (a.KP > kHdMaxDim || a.VP > kHdMaxDim) return run_any<uint16_t>(a, tile_seq, tile_q0, num_tiles, 1, st);
+  const bool latent = a.KP == a.VP && a.KP <= kHdMaxLatent;
+  if ((a.KP > kHdMaxDim || a.VP > kHdMaxDim) && !latent) return run_any<uint16_t>(a, tile_seq, tile_q0, num_tiles, 1, st);
   const dim3 grid(num_tiles, a.G * cdiv(a.H / a.G, 16), nparts);
 #define MLOP_RUN(K, V) \
   paged_hd_kernel<K, V><<<grid, 256, 0, st>>>(a, part_o, part_ml, sem, tile_seq, tile_q0, part_tokens, nparts)
+  if (a.KP > kHdMaxDim) {
+    switch (a.KP / 64) {
+      case 5: MLOP_RUN(5, 5); break;
+      case 6: MLOP_RUN(6, 6); break;
+      case 7: MLOP_RUN(7, 7); break;
+      default: MLOP_RUN(8, 8); break;
+    }
+    return;
+  }
   MLOP_HD(MLOP_RUN)
 #undef MLOP_RUN
 }

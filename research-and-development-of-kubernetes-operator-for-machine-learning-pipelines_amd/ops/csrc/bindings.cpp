@@ -264,7 +264,7 @@ int64_t gemm_workspace(int64_t M, int64_t N, int64_t K, int64_t epi) {
 }
 
 // out[M, N or N/2] = epi(a[M, K] . w[N, K]^T)
-void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi) {
+void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi, double glu_alpha, double glu_limit) {
   TORCH_CHECK(a.is_cuda() && a.scalar_type() == at::kBFloat16 && a.dim() == 2 && a.stride(1) == 1,
               "a must be bf16 [M, K] with unit inner stride");
   check_bf16(w, "w");
@@ -288,7 +288,8 @@ void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi) {
   }
   c10::DeviceGuard g(a.device());
   mlop::launch_gemm(a.data_ptr(), (int)a.stride(0), w.data_ptr(), (int)K, out.data_ptr(),
-                    (int)out.stride(0), wsp, wsn, (int)M, (int)N, (int)K, (int)epi, cur_stream());
+                    (int)out.stride(0), wsp, wsn, (int)M, (int)N, (int)K, (int)epi, cur_stream(), (float)glu_alpha,
+                    (float)glu_limit);
 }
 
 // QKV projection with RoPE + paged-cache stores in the GEMM epilogue; false = this M
@@ -928,7 +929,7 @@ TORCH_LIBRARY(mlop, m) {
         "Tensor pos, Tensor cos_sin, Tensor slots, Tensor ss_in, float eps) -> bool");
   m.def("gemm_rope_cache(Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor a, Tensor w, "
         "Tensor pos, Tensor cos_sin, Tensor slots) -> bool");
-  m.def("gemm(Tensor(a!) out, Tensor a, Tensor w, Tensor(b!) ws, int epi) -> ()");
+  m.def("gemm(Tensor(a!) out, Tensor a, Tensor w, Tensor(b!) ws, int epi, float glu_alpha=0., float glu_limit=0.) -> ()");
   m.def("grouped_gemm(Tensor(a!) out, Tensor a, Tensor w, Tensor offsets, int max_rows, "
         "int epi, Tensor? a_rows=None) -> ()");
   m.def("gemm_add_rmsnorm(Tensor(a!) out, Tensor(b!) residual, Tensor a, Tensor w, Tensor norm_w, "

@@ -1,47 +1,12 @@
 // torch.ops.mlop.* registrations of the hybrid-decoder kernels (hybrid.h): hyper-connections,
 // query / key norm + rotary + paged stores, paged attention of any head sizes, gated linear
 // attention.  As in bindings.cpp every op checks types and shapes on the host before it launches.
-#include <torch/library.h>
-#include <ATen/ATen.h>
-#include <c10/hip/HIPStream.h>
-#include <c10/core/DeviceGuard.h>
-
 #include <cmath>
-#include <optional>
 
+#include "bind_util.h"
 #include "hybrid.h"
 
 namespace {
-
-using at::Tensor;
-using OptT = std::optional<Tensor>;
-
-hipStream_t cur() { return c10::hip::getCurrentHIPStream().stream(); }
-
-// model dtype: bf16 or fp32, unit inner stride
-bool model_f32(const Tensor& t, const char* n) {
-  TORCH_CHECK(t.is_cuda(), n, " must be a GPU tensor");
-  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat, n, " must be bf16 or fp32");
-  TORCH_CHECK(t.dim() == 0 || t.stride(-1) == 1, n, " needs a unit inner stride");
-  return t.scalar_type() == at::kFloat;
-}
-void like(const Tensor& t, const Tensor& ref, const char* n) {
-  model_f32(t, n);
-  TORCH_CHECK(t.scalar_type() == ref.scalar_type(), n, " has another dtype than its operands");
-}
-const float* f32_of(const Tensor& t, int64_t numel, const char* n) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() == numel, n,
-              " must be a contiguous fp32 GPU tensor of ", numel, " elements");
-  return t.data_ptr<float>();
-}
-const int* i32_of(const Tensor& t, const char* n) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kInt && t.is_contiguous(), n, " must be contiguous int32 on the GPU");
-  return t.data_ptr<int>();
-}
-// rows of 16-B aligned vectors (the kernels' widest loads)
-void aligned16(const Tensor& t, const char* n) {
-  TORCH_CHECK(reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0, n, " must be 16-B aligned");
-}
 
 void hyper_common(mlop::HyperArgs& a, const Tensor& xn, const Tensor& streams, const Tensor& w_in, const Tensor& norm_w,
                   double eps) {
@@ -173,33 +138,61 @@ void qk_norm_rope(Tensor q_out, Tensor k_cache, Tensor v_cache, Tensor proj, int
   mlop::launch_qk_norm(a, f32, cur());
 }
 
-// decode tiles (one query token each) and prompt tiles (128 tokens of a head) of one step
+// decode tiles (one query token each) and prompt tiles (128 tokens of a head) of one step.  k, v: paged
+// caches [NB, G, 16, KP]; or, with xbase, dense rows [rows, G, KP] of prompt tiles.  by_tile: q [tiles, H,
+// KP] and out by decode tile
 void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Tensor q, Tensor k_cache, Tensor v_cache,
                   Tensor block_tables, Tensor tile_seq, Tensor tile_q0, Tensor ptile_seq, Tensor ptile_q0,
                   Tensor q_start, Tensor q_len, Tensor ctx_len, int64_t D, double scale, OptT sink, OptT gate,
-                  int64_t part_tokens, int64_t nparts) {
+                  int64_t part_tokens, int64_t nparts, int64_t window, OptT xbase, bool by_tile) {
   mlop::AttnHdArgs a{};
   const bool f32 = model_f32(q, "q");
   like(out, q, "out");
   like(k_cache, q, "k_cache");
   like(v_cache, q, "v_cache");
-  TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && out.dim() == 3 && out.is_contiguous(), "q, out ranks");
-  TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous() && v_cache.dim() == 4 && v_cache.is_contiguous(), "cache ranks");
+  const int64_t num_tiles = tile_seq.numel(), num_ptiles = ptile_seq.numel();
+  TORCH_CHECK(q.dim() == 3 && out.dim() == 3 && out.is_contiguous(), "q, out ranks");
   a.H = (int)q.size(1);
   a.KP = (int)q.size(2);
-  a.G = (int)k_cache.size(1);
-  a.VP = (int)v_cache.size(3);
   a.V = (int)out.size(2);
   a.D = (int)D;
-  TORCH_CHECK(out.size(0) == q.size(0) && out.size(1) == a.H, "out must be [T, H, V]");
+  a.q_row = q.stride(0);
+  a.q_head = q.stride(1);
+  const int kd = (int)k_cache.dim();
+  TORCH_CHECK(kd == (xbase ? 3 : 4) && v_cache.dim() == kd, "key / value ranks");
+  a.G = (int)k_cache.size(1);
+  a.VP = (int)v_cache.size(kd - 1);
+  TORCH_CHECK(out.size(1) == a.H && out.size(0) == q.size(0), "out must be [T, H, V]");
   TORCH_CHECK(a.KP % 64 == 0 && a.VP % 64 == 0 && D >= 1 && D <= a.KP && a.V >= 1 && a.V <= a.VP &&
                   a.VP <= mlop::kHdMaxV && D <= 4096,
               "head sizes");
-  TORCH_CHECK(k_cache.size(2) == 16 && k_cache.size(3) == a.KP && v_cache.size(0) == k_cache.size(0) &&
-                  v_cache.size(1) == a.G && v_cache.size(2) == 16,
-              "caches must be [NB, G, 16, KP] and [NB, G, 16, VP]");
+  TORCH_CHECK(k_cache.size(kd - 1) == a.KP && v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == a.G, "key / value sizes");
   TORCH_CHECK(a.G >= 1 && a.H % a.G == 0, "query heads must be a multiple of kv heads");
+  if (xbase) {
+    TORCH_CHECK(num_tiles == 0 && !by_tile, "dense keys are for prompt tiles");
+    a.xbase = i32_of(*xbase, "xbase");
+    TORCH_CHECK(xbase->numel() >= q_len.numel(), "xbase length");
+    a.k_pitch = a.k_row = k_cache.stride(0);
+    a.v_pitch = a.v_row = v_cache.stride(0);
+    a.k_head = k_cache.stride(1);
+    a.v_head = v_cache.stride(1);
+    TORCH_CHECK(a.k_row % 8 == 0 && a.v_row % 8 == 0 && a.k_head % 8 == 0 && a.v_head % 8 == 0, "16-B aligned rows");
+  } else {
+    TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() && k_cache.size(2) == 16 && v_cache.size(2) == 16,
+                "caches must be [NB, G, 16, KP] and [NB, G, 16, VP]");
+    a.k_pitch = (long)a.G * a.KP;
+    a.v_pitch = (long)a.G * a.VP;
+    a.k_row = a.KP;
+    a.v_row = a.VP;
+    a.k_head = 16l * a.KP;
+    a.v_head = 16l * a.VP;
+  }
+  TORCH_CHECK(!by_tile || (num_ptiles == 0 && q.size(0) >= num_tiles), "by_tile is for decode tiles");
+  TORCH_CHECK(a.q_row % 8 == 0 && a.q_head % 8 == 0, "16-B aligned query rows");
   TORCH_CHECK(scale > 0, "score scale must be positive");
+  TORCH_CHECK(window >= 0 && window < (1 << 30), "window");
+  a.window = (int)window;
+  a.by_tile = by_tile;
   for (const Tensor* t : {&q, &k_cache, &v_cache, &out}) aligned16(*t, "attention operand");
   a.bt = i32_of(block_tables, "block_tables");
   a.bt_stride = (int)block_tables.stride(0);
@@ -212,9 +205,12 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
   if (sink) a.sink = f32_of(*sink, a.H, "sink");
   if (gate) {
     like(*gate, q, "gate");
-    TORCH_CHECK(gate->dim() == 2 && gate->size(0) == q.size(0) && gate->size(1) == a.H, "gate must be [T, H]");
+    TORCH_CHECK(gate->dim() == 2 && !by_tile && gate->size(0) == q.size(0) &&
+                    (gate->size(1) == a.H || gate->size(1) == (int64_t)a.H * a.V),
+                "gate must be [T, H] or [T, H * V]");
     a.gate = gate->data_ptr();
     a.gate_stride = gate->stride(0);
+    a.gate_elem = gate->size(1) != a.H;
   }
   a.scale_log2 = (float)(scale * 1.4426950408889634);
   a.num_blocks = (int)k_cache.size(0);
@@ -222,13 +218,13 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
   a.q = q.data_ptr();
   a.k_cache = k_cache.data_ptr();
   a.v_cache = v_cache.data_ptr();
-  const int num_tiles = (int)tile_seq.numel();
-  const bool plain = f32 || a.KP > mlop::kHdMaxDim || a.VP > mlop::kHdMaxDim;
+  const bool plain = f32 || ((a.KP > mlop::kHdMaxDim || a.VP > mlop::kHdMaxDim) &&
+                             !(a.KP == a.VP && a.KP <= mlop::kHdMaxLatent));
   TORCH_CHECK(part_tokens > 0 && part_tokens % 32 == 0 && nparts >= 1, "partition size");
   float *po = nullptr, *pml = nullptr;
   int* sem = nullptr;
   if (nparts > 1 && num_tiles && !plain) {
-    const int64_t units = (int64_t)num_tiles * a.G * ((a.H / a.G + 15) / 16);
+    const int64_t units = num_tiles * a.G * ((a.H / a.G + 15) / 16);
     TORCH_CHECK(part_o.scalar_type() == at::kFloat && part_ml.scalar_type() == at::kFloat &&
                     part_o.numel() >= units * nparts * 16 * a.VP && part_ml.numel() >= units * nparts * 16 * 2,
                 "partial workspace too small");
@@ -239,10 +235,9 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
     sem = part_sem.data_ptr<int>();
   }
   c10::DeviceGuard g(q.device());
-  mlop::launch_paged_hd(a, f32, po, pml, sem, i32_of(tile_seq, "tile_seq"), i32_of(tile_q0, "tile_q0"), num_tiles,
+  mlop::launch_paged_hd(a, f32, po, pml, sem, i32_of(tile_seq, "tile_seq"), i32_of(tile_q0, "tile_q0"), (int)num_tiles,
                         (int)part_tokens, (int)nparts, cur());
-  mlop::launch_flash_hd(a, f32, i32_of(ptile_seq, "ptile_seq"), i32_of(ptile_q0, "ptile_q0"), (int)ptile_seq.numel(),
-                        cur());
+  mlop::launch_flash_hd(a, f32, i32_of(ptile_seq, "ptile_seq"), i32_of(ptile_q0, "ptile_q0"), (int)num_ptiles, cur());
 }
 
 void gla(Tensor out, Tensor state, Tensor proj, int64_t H, int64_t dk, int64_t dv, Tensor a2, Tensor a2_b, Tensor norm_w,
@@ -313,7 +308,7 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
   m.def("attention_hd(Tensor(a!) out, Tensor(b!) part_o, Tensor(c!) part_ml, Tensor(d!) part_sem, Tensor q, "
         "Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_q0, Tensor ptile_seq, "
         "Tensor ptile_q0, Tensor q_start, Tensor q_len, Tensor ctx_len, int D, float scale, Tensor? sink, Tensor? gate, "
-        "int part_tokens, int nparts) -> ()");
+        "int part_tokens, int nparts, int window=0, Tensor? xbase=None, bool by_tile=False) -> ()");
   m.def("gla(Tensor(a!) out, Tensor(b!) state, Tensor proj, int H, int dk, int dv, Tensor a2, Tensor a2_b, "
         "Tensor norm_w, float tau, float eps, Tensor q_start, Tensor q_len, Tensor ctx_len, Tensor rows, "
         "Tensor item_seq, Tensor item_t0, Tensor crow_seq, Tensor crow_item0, int chunk) -> ()");

@@ -1,0 +1,341 @@
+// torch.ops.mlop.* registrations of the mixers and norms in mixers.h.  Every op checks types and shapes
+// on the host before it launches.
+#include <cmath>
+
+#include "bind_util.h"
+#include "mixers.h"
+
+namespace {
+
+// a step's row lists; T: tokens the per-token operands hold
+mlop::StepRows step_rows(const Tensor& q_start, const Tensor& q_len, const Tensor& ctx_len, const Tensor& rows,
+                         const Tensor& item_seq, const Tensor& item_t0, const Tensor& crow_seq, const Tensor& crow_item0,
+                         int64_t chunk, int64_t n_slots) {
+  mlop::StepRows s{};
+  s.q_start = i32_of(q_start, "q_start");
+  s.q_len = i32_of(q_len, "q_len");
+  s.ctx_len = i32_of(ctx_len, "ctx_len");
+  TORCH_CHECK(q_start.numel() == q_len.numel() && q_len.numel() == ctx_len.numel(), "per-sequence arrays");
+  s.rows = i32_of(rows, "rows");
+  s.n_rows = (int)rows.numel();
+  s.item_seq = i32_of(item_seq, "item_seq");
+  s.item_t0 = i32_of(item_t0, "item_t0");
+  s.n_items = (int)item_seq.numel();
+  s.crow_seq = i32_of(crow_seq, "crow_seq");
+  s.crow_item0 = i32_of(crow_item0, "crow_item0");
+  s.n_crows = (int)crow_seq.numel();
+  TORCH_CHECK(item_t0.numel() == s.n_items && crow_item0.numel() == s.n_crows, "chunk lists");
+  TORCH_CHECK((s.n_items == 0) == (s.n_crows == 0) && (s.n_items == 0 || (chunk >= 16 && chunk % 16 == 0)), "chunk size");
+  s.chunk = (int)chunk;
+  s.n_slots = (int)n_slots;
+  return s;
+}
+
+void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, const Tensor& norm_w, double eps) {
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.is_cuda() && x.scalar_type() == at::kFloat, "x must be [T, W] fp32");
+  a.T = (int)x.size(0);
+  a.W = (int)x.size(1);
+  TORCH_CHECK(a.W >= 1 && a.W <= mlop::kResidualMaxW, "row width 1 .. ", mlop::kResidualMaxW);
+  TORCH_CHECK(xn.is_contiguous() && xn.numel() == x.numel(), "xn must be [T, W]");
+  a.x = x.data_ptr<float>();
+  a.xn = xn.data_ptr();
+  a.norm_w = f32_of(norm_w, a.W, "norm_w");
+  a.eps = (float)eps;
+  for (const Tensor* t : {&x, &xn, &norm_w}) aligned16(*t, "residual operand");
+}
+
+void residual_begin(Tensor xn, Tensor x, Tensor ids, Tensor table, double scale, OptT pos_table, Tensor pos, Tensor norm_w,
+                    double eps) {
+  mlop::ResidualArgs a{};
+  const bool f32 = model_f32(table, "table");
+  like(xn, table, "xn");
+  residual_common(a, xn, x, norm_w, eps);
+  TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.numel() == a.T, "ids int64 [T]");
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && table.size(1) == a.W, "table must be [vocab, W]");
+  aligned16(table, "table");
+  a.ids = ids.data_ptr<int64_t>();
+  a.table = table.data_ptr();
+  a.vocab = table.size(0);
+  a.embed_scale = (float)scale;
+  if (pos_table) {
+    like(*pos_table, table, "pos_table");
+    TORCH_CHECK(pos_table->dim() == 2 && pos_table->is_contiguous() && pos_table->size(1) == a.W, "pos_table [n, W]");
+    aligned16(*pos_table, "pos_table");
+    a.pos_table = pos_table->data_ptr();
+    a.n_pos = pos_table->size(0);
+    a.pos = i32_of(pos, "pos");
+    TORCH_CHECK(pos.numel() == a.T, "pos length");
+  }
+  a.store = true;
+  c10::DeviceGuard g(table.device());
+  mlop::launch_residual(a, f32, cur());
+}
+
+void residual_step(Tensor xn, Tensor x, Tensor y, OptT post_w, Tensor norm_w, double eps, bool store) {
+  mlop::ResidualArgs a{};
+  const bool f32 = model_f32(y, "y");
+  like(xn, y, "xn");
+  residual_common(a, xn, x, norm_w, eps);
+  TORCH_CHECK(y.is_contiguous() && y.numel() == x.numel(), "y must be [T, W]");
+  aligned16(y, "y");
+  a.y = y.data_ptr();
+  if (post_w) {
+    a.post_w = f32_of(*post_w, a.W, "post_w");
+    aligned16(*post_w, "post_w");
+  }
+  a.store = store;
+  c10::DeviceGuard g(y.device());
+  mlop::launch_residual(a, f32, cur());
+}
+
+void gated_norm(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t groups, double eps, int64_t act, bool gate_first) {
+  mlop::GatedNormArgs a{};
+  const bool f32 = model_f32(y, "y");
+  like(out, y, "out");
+  like(gate, y, "gate");
+  TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && out.is_contiguous() && out.numel() == y.numel(), "y, out must be [T, n]");
+  a.T = (int)y.size(0);
+  a.n = (int)y.size(1);
+  TORCH_CHECK(gate.dim() == 2 && gate.size(0) == a.T && gate.size(1) == a.n, "gate must be [T, n]");
+  TORCH_CHECK(groups >= 1 && a.n % groups == 0, "groups must divide the row");
+  TORCH_CHECK(act == mlop::kGateSilu || act == mlop::kGateSigmoid, "gate activation");
+  a.groups = (int)groups;
+  a.out = out.data_ptr();
+  a.y = y.data_ptr();
+  a.gate = gate.data_ptr();
+  a.ldg = gate.stride(0);
+  a.w = f32_of(w, a.n, "w");
+  a.eps = (float)eps;
+  a.act = (int)act;
+  a.gate_first = gate_first;
+  c10::DeviceGuard g(y.device());
+  mlop::launch_gated_norm(a, f32, cur());
+}
+
+void clamp_glu(Tensor out, Tensor x, double alpha, double limit) {
+  const bool f32 = model_f32(x, "x");
+  like(out, x, "out");
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && out.is_contiguous() && x.size(1) % 32 == 0 &&
+                  out.numel() * 2 == x.numel(),
+              "x must be [T, 2 I] with columns interleaved in groups of 16, out [T, I]");
+  aligned16(x, "x");
+  aligned16(out, "out");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_clamp_glu(out.data_ptr(), x.data_ptr(), (int)x.size(0), (int)(x.size(1) / 2), (float)alpha, (float)limit, f32,
+                         cur());
+}
+
+void short_conv(Tensor out, Tensor tail, Tensor x, Tensor w, OptT b, Tensor q_start, Tensor q_len, Tensor ctx_len,
+                Tensor rows, Tensor item_seq, Tensor item_t0, Tensor crow_seq, Tensor crow_item0, int64_t chunk) {
+  mlop::ConvArgs a{};
+  const bool f32 = model_f32(x, "x");
+  like(out, x, "out");
+  TORCH_CHECK(w.dim() == 2, "w must be [C, taps]");
+  a.C = (int)w.size(0);
+  a.taps = (int)w.size(1);
+  TORCH_CHECK(a.taps >= 1 && a.taps <= mlop::kConvMaxTaps, "1 .. ", mlop::kConvMaxTaps, " taps");
+  TORCH_CHECK(x.dim() == 2 && x.size(1) == a.C && out.is_contiguous() && out.numel() == x.size(0) * a.C, "x, out must be [T, C]");
+  TORCH_CHECK(tail.is_cuda() && tail.scalar_type() == at::kFloat && tail.is_contiguous() && tail.dim() == 3 &&
+                  tail.size(1) == a.taps - 1 && tail.size(2) == a.C,
+              "tail must be [slots, taps - 1, C] fp32");
+  a.out = out.data_ptr();
+  a.x = x.data_ptr();
+  a.ldx = x.stride(0);
+  a.w = f32_of(w, (int64_t)a.C * a.taps, "w");
+  if (b) a.b = f32_of(*b, a.C, "b");
+  a.tail = tail.data_ptr<float>();
+  const auto s = step_rows(q_start, q_len, ctx_len, rows, item_seq, item_t0, crow_seq, crow_item0, chunk, tail.size(0));
+  c10::DeviceGuard g(x.device());
+  mlop::launch_short_conv(a, s, f32, cur());
+}
+
+void ssd(Tensor y, Tensor state, Tensor xbc, Tensor dt, int64_t G, Tensor dt_bias, Tensor a_neg, Tensor d_skip,
+         Tensor q_start, Tensor q_len, Tensor ctx_len, Tensor rows, Tensor item_seq, Tensor item_t0, Tensor crow_seq,
+         Tensor crow_item0, int64_t chunk) {
+  mlop::SsdArgs a{};
+  const bool f32 = model_f32(xbc, "xbc");
+  like(y, xbc, "y");
+  like(dt, xbc, "dt");
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() && state.dim() == 4,
+              "state must be [slots, H, N, V] fp32");
+  aligned16(state, "state");
+  a.H = (int)state.size(1);
+  a.N = (int)state.size(2);
+  a.V = (int)state.size(3);
+  a.G = (int)G;
+  TORCH_CHECK(a.H >= 1 && G >= 1 && a.H % G == 0 && a.N >= 1 && a.N <= 4096 && a.V >= 1 && a.V <= 4096, "ssd sizes");
+  TORCH_CHECK(xbc.dim() == 2 && xbc.size(1) == (int64_t)a.H * a.V + 2 * G * a.N, "xbc must be [T, H V + 2 G N]");
+  const int64_t T = xbc.size(0);
+  TORCH_CHECK(y.is_contiguous() && y.numel() == T * a.H * a.V, "y must be [T, H * V]");
+  TORCH_CHECK(dt.dim() == 2 && dt.size(0) == T && dt.size(1) == a.H, "dt must be [T, H]");
+  aligned16(xbc, "xbc");
+  a.y = y.data_ptr();
+  a.xbc = xbc.data_ptr();
+  a.ldx = xbc.stride(0);
+  a.dt = dt.data_ptr();
+  a.ldt = dt.stride(0);
+  a.dt_bias = f32_of(dt_bias, a.H, "dt_bias");
+  a.a_neg = f32_of(a_neg, a.H, "a_neg");
+  a.d_skip = f32_of(d_skip, a.H, "d_skip");
+  a.state = state.data_ptr<float>();
+  const auto s = step_rows(q_start, q_len, ctx_len, rows, item_seq, item_t0, crow_seq, crow_item0, chunk, state.size(0));
+  c10::DeviceGuard g(xbc.device());
+  mlop::launch_ssd(a, s, f32, cur());
+}
+
+void delta(Tensor o, Tensor state, Tensor proj, Tensor w2, Tensor w0, Tensor a_b, double decay_scale, double unit_eps,
+           Tensor q_start, Tensor q_len, Tensor ctx_len, Tensor rows, Tensor item_seq, Tensor item_t0, Tensor crow_seq,
+           Tensor crow_item0, int64_t chunk) {
+  mlop::DeltaArgs a{};
+  const bool f32 = model_f32(proj, "proj");
+  like(o, proj, "o");
+  like(w2, proj, "w2");
+  TORCH_CHECK(state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() && state.dim() == 4,
+              "state must be [slots, H, dk, dv] fp32");
+  aligned16(state, "state");
+  a.H = (int)state.size(1);
+  a.dk = (int)state.size(2);
+  a.dv = (int)state.size(3);
+  TORCH_CHECK(a.H >= 1 && a.dk >= 1 && a.dk <= 1024 && a.dv >= 1 && a.dv <= 4096 && decay_scale >= 0, "delta sizes");
+  TORCH_CHECK(w2.dim() == 2 && w2.is_contiguous() && w2.size(0) == (int64_t)a.H * a.dk, "w2 must be [H * dk, rank]");
+  a.rank = (int)w2.size(1);
+  const int64_t T = proj.size(0);
+  TORCH_CHECK(proj.dim() == 2 && proj.size(1) >= (int64_t)a.H * (3 * a.dk + a.dv) + a.rank, "proj is too narrow");
+  TORCH_CHECK(o.is_contiguous() && o.numel() == T * a.H * a.dv, "o must be [T, H * dv]");
+  TORCH_CHECK((size_t)(a.rank + 5 * a.dk + 3 * 512 * 4) * 4 <= 60 * 1024, "delta: sizes past the kernels' LDS");
+  aligned16(proj, "proj");
+  aligned16(w2, "w2");
+  a.o = o.data_ptr();
+  a.proj = proj.data_ptr();
+  a.ldp = proj.stride(0);
+  a.w2 = w2.data_ptr();
+  a.w0 = f32_of(w0, (int64_t)a.H * a.dk, "w0");
+  a.a_b = f32_of(a_b, (int64_t)a.H * a.dk, "a_b");
+  a.state = state.data_ptr<float>();
+  a.decay_scale = (float)decay_scale;
+  a.unit_eps = (float)unit_eps;
+  const auto s = step_rows(q_start, q_len, ctx_len, rows, item_seq, item_t0, crow_seq, crow_item0, chunk, state.size(0));
+  c10::DeviceGuard g(proj.device());
+  Tensor ws;
+  if (s.n_items && mlop::delta_blocks_ok(a.dk, a.decay_scale))
+    ws = at::empty({mlop::delta_ws_floats(s.n_items, s.chunk, a.H, a.dk)}, proj.options().dtype(at::kFloat));
+  mlop::launch_delta(a, s, ws.defined() ? ws.data_ptr<float>() : nullptr, f32, cur());
+}
+
+void latent_store(Tensor cache, Tensor l, Tensor w, double eps, Tensor slots) {
+  const bool f32 = model_f32(l, "l");
+  like(cache, l, "cache");
+  TORCH_CHECK(cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == 1, "cache must be [NB, 1, BS, RP]");
+  TORCH_CHECK(l.dim() == 2 && l.size(1) <= cache.size(3) && slots.numel() == l.size(0), "latents must be [T, R]");
+  aligned16(cache, "cache");
+  c10::DeviceGuard g(l.device());
+  mlop::launch_latent_store(cache.data_ptr(), l.data_ptr(), l.stride(0), f32_of(w, l.size(1), "w"), (float)eps,
+                            i32_of(slots, "slots"), (int)l.size(0), (int)l.size(1), (int)cache.size(3), (int)cache.size(2),
+                            f32, cur());
+}
+
+void latent_gather(Tensor out, Tensor cache, Tensor block_tables, Tensor xbase, Tensor q_len, Tensor ctx_len,
+                   Tensor crow_seq, int64_t rows, int64_t x_max, int64_t window) {
+  mlop::LatentGatherArgs a{};
+  const bool f32 = model_f32(cache, "cache");
+  like(out, cache, "out");
+  TORCH_CHECK(cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == 1, "cache must be [NB, 1, BS, RP]");
+  a.RP = (int)cache.size(3);
+  TORCH_CHECK(out.dim() == 2 && out.is_contiguous() && out.size(1) == a.RP && out.size(0) >= rows && a.RP % 64 == 0,
+              "out must be [rows + pad, RP]");
+  aligned16(out, "out");
+  aligned16(cache, "cache");
+  a.out = out.data_ptr();
+  a.cache = cache.data_ptr();
+  a.bt = i32_of(block_tables, "block_tables");
+  a.bt_stride = (int)block_tables.stride(0);
+  a.xbase = i32_of(xbase, "xbase");
+  a.q_len = i32_of(q_len, "q_len");
+  a.ctx_len = i32_of(ctx_len, "ctx_len");
+  a.crow_seq = i32_of(crow_seq, "crow_seq");
+  a.n_crows = (int)crow_seq.numel();
+  a.x_max = (int)x_max;
+  a.rows = (int)rows;
+  a.pad = (int)(out.size(0) - rows);
+  a.BS = (int)cache.size(2);
+  a.num_blocks = (int)cache.size(0);
+  a.window = (int)window;
+  c10::DeviceGuard g(cache.device());
+  mlop::launch_latent_gather(a, f32, cur());
+}
+
+void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Tensor q_start, Tensor q_len, bool x_tok,
+             bool out_tok, OptT gate) {
+  mlop::HeadMmArgs a{};
+  const bool f32 = model_f32(x, "x");
+  like(out, x, "out");
+  like(w, x, "w");
+  TORCH_CHECK(w.dim() == 3 && w.is_contiguous() && x.dim() == 3 && out.dim() == 3, "w [H, N, K], x [rows, H, K], out [rows, H, N]");
+  a.H = (int)w.size(0);
+  a.N = (int)w.size(1);
+  a.K = (int)w.size(2);
+  TORCH_CHECK(a.K % 64 == 0 && x.size(1) == a.H && x.size(2) == a.K && out.size(1) == a.H && out.size(2) == a.N, "head_mm sizes");
+  a.n_tiles = (int)tile_seq.numel();
+  TORCH_CHECK((x_tok || x.size(0) >= a.n_tiles) && (out_tok || out.size(0) >= a.n_tiles) && a.n_tiles <= 65535, "head_mm rows");
+  a.out = out.data_ptr();
+  a.x = x.data_ptr();
+  a.w = w.data_ptr();
+  a.ldx = x.stride(0);
+  a.hx = x.stride(1);
+  a.ldo = out.stride(0);
+  a.ho = out.stride(1);
+  TORCH_CHECK(a.ldx % 8 == 0 && a.hx % 8 == 0, "16-B aligned rows");
+  aligned16(x, "x");
+  aligned16(w, "w");
+  a.tile_seq = i32_of(tile_seq, "tile_seq");
+  a.tile_q0 = i32_of(tile_q0, "tile_q0");
+  a.q_start = i32_of(q_start, "q_start");
+  a.q_len = i32_of(q_len, "q_len");
+  a.x_tok = x_tok;
+  a.out_tok = out_tok;
+  if (gate) {
+    like(*gate, x, "gate");
+    TORCH_CHECK(gate->dim() == 2 && gate->size(1) == (int64_t)a.H * a.N, "gate must be [T, H * N]");
+    a.gate = gate->data_ptr();
+    a.ldg = gate->stride(0);
+  }
+  c10::DeviceGuard g(x.device());
+  mlop::launch_head_mm(a, f32, cur());
+}
+
+}  // namespace
+
+#define MLOP_ROWS                                                                                                \
+  "Tensor q_start, Tensor q_len, Tensor ctx_len, Tensor rows, Tensor item_seq, Tensor item_t0, Tensor crow_seq, " \
+  "Tensor crow_item0, int chunk"
+
+TORCH_LIBRARY_FRAGMENT(mlop, m) {
+  m.def("residual_begin(Tensor(a!) xn, Tensor(b!) x, Tensor ids, Tensor table, float scale, Tensor? pos_table, Tensor pos, "
+        "Tensor norm_w, float eps) -> ()");
+  m.def("residual_step(Tensor(a!) xn, Tensor(b!) x, Tensor y, Tensor? post_w, Tensor norm_w, float eps, bool store) -> ()");
+  m.def("gated_norm(Tensor(a!) out, Tensor y, Tensor gate, Tensor w, int groups, float eps, int act, bool gate_first) -> ()");
+  m.def("clamp_glu(Tensor(a!) out, Tensor x, float alpha, float limit) -> ()");
+  m.def("short_conv(Tensor(a!) out, Tensor(b!) tail, Tensor x, Tensor w, Tensor? b, " MLOP_ROWS ") -> ()");
+  m.def("ssd(Tensor(a!) y, Tensor(b!) state, Tensor xbc, Tensor dt, int G, Tensor dt_bias, Tensor a_neg, Tensor d_skip, "
+        MLOP_ROWS ") -> ()");
+  m.def("delta(Tensor(a!) o, Tensor(b!) state, Tensor proj, Tensor w2, Tensor w0, Tensor a_b, float decay_scale, "
+        "float unit_eps, " MLOP_ROWS ") -> ()");
+  m.def("latent_store(Tensor(a!) cache, Tensor l, Tensor w, float eps, Tensor slots) -> ()");
+  m.def("latent_gather(Tensor(a!) out, Tensor cache, Tensor block_tables, Tensor xbase, Tensor q_len, Tensor ctx_len, "
+        "Tensor crow_seq, int rows, int x_max, int window) -> ()");
+  m.def("head_mm(Tensor(a!) out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Tensor q_start, Tensor q_len, "
+        "bool x_tok, bool out_tok, Tensor? gate) -> ()");
+}
+
+TORCH_LIBRARY_IMPL(mlop, CUDA, m) {
+  m.impl("residual_begin", &residual_begin);
+  m.impl("residual_step", &residual_step);
+  m.impl("gated_norm", &gated_norm);
+  m.impl("clamp_glu", &clamp_glu);
+  m.impl("short_conv", &short_conv);
+  m.impl("ssd", &ssd);
+  m.impl("delta", &delta);
+  m.impl("latent_store", &latent_store);
+  m.impl("latent_gather", &latent_gather);
+  m.impl("head_mm", &head_mm);
+}

@@ -125,6 +125,13 @@ __device__ __forceinline__ float silu_bf(float g) {
   return bf2f(f2bf(gb * __builtin_amdgcn_rcpf(1.f + __expf(-gb))));
 }
 
+// clamped gated unit: g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)
+__device__ __forceinline__ float clamp_glu_f(float g, float u, float alpha, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * (u + 1.f) / (1.f + __expf(-alpha * g));
+}
+
 __device__ __forceinline__ float relu2_f(float x) {
   const float r = fmaxf(x, 0.f);
   return r * r;

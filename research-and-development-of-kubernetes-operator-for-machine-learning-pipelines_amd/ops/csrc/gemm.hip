@@ -393,8 +393,7 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
         u32x4 o;
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-          o[j] = pack2(silu_bf(g[2 * j] * f) * bf2f(f2bf(u[2 * j] * f)),
-                       silu_bf(g[2 * j + 1] * f) * bf2f(f2bf(u[2 * j + 1] * f)));
+          o[j] = pack2(glu_out(re, g[2 * j] * f, u[2 * j] * f), glu_out(re, g[2 * j + 1] * f, u[2 * j + 1] * f));
         *reinterpret_cast<u32x4*>(C + (size_t)(m0 + r) * ldc + (n0 + c0) / 2 + j0) = o;
       }
     }
@@ -406,10 +405,14 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
 template <int EPI>
 __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict__ C, int ldc,
                                                            const float* __restrict__ ws, int M,
-                                                           int N, int splits, int relu2 = 0) {
+                                                           int N, int splits, int relu2 = 0, float glu_alpha = 0.f,
+                                                           float glu_limit = 0.f) {
   const int outw = EPI == EPI_NONE ? N : N / 2;
   const int vpr = outw / 8;
   const long total = (long)M * vpr;
+  RopeEpi re{};
+  re.glu_alpha = glu_alpha;
+  re.glu_limit = glu_limit;
   for (long v = blockIdx.x * (long)blockDim.x + threadIdx.x; v < total;
        v += (long)gridDim.x * blockDim.x) {
     const int r = (int)(v / vpr), j0 = (int)(v % vpr) * 8;
@@ -433,8 +436,7 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict
       if (EPI == EPI_NONE)
         o[j] = relu2 ? pack2(relu2_f(a[2 * j]), relu2_f(a[2 * j + 1])) : pack2(a[2 * j], a[2 * j + 1]);
       else
-        o[j] = pack2(silu_bf(a[2 * j]) * bf2f(f2bf(b[2 * j])),
-                     silu_bf(a[2 * j + 1]) * bf2f(f2bf(b[2 * j + 1])));
+        o[j] = pack2(glu_out(re, a[2 * j], b[2 * j]), glu_out(re, a[2 * j + 1], b[2 * j + 1]));
     }
     *reinterpret_cast<u32x4*>(C + (size_t)r * ldc + j0) = o;
   }
@@ -1112,7 +1114,7 @@ __global__ void __launch_bounds__(512, 1) gemm_pp_kernel(
 #pragma unroll
           for (int jp = 0; jp < 2; ++jp) {
             const float g = acc[i][2 * jp][r], u = acc[i][2 * jp + 1][r];
-            sC[row * LD + jp * 16 + (lane & 15)] = f2bf(silu_bf(g) * bf2f(f2bf(u)));
+            sC[row * LD + jp * 16 + (lane & 15)] = f2bf(glu_out(re, g, u));
           }
         }
       }
@@ -1723,13 +1725,15 @@ long gemm_workspace_floats(int M, int N, int K, int epi) {
 }
 
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
-                 long ws_floats, int M, int N, int K, int epi, hipStream_t st) {
+                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float glu_alpha, float glu_limit) {
   if (M == 0) return;
   RopeEpi re{};
+  re.glu_alpha = glu_alpha;
+  re.glu_limit = glu_limit;
   re.relu2 = epi == kEpiRelu2;
   if (re.relu2) epi = EPI_NONE;
   if (gemv_takes(M, N, K, epi) && lda % 8 == 0 && ldb % 8 == 0) {
-    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, re.relu2 ? kEpiRelu2 : epi, st);
+    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, re.relu2 ? kEpiRelu2 : epi, st, glu_alpha, glu_limit);
     return;
   }
   Plan p = plan(M, N, K, false, 0, 0);
@@ -1739,7 +1743,7 @@ void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ld
                                  ldc, ws, M, N, K, nullptr, 0, st, re);
   else
     launch_plan<EPI_SILU_MUL, false>(p, (const uint16_t*)A, lda, (const uint16_t*)B, ldb,
-                                     (uint16_t*)C, ldc, ws, M, N, K, nullptr, 0, st);
+                                     (uint16_t*)C, ldc, ws, M, N, K, nullptr, 0, st, re);
   if (p.splits > 1) {
     const int outw = epi == EPI_NONE ? N : N / 2;
     const long total = (long)M * (outw / 8);
@@ -1747,7 +1751,7 @@ void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ld
     if (epi == EPI_NONE)
       splitk_reduce_kernel<EPI_NONE><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, re.relu2);
     else
-      splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits);
+      splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, 0, glu_alpha, glu_limit);
   }
 }
 

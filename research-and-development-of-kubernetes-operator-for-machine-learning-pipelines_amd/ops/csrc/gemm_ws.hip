@@ -181,7 +181,7 @@ __global__ void __launch_bounds__(256) gemm_ws_kernel(const uint16_t* __restrict
     if constexpr (EPI == WS_SILU_MUL) {
 #pragma unroll
       for (int g = 0; g < RB / 2; ++g)
-        C[(size_t)m * ldc + (blk * (RB / 2) + g) * 16 + col] = f2bf(silu_bf(y[2 * g]) * bf2f(f2bf(y[2 * g + 1])));
+        C[(size_t)m * ldc + (blk * (RB / 2) + g) * 16 + col] = f2bf(glu_out(re, y[2 * g], y[2 * g + 1]));
     } else if constexpr (EPI == WS_ROPE) {
       const int slot = re.slots[m];
       const int pblk = slot >= 0 ? slot / re.BS : 0, poff = slot >= 0 ? slot % re.BS : 0;

@@ -258,7 +258,7 @@ __global__ void __launch_bounds__(256) gemv_kernel(const uint16_t* __restrict__ 
 #pragma unroll
       for (int p = 0; p < RP; ++p)
         if (lane == m * RP + p && m < mc)
-          C[(size_t)m * ldc + set * RP + p] = f2bf(silu_bf(acc[p][m]) * bf2f(f2bf(acc[RP + p][m])));
+          C[(size_t)m * ldc + set * RP + p] = f2bf(glu_out(re, acc[p][m], acc[RP + p][m]));
   } else if constexpr (EPI == EPI_ROPE) {
     const int rope_sets = (re.Hq + re.Hkv) * (kHeadD / 2);
 #pragma unroll
@@ -376,12 +376,14 @@ bool gemv_takes(int M, int N, int K, int epi) {
 }
 
 void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ldc, int M, int N, int K,
-                 int epi, hipStream_t st) {
+                 int epi, hipStream_t st, float glu_alpha, float glu_limit) {
   auto* a = (const uint16_t*)A;
   auto* b = (const uint16_t*)B;
   auto* c = (uint16_t*)C;
   RopeEpi none{};
   none.relu2 = epi == kEpiRelu2;
+  none.glu_alpha = glu_alpha;
+  none.glu_limit = glu_limit;
   if (epi == EPI_SILU_MUL) run_gemv<EPI_SILU_MUL>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
   else run_gemv<EPI_NONE>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
 }

@@ -51,16 +51,24 @@ void launch_qk_norm(const QkNormArgs& a, bool f32, hipStream_t st);
 
 // ---- paged attention of any head sizes (attention_hd.hip)
 struct AttnHdArgs {
-  void* out;             // [T, H, V]
-  const void* q;         // [T, H, KP]
-  const void* k_cache;   // [NB, G, 16, KP]
-  const void* v_cache;   // [NB, G, 16, VP]
+  void* out;             // [T, H, V] (by_tile: [tiles, H, V])
+  const void* q;         // rows of KP per token (by_tile: per tile) and head
+  long q_row, q_head;    // strides of q (elements)
+  // keys and values, 16-token pages: row t of page p, head g at p * 16 * pitch + t * row + g * head.  Paged
+  // caches [NB, G, 16, KP]; or dense rows (xbase: row of a sequence's position 0), where pitch = row
+  const void* k_cache;
+  const void* v_cache;
+  long k_pitch, k_row, k_head, v_pitch, v_row, v_head;
+  const int* xbase;      // dense: [sequences]; null: paged
   const int* bt;
   int bt_stride;
   const int *q_start, *q_len, *ctx_len;
   const float* sink;     // [H] or null
-  const void* gate;      // [T, gate_stride] pre-sigmoid, one per head, or null
+  const void* gate;      // [T, gate_stride] pre-sigmoid, or null
   long gate_stride;
+  bool gate_elem;        // one gate per head and value element (H x V); else one per head
+  bool by_tile;          // q and out rows are decode tiles, not tokens
+  int window;            // a token sees itself and the window - 1 tokens before it (0: all)
   int H, G, D, V, KP, VP;
   float scale_log2;
   int num_blocks;
@@ -73,6 +81,7 @@ void launch_flash_hd(const AttnHdArgs& a, bool f32, const int* tile_seq, const i
                      hipStream_t st);
 constexpr int kHdTile = 128;      // query tokens of a flash tile
 constexpr int kHdMaxDim = 256;    // head sizes of the MFMA kernels (larger ones take the plain kernel)
+constexpr int kHdMaxLatent = 512; // same, decode with keys and values of one size
 constexpr int kHdMaxV = 1024;     // value size of the plain kernel
 
 // ---- gated linear attention (gla.hip)

@@ -74,7 +74,15 @@ struct RopeEpi {
   int mid_acq = 0;
   // plain epilogue only: C = bf16(max(acc, 0)^2) instead of bf16(acc) (EPI_RELU2 of launch_gemm)
   int relu2 = 0;
+  // SiLU-mul epilogue: alpha > 0 makes it the clamped gated unit (common.h clamp_glu_f) instead
+  float glu_alpha = 0.f, glu_limit = 0.f;
 };
+#ifdef __HIP__
+// one output of the gate / up epilogue
+__device__ __forceinline__ float glu_out(const RopeEpi& re, float g, float u) {
+  return re.glu_alpha > 0.f ? clamp_glu_f(g, u, re.glu_alpha, re.glu_limit) : silu_bf(g) * bf2f(f2bf(u));
+}
+#endif
 constexpr int kEpiRelu2 = 6;  // launch_gemm: plain product with the squared-relu epilogue
 // RoPE + paged-cache stores from the QKV projection's fp32 split-K slabs ws[splits][T][N] (the
 // split-K reduce fused in: small-M launch_gemm_rope)
@@ -119,7 +127,7 @@ int gemm_sk_workgroups(int M, int N, int K);
 // K2 skinny GEMV (gemv.hip): decode projections at M <= 8 (epi 0 none, 1 silu-mul, 3 rope)
 bool gemv_takes(int M, int N, int K, int epi);
 void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ldc, int M, int N, int K,
-                 int epi, hipStream_t st);
+                 int epi, hipStream_t st, float glu_alpha = 0.f, float glu_limit = 0.f);
 void launch_gemv_rope(const void* A, int lda, const void* B, int M, int N, int K, const RopeEpi& re,
                       hipStream_t st);
 // the decode norm chain's row-scale prologue parameters (gemv.hip PRO_RS)
@@ -165,7 +173,8 @@ bool gemm_rope_supported(int M, int N, int K);
 bool launch_gemm_rope(const void* A, int lda, const void* B, int M, int N, int K, const RopeEpi& re,
                       hipStream_t st);
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
-                 long ws_floats, int M, int N, int K, int epi, hipStream_t st);
+                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float glu_alpha = 0.f,
+                 float glu_limit = 0.f);
 bool launch_gemm_add_rmsnorm(const void* A, int lda, const void* B, void* out, void* residual,
                              const void* w, float eps, float* ws, long ws_floats, int M, int N,
                              int K, hipStream_t st);

@@ -208,6 +208,120 @@ def gla(proj, H, D, V, a2, a2_b, norm_w, tau, eps, state, meta):
     return o.to(proj.dtype)
 
 
+def residual_begin(ids, table, scale, pos_table, positions, norm_w, eps):
+    x = table[ids.reshape(-1).long()].float() * scale
+    if pos_table is not None:
+        x = x + pos_table[positions.long()].float()
+    return x, (_unit(x, eps) * norm_w).to(table.dtype)
+
+
+def residual_step(x, y, post_w, norm_w, eps):
+    x.add_(_unit(y.float(), eps) * post_w if post_w is not None else y.float())
+    return (_unit(x, eps) * norm_w).to(y.dtype)
+
+
+def gated_norm(y, gate, w, groups, eps, silu, gate_first):
+    T, n = y.shape
+    v, g = y.float(), gate.float()
+    g = torch.nn.functional.silu(g) if silu else torch.sigmoid(g)
+    if gate_first:
+        v = v * g
+    v = _unit(v.reshape(T, groups, -1), eps).reshape(T, n) * w
+    return (v if gate_first else v * g).to(y.dtype)
+
+
+def clamp_glu(x, alpha, limit):
+    """x [T, 2 I] = [gate | up]."""
+    g, u = x.float().chunk(2, -1)
+    g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+    return (g * torch.sigmoid(alpha * g) * (u + 1)).to(x.dtype)
+
+
+def short_conv(x, w, b, tail, meta):
+    out = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
+    P = w.shape[1] - 1
+    for row, s, n, ctx in _live_rows(meta):
+        old = torch.zeros_like(tail[row]) if ctx == n else tail[row]
+        seq = torch.cat([old, x[s:s + n].float()], 0)
+        for j in range(P + 1):
+            out[s:s + n] += seq[j:j + n] * w[:, j]
+        tail[row] = seq[len(seq) - P:]
+    if b is not None:
+        out = out + b
+    return torch.nn.functional.silu(out).to(x.dtype)
+
+
+def ssd(xbc, dt, G, dt_bias, a_neg, d_skip, state, meta):
+    _, H, N, V = state.shape
+    T = xbc.shape[0]
+    v = xbc.float()
+    x = v[:, :H * V].reshape(T, H, V)
+    B = v[:, H * V:H * V + G * N].reshape(T, G, N).repeat_interleave(H // G, 1)
+    C = v[:, H * V + G * N:].reshape(T, G, N).repeat_interleave(H // G, 1)
+    d = torch.nn.functional.softplus(dt.float() + dt_bias, threshold=1e9)
+    y = torch.zeros(T, H, V, dtype=torch.float32, device=xbc.device)
+    for row, s, n, ctx in _live_rows(meta):
+        S = torch.zeros_like(state[row]) if ctx == n else state[row]
+        for t in range(s, s + n):
+            S = torch.exp(a_neg * d[t])[:, None, None] * S + (d[t][:, None] * B[t])[:, :, None] * x[t][:, None, :]
+            y[t] = torch.einsum("hnv,hn->hv", S, C[t]) + d_skip[:, None] * x[t]
+        state[row] = S
+    return y.reshape(T, H * V).to(xbc.dtype)
+
+
+def delta(proj, w2, w0, a_b, decay_scale, unit_eps, state, meta):
+    _, H, D, V = state.shape
+    T, hk, hv = proj.shape[0], H * D, H * V
+    x = proj.float()
+    r, k = x[:, :hk].reshape(T, H, D), x[:, hk:2 * hk].reshape(T, H, D)
+    v = x[:, 2 * hk:2 * hk + hv].reshape(T, H, V)
+    a = torch.sigmoid(x[:, 2 * hk + hv:3 * hk + hv] + a_b).reshape(T, H, D)
+    z = torch.tanh(x[:, 3 * hk + hv:3 * hk + hv + w2.shape[1]]) @ w2.float().t() + w0
+    w = torch.exp(-decay_scale * torch.sigmoid(z)).reshape(T, H, D)
+    u = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + unit_eps)
+    o = torch.zeros(T, H, V, dtype=torch.float32, device=proj.device)
+    for row, s, n, ctx in _live_rows(meta):
+        S = torch.zeros_like(state[row]) if ctx == n else state[row]
+        for t in range(s, s + n):
+            z_t = torch.einsum("hd,hdv->hv", u[t], S)
+            S = w[t][:, :, None] * S - (a[t] * u[t])[:, :, None] * z_t[:, None, :] + k[t][:, :, None] * v[t][:, None, :]
+            o[t] = torch.einsum("hdv,hd->hv", S, r[t])
+        state[row] = S
+    return o.reshape(T, hv).to(proj.dtype)
+
+
+def latent_store(latents, w, eps, slots, cache):
+    c = (_unit(latents.float(), eps) * w).to(cache.dtype)
+    keep = slots >= 0
+    cache.view(-1, cache.shape[-1])[slots[keep].long(), :c.shape[1]] = c[keep]
+
+
+def latent_attention(q, gate, cache, w_kv, H, V, scale, window, sink, meta):
+    """q [T, H, KP]; w_kv [H (KP + VP), RP]: a head's keys, then values, of a latent row."""
+    T, KP = q.shape[0], q.shape[2]
+    VP = w_kv.shape[0] // H - KP
+    out = torch.zeros(T, H, V, dtype=torch.float32, device=q.device)
+    for row, s, n, ctx in _live_rows(meta):
+        c, _ = gather_kv(cache, cache, meta.block_tables[row], ctx)
+        kv = c[:, 0].float() @ w_kv.float().t()
+        k = kv[:, :H * KP].reshape(ctx, H, KP)
+        v = kv[:, H * KP:].reshape(ctx, H, VP)[..., :V]
+        sc = torch.einsum("qhd,khd->hqk", q[s:s + n].float(), k) * scale
+        pos = torch.arange(ctx - n, ctx, device=q.device)[:, None]
+        keys = torch.arange(ctx, device=q.device)[None]
+        hidden = keys > pos
+        if window:
+            hidden = hidden | (keys <= pos - window)
+        sc = sc.masked_fill(hidden[None], float("-inf"))
+        if sink is not None:
+            sc = torch.cat([sc, sink.float().view(H, 1, 1).expand(H, n, 1)], -1)
+        out[s:s + n] = torch.einsum("hqk,khd->qhd", torch.softmax(sc, -1)[..., :ctx], v)
+    out = out.reshape(T, H * V)
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float())
+    return out.to(q.dtype)
+
+
 # ------------------------------------------------------------------ MoE --
 
 def moe_route(logits, top_k):

@@ -52,6 +52,12 @@ class AttnMeta:
     crow_seq: torch.Tensor | None = None
     crow_item0: torch.Tensor | None = None
     chunk: int = 0
+    # layers that expand a portion's keys to dense rows: row of position p of sequence s is xbase[s] + p,
+    # x_rows rows in all, x_max of the longest sequence; the keys start at key_region_start
+    xbase: torch.Tensor | None = None
+    x_rows: int = 0
+    x_max: int = 0
+    x_window: int = 0
 
 
 # 128-token partitions: one 32-token page pair per wave at batch 1 (256: 312 tok/s, 128: 322,
@@ -104,16 +110,25 @@ def plan_partitions(num_tiles: int, n_kv: int, max_ctx: int, min_part: int | Non
     return part, nparts
 
 
+def key_region_start(start: int, window: int) -> int:
+    """First position of the keys a portion that starts at ``start`` needs (``window`` 0: all), on a
+    pair of pages."""
+    return max(0, start - window + 1) // 32 * 32 if window else 0
+
+
 class MetaBuffers:
     """Fixed-layout pinned host + device buffers for up to ``max_tokens`` tokens
     and ``max_seqs`` concurrent sequences."""
 
     def __init__(self, max_tokens: int, max_seqs: int, max_blocks_per_seq: int, group: int,
                  n_kv: int, max_model_len: int, device, flash_min_q: int = 17, flash_tile: int | None = None,
-                 part_dim: int = 128, chunk: int = 0, max_logits: int | None = None):
+                 part_dim: int = 128, chunk: int = 0, max_logits: int | None = None,
+                 expand_window: int | None = None):
         """``flash_tile``: query tokens of a prompt tile (default: 128 MFMA rows of the GQA group);
         ``part_dim``: value size of the split-KV partials; ``chunk``: prompt chunk of recurrent
-        layers (0: none); ``max_logits``: logits rows of a step (default: one per sequence)."""
+        layers (0: none); ``max_logits``: logits rows of a step (default: one per sequence);
+        ``expand_window``: the widest window of layers that expand a portion's keys (0: unbounded,
+        None: no such layer)."""
         self.device = torch.device(device)
         self.max_tokens, self.max_seqs, self.mb = max_tokens, max_seqs, max_blocks_per_seq
         self.G, self.n_kv, self.max_model_len = group, n_kv, max_model_len
@@ -129,6 +144,10 @@ class MetaBuffers:
                  ("q_start", max_seqs), ("q_len", max_seqs), ("ctx_len", max_seqs)]
         self.chunk = self.step_chunk = chunk
         self.n_items = self.n_crows = 0  # recurrent chunk items / rows of the last fill
+        self.expand_window = expand_window
+        self.x_rows = self.x_max = 0
+        if expand_window is not None:
+            sizes.append(("xbase", max_seqs))
         if chunk:
             ni = max_tokens // chunk + min(max_seqs, max_tokens // 2) + 1
             sizes += [("citem_seq", ni), ("citem_t0", ni), ("crow_seq", max_seqs), ("crow_item0", max_seqs)]
@@ -217,10 +236,14 @@ class MetaBuffers:
             logits_idx=self.lidx_d[:n_logits], num_tokens=num_tokens, part_sem=self.part_sem, **self._chunk_views())
 
     def _chunk_views(self) -> dict:
+        d = {}
+        if self.expand_window is not None:
+            d = {"xbase": self.view_d("xbase"), "x_rows": self.x_rows, "x_max": self.x_max,
+                 "x_window": self.expand_window}
         if not self.chunk:
-            return {}
+            return d
         n, r = self.n_items, self.n_crows
-        return {"citem_seq": self.view_d("citem_seq", n), "citem_t0": self.view_d("citem_t0", n),
+        return {**d, "citem_seq": self.view_d("citem_seq", n), "citem_t0": self.view_d("citem_t0", n),
                 "crow_seq": self.view_d("crow_seq", r), "crow_item0": self.view_d("crow_item0", r), "chunk": self.step_chunk}
 
     def fill(self, rows, q_lens, ctx_lens, token_ids_per_seq, want_logits=None):
@@ -249,7 +272,7 @@ class MetaBuffers:
         ts_h, tq_h = self.view_h("tile_seq"), self.view_h("tile_q0")
         pts_h, ptq_h = self.view_h("ptile_seq"), self.view_h("ptile_q0")
         npt, pqt = 0, self.pqt
-        ni = nr = 0
+        ni = nr = xr = xm = 0
         if self.chunk:
             # enough chunks to fill the chip either way: longer ones halve the chunk states' traffic
             self.step_chunk = self.chunk * (2 if sum(int(q) for q in q_lens) >= 64 * self.chunk else 1)
@@ -281,6 +304,10 @@ class MetaBuffers:
                 self.view_h("citem_seq")[ni:ni + n] = row
                 self.view_h("citem_t0")[ni:ni + n] = np.arange(n, dtype=np.int32) * self.step_chunk
                 ni, nr = ni + n, nr + 1
+            if self.expand_window is not None and ql > 1:
+                p0 = key_region_start(cl - ql, self.expand_window)
+                self.view_h("xbase")[row] = xr - p0
+                xr, xm = xr + cl - p0, max(xm, cl - p0)
             w = True if want_logits is None else want_logits[i]
             if isinstance(w, (list, tuple)):
                 self.lidx_hn[nl:nl + len(w)] = np.asarray(w, dtype=np.int64) + t
@@ -293,13 +320,14 @@ class MetaBuffers:
             order_flash_tiles(pts_h[:npt], ptq_h[:npt], self._pwork[:npt])
         self.npt = npt
         self.n_items, self.n_crows = ni, nr
+        self.x_rows, self.x_max = xr, xm
         return t, nt, nl
 
     def fill_decode(self, rows: np.ndarray, ctx_lens: np.ndarray, last_tokens: np.ndarray, pad_to: int):
         """Vectorised decode fill: one query token per sequence, padded to the
         graph bucket ``pad_to`` with rows that attend to nothing."""
         B = len(rows)
-        self.npt = self.n_items = self.n_crows = 0
+        self.npt = self.n_items = self.n_crows = self.x_rows = self.x_max = 0
         pos_h, slot_h = self.view_h("positions"), self.view_h("slots")
         ts_h, tq_h = self.view_h("tile_seq"), self.view_h("tile_q0")
         qs_h, ql_h, cl_h = self.view_h("q_start"), self.view_h("q_len"), self.view_h("ctx_len")
