@@ -1,8 +1,8 @@
-"""Prefill and decode throughput of the hybrid design beside the closest model of the package, at
+"""Prefill and decode throughput of the hybrid designs beside the closest models of the package, at
 equal layer sizes (``bench.py --hybrid``).
 
-Each pair is a Kosesun preset cut to a few layers and a Llama of the same width, head sizes, layer
-count, vocabulary and feed-forward parameters.  Both run through the engine's own scheduler
+Each size has a Regesun and a Kosesun preset cut to a few layers and a Llama, all of the same width,
+layer count, vocabulary and feed-forward parameters.  Both run through the engine's own scheduler
 (``add_request`` / ``step``; decode replays the captured graphs), random weights, random prompts,
 greedy sampling.  One JSON line per (model, workload); ``--hybrid-kernels`` adds each kernel's share
 of a profiled run.
@@ -26,14 +26,15 @@ PREFILL = ((1, 8192), (4, 2048), (16, 512))       # prompts x tokens, one step
 DECODE = ((1, 1024), (32, 1024), (256, 1024))     # sequences x context
 
 
-def pairs() -> list:
+def sizes() -> list:
     k8, k1 = get_config("kosesun-8b", num_layers=LAYERS), get_config("kosesun-1b", num_layers=LAYERS)
     l8 = get_config("llama3-8b", num_layers=LAYERS)
     # 3 W I = 2 W ff: the same feed-forward parameters (I in whole GEMM tiles)
     l1 = replace(LLAMA3_8B, name="llama-1b", num_layers=LAYERS, hidden_size=2048, intermediate_size=5376, num_heads=16,
                  num_kv_heads=4)
-    return [("8b", replace(k8, max_position=16384), replace(l8, max_position=16384)),
-            ("1b", replace(k1, max_position=16384), replace(l1, max_position=16384))]
+    r8, r1 = get_config("regesun-8b", num_layers=LAYERS), get_config("regesun-1b", num_layers=LAYERS)
+    return [("8b", *(replace(c, max_position=16384) for c in (r8, k8, l8))),
+            ("1b", *(replace(c, max_position=16384) for c in (r1, k1, l1)))]
 
 
 def _kernels(fn) -> list:
@@ -103,7 +104,7 @@ def _decode(eng, n, ctx, steps, kernels) -> dict:
 def main(device=None, steps: int = 64, kernels: bool = False, only: str = "") -> list:
     device = device or torch.device("cuda", 0)
     lines = []
-    for size, *cfgs in pairs():
+    for size, *cfgs in sizes():
         for cfg in cfgs:
             if only and only not in f"{size} {cfg.name}":
                 continue

@@ -1,5 +1,5 @@
-"""Shared helpers of the hybrid-decoder tests: small random Kosesun checkpoints, and one attention
-step's metadata with scattered pages."""
+"""Shared helpers of the hybrid decoders' tests: small random Kosesun checkpoints, and one step's metadata
+with scattered pages."""
 import json
 import math
 
@@ -20,7 +20,7 @@ class Step:
     """Rows with ``q_lens[i]`` new tokens on top of a context that ends at ``ctx[i]`` tokens, on
     shuffled pages, one-token rows first (as the engine orders them)."""
 
-    def __init__(self, q_lens, ctx, device, n_kv=1, chunk=64, min_part=None, part_dim=64, seed=0):
+    def __init__(self, q_lens, ctx, device, n_kv=1, chunk=64, min_part=None, part_dim=64, seed=0, expand_window=None):
         order = sorted(range(len(q_lens)), key=lambda i: q_lens[i] != 1)
         self.q_lens, self.ctx = [q_lens[i] for i in order], [ctx[i] for i in order]
         n = len(q_lens)
@@ -28,7 +28,7 @@ class Step:
         self.rows = rng.permutation(n + 2)[:n].astype(np.int32)
         longest = max(self.ctx)
         mb = MetaBuffers(max(sum(q_lens), 4), n + 2, blocks_needed(longest), 16, n_kv, longest, device, flash_min_q=2,
-                         flash_tile=128, part_dim=part_dim, chunk=chunk)
+                         flash_tile=128, part_dim=part_dim, chunk=chunk, expand_window=expand_window)
         pages = rng.permutation(sum(blocks_needed(c) for c in self.ctx)) + 1
         self.num_blocks = len(pages) + 1
         o = 0
