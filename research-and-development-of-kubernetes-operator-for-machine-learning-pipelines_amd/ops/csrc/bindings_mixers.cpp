@@ -180,7 +180,10 @@ void ssd(Tensor y, Tensor state, Tensor xbc, Tensor dt, int64_t G, Tensor dt_bia
   a.state = state.data_ptr<float>();
   const auto s = step_rows(q_start, q_len, ctx_len, rows, item_seq, item_t0, crow_seq, crow_item0, chunk, state.size(0));
   c10::DeviceGuard g(xbc.device());
-  mlop::launch_ssd(a, s, f32, cur());
+  Tensor ws;
+  if (s.n_items && a.N <= mlop::kSsdMaxN)
+    ws = at::empty({mlop::ssd_ws_floats(s.n_items, s.chunk, a.H)}, xbc.options().dtype(at::kFloat));
+  mlop::launch_ssd(a, s, ws.defined() ? ws.data_ptr<float>() : nullptr, f32, cur());
 }
 
 void delta(Tensor o, Tensor state, Tensor proj, Tensor w2, Tensor w0, Tensor a_b, double decay_scale, double unit_eps,

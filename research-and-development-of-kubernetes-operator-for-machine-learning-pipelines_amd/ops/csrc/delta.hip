@@ -371,17 +371,20 @@ __global__ void __launch_bounds__(256) delta_block_kernel(DeltaArgs a, StepRows 
   }
 }
 
-template <typename E, int KT>
-__global__ void __launch_bounds__(256, KT <= 1 ? 2 : 1) delta_walk_kernel(DeltaArgs a, StepRows r,
-                                                                         const float* __restrict__ ws) {
-  constexpr int NW = 4, DEPTH = 3;
+template <typename E, int NW, int KT>
+__global__ void __launch_bounds__(64 * NW) delta_walk_kernel(DeltaArgs a, StepRows r, const float* __restrict__ ws,
+                                                             int n_cols) {
+  constexpr int DEPTH = 3;
   __shared__ __attribute__((aligned(16))) f32x4 part[2][NW][2][64];
-  const int crow = blockIdx.x / a.H, h = blockIdx.x % a.H, s = r.crow_seq[crow];
+  // units: head by head, then portion, then columns: a head's columns read its blocks from one L2
+  const int unit = xcd_unit(blockIdx.x, a.H * r.n_crows * n_cols);
+  if (unit < 0) return;
+  const int h = unit / (r.n_crows * n_cols), crow = unit / n_cols % r.n_crows, s = r.crow_seq[crow];
   if (s >= r.n_slots) return;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l15 = lane & 15, g4 = lane >> 4;
   const int dk = a.dk, dv = a.dv, dkp = delta_dkp(dk), HK = a.H * dk, HV = a.H * dv;
   const int ql = r.q_len[s], ctx = r.ctx_len[s], q0 = r.q_start[s], nblk = cdiv(ql, kBlk);
-  const int col = (int)blockIdx.y * 16 + l15, colc = min(col, dv - 1), n0 = wid * KT * 16;
+  const int col = unit % n_cols * 16 + l15, colc = min(col, dv - 1), n0 = wid * KT * 16;
   const E* vp = reinterpret_cast<const E*>(a.proj) + (size_t)q0 * a.ldp + 2 * HK + h * dv + colc;
   const size_t per = (size_t)delta_per(dkp), stride = per * a.H;
   const float* base = ws + ((size_t)r.crow_item0[crow] * (r.chunk / kBlk) * a.H + h) * per;
@@ -400,7 +403,8 @@ __global__ void __launch_bounds__(256, KT <= 1 ? 2 : 1) delta_walk_kernel(DeltaA
     }
   }
   struct Ops {
-    f32x4 w[KT], r[KT], k[KT], a[KT], e[KT], m, am, v;
+    f32x4 w[KT], r[KT], k[KT], a[KT], e[KT], m, am;
+    E v[4];  // (as stored: converting here would wait for every load before)
   };
   auto fetch = [&](int blk, Ops& o) {
     const float* b = base + stride * blk;
@@ -417,15 +421,16 @@ __global__ void __launch_bounds__(256, KT <= 1 ? 2 : 1) delta_walk_kernel(DeltaA
     o.m = *reinterpret_cast<const f32x4*>(m + l15 * kBlk + 4 * g4);
     o.am = *reinterpret_cast<const f32x4*>(m + 256 + l15 * kBlk + 4 * g4);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) o.v[i] = ld1(vp + (size_t)min(blk * kBlk + 4 * g4 + i, ql - 1) * a.ldp);
+    for (int i = 0; i < 4; ++i) o.v[i] = vp[(size_t)min(blk * kBlk + 4 * g4 + i, ql - 1) * a.ldp];
   };
   auto step = [&](int blk, const Ops& o, Ops& fill) {
     if (blk + DEPTH - 1 < nblk) fetch(blk + DEPTH - 1, fill);
     const int buf = blk & 1;
+    const f32x4 v = {ld1(&o.v[0]), ld1(&o.v[1]), ld1(&o.v[2]), ld1(&o.v[3])};
     f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
     if (wid == 0) {
-      x = mfma_f32x16(o.m, o.v, x);
-      y = mfma_f32x16(o.am, o.v, y);
+      x = mfma_f32x16(o.m, v, x);
+      y = mfma_f32x16(o.am, v, y);
     }
 #pragma unroll
     for (int k = 0; k < KT; ++k) {
@@ -441,7 +446,7 @@ __global__ void __launch_bounds__(256, KT <= 1 ? 2 : 1) delta_walk_kernel(DeltaA
     part[buf][wid][1][lane] = y;
 #pragma unroll
     for (int k = 0; k < KT; ++k)
-      if (n0 + 16 * k < dkp) S[k] = mfma_f32x16(o.k[k], o.v, S[k] * o.e[k]);
+      if (n0 + 16 * k < dkp) S[k] = mfma_f32x16(o.k[k], v, S[k] * o.e[k]);
     lds_sync();
     x = part[buf][0][0][lane];
 #pragma unroll
@@ -515,16 +520,16 @@ static void delta_all(const DeltaArgs& a, const StepRows& s, float* ws, hipStrea
   delta_rows<E>(a, s, s.rows, s.n_rows, st);
   if (s.n_crows == 0) return;
   if (!delta_blocks_ok(a.dk, a.decay_scale)) return delta_rows<E>(a, s, s.crow_seq, s.n_crows, st);
-  const dim3 grid(s.n_crows * a.H, cdiv(a.dv, 16));
+  const int cols = cdiv(a.dv, 16), grid = xcd_grid(a.H * s.n_crows * cols);
   if (a.dk <= 64) {
     delta_blocks<E, 1>(a, s, ws, st);
-    delta_walk_kernel<E, 1><<<grid, 256, 0, st>>>(a, s, ws);
+    delta_walk_kernel<E, 4, 1><<<grid, 256, 0, st>>>(a, s, ws, cols);
   } else if (a.dk <= 128) {
     delta_blocks<E, 2>(a, s, ws, st);
-    delta_walk_kernel<E, 2><<<grid, 256, 0, st>>>(a, s, ws);
+    delta_walk_kernel<E, 8, 1><<<grid, 512, 0, st>>>(a, s, ws, cols);
   } else {
     delta_blocks<E, 4>(a, s, ws, st);
-    delta_walk_kernel<E, 4><<<grid, 256, 0, st>>>(a, s, ws);
+    delta_walk_kernel<E, 8, 2><<<grid, 512, 0, st>>>(a, s, ws, cols);
   }
 }
 

@@ -84,7 +84,9 @@ struct SsdArgs {
   float* state;           // [slots, H, N, V]
   int H, V, N, G;
 };
-void launch_ssd(const SsdArgs& a, const StepRows& s, bool f32, hipStream_t st);
+// one-token rows in place; portions in blocks of 16 tokens over `ws` (ssd_ws_floats)
+void launch_ssd(const SsdArgs& a, const StepRows& s, float* ws, bool f32, hipStream_t st);
+long ssd_ws_floats(int n_items, int chunk, int H);
 constexpr int kSsdMaxN = 256;    // state size of the prompt kernel (larger: token by token)
 
 // ---- generalized delta rule (delta.hip)

@@ -17,6 +17,22 @@ __device__ __forceinline__ f32x4 mfma_f32x16(const f32x4& a, const f32x4& b, f32
   return c;
 }
 
+// bf16 operands in the same 16-deep layout (lane: k = 4 (l >> 4) + i), exact products, fp32 sums
+using s16x4 = __attribute__((ext_vector_type(4))) short;
+__device__ __forceinline__ f32x4 mfma_bf16x16(const u32x2& a, const u32x2& b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(s16x4, a), __builtin_bit_cast(s16x4, b), c, 0, 0, 0);
+}
+// x = hi + mid + lo in bf16, to fp32 accuracy: with an exact bf16 operand, three bf16 products stand for an
+// fp32 one
+__device__ __forceinline__ void split3(const f32x4& x, u32x2 (&p)[3]) {
+  f32x4 r = x;
+#pragma unroll
+  for (int t = 0; t < 3; ++t) {
+    p[t] = u32x2{pack2(r[0], r[1]), pack2(r[2], r[3])};
+    if (t < 2) r -= f32x4{lo_bf(p[t][0]), hi_bf(p[t][0]), lo_bf(p[t][1]), hi_bf(p[t][1])};
+  }
+}
+
 // workgroup barrier for LDS hand-offs: global loads and stores stay in flight across it
 __device__ __forceinline__ void lds_sync() {
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -28,6 +44,27 @@ constexpr float kLog2E = 1.4426950408889634f;
 
 __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float sigmoid_acc(float x) { return 1.f / (1.f + expf(-x)); }
+
+// inclusive running sum over each row of 16 lanes
+__device__ __forceinline__ float scan16(float x) {
+#define MLOP_SHR(N)                                                                                            \
+  x += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x110 + N /* row_shr */, 0xF, 0xF, true))
+  MLOP_SHR(1);
+  MLOP_SHR(2);
+  MLOP_SHR(4);
+  MLOP_SHR(8);
+#undef MLOP_SHR
+  return x;
+}
+
+// Work units dealt to the 8 XCDs in contiguous ranges (workgroups go round them by their index), so that
+// neighbours share an L2.  Grid: xcd_grid(units); -1: no unit.
+constexpr int kXcds = 8;
+__host__ __device__ inline int xcd_grid(int units) { return (units + kXcds - 1) / kXcds * kXcds; }
+__device__ __forceinline__ int xcd_unit(int id, int units) {
+  const int per = (units + kXcds - 1) / kXcds, u = (id % kXcds) * per + id / kXcds;
+  return u < units ? u : -1;
+}
 
 // four elements p[0 .. 3], those past `left` zero; `vec`: the address is aligned to four elements
 template <typename E>
@@ -42,5 +79,41 @@ __device__ __forceinline__ f32x4 ld4m(const E* p, int left, bool vec) {
   }
   return f32x4{v[0], v[1], v[2], v[3]};
 }
+
+// Operands are kept as stored and converted where they are used, not where they are loaded, so that a
+// block's loads stay in flight together.  Eight consecutive elements; `last`: p[min(e, last)].
+template <typename E>
+struct Raw8;
+template <>
+struct Raw8<uint16_t> {
+  u32x4 v;
+  template <bool VEC>
+  __device__ __forceinline__ void load(const uint16_t* p, int last) {
+    if constexpr (VEC) {
+      v = *reinterpret_cast<const u32x4*>(p);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = (uint32_t)p[min(2 * e, last)] | (uint32_t)p[min(2 * e + 1, last)] << 16;
+    }
+  }
+  __device__ __forceinline__ f32x4 f(int k) const {  // elements 4 k .. + 3
+    return f32x4{lo_bf(v[2 * k]), hi_bf(v[2 * k]), lo_bf(v[2 * k + 1]), hi_bf(v[2 * k + 1])};
+  }
+};
+template <>
+struct Raw8<float> {
+  f32x4 v[2];
+  template <bool VEC>
+  __device__ __forceinline__ void load(const float* p, int last) {
+    if constexpr (VEC) {
+      v[0] = *reinterpret_cast<const f32x4*>(p);
+      v[1] = *reinterpret_cast<const f32x4*>(p + 4);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e >> 2][e & 3] = p[min(e, last)];
+    }
+  }
+  __device__ __forceinline__ f32x4 f(int k) const { return v[k]; }
+};
 
 }  // namespace mlop

@@ -15,6 +15,7 @@
 //                     per block.
 //
 // A sequence's first token starts from the zero state whatever its slot holds.
+#include <cstdlib>
 #include "mixers.h"
 #include "recur.h"
 
@@ -90,114 +91,174 @@ __global__ void __launch_bounds__(BT) ssd_rows_kernel(SsdArgs a, StepRows r, con
   }
 }
 
-template <typename E, int KT, int NC>
-__global__ void __launch_bounds__(256) ssd_walk_kernel(SsdArgs a, StepRows r) {
-  constexpr int NW = 4, M = 1 + NC;
+// Decays of a portion's blocks, per (block, head): running log2 decay b of the block's tokens, their step
+// sizes dt (0 past the portion), e^{b_16 - b} dt, e^b.  Lane = token, 16 heads per workgroup.
+constexpr int kSsdBlk = 16, kSsdDec = 4 * kSsdBlk;
+
+template <typename E>
+__global__ void __launch_bounds__(256) ssd_decay_kernel(SsdArgs a, StepRows r, float* __restrict__ ws) {
+  const int nb = r.chunk / kSsdBlk, item = blockIdx.x / nb, h = blockIdx.y * 16 + (threadIdx.x >> 4), l15 = threadIdx.x & 15;
+  const int s = r.item_seq[item], t = r.item_t0[item] + (int)blockIdx.x % nb * kSsdBlk + l15;
+  const bool in = t < r.q_len[s];
+  const int hc = min(h, a.H - 1);
+  const size_t row = (size_t)r.q_start[s] + (in ? t : 0);
+  const float raw = ld1(reinterpret_cast<const E*>(a.dt) + row * a.ldt + hc);
+  const float dt = in ? softplus_f(raw + a.dt_bias[hc]) : 0.f;
+  const float b = scan16(a.a_neg[hc] * kLog2E * dt), all = __shfl(b, 15, 16);
+  if (h >= a.H) return;
+  float* o = ws + ((size_t)blockIdx.x * a.H + h) * kSsdDec + l15;
+  o[0] = b;
+  o[16] = dt;
+  o[32] = exp2_f(all - b) * dt;
+  o[48] = exp2_f(b);
+}
+
+// State rows per wave: 32, in two accumulator tiles; tile k's row r is state row 8 (r >> 2) + 4 k + (r & 3), so
+// that a lane's eight consecutive elements of B or C are the operands of both.
+template <typename E, int NW, int NC, bool VEC>
+__global__ void __launch_bounds__(64 * NW) ssd_walk_kernel(SsdArgs a, StepRows r, const float* __restrict__ ws,
+                                                           int n_cols) {
+  constexpr int M = 1 + NC;
+  constexpr bool BF = sizeof(E) == 2;
   __shared__ __attribute__((aligned(16))) f32x4 part[2][NW][M][64];
-  const int crow = blockIdx.x / a.H, h = blockIdx.x % a.H, s = r.crow_seq[crow];
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l15 = lane & 15, g4 = lane >> 4;
+  // units: head by head (a group's heads share B and C in one L2), then portion, then columns
+  const int unit = xcd_unit(blockIdx.x, a.H * r.n_crows * n_cols);
+  if (unit < 0) return;
+  const int h = unit / (r.n_crows * n_cols), crow = unit / n_cols % r.n_crows, s = r.crow_seq[crow];
+  const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6)), l15 = lane & 15, g4 = lane >> 4;
   const int N = a.N, V = a.V, HV = a.H * V, grp = h / (a.H / a.G);
   const int ql = r.q_len[s], ctx = r.ctx_len[s], q0 = r.q_start[s];
   if (s >= r.n_slots) return;
-  const int col0 = (int)blockIdx.y * 16 * NC, n0 = wid * KT * 16;
-  const E* xr = reinterpret_cast<const E*>(a.xbc) + (size_t)q0 * a.ldx;
-  const E* xp = xr + h * V;
-  const E* bp = xr + HV + grp * N;
-  const E* cp = xr + HV + (a.G + grp) * N;
-  const E* dtp = reinterpret_cast<const E*>(a.dt) + (size_t)q0 * a.ldt + h;
-  const bool vec = HV % 4 == 0 && N % 4 == 0 && a.ldx % 4 == 0;
-  const float a2 = a.a_neg[h] * kLog2E, bias = a.dt_bias[h], dsk = a.d_skip[h];
+  const int col0 = unit % n_cols * 16 * NC, n0 = wid * 32;
+  const float dsk = a.d_skip[h];
   float* st = a.state + ((size_t)s * a.H + h) * N * V;
+  // this lane's state rows: 8 g4 + 4 k + i of the wave's (accumulators), and the one it feeds tile k (B^T)
+  const int d8 = n0 + 8 * g4, dt_row = n0 + 8 * (l15 >> 2) + (l15 & 3);
 
-  f32x4 S[KT][NC];
+  f32x4 S[2][NC];
 #pragma unroll
-  for (int k = 0; k < KT; ++k)
+  for (int k = 0; k < 2; ++k)
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       S[k][c] = f32x4{0.f, 0.f, 0.f, 0.f};
       const int col = col0 + 16 * c + l15;
       if (ctx != ql && col < V) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int d = n0 + 16 * k + 4 * g4 + i;
-          if (d < N) S[k][c][i] = st[(size_t)d * V + col];
-        }
+        for (int i = 0; i < 4; ++i)
+          if (d8 + 4 * k + i < N) S[k][c][i] = st[(size_t)(d8 + 4 * k + i) * V + col];
       }
     }
 
-  // a block's operands; rows past the portion repeat its last one (their dt is zero)
+  // A block's operands as stored.  Offsets from the block's first row are per lane and fixed but for a
+  // portion's last block, whose missing rows repeat its last one (their dt is zero); state rows past N
+  // repeat the last ones (zeroed where they are used).
   struct Ops {
-    f32x4 b[KT], c[KT], bt[KT], x[NC];
-    float dt;
+    Raw8<E> b, c;
+    E bt[2][4], x[NC][4];
+    float b1;
+    f32x4 bj, dj, sj, eb;
   };
+  const E* base = reinterpret_cast<const E*>(a.xbc) + (size_t)q0 * a.ldx;
+  const uint32_t ldx = (uint32_t)a.ldx, ob = HV + grp * N, oc = HV + (a.G + grp) * N;
+  const int dd = min(d8, VEC ? N - 8 : N - 1), last = N - 1 - dd;
+  uint32_t row1, rows[4];
+  auto offsets = [&](int n) {
+    row1 = (uint32_t)min(l15, n - 1) * ldx;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) rows[i] = (uint32_t)min(4 * g4 + i, n - 1) * ldx;
+  };
+  const float* dec = ws + ((size_t)r.crow_item0[crow] * (r.chunk / kSsdBlk) * a.H + h) * kSsdDec;
   auto fetch = [&](int t, Ops& o) {
-    const E* br = bp + (size_t)min(t + l15, ql - 1) * a.ldx;
-    const E* cr = cp + (size_t)min(t + l15, ql - 1) * a.ldx;
+    if (t + 16 > ql) offsets(ql - t);
+    const E* p = base + (size_t)t * ldx;
+    o.b.template load<VEC>(p + (row1 + ob + dd), last);
+    o.c.template load<VEC>(p + (row1 + oc + dd), last);
 #pragma unroll
-    for (int k = 0; k < KT; ++k) {
-      const int d = n0 + 16 * k + 4 * g4, dd = min(d, N - 1);
-      o.b[k] = ld4m(br + dd, N - d, vec);
-      o.c[k] = ld4m(cr + dd, N - d, vec);
-      const int dl = n0 + 16 * k + l15;
+    for (int k = 0; k < 2; ++k) {
+      const uint32_t dl = ob + min(dt_row + 4 * k, N - 1);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        o.bt[k][i] = dl < N ? ld1(bp + (size_t)min(t + 4 * g4 + i, ql - 1) * a.ldx + dl) : 0.f;
+      for (int i = 0; i < 4; ++i) o.bt[k][i] = p[rows[i] + dl];
     }
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
-      const int col = min(col0 + 16 * c + l15, V - 1);
+      const uint32_t col = h * V + min(col0 + 16 * c + l15, V - 1);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o.x[c][i] = ld1(xp + (size_t)min(t + 4 * g4 + i, ql - 1) * a.ldx + col);
+      for (int i = 0; i < 4; ++i) o.x[c][i] = p[rows[i] + col];
     }
-    o.dt = ld1(dtp + (size_t)min(t + l15, ql - 1) * a.ldt);
+    const float* d = dec + (size_t)(t / kSsdBlk) * a.H * kSsdDec;
+    o.b1 = d[l15];
+    o.bj = *reinterpret_cast<const f32x4*>(d + 4 * g4);
+    o.dj = *reinterpret_cast<const f32x4*>(d + 16 + 4 * g4);
+    o.sj = *reinterpret_cast<const f32x4*>(d + 32 + 4 * g4);
+    o.eb = *reinterpret_cast<const f32x4*>(d + 48 + 4 * g4);
   };
+  offsets(16);
   Ops cur, nxt;
   fetch(0, cur);
   for (int t = 0, blk = 0; t < ql; t += 16, ++blk) {
     if (t + 16 < ql) fetch(t + 16, nxt);
     const int buf = blk & 1;
-    // dt of token l15, running log2 decay over the block
-    const float dt = t + l15 < ql ? softplus_f(cur.dt + bias) : 0.f;
-    float b = a2 * dt;
-#pragma unroll
-    for (int d = 1; d < 16; d <<= 1) {
-      const float up = __shfl_up(b, d, 16);
-      if (l15 >= d) b += up;
-    }
-    const float ball = __shfl(b, 15);
-    float bj[4], dj[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      bj[i] = __shfl(b, 4 * g4 + i);
-      dj[i] = __shfl(dt, 4 * g4 + i);
-    }
-    f32x4 sc = {0.f, 0.f, 0.f, 0.f};  // row j = 4 g4 + i, column = token l15
+    f32x4 sc = {0.f, 0.f, 0.f, 0.f};  // B C^T: row j = 4 g4 + i, column = token l15
     f32x4 yp[NC];
 #pragma unroll
     for (int c = 0; c < NC; ++c) yp[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if constexpr (BF) {
+      u32x4 b = cur.b.v;
+      if (n0 + 32 > N) {  // (one side zero is enough)
 #pragma unroll
-    for (int k = 0; k < KT; ++k) {
-      sc = mfma_f32x16(cur.b[k], cur.c[k], sc);
+        for (int e = 0; e < 4; ++e)
+          b[e] = d8 + 2 * e + 1 < N ? b[e] : d8 + 2 * e < N ? b[e] & 0xffffu : 0u;
+      }
+      sc = mfma16(__builtin_bit_cast(bf16x8, b), __builtin_bit_cast(bf16x8, cur.c.v), sc);
+    }
 #pragma unroll
-      for (int c = 0; c < NC; ++c) yp[c] = mfma_f32x16(cur.c[k], S[k][c], yp[c]);
+    for (int k = 0; k < 2; ++k) {
+      const f32x4 ck = cur.c.f(k);
+      if constexpr (!BF) {
+        f32x4 bk = cur.b.f(k);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (d8 + 4 * k + i >= N) bk[i] = 0.f;
+        sc = mfma_f32x16(bk, ck, sc);
+      }
+#pragma unroll
+      for (int c = 0; c < NC; ++c) yp[c] = mfma_f32x16(ck, S[k][c], yp[c]);
     }
     part[buf][wid][0][lane] = sc;
 #pragma unroll
     for (int c = 0; c < NC; ++c) part[buf][wid][1 + c][lane] = yp[c];
     // the state behind the block
-    const float eall = exp2_f(ball);
-    float sj[4];
+    const float eall = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(cur.eb[3]), 63));
+    f32x4 x[NC];
+    u32x2 btp[2];
+    if constexpr (BF) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) sj[i] = exp2_f(ball - bj[i]) * dj[i];
+      for (int k = 0; k < 2; ++k) {
+        btp[k] = u32x2{(uint32_t)cur.bt[k][0] | (uint32_t)cur.bt[k][1] << 16, (uint32_t)cur.bt[k][2] | (uint32_t)cur.bt[k][3] << 16};
+        if (dt_row + 4 * k >= N) btp[k] = u32x2{0u, 0u};
+      }
+    }
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
-      f32x4 xs;
+      x[c] = f32x4{ld1(&cur.x[c][0]), ld1(&cur.x[c][1]), ld1(&cur.x[c][2]), ld1(&cur.x[c][3])};
+      const f32x4 xs = x[c] * cur.sj;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) xs[i] = cur.x[c][i] * sj[i];
+      for (int k = 0; k < 2; ++k) S[k][c] *= eall;
+      if constexpr (BF) {
+        u32x2 xp[3];
+        split3(xs, xp);
 #pragma unroll
-      for (int k = 0; k < KT; ++k) {
-        S[k][c] *= eall;
-        S[k][c] = mfma_f32x16(cur.bt[k], xs, S[k][c]);
+        for (int p = 2; p >= 0; --p)
+#pragma unroll
+          for (int k = 0; k < 2; ++k) S[k][c] = mfma_bf16x16(btp[k], xp[p], S[k][c]);
+      } else {
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+          f32x4 bt;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) bt[i] = dt_row + 4 * k < N ? ld1(&cur.bt[k][i]) : 0.f;
+          S[k][c] = mfma_f32x16(bt, xs, S[k][c]);
+        }
       }
     }
     lds_sync();
@@ -212,10 +273,10 @@ __global__ void __launch_bounds__(256) ssd_walk_kernel(SsdArgs a, StepRows r) {
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        G[i] = 4 * g4 + i <= l15 ? G[i] * dj[i] * exp2_f(b - bj[i]) : 0.f;
-        y[i] = fmaf(y[i], exp2_f(bj[i]), dsk * cur.x[c][i]);
+        G[i] = 4 * g4 + i <= l15 ? G[i] * cur.dj[i] * exp2_f(cur.b1 - cur.bj[i]) : 0.f;
+        y[i] = fmaf(y[i], cur.eb[i], dsk * x[c][i]);
       }
-      y = mfma_f32x16(G, cur.x[c], y);
+      y = mfma_f32x16(G, x[c], y);
       const int col = col0 + 16 * c + l15;
       E* out = reinterpret_cast<E*>(a.y) + (size_t)(q0 + t) * HV + h * V + col;
       if (col < V) {
@@ -227,15 +288,17 @@ __global__ void __launch_bounds__(256) ssd_walk_kernel(SsdArgs a, StepRows r) {
     cur = nxt;
   }
 #pragma unroll
-  for (int k = 0; k < KT; ++k)
+  for (int k = 0; k < 2; ++k)
 #pragma unroll
     for (int c = 0; c < NC; ++c)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int d = n0 + 16 * k + 4 * g4 + i, col = col0 + 16 * c + l15;
+        const int d = d8 + 4 * k + i, col = col0 + 16 * c + l15;
         if (d < N && col < V) st[(size_t)d * V + col] = S[k][c][i];
       }
 }
+
+static int g_ssd_wide = getenv("SSDW") ? atoi(getenv("SSDW")) : 256;
 
 template <typename E, int BT>
 static void ssd_rows_t(const SsdArgs& a, const StepRows& s, const int* rows, int n, hipStream_t st) {
@@ -254,25 +317,32 @@ static void ssd_rows(const SsdArgs& a, const StepRows& s, const int* rows, int n
 }
 
 template <typename E>
-static void ssd_all(const SsdArgs& a, const StepRows& s, hipStream_t st) {
+static void ssd_all(const SsdArgs& a, const StepRows& s, float* ws, hipStream_t st) {
   ssd_rows<E>(a, s, s.rows, s.n_rows, st);
   if (s.n_crows == 0) return;
   if (a.N > kSsdMaxN) return ssd_rows<E>(a, s, s.crow_seq, s.n_crows, st);
-  const bool wide = a.V > 16 && s.n_crows * a.H * cdiv(a.V, 32) >= 256;
-#define MLOP_WALK(KT)                                                                                             \
-  do {                                                                                                            \
-    if (wide) ssd_walk_kernel<E, KT, 2><<<dim3(s.n_crows * a.H, cdiv(a.V, 32)), 256, 0, st>>>(a, s);              \
-    else ssd_walk_kernel<E, KT, 1><<<dim3(s.n_crows * a.H, cdiv(a.V, 16)), 256, 0, st>>>(a, s);                   \
+  ssd_decay_kernel<E><<<dim3(s.n_items * (s.chunk / kSsdBlk), cdiv(a.H, 16)), 256, 0, st>>>(a, s, ws);
+  const bool vec = a.N % 8 == 0 && a.H * a.V % 8 == 0 && a.ldx % 8 == 0;
+  const int c1 = cdiv(a.V, 16), c2 = cdiv(a.V, 32), u1 = a.H * s.n_crows * c1, u2 = a.H * s.n_crows * c2;
+  const bool wide = a.V > 16 && u2 >= g_ssd_wide;  // (32 columns share the scores; 16 fill the chip sooner)
+#define MLOP_WALK(NW)                                                                                        \
+  do {                                                                                                       \
+    if (!vec) ssd_walk_kernel<E, NW, 1, false><<<xcd_grid(u1), 64 * NW, 0, st>>>(a, s, ws, c1);              \
+    else if (wide) ssd_walk_kernel<E, NW, 2, true><<<xcd_grid(u2), 64 * NW, 0, st>>>(a, s, ws, c2);          \
+    else ssd_walk_kernel<E, NW, 1, true><<<xcd_grid(u1), 64 * NW, 0, st>>>(a, s, ws, c1);                    \
   } while (0)
-  if (a.N <= 64) MLOP_WALK(1);
-  else if (a.N <= 128) MLOP_WALK(2);
-  else MLOP_WALK(4);
+  if (a.N <= 32) MLOP_WALK(1);
+  else if (a.N <= 64) MLOP_WALK(2);
+  else if (a.N <= 128) MLOP_WALK(4);
+  else MLOP_WALK(8);
 #undef MLOP_WALK
 }
 
-void launch_ssd(const SsdArgs& a, const StepRows& s, bool f32, hipStream_t st) {
-  if (f32) ssd_all<float>(a, s, st);
-  else ssd_all<uint16_t>(a, s, st);
+long ssd_ws_floats(int n_items, int chunk, int H) { return (long)n_items * (chunk / kSsdBlk) * H * kSsdDec; }
+
+void launch_ssd(const SsdArgs& a, const StepRows& s, float* ws, bool f32, hipStream_t st) {
+  if (f32) ssd_all<float>(a, s, ws, st);
+  else ssd_all<uint16_t>(a, s, ws, st);
 }
 
 }  // namespace mlop
