@@ -406,7 +406,10 @@ __global__ void __launch_bounds__(64 * NW) delta_walk_kernel(DeltaArgs a, StepRo
     f32x4 w[KT], r[KT], k[KT], a[KT], e[KT], m, am;
     E v[4];  // (as stored: converting here would wait for every load before)
   };
+  // (never conditional: a branch around loads makes every later wait drain them all; past the last block
+  // it repeats that one)
   auto fetch = [&](int blk, Ops& o) {
+    blk = min(blk, nblk - 1);
     const float* b = base + stride * blk;
 #pragma unroll
     for (int k = 0; k < KT; ++k) {
@@ -424,7 +427,7 @@ __global__ void __launch_bounds__(64 * NW) delta_walk_kernel(DeltaArgs a, StepRo
     for (int i = 0; i < 4; ++i) o.v[i] = vp[(size_t)min(blk * kBlk + 4 * g4 + i, ql - 1) * a.ldp];
   };
   auto step = [&](int blk, const Ops& o, Ops& fill) {
-    if (blk + DEPTH - 1 < nblk) fetch(blk + DEPTH - 1, fill);
+    fetch(blk + DEPTH - 1, fill);
     const int buf = blk & 1;
     const f32x4 v = {ld1(&o.v[0]), ld1(&o.v[1]), ld1(&o.v[2]), ld1(&o.v[3])};
     f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
@@ -468,12 +471,15 @@ __global__ void __launch_bounds__(64 * NW) delta_walk_kernel(DeltaArgs a, StepRo
   };
   Ops o0, o1, o2;
   fetch(0, o0);
-  if (nblk > 1) fetch(1, o1);
-  for (int blk = 0; blk < nblk; blk += DEPTH) {
+  fetch(1, o1);
+  int blk = 0;
+  for (; blk + DEPTH <= nblk; blk += DEPTH) {
     step(blk, o0, o2);
-    if (blk + 1 < nblk) step(blk + 1, o1, o0);
-    if (blk + 2 < nblk) step(blk + 2, o2, o1);
+    step(blk + 1, o1, o0);
+    step(blk + 2, o2, o1);
   }
+  if (blk < nblk) step(blk, o0, o2);
+  if (blk + 1 < nblk) step(blk + 1, o1, o0);
 #pragma unroll
   for (int k = 0; k < KT; ++k)
 #pragma unroll

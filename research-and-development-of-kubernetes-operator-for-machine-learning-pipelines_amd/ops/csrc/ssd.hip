@@ -168,7 +168,11 @@ __global__ void __launch_bounds__(64 * NW) ssd_walk_kernel(SsdArgs a, StepRows r
     for (int i = 0; i < 4; ++i) rows[i] = (uint32_t)min(4 * g4 + i, n - 1) * ldx;
   };
   const float* dec = ws + ((size_t)r.crow_item0[crow] * (r.chunk / kSsdBlk) * a.H + h) * kSsdDec;
+  const int t_last = (ql - 1) / kSsdBlk * kSsdBlk;
+  // (never conditional: a branch around loads makes every later wait drain them all; past the last block
+  // it repeats that one)
   auto fetch = [&](int t, Ops& o) {
+    t = min(t, t_last);
     if (t + 16 > ql) offsets(ql - t);
     const E* p = base + (size_t)t * ldx;
     o.b.template load<VEC>(p + (row1 + ob + dd), last);
@@ -193,11 +197,9 @@ __global__ void __launch_bounds__(64 * NW) ssd_walk_kernel(SsdArgs a, StepRows r
     o.eb = *reinterpret_cast<const f32x4*>(d + 48 + 4 * g4);
   };
   offsets(16);
-  Ops cur, nxt;
-  fetch(0, cur);
-  for (int t = 0, blk = 0; t < ql; t += 16, ++blk) {
-    if (t + 16 < ql) fetch(t + 16, nxt);
-    const int buf = blk & 1;
+  auto step = [&](int blk, const Ops& cur, Ops& fill) {
+    const int t = blk * kSsdBlk, buf = blk & 1;
+    fetch(t + 2 * kSsdBlk, fill);
     f32x4 sc = {0.f, 0.f, 0.f, 0.f};  // B C^T: row j = 4 g4 + i, column = token l15
     f32x4 yp[NC];
 #pragma unroll
@@ -285,8 +287,19 @@ __global__ void __launch_bounds__(64 * NW) ssd_walk_kernel(SsdArgs a, StepRows r
           if (t + 4 * g4 + i < ql) st1(out + (size_t)(4 * g4 + i) * HV, y[i]);
       }
     }
-    cur = nxt;
+  };
+  Ops o0, o1, o2;
+  fetch(0, o0);
+  fetch(kSsdBlk, o1);
+  const int nblk = cdiv(ql, kSsdBlk);
+  int blk = 0;
+  for (; blk + 3 <= nblk; blk += 3) {
+    step(blk, o0, o2);
+    step(blk + 1, o1, o0);
+    step(blk + 2, o2, o1);
   }
+  if (blk < nblk) step(blk, o0, o2);
+  if (blk + 1 < nblk) step(blk + 1, o1, o0);
 #pragma unroll
   for (int k = 0; k < 2; ++k)
 #pragma unroll
