@@ -86,7 +86,8 @@ def _stale(obj: Path, src: Path, headers, cmd) -> tuple[bool, str]:
 # forms have returned wrong results on this hardware, without an error.
 KERNEL_FLAGS = ["-ffp-contract=fast", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 FILE_FLAGS = {"attention": ["-fno-honor-nans", "-fno-slp-vectorize"],
-              "attention_hd": ["-fno-honor-nans", "-fno-slp-vectorize"]}
+              "attention_hd": ["-fno-honor-nans", "-fno-slp-vectorize"],
+              "latent_decode": ["-fno-honor-nans", "-fno-slp-vectorize"]}
 
 
 def _run(cmd):

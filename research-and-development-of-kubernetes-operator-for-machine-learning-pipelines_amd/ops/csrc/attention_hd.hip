@@ -13,8 +13,7 @@
 //   * sink: a number per head that joins the softmax's denominator once, with no key and no value;
 //   * gate: head h's output times sigmoid(gate[t, h]), or an element's with its own gate, in the epilogue;
 //   * window: a token sees itself and the window - 1 tokens before it; pages in front are not read;
-//   * a prompt's keys and values may also come from dense rows (latent attention's expanded keys), and
-//     decode's keys and values may be the same rows (its latents).
+//   * a prompt's keys and values may also come from dense rows (latent attention's expanded keys).
 // The sizes above 256 and fp32 operands take attn_any_kernel (one wave per query and head).
 //
 // REQUIREMENT: the cache is zero-initialised at allocation (as attention.hip's) and the pad
@@ -659,20 +658,14 @@ void launch_paged_hd(const AttnHdArgs& a, bool f32, float* part_o, float* part_m
                      const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st) {
   if (num_tiles == 0) return;
   if (f32) return run_any<float>(a, tile_seq, tile_q0, num_tiles, 1, st);
-  const bool latent = a.KP == a.VP && a.KP <= kHdMaxLatent;
-  if ((a.KP > kHdMaxDim || a.VP > kHdMaxDim) && !latent) return run_any<uint16_t>(a, tile_seq, tile_q0, num_tiles, 1, st);
+  if (latent_decode_ok(a, f32)) {
+    launch_latent_decode(a, part_o, part_ml, tile_seq, tile_q0, num_tiles, part_tokens, nparts, st);
+    return;
+  }
+  if (a.KP > kHdMaxDim || a.VP > kHdMaxDim) return run_any<uint16_t>(a, tile_seq, tile_q0, num_tiles, 1, st);
   const dim3 grid(num_tiles, a.G * cdiv(a.H / a.G, 16), nparts);
 #define MLOP_RUN(K, V) \
   paged_hd_kernel<K, V><<<grid, 256, 0, st>>>(a, part_o, part_ml, sem, tile_seq, tile_q0, part_tokens, nparts)
-  if (a.KP > kHdMaxDim) {
-    switch (a.KP / 64) {
-      case 5: MLOP_RUN(5, 5); break;
-      case 6: MLOP_RUN(6, 6); break;
-      case 7: MLOP_RUN(7, 7); break;
-      default: MLOP_RUN(8, 8); break;
-    }
-    return;
-  }
   MLOP_HD(MLOP_RUN)
 #undef MLOP_RUN
 }

@@ -218,13 +218,14 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
   a.q = q.data_ptr();
   a.k_cache = k_cache.data_ptr();
   a.v_cache = v_cache.data_ptr();
-  const bool plain = f32 || ((a.KP > mlop::kHdMaxDim || a.VP > mlop::kHdMaxDim) &&
-                             !(a.KP == a.VP && a.KP <= mlop::kHdMaxLatent));
+  const bool latent = mlop::latent_decode_ok(a, f32);
+  const bool plain = f32 || ((a.KP > mlop::kHdMaxDim || a.VP > mlop::kHdMaxDim) && !latent);
   TORCH_CHECK(part_tokens > 0 && part_tokens % 32 == 0 && nparts >= 1, "partition size");
   float *po = nullptr, *pml = nullptr;
   int* sem = nullptr;
   if (nparts > 1 && num_tiles && !plain) {
-    const int64_t units = num_tiles * a.G * ((a.H / a.G + 15) / 16);
+    // 16-head groups (the latent kernel: pairs of them)
+    const int64_t units = num_tiles * (latent ? (a.H + 31) / 32 * 2 : a.G * ((a.H / a.G + 15) / 16));
     TORCH_CHECK(part_o.scalar_type() == at::kFloat && part_ml.scalar_type() == at::kFloat &&
                     part_o.numel() >= units * nparts * 16 * a.VP && part_ml.numel() >= units * nparts * 16 * 2,
                 "partial workspace too small");

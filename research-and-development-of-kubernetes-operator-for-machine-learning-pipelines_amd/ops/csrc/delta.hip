@@ -39,7 +39,7 @@ __host__ __device__ constexpr int delta_dkp(int dk) { return (dk + 15) / 16 * 16
 __host__ __device__ constexpr long delta_per(int dkp) { return (long)dkp * 65 + 512; }
 
 // log2 decay of a channel from its logit
-__device__ __forceinline__ float log2_decay(const DeltaArgs& a, float z) { return -a.decay_scale * kLog2E * sigmoid_acc(z); }
+__device__ __forceinline__ float log2_decay(const DeltaArgs& a, float z) { return -a.decay_scale * kLog2E * sigmoid_hw(z); }
 
 }  // namespace
 
@@ -70,7 +70,7 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
   for (int t = 0; t < ql; ++t) {
     const E* row = reinterpret_cast<const E*>(a.proj) + (size_t)(q0 + t) * a.ldp;
     const bool fresh = ctx - ql + t == 0;
-    for (int i = tid; i < a.rank; i += BT) w1[i] = tanhf(ld1(row + 3 * HK + HV + i));
+    for (int i = tid; i < a.rank; i += BT) w1[i] = tanh_hw(ld1(row + 3 * HK + HV + i));
     __syncthreads();
     float ss = 0.f, rk = 0.f;
     for (int d = tid; d < dk; d += BT) {
@@ -80,7 +80,7 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
       const E* w2 = reinterpret_cast<const E*>(a.w2) + (size_t)n * a.rank;
       for (int i = 0; i < a.rank; ++i) z = fmaf(ld1(w2 + i), w1[i], z);
       wv[d] = exp2_f(log2_decay(a, z));
-      au[d] = sigmoid_acc(ld1(row + 2 * HK + HV + n) + a.a_b[n]);
+      au[d] = sigmoid_hw(ld1(row + 2 * HK + HV + n) + a.a_b[n]);
       kv[d] = k;
       rv[d] = rr;
       ss = fmaf(k, k, ss);
@@ -211,20 +211,51 @@ __global__ void __launch_bounds__(256) delta_block_kernel(DeltaArgs a, StepRows 
   float* oE = oA + kBlk * dkp;
   float* oM = oE + dkp;
 
-  float k[NP][4], rr[NP][4], aa[NP][4];
-  float ss[4] = {0.f, 0.f, 0.f, 0.f};
+  // every operand's loads first, as stored (the decay projection in steps of 16 RK ranks)
+  constexpr int RK = 4;
+  E rk[NP][4], rq[NP][4], ra_[NP][4];
   const E* rows[4];
 #pragma unroll
   for (int i = 0; i < 4; ++i) rows[i] = proj + (size_t)min(4 * g4 + i, nt - 1) * a.ldp;
+  int ch[NP];
+  float b0[NP], ab[NP];
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
-    const int d = (p * NW + wid) * 16 + l15, n = h * dk + min(d, dk - 1);
+    ch[p] = h * dk + min((p * NW + wid) * 16 + l15, dk - 1);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      rk[p][i] = rows[i][HK + ch[p]];
+      rq[p][i] = rows[i][ch[p]];
+      ra_[p][i] = rows[i][2 * HK + HV + ch[p]];
+    }
+    b0[p] = a.w0[ch[p]];
+    ab[p] = a.a_b[ch[p]];
+  }
+  const E* w1 = proj + (size_t)min(l15, nt - 1) * a.ldp + 3 * HK + HV;
+  const bool v1 = (3 * HK + HV) % 4 == 0 && a.ldp % 4 == 0 && rank % 4 == 0, v2 = rank % 4 == 0;
+  Raw4<E> x1[RK], w2[RK][NP];
+  auto fetch = [&](int r0) {
+#pragma unroll
+    for (int j = 0; j < RK; ++j) {
+      const int rc = min(r0 + 16 * j + 4 * g4, v2 ? rank - 4 : rank - 1);
+      x1[j].load(w1 + rc, rank - 1 - rc, v1);
+#pragma unroll
+      for (int p = 0; p < NP; ++p)
+        w2[j][p].load(reinterpret_cast<const E*>(a.w2) + (size_t)ch[p] * rank + rc, rank - 1 - rc, v2);
+    }
+  };
+  fetch(0);
+  float k[NP][4], rr[NP][4], aa[NP][4];
+  float ss[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int p = 0; p < NP; ++p) {
+    const int d = (p * NW + wid) * 16 + l15;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const bool ok = d < dk && 4 * g4 + i < nt;
-      k[p][i] = ok ? ld1(rows[i] + HK + n) : 0.f;
-      rr[p][i] = ok ? ld1(rows[i] + n) : 0.f;
-      aa[p][i] = ok ? ld1(rows[i] + 2 * HK + HV + n) : 0.f;
+      k[p][i] = ok ? ld1(&rk[p][i]) : 0.f;
+      rr[p][i] = ok ? ld1(&rq[p][i]) : 0.f;
+      aa[p][i] = ok ? ld1(&ra_[p][i]) : 0.f;
       ss[i] = fmaf(k[p][i], k[p][i], ss[i]);
     }
   }
@@ -239,22 +270,17 @@ __global__ void __launch_bounds__(256) delta_block_kernel(DeltaArgs a, StepRows 
   // decay logits of this wave's channels: rows = tokens, columns = channels
   f32x4 z[NP];
 #pragma unroll
-  for (int p = 0; p < NP; ++p) {
-    const int d = (p * NW + wid) * 16 + l15, n = h * dk + min(d, dk - 1);
-    const float b0 = a.w0[n];
-    z[p] = f32x4{b0, b0, b0, b0};
-  }
-  const E* w1 = proj + (size_t)min(l15, nt - 1) * a.ldp + 3 * HK + HV;
-  const bool v1 = (3 * HK + HV) % 4 == 0 && a.ldp % 4 == 0, v2 = rank % 4 == 0;
-  for (int r0 = 0; r0 < rank; r0 += 16) {
-    const int rc = r0 + 4 * g4;
-    f32x4 x = ld4m(w1 + rc, rank - rc, v1);
+  for (int p = 0; p < NP; ++p) z[p] = f32x4{b0[p], b0[p], b0[p], b0[p]};
+  for (int r0 = 0; r0 < rank; r0 += 16 * RK) {
+    if (r0) fetch(r0);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) x[i] = tanhf(x[i]);
+    for (int j = 0; j < RK; ++j) {
+      const int left = rank - (r0 + 16 * j + 4 * g4);
+      f32x4 x = x1[j].f(left);
 #pragma unroll
-    for (int p = 0; p < NP; ++p) {
-      const int d = (p * NW + wid) * 16 + l15, n = h * dk + min(d, dk - 1);
-      z[p] = mfma_f32x16(x, ld4m(reinterpret_cast<const E*>(a.w2) + (size_t)n * rank + rc, rank - rc, v2), z[p]);
+      for (int i = 0; i < 4; ++i) x[i] = tanh_hw(x[i]);
+#pragma unroll
+      for (int p = 0; p < NP; ++p) z[p] = mfma_f32x16(x, w2[j][p].f(left), z[p]);
     }
   }
   lds_sync();
@@ -268,7 +294,7 @@ __global__ void __launch_bounds__(256) delta_block_kernel(DeltaArgs a, StepRows 
   }
 #pragma unroll
   for (int p = 0; p < NP; ++p) {
-    const int d = (p * NW + wid) * 16 + l15, n = h * dk + min(d, dk - 1);
+    const int d = (p * NW + wid) * 16 + l15;
     if ((p * NW + wid) * 16 >= dkp) continue;  // whole waves
     float lw[4], b[4], sum = 0.f;
 #pragma unroll
@@ -284,13 +310,12 @@ __global__ void __launch_bounds__(256) delta_block_kernel(DeltaArgs a, StepRows 
       if (g < g4) before += x;
       all += x;
     }
-    const float ab = a.a_b[n];
     f32x4 kh, ah;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       b[i] += before;
       const int t = 4 * g4 + i;
-      const float u = k[p][i] * inv[i], au = sigmoid_acc(aa[p][i] + ab) * u;
+      const float u = k[p][i] * inv[i], au = sigmoid_hw(aa[p][i] + ab[p]) * u;
       const float eb = exp2_f(b[i]), en = exp2_f(-b[i]), el = exp2_f(all - b[i]);
       Bt[t * LD + d] = u * exp2_f(b[i] - lw[i]);
       At[t * LD + d] = -au * en;
@@ -371,10 +396,10 @@ __global__ void __launch_bounds__(256) delta_block_kernel(DeltaArgs a, StepRows 
   }
 }
 
-template <typename E, int NW, int KT>
+// DEPTH: blocks whose operands are in registers or on their way
+template <typename E, int NW, int KT, int DEPTH>
 __global__ void __launch_bounds__(64 * NW) delta_walk_kernel(DeltaArgs a, StepRows r, const float* __restrict__ ws,
                                                              int n_cols) {
-  constexpr int DEPTH = 3;
   __shared__ __attribute__((aligned(16))) f32x4 part[2][NW][2][64];
   // units: head by head, then portion, then columns: a head's columns read its blocks from one L2
   const int unit = xcd_unit(blockIdx.x, a.H * r.n_crows * n_cols);
@@ -469,17 +494,17 @@ __global__ void __launch_bounds__(64 * NW) delta_walk_kernel(DeltaArgs a, StepRo
       }
     }
   };
-  Ops o0, o1, o2;
-  fetch(0, o0);
-  fetch(1, o1);
+  Ops o[DEPTH];
+#pragma unroll
+  for (int j = 0; j < DEPTH - 1; ++j) fetch(j, o[j]);
   int blk = 0;
   for (; blk + DEPTH <= nblk; blk += DEPTH) {
-    step(blk, o0, o2);
-    step(blk + 1, o1, o0);
-    step(blk + 2, o2, o1);
+#pragma unroll
+    for (int j = 0; j < DEPTH; ++j) step(blk + j, o[j], o[(j + DEPTH - 1) % DEPTH]);
   }
-  if (blk < nblk) step(blk, o0, o2);
-  if (blk + 1 < nblk) step(blk + 1, o1, o0);
+#pragma unroll
+  for (int j = 0; j < DEPTH - 1; ++j)
+    if (blk + j < nblk) step(blk + j, o[j], o[(j + DEPTH - 1) % DEPTH]);
 #pragma unroll
   for (int k = 0; k < KT; ++k)
 #pragma unroll
@@ -529,13 +554,15 @@ static void delta_all(const DeltaArgs& a, const StepRows& s, float* ws, hipStrea
   const int cols = cdiv(a.dv, 16), grid = xcd_grid(a.H * s.n_crows * cols);
   if (a.dk <= 64) {
     delta_blocks<E, 1>(a, s, ws, st);
-    delta_walk_kernel<E, 4, 1><<<grid, 256, 0, st>>>(a, s, ws, cols);
+    delta_walk_kernel<E, 4, 1, 3><<<grid, 256, 0, st>>>(a, s, ws, cols);
   } else if (a.dk <= 128) {
     delta_blocks<E, 2>(a, s, ws, st);
-    delta_walk_kernel<E, 8, 1><<<grid, 512, 0, st>>>(a, s, ws, cols);
+    // few units: more waves on each (latency); many: fewer, with more in flight per CU
+    if (grid < 1024) delta_walk_kernel<E, 8, 1, 3><<<grid, 512, 0, st>>>(a, s, ws, cols);
+    else delta_walk_kernel<E, 4, 2, 3><<<grid, 256, 0, st>>>(a, s, ws, cols);
   } else {
     delta_blocks<E, 4>(a, s, ws, st);
-    delta_walk_kernel<E, 8, 2><<<grid, 512, 0, st>>>(a, s, ws, cols);
+    delta_walk_kernel<E, 8, 2, 2><<<grid, 512, 0, st>>>(a, s, ws, cols);
   }
 }
 

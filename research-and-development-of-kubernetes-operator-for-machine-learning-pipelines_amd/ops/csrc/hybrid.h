@@ -76,12 +76,17 @@ struct AttnHdArgs {
 // one query token per tile, split over `nparts` ranges of `part_tokens` keys
 void launch_paged_hd(const AttnHdArgs& a, bool f32, float* part_o, float* part_ml, int* sem, const int* tile_seq,
                      const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st);
+// the same with keys and values the same latent rows (latent_decode.hip): by_tile, one head of KP = VP <=
+// 512 elements; partials per 16 heads
+void launch_latent_decode(const AttnHdArgs& a, float* part_o, float* part_ml, const int* tile_seq, const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st);
+inline bool latent_decode_ok(const AttnHdArgs& a, bool f32) {
+  return !f32 && a.by_tile && a.G == 1 && a.k_cache == a.v_cache && a.KP == a.VP && a.V == a.VP && a.KP <= 512;
+}
 // tiles of up to 128 query tokens of one head
 void launch_flash_hd(const AttnHdArgs& a, bool f32, const int* tile_seq, const int* tile_q0, int num_tiles,
                      hipStream_t st);
 constexpr int kHdTile = 128;      // query tokens of a flash tile
 constexpr int kHdMaxDim = 256;    // head sizes of the MFMA kernels (larger ones take the plain kernel)
-constexpr int kHdMaxLatent = 512; // same, decode with keys and values of one size
 constexpr int kHdMaxV = 1024;     // value size of the plain kernel
 
 // ---- gated linear attention (gla.hip)

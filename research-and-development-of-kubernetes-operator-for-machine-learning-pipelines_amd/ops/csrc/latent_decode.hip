@@ -1,0 +1,297 @@
+// Decode attention over cached latents: one query token per tile, keys and values are the SAME rows of RP
+// elements (one latent head), so a step reads each latent once.
+//
+// A workgroup takes one tile, up to 32 heads and a partition of the keys, 32 keys (a page pair) at a
+// time through a two-stage LDS ring (LDS-DMA, one pair ahead).  Wave w works on head group w & 1 (16
+// heads, the MFMA columns) and half w >> 1 of the RP dims:
+//   S^T = C . Q^T over its half, the halves' partial scores meet in LDS, both waves run the same softmax,
+//   O^T += C^T . P^T for its half of the dims.
+// Every LDS row is read as K (ds_read_b128 along dims) and as V (ds_read_b64_tr_b16 along keys), so the
+// image [32 keys][128 B] per 64 dims has one swizzle for both: 16-B chunk c of key t at slot c ^ sw(t),
+// sw = (bit 1, bit 3, bit 2) of t, conflict-free for either kind of read.
+// Key partitions leave (O, max, sum), which a second launch joins head by head (one workgroup that joined
+// all of a token's heads would take longer than the attention itself).
+#include "elem.h"
+#include "hybrid.h"
+
+namespace mlop {
+
+namespace {
+
+constexpr int kPg = 16;
+constexpr float kLow = -1.0e30f;
+constexpr float kLog2e = 1.4426950408889634f;
+typedef short v4s16 __attribute__((ext_vector_type(4)));
+
+// LDS reads by hand: the compiler would make every one of them wait for the LDS-DMA in flight
+__device__ __forceinline__ void lds_read16(bf16x8& f, uint32_t ad) {
+  asm volatile("ds_read_b128 %0, %1" : "=v"(f) : "v"(ad));
+}
+__device__ __forceinline__ void lds_read_tr(v4s16& f, uint32_t ad) {
+  asm volatile("ds_read_b64_tr_b16 %0, %1" : "=v"(f) : "v"(ad));
+}
+// the reads older than the last `left` have arrived, a and b among them
+template <typename T>
+__device__ __forceinline__ void lds_wait(int left, T& a, T& b) {
+  switch (left) {  // (a constant at every call)
+    case 0: asm volatile("s_waitcnt lgkmcnt(0)" : "+v"(a), "+v"(b)); break;
+    case 2: asm volatile("s_waitcnt lgkmcnt(2)" : "+v"(a), "+v"(b)); break;
+    case 4: asm volatile("s_waitcnt lgkmcnt(4)" : "+v"(a), "+v"(b)); break;
+    default: asm volatile("s_waitcnt lgkmcnt(6)" : "+v"(a), "+v"(b)); break;
+  }
+}
+constexpr int kAhead = 4;  // pairs of reads in flight
+
+__device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ int sw(int t) { return ((t & 2) << 1) | ((t >> 2) & 2) | ((t >> 2) & 1); }
+
+}  // namespace
+
+// NB: 64-element blocks of a latent row
+template <int NB>
+__global__ void __launch_bounds__(256, 2) latent_decode_kernel(AttnHdArgs a, float* __restrict__ part_o,
+                                                              float* __restrict__ part_ml,
+                                                              const int* __restrict__ tile_seq,
+                                                              const int* __restrict__ tile_q0, int part_tokens, int nparts) {
+  constexpr int RP = 64 * NB, NH = (NB + 1) / 2, NK = 2 * NH, ND = 4 * NH;
+  constexpr uint32_t STAGE = NB * 4096u;  // bytes
+  __shared__ __attribute__((aligned(256))) uint16_t smem[2 * STAGE / 2];
+  __shared__ __attribute__((aligned(16))) f32x4 sx[2][2][2][64];  // partial scores [group][half][product]
+  const uint16_t* cc = reinterpret_cast<const uint16_t*>(a.k_cache);
+  uint16_t* out = reinterpret_cast<uint16_t*>(a.out);
+  const int tile = blockIdx.x, part = blockIdx.z, ny = gridDim.y;
+  const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
+  const int grp = wid & 1, half = wid >> 1, r = lane & 15, g4 = lane >> 4;
+  const int head0 = blockIdx.y * 32 + 16 * grp, nh = min(16, a.H - head0);  // (<= 0: no such group)
+  const int b0 = half * NH;                                                 // first block of this half
+  const int nb = min(NH, NB - b0);  // an odd NB leaves one less: the last block stands in, with zero queries
+  // (uniform, so that the page table is read through the scalar cache, not behind the LDS-DMA)
+  const int s = __builtin_amdgcn_readfirstlane(tile_seq[tile]), qi = __builtin_amdgcn_readfirstlane(tile_q0[tile]);
+  const int ql = __builtin_amdgcn_readfirstlane(a.q_len[s]), ctx = __builtin_amdgcn_readfirstlane(a.ctx_len[s]);
+  const int* bt = a.bt + (size_t)s * a.bt_stride;
+  const bool live = qi < ql;
+  const int kv_end = live ? max(0, ctx - ql + qi + 1) : 0;
+  const int k_lo = a.window > 0 ? max(0, kv_end - a.window) : 0, k_base = k_lo & ~31;
+  const int p_begin = k_base + part * part_tokens;
+  const int p_end = min(kv_end, p_begin + part_tokens);
+  const int h_all = min(32, a.H - (int)blockIdx.y * 32);
+  uint16_t* orow = out + ((size_t)tile * a.H + blockIdx.y * 32) * RP;
+  if (p_begin >= p_end) {  // nothing here; an empty row (graph padding) gives zeros
+    if (part == 0 && kv_end <= 0 && live)
+      for (int e = threadIdx.x; e < h_all * RP; e += 256) orow[e] = 0;
+    return;
+  }
+
+  bf16x8 qf[NK];
+  {
+    const bool ok = r < nh;
+    const uint16_t* qrow = reinterpret_cast<const uint16_t*>(a.q) + (size_t)tile * a.q_row + (ok ? head0 + r : 0) * a.q_head +
+                           b0 * 64 + g4 * 8;
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk) {
+      bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (ok && (kk >> 1) < nb) v = *reinterpret_cast<const bf16x8*>(qrow + kk * 32);
+      qf[kk] = v;
+    }
+  }
+  f32x4 o[ND];
+#pragma unroll
+  for (int d = 0; d < ND; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = kLow, l = 0.f;
+  const int pp0 = p_begin >> 5, pp_end = (p_end + 31) >> 5, n_pages = (p_end + kPg - 1) / kPg;
+  // LDS-DMA: wave w brings rows 8 w .. 8 w + 7 of every block (page A: waves 0, 1; page B: 2, 3)
+  const int row32 = 8 * wid + (lane >> 3), row = row32 & 15;
+  const uint32_t src_off = row * RP + (((lane & 7) ^ sw(row)) << 3);
+  auto page_of = [&](int pp) {
+    const auto* pages = (const __attribute__((address_space(4))) int*)(uintptr_t)bt;  // (constant: scalar loads)
+    return min(max(pages[min(2 * pp + (wid >> 1), n_pages - 1)], 0), a.num_blocks - 1);
+  };
+  auto issue = [&](int buf, int pg) {
+    uint16_t* base = smem + buf * (STAGE / 2) + wid * 512;
+    const uint16_t* src = cc + (size_t)pg * (kPg * RP) + src_off;
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
+      __builtin_amdgcn_global_load_lds((const void*)(src + b * 64), (lds_void_t*)(base + b * 2048), 16, 0, 0);
+  };
+  const uint32_t lds0 = (uint32_t)(uintptr_t)smem;
+  auto block = [&](int b) { return 4096u * (NB % 2 ? min(b0 + b, NB - 1) : b0 + b); };
+  // K: MFMA row r is key 8 (r >> 2) + (r & 3) of the pair in the first product, + 4 in the second
+  const int kt = 8 * (r >> 2) + (r & 3);
+  const uint32_t ka0 = lds0 + 128u * kt + 16u * (g4 ^ sw(kt & 15)), kb0 = lds0 + 128u * (kt + 4) + 16u * (g4 ^ sw((kt + 4) & 15));
+  // V: transposed reads of keys 8 g4 + q (first) and + 4 (second), 16 dims at a time
+  const int q = (lane >> 2) & 3, p4 = lane & 3, vt = 8 * g4 + q;
+  const uint32_t va0 = lds0 + 128u * vt + 16u * ((p4 >> 1) ^ sw(vt & 15)) + 8u * (p4 & 1);
+  const uint32_t vb0 = lds0 + 128u * (vt + 4) + 16u * ((p4 >> 1) ^ sw((vt + 4) & 15)) + 8u * (p4 & 1);
+
+  const uint32_t sx_own = (uint32_t)(uintptr_t)&sx[grp][half][0][lane], sx_other = (uint32_t)(uintptr_t)&sx[grp][half ^ 1][0][lane];
+  issue(0, page_of(pp0));
+  int nxt = page_of(pp0 + 1), buf = 0;
+  for (int pp = pp0; pp < pp_end; ++pp) {
+    wait_vmcnt<0>();
+    raw_barrier();  // the pair is in LDS for every wave; the other stage is free, and so is sx
+    if (pp + 1 < pp_end) {
+      issue(buf ^ 1, nxt);
+      nxt = page_of(pp + 2);
+    }
+    const uint32_t so = buf * STAGE;
+    f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = sa;
+    {
+      bf16x8 fa[kAhead], fb[kAhead];
+      auto rd = [&](int kk) {
+        const uint32_t off = so + block(kk >> 1), x = 64u * (kk & 1);
+        lds_read16(fa[kk % kAhead], (ka0 ^ x) + off);
+        lds_read16(fb[kk % kAhead], (kb0 ^ x) + off);
+      };
+#pragma unroll
+      for (int kk = 0; kk < kAhead && kk < NK; ++kk) rd(kk);
+#pragma unroll
+      for (int kk = 0; kk < NK; ++kk) {
+        lds_wait(2 * (NK - 1 - kk < kAhead - 1 ? NK - 1 - kk : kAhead - 1), fa[kk % kAhead], fb[kk % kAhead]);
+        sa = mfma16(fa[kk % kAhead], qf[kk], sa);
+        sb = mfma16(fb[kk % kAhead], qf[kk], sb);
+        if (kk + kAhead < NK) rd(kk + kAhead);
+      }
+    }
+    asm volatile("ds_write_b128 %0, %1\n\tds_write_b128 %0, %2 offset:1024\n\ts_waitcnt lgkmcnt(0)" ::"v"(sx_own), "v"(sa), "v"(sb)
+                 : "memory");
+    raw_barrier();
+    {
+      f32x4 ta, tb;
+      asm volatile("ds_read_b128 %0, %2\n\tds_read_b128 %1, %2 offset:1024\n\ts_waitcnt lgkmcnt(0)"
+                   : "=&v"(ta), "=&v"(tb)
+                   : "v"(sx_other)
+                   : "memory");
+      sa += ta;
+      sb += tb;
+    }
+    const int tokA = pp * 32 + g4 * 8, tokB = tokA + 4;
+    float pa[4], pb[4], mx = kLow;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      pa[i] = tokA + i < p_end && tokA + i >= k_lo ? sa[i] * a.scale_log2 : -INFINITY;
+      pb[i] = tokB + i < p_end && tokB + i >= k_lo ? sb[i] * a.scale_log2 : -INFINITY;
+      mx = fmaxf(mx, fmaxf(pa[i], pb[i]));
+    }
+    mx = max_x16_x32(mx);
+    const float m_new = fmaxf(m, mx), alpha = exp2_hw(m - m_new);
+    m = m_new;
+    float rs = 0.f;
+    bf16x8 pf;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      pa[i] = exp2_hw(pa[i] - m_new);
+      pb[i] = exp2_hw(pb[i] - m_new);
+      rs += pa[i] + pb[i];
+      pf[i] = (short)f2bf(pa[i]);
+      pf[4 + i] = (short)f2bf(pb[i]);
+    }
+    l = l * alpha + rs;
+    if (__ballot(alpha != 1.f)) {
+#pragma unroll
+      for (int d = 0; d < ND; ++d) o[d] *= alpha;
+    }
+    {
+      v4s16 lo[kAhead], hi[kAhead];
+      auto rd = [&](int d) {
+        const uint32_t off = so + block(d >> 2), x = 32u * (d & 3);
+        lds_read_tr(lo[d % kAhead], (va0 ^ x) + off);
+        lds_read_tr(hi[d % kAhead], (vb0 ^ x) + off);
+      };
+#pragma unroll
+      for (int d = 0; d < kAhead; ++d) rd(d);
+#pragma unroll
+      for (int d = 0; d < ND; ++d) {
+        lds_wait(2 * (ND - 1 - d < kAhead - 1 ? ND - 1 - d : kAhead - 1), lo[d % kAhead], hi[d % kAhead]);
+        bf16x8 f;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          f[e] = lo[d % kAhead][e];
+          f[4 + e] = hi[d % kAhead][e];
+        }
+        o[d] = mfma16(f, pf, o[d]);
+        if (d + kAhead < ND) rd(d + kAhead);
+      }
+    }
+    buf ^= 1;
+  }
+  l = sum_x16_x32(l);
+  const bool ok = r < nh;
+  const size_t slab = (((size_t)tile * ny + blockIdx.y) * 2 + grp) * nparts;  // 16 heads each
+  if (nparts == 1) {
+    float L = l, f = 1.f;
+    if (a.sink && ok) {
+      const float s2 = a.sink[head0 + r] * kLog2e, M = fmaxf(m, s2);
+      f = exp2f(m - M);
+      L = l * f + exp2f(s2 - M);
+    }
+    const float inv = L > 0.f ? f / L : 0.f;
+    if (ok) {
+#pragma unroll
+      for (int d = 0; d < ND; ++d)
+        if ((d >> 2) < nb) {
+          const float v[4] = {o[d][0] * inv, o[d][1] * inv, o[d][2] * inv, o[d][3] * inv};
+          stn<4>(orow + (size_t)(16 * grp + r) * RP + b0 * 64 + 16 * d + 4 * g4, v);
+        }
+    }
+    return;
+  }
+  // partial (O, m, l) of this key range
+  if (ok) {
+    float* po = part_o + ((slab + part) * 16 + r) * RP + b0 * 64 + 4 * g4;
+#pragma unroll
+    for (int d = 0; d < ND; ++d)
+      if ((d >> 2) < nb) *reinterpret_cast<f32x4*>(po + 16 * d) = o[d];
+    if (half == 0 && g4 == 0) {
+      float* ml = part_ml + ((slab + part) * 16 + r) * 2;
+      ml[0] = m;
+      ml[1] = l;
+    }
+  }
+}
+
+// the partitions of one (tile, head): 4 elements per thread
+__global__ void __launch_bounds__(128) latent_combine_kernel(AttnHdArgs a, const float* __restrict__ part_o,
+                                                             const float* __restrict__ part_ml,
+                                                             const int* __restrict__ tile_seq,
+                                                             const int* __restrict__ tile_q0, int part_tokens, int nparts) {
+  const int tile = blockIdx.x, head = blockIdx.y, c = threadIdx.x * 4, RP = a.KP;
+  const int s = tile_seq[tile], qi = tile_q0[tile], ql = a.q_len[s], ctx = a.ctx_len[s];
+  const int kv_end = qi < ql ? max(0, ctx - ql + qi + 1) : 0;
+  if (kv_end == 0 || c >= RP) return;  // (an empty row was zeroed)
+  const int k_base = (a.window > 0 ? max(0, kv_end - a.window) : 0) & ~31;
+  const int nvalid = min(nparts, (kv_end - k_base + part_tokens - 1) / part_tokens);
+  const size_t slab = ((size_t)tile * (cdiv(a.H, 32) * 2) + (head >> 4)) * nparts * 16 + (head & 15);
+  const float* ml = part_ml + slab * 2;
+  const float* po = part_o + slab * RP + c;
+  const float s2 = a.sink ? a.sink[head] * kLog2e : kLow;
+  float M = s2;
+  for (int p = 0; p < nvalid; ++p) M = fmaxf(M, ml[p * 32]);
+  float L = a.sink ? exp2f(s2 - M) : 0.f;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int p = 0; p < nvalid; ++p) {
+    const float f = exp2f(ml[p * 32] - M);
+    L += f * ml[p * 32 + 1];
+    acc += f * *reinterpret_cast<const f32x4*>(po + (size_t)p * 16 * RP);
+  }
+  const float inv = L > 0.f ? 1.f / L : 0.f;
+  const float v[4] = {acc[0] * inv, acc[1] * inv, acc[2] * inv, acc[3] * inv};
+  stn<4>(reinterpret_cast<uint16_t*>(a.out) + ((size_t)tile * a.H + head) * RP + c, v);
+}
+
+void launch_latent_decode(const AttnHdArgs& a, float* part_o, float* part_ml, const int* tile_seq,
+                          const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st) {
+  const dim3 grid(num_tiles, cdiv(a.H, 32), nparts);
+#define MLOP_LD(N) \
+  case N: latent_decode_kernel<N><<<grid, 256, 0, st>>>(a, part_o, part_ml, tile_seq, tile_q0, part_tokens, nparts); break;
+  switch (a.KP / 64) {
+    MLOP_LD(1) MLOP_LD(2) MLOP_LD(3) MLOP_LD(4) MLOP_LD(5) MLOP_LD(6) MLOP_LD(7) MLOP_LD(8)
+    default: break;
+  }
+#undef MLOP_LD
+  if (nparts > 1)
+    latent_combine_kernel<<<dim3(num_tiles, a.H), cdiv(a.KP, 256) * 64, 0, st>>>(a, part_o, part_ml, tile_seq, tile_q0,
+                                                                                part_tokens, nparts);
+}
+
+}  // namespace mlop

@@ -43,7 +43,9 @@ __device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f
 constexpr float kLog2E = 1.4426950408889634f;
 
 __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
-__device__ __forceinline__ float sigmoid_acc(float x) { return 1.f / (1.f + expf(-x)); }
+// to a few fp32 ulp (of 1 for tanh), by the hardware's exp2 and reciprocal
+__device__ __forceinline__ float sigmoid_hw(float x) { return __builtin_amdgcn_rcpf(1.f + exp2_f(-kLog2E * x)); }
+__device__ __forceinline__ float tanh_hw(float x) { return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + exp2_f(2.f * kLog2E * x)); }
 
 // inclusive running sum over each row of 16 lanes
 __device__ __forceinline__ float scan16(float x) {
@@ -65,6 +67,31 @@ __device__ __forceinline__ int xcd_unit(int id, int units) {
   const int per = (units + kXcds - 1) / kXcds, u = (id % kXcds) * per + id / kXcds;
   return u < units ? u : -1;
 }
+
+// four elements as stored (see Raw8); the address is aligned to four elements if `vec`
+template <typename E>
+struct Raw4 {
+  E v[4];
+  __device__ __forceinline__ void load(const E* p, int last, bool vec) {  // p[min(e, last)]
+    if (vec) {
+      if constexpr (sizeof(E) == 2) {
+        const u32x2 t = *reinterpret_cast<const u32x2*>(p);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = (E)(t[e >> 1] >> (16 * (e & 1)));
+      } else {
+        const f32x4 t = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = (E)t[e];
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = p[min(e, last)];
+    }
+  }
+  __device__ __forceinline__ f32x4 f(int n) const {  // the first n, zeros behind them
+    return f32x4{n > 0 ? ld1(&v[0]) : 0.f, n > 1 ? ld1(&v[1]) : 0.f, n > 2 ? ld1(&v[2]) : 0.f, n > 3 ? ld1(&v[3]) : 0.f};
+  }
+};
 
 // four elements p[0 .. 3], those past `left` zero; `vec`: the address is aligned to four elements
 template <typename E>

@@ -15,7 +15,6 @@
 //                     per block.
 //
 // A sequence's first token starts from the zero state whatever its slot holds.
-#include <cstdlib>
 #include "mixers.h"
 #include "recur.h"
 
@@ -311,8 +310,6 @@ __global__ void __launch_bounds__(64 * NW) ssd_walk_kernel(SsdArgs a, StepRows r
       }
 }
 
-static int g_ssd_wide = getenv("SSDW") ? atoi(getenv("SSDW")) : 256;
-
 template <typename E, int BT>
 static void ssd_rows_t(const SsdArgs& a, const StepRows& s, const int* rows, int n, hipStream_t st) {
   const bool v4 = a.V % 4 == 0;
@@ -337,7 +334,7 @@ static void ssd_all(const SsdArgs& a, const StepRows& s, float* ws, hipStream_t 
   ssd_decay_kernel<E><<<dim3(s.n_items * (s.chunk / kSsdBlk), cdiv(a.H, 16)), 256, 0, st>>>(a, s, ws);
   const bool vec = a.N % 8 == 0 && a.H * a.V % 8 == 0 && a.ldx % 8 == 0;
   const int c1 = cdiv(a.V, 16), c2 = cdiv(a.V, 32), u1 = a.H * s.n_crows * c1, u2 = a.H * s.n_crows * c2;
-  const bool wide = a.V > 16 && u2 >= g_ssd_wide;  // (32 columns share the scores; 16 fill the chip sooner)
+  const bool wide = a.V > 16 && u2 >= 256;  // (32 columns share the scores; 16 fill the chip sooner)
 #define MLOP_WALK(NW)                                                                                        \
   do {                                                                                                       \
     if (!vec) ssd_walk_kernel<E, NW, 1, false><<<xcd_grid(u1), 64 * NW, 0, st>>>(a, s, ws, c1);              \
