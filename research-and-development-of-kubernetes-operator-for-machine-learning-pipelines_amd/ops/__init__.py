@@ -917,7 +917,7 @@ def latent_attention(q, gate, cache, w_kv, w_qk, w_vo, vdim: int, scale: float, 
         ol = torch.empty_like(ql)
         keys = meta.part_tokens * meta.nparts
         part, nparts = plan_partitions(nt, -(-H // 32), min(keys, window + 31) if window else keys,
-                                       min_part=int(os.environ.get('LMP', '128')))
+                                       target_wgs=512)
         op.attention_hd(ol, meta.part_o, meta.part_ml, meta.part_sem, ql, cache, cache, meta.block_tables, meta.tile_seq,
                         meta.tile_q0, none, none, *step, RP, scale, sink, None, part, nparts, window, None, True)
         op.head_mm(out.view(T, H, vdim), ol, w_vo, meta.tile_seq, meta.tile_q0, meta.q_start, meta.q_len, False, True, gate)

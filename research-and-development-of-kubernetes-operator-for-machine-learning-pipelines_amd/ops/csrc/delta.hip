@@ -43,15 +43,16 @@ __device__ __forceinline__ float log2_decay(const DeltaArgs& a, float z) { retur
 
 }  // namespace
 
-// NR: key rows of a strip that stay in a thread's registers between the two passes (0: read twice)
+// NR: key rows of a strip that a thread keeps in registers from their loads, in front of everything else,
+// to the stores (one strip per thread, then); 0: the state is read twice.
 template <typename E, int VEC, int BT, int NR>
 __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r, const int* __restrict__ rows) {
   extern __shared__ float sm[];
-  __shared__ float scratch[16];
+  __shared__ float scratch[3][BT / 64];
   const int s = rows[blockIdx.x], h = blockIdx.y, tid = threadIdx.x;
   const int dk = a.dk, dv = a.dv, HK = a.H * dk, HV = a.H * dv;
   float* w1 = sm;                  // [rank]
-  float* wv = w1 + a.rank;         // [dk] each
+  float* wv = w1 + a.rank;         // [dk] each: decay, unit key, removal, key, w r
   float* uv = wv + dk;
   float* au = uv + dk;
   float* kv = au + dk;
@@ -66,54 +67,86 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
     return;
   }
   float* S = a.state + ((size_t)s * a.H + h) * dk * dv;
-  const int nstrip = dv / VEC, per = min(nstrip, BT), RG = BT / per;
+  const int nstrip = dv / VEC, per = min(nstrip, BT), RG = BT / per, rg = tid / per;
   for (int t = 0; t < ql; ++t) {
     const E* row = reinterpret_cast<const E*>(a.proj) + (size_t)(q0 + t) * a.ldp;
     const bool fresh = ctx - ql + t == 0;
+    float x[NR ? NR : 1][VEC];
+    auto get = [&](int strip, int d, float (&v)[VEC]) {
+      if (fresh) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) v[e] = 0.f;
+      } else {
+        ldn<VEC>(S + strip * VEC + (size_t)d * dv, v);
+      }
+    };
+    if constexpr (NR > 0) {
+      if (rg < RG) {
+#pragma unroll
+        for (int i = 0; i < NR; ++i)
+          if (rg + i * RG < dk) get(tid % per, rg + i * RG, x[i]);
+      }
+    }
     for (int i = tid; i < a.rank; i += BT) w1[i] = tanh_hw(ld1(row + 3 * HK + HV + i));
     __syncthreads();
-    float ss = 0.f, rk = 0.f;
+    float ss = 0.f, rk = 0.f, ra = 0.f;
     for (int d = tid; d < dk; d += BT) {
       const int n = h * dk + d;
       const float k = ld1(row + HK + n), rr = ld1(row + n);
+      const float al = sigmoid_hw(ld1(row + 2 * HK + HV + n) + a.a_b[n]);
       float z = a.w0[n];
       const E* w2 = reinterpret_cast<const E*>(a.w2) + (size_t)n * a.rank;
-      for (int i = 0; i < a.rank; ++i) z = fmaf(ld1(w2 + i), w1[i], z);
-      wv[d] = exp2_f(log2_decay(a, z));
-      au[d] = sigmoid_hw(ld1(row + 2 * HK + HV + n) + a.a_b[n]);
+      if (a.rank % 8 == 0) {
+        for (int i = 0; i < a.rank; i += 8) {
+          float wr[8];
+          ldn<8>(w2 + i, wr);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) z = fmaf(wr[e], w1[i + e], z);
+        }
+      } else {
+        for (int i = 0; i < a.rank; ++i) z = fmaf(ld1(w2 + i), w1[i], z);
+      }
+      const float w = exp2_f(log2_decay(a, z));
+      wv[d] = w;
       kv[d] = k;
-      rv[d] = rr;
+      rv[d] = rr * w;
+      au[d] = al;
       ss = fmaf(k, k, ss);
       rk = fmaf(rr, k, rk);
+      ra = fmaf(rr, al * k, ra);
     }
-    ss = block_sum(ss, scratch);
-    rk = block_sum(rk, scratch);
+    ss = wave_sum(ss);
+    rk = wave_sum(rk);
+    ra = wave_sum(ra);
+    if ((tid & 63) == 0) {
+      scratch[0][tid >> 6] = ss;
+      scratch[1][tid >> 6] = rk;
+      scratch[2][tid >> 6] = ra;
+    }
+    __syncthreads();
+    ss = rk = ra = 0.f;
+#pragma unroll
+    for (int w = 0; w < BT / 64; ++w) {
+      ss += scratch[0][w];
+      rk += scratch[1][w];
+      ra += scratch[2][w];
+    }
     const float inv = 1.f / sqrtf(ss + a.unit_eps);
-    float ra = 0.f;
-    for (int d = tid; d < dk; d += BT) {  // this thread's own entries
+    ra *= inv;  // r . (a u)
+    for (int d = tid; d < dk; d += BT) {
       const float u = kv[d] * inv;
       uv[d] = u;
       au[d] *= u;
-      ra = fmaf(rv[d], au[d], ra);
     }
-    ra = block_sum(ra, scratch);
+    __syncthreads();
     for (int s0 = 0; s0 < nstrip; s0 += per) {
-      const int strip = s0 + tid % per, rg = tid / per;
+      const int strip = s0 + tid % per;
       const bool on = rg < RG && strip < nstrip;
-      float* col = S + strip * VEC;
-      float x[NR ? NR : 1][VEC], z[VEC], y[VEC];
+      float z[VEC], y[VEC];
 #pragma unroll
       for (int e = 0; e < VEC; ++e) z[e] = y[e] = 0.f;
-      auto get = [&](int d, float (&v)[VEC]) {
-        if (fresh) {
-#pragma unroll
-          for (int e = 0; e < VEC; ++e) v[e] = 0.f;
-        } else {
-          ldn<VEC>(col + (size_t)d * dv, v);
-        }
-      };
       auto sums = [&](int d, const float (&v)[VEC]) {
-        const float u = uv[d], rw = rv[d] * wv[d];
+        const float u = uv[d], rw = rv[d];
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
           z[e] = fmaf(u, v[e], z[e]);
@@ -124,13 +157,10 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
         if constexpr (NR > 0) {
 #pragma unroll
           for (int i = 0; i < NR; ++i)
-            if (rg + i * RG < dk) get(rg + i * RG, x[i]);
-#pragma unroll
-          for (int i = 0; i < NR; ++i)
             if (rg + i * RG < dk) sums(rg + i * RG, x[i]);
         } else {
           for (int d = rg; d < dk; d += RG) {
-            get(d, x[0]);
+            get(strip, d, x[0]);
             sums(d, x[0]);
           }
         }
@@ -165,7 +195,7 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
           const float w = wv[d], k = kv[d], ad = au[d];
 #pragma unroll
           for (int e = 0; e < VEC; ++e) xx[e] = fmaf(w, xx[e], fmaf(k, v[e], -ad * zz[e]));
-          stn<VEC>(col + (size_t)d * dv, xx);
+          stn<VEC>(S + strip * VEC + (size_t)d * dv, xx);
         };
         if constexpr (NR > 0) {
 #pragma unroll
@@ -173,7 +203,7 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
             if (rg + i * RG < dk) put(rg + i * RG, x[i]);
         } else {
           for (int d = rg; d < dk; d += RG) {
-            get(d, x[0]);
+            get(strip, d, x[0]);
             put(d, x[0]);
           }
         }
@@ -519,7 +549,8 @@ static void delta_rows_nr(const DeltaArgs& a, const StepRows& s, const int* rows
   const int per = std::min(a.dv / VEC, BT), rg = BT / per, nr = cdiv(a.dk, rg);
   const size_t lds = (size_t)(a.rank + 5 * a.dk + 3 * BT * VEC) * 4;
   const dim3 grid(n, a.H);
-  if (nr <= 4) delta_rows_kernel<E, VEC, BT, 4><<<grid, BT, lds, st>>>(a, s, rows);
+  if (a.dv / VEC > BT) delta_rows_kernel<E, VEC, BT, 0><<<grid, BT, lds, st>>>(a, s, rows);
+  else if (nr <= 4) delta_rows_kernel<E, VEC, BT, 4><<<grid, BT, lds, st>>>(a, s, rows);
   else if (nr <= 16) delta_rows_kernel<E, VEC, BT, 16><<<grid, BT, lds, st>>>(a, s, rows);
   else delta_rows_kernel<E, VEC, BT, 0><<<grid, BT, lds, st>>>(a, s, rows);
 }
@@ -559,7 +590,7 @@ static void delta_all(const DeltaArgs& a, const StepRows& s, float* ws, hipStrea
     delta_blocks<E, 2>(a, s, ws, st);
     // few units: more waves on each (latency); many: fewer, with more in flight per CU
     if (grid < 1024) delta_walk_kernel<E, 8, 1, 3><<<grid, 512, 0, st>>>(a, s, ws, cols);
-    else delta_walk_kernel<E, 4, 2, 3><<<grid, 256, 0, st>>>(a, s, ws, cols);
+    else delta_walk_kernel<E, 4, 2, 2><<<grid, 256, 0, st>>>(a, s, ws, cols);
   } else {
     delta_blocks<E, 4>(a, s, ws, st);
     delta_walk_kernel<E, 8, 2, 2><<<grid, 512, 0, st>>>(a, s, ws, cols);

@@ -94,48 +94,72 @@ __device__ __forceinline__ float gate_f(float g) { return 1.f / (1.f + __expf(-g
 
 }  // namespace
 
-// A workgroup: one head, 64 output columns (16 per wave), 16 MT tiles.
-template <int MT>
+// A workgroup: one head, 64 NT output columns (16 NT per wave), 16 MT tiles.
+template <int MT, int NT>
 __global__ void __launch_bounds__(256) head_mm_kernel(HeadMmArgs a) {
   const int h = blockIdx.x, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l15 = lane & 15, g4 = lane >> 4;
-  const int n0 = blockIdx.y * 64 + wid * 16, m0 = blockIdx.z * 16 * MT;
+  const int n0 = (blockIdx.y * 4 + wid) * 16 * NT, m0 = blockIdx.z * 16 * MT;
   if (n0 >= a.N) return;
-  const uint16_t* w = reinterpret_cast<const uint16_t*>(a.w) + ((size_t)h * a.N + min(n0 + l15, a.N - 1)) * a.K + 8 * g4;
+  const uint16_t* w[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n)
+    w[n] = reinterpret_cast<const uint16_t*>(a.w) + ((size_t)h * a.N + min(n0 + 16 * n + l15, a.N - 1)) * a.K + 8 * g4;
   const uint16_t* x[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
     const int i = min(m0 + 16 * m + l15, a.n_tiles - 1);
     x[m] = reinterpret_cast<const uint16_t*>(a.x) + (size_t)(a.x_tok ? tile_token(a, i) : i) * a.ldx + h * a.hx + 8 * g4;
   }
-  f32x4 acc[MT];
+  f32x4 acc[MT][NT];
 #pragma unroll
-  for (int m = 0; m < MT; ++m) acc[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[m][n] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k = 0; k < a.K; k += 64) {
-    bf16x8 wf[2], xf[2][MT];
+    bf16x8 wf[2][NT], xf[2][MT];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      wf[u] = *reinterpret_cast<const bf16x8*>(w + k + 32 * u);
+#pragma unroll
+      for (int n = 0; n < NT; ++n) wf[u][n] = *reinterpret_cast<const bf16x8*>(w[n] + k + 32 * u);
 #pragma unroll
       for (int m = 0; m < MT; ++m) xf[u][m] = *reinterpret_cast<const bf16x8*>(x[m] + k + 32 * u);
     }
 #pragma unroll
     for (int u = 0; u < 2; ++u)
 #pragma unroll
-      for (int m = 0; m < MT; ++m) acc[m] = mfma16(xf[u][m], wf[u], acc[m]);
+      for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[m][n] = mfma16(wf[u][n], xf[u][m], acc[m][n]);
   }
-  const int n = n0 + l15;
-  if (n >= a.N) return;
+  // row 4 g4 + e of a product = output column, column l15 = tile
+  const bool vec = a.N % 4 == 0 && (a.ldo | a.ho) % 4 == 0 && (!a.gate || a.ldg % 4 == 0);
 #pragma unroll
-  for (int m = 0; m < MT; ++m)
+  for (int m = 0; m < MT; ++m) {
+    const int i = m0 + 16 * m + l15;
+    if (i >= a.n_tiles) continue;
+    const int tok = a.out_tok || a.gate ? tile_token(a, i) : 0;
+    const uint16_t* gate = reinterpret_cast<const uint16_t*>(a.gate) + (size_t)tok * a.ldg + (size_t)h * a.N;
+    uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + (size_t)(a.out_tok ? tok : i) * a.ldo + h * a.ho;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int i = m0 + 16 * m + 4 * g4 + e;
-      if (i >= a.n_tiles) continue;
-      const int tok = a.out_tok || a.gate ? tile_token(a, i) : 0;
-      float v = acc[m][e];
-      if (a.gate) v *= gate_f(bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)tok * a.ldg + (size_t)h * a.N + n]));
-      reinterpret_cast<uint16_t*>(a.out)[(size_t)(a.out_tok ? tok : i) * a.ldo + h * a.ho + n] = f2bf(v);
+    for (int t = 0; t < NT; ++t) {
+      const int n = n0 + 16 * t + 4 * g4;
+      if (n >= a.N) continue;
+      float v[4] = {acc[m][t][0], acc[m][t][1], acc[m][t][2], acc[m][t][3]};
+      if (vec) {
+        if (a.gate) {
+          float g[4];
+          ldn<4>(gate + n, g);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] *= gate_f(g[e]);
+        }
+        stn<4>(out + n, v);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (n + e < a.N) out[n + e] = f2bf(a.gate ? v[e] * gate_f(bf2f(gate[n + e])) : v[e]);
+      }
     }
+  }
 }
 
 // plain form (fp32): one thread per output
@@ -155,10 +179,12 @@ void launch_head_mm(const HeadMmArgs& a, bool f32, hipStream_t st) {
   if (a.n_tiles == 0) return;
   if (f32) {
     head_mm_plain_kernel<<<dim3(a.H, cdiv(a.N, 256), a.n_tiles), 256, 0, st>>>(a);
+  } else if (a.n_tiles > 64) {
+    head_mm_kernel<4, 2><<<dim3(a.H, cdiv(a.N, 128), cdiv(a.n_tiles, 64)), 256, 0, st>>>(a);
   } else if (a.n_tiles > 16) {
-    head_mm_kernel<4><<<dim3(a.H, cdiv(a.N, 64), cdiv(a.n_tiles, 64)), 256, 0, st>>>(a);
+    head_mm_kernel<2, 1><<<dim3(a.H, cdiv(a.N, 64), cdiv(a.n_tiles, 32)), 256, 0, st>>>(a);
   } else {
-    head_mm_kernel<1><<<dim3(a.H, cdiv(a.N, 64), 1), 256, 0, st>>>(a);
+    head_mm_kernel<1, 1><<<dim3(a.H, cdiv(a.N, 64), 1), 256, 0, st>>>(a);
   }
 }
 

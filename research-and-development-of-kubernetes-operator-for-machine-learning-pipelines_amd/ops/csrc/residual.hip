@@ -116,16 +116,17 @@ void launch_residual(const ResidualArgs& a, bool f32, hipStream_t st) {
   }
 }
 
-__device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ __forceinline__ float sigmoid_f(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
-// WPG waves per (token, group); NI > 0: the group's values stay in registers, 0: they are read twice
-template <typename E, int VEC, int WPG, int NI>
+// BT threads (16, 64 or 256) per (token, group); NI > 0: the group's values stay in registers, 0: they are
+// read twice
+template <typename E, int VEC, int BT, int NI>
 __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a) {
   __shared__ float scratch[16];
-  constexpr int BT = 64 * WPG, N = NI ? NI : 1;
+  constexpr int N = NI ? NI : 1;
   const int gw = a.n / a.groups;
-  const long unit = WPG == 1 ? (long)blockIdx.x * 4 + (threadIdx.x >> 6) : (long)blockIdx.x;
-  if (unit >= (long)a.T * a.groups) return;  // whole waves, and no barrier below when WPG == 1
+  const long unit = (long)blockIdx.x * (256 / BT) + threadIdx.x / BT;
+  if (unit >= (long)a.T * a.groups) return;  // whole groups of BT threads, and no barrier below when BT < 256
   const int t = (int)(unit / a.groups), g = (int)(unit % a.groups), tid = threadIdx.x % BT;
   const E* y = reinterpret_cast<const E*>(a.y) + (size_t)t * a.n + (size_t)g * gw;
   const E* gt = reinterpret_cast<const E*>(a.gate) + (size_t)t * a.ldg + (size_t)g * gw;
@@ -160,7 +161,14 @@ __global__ void __launch_bounds__(256) gated_norm_kernel(GatedNormArgs a) {
       for (int e = 0; e < VEC; ++e) ss = fmaf(v[0][e], v[0][e], ss);
     }
   }
-  ss = WPG == 1 ? wave_sum(ss) : block_sum(ss, scratch);
+  if constexpr (BT == 16) {
+    ss += detail::dpp<0xB1>(ss);
+    ss += detail::dpp<0x4E>(ss);
+    ss += detail::dpp<0x141>(ss);
+    ss += detail::dpp<0x140>(ss);
+  } else {
+    ss = BT == 64 ? wave_sum(ss) : block_sum(ss, scratch);
+  }
   const float inv = 1.f / sqrtf(ss / (float)gw + a.eps);
   auto put = [&](int c, float (&vv)[VEC], float (&zz)[VEC]) {
     float wv[VEC];
@@ -187,17 +195,15 @@ template <typename E, int VEC>
 static void gated_norm_vec(const GatedNormArgs& a, hipStream_t st) {
   const int gw = a.n / a.groups;
   const long units = (long)a.T * a.groups;
-  if (gw <= 64 * VEC * 2) {
-    const int grid = (int)((units + 3) / 4);
-    if (gw <= 64 * VEC) gated_norm_kernel<E, VEC, 1, 1><<<grid, 256, 0, st>>>(a);
-    else gated_norm_kernel<E, VEC, 1, 2><<<grid, 256, 0, st>>>(a);
-  } else if (gw <= 256 * VEC) {
-    gated_norm_kernel<E, VEC, 4, 1><<<(int)units, 256, 0, st>>>(a);
-  } else if (gw <= 256 * VEC * 4) {
-    gated_norm_kernel<E, VEC, 4, 4><<<(int)units, 256, 0, st>>>(a);
-  } else {
-    gated_norm_kernel<E, VEC, 4, 0><<<(int)units, 256, 0, st>>>(a);
-  }
+#define MLOP_GN(BT, NI) gated_norm_kernel<E, VEC, BT, NI><<<(int)((units * BT + 255) / 256), 256, 0, st>>>(a)
+  if (gw <= 16 * VEC) MLOP_GN(16, 1);
+  else if (gw <= 32 * VEC) MLOP_GN(16, 2);
+  else if (gw <= 64 * VEC) MLOP_GN(64, 1);
+  else if (gw <= 128 * VEC) MLOP_GN(64, 2);
+  else if (gw <= 256 * VEC) MLOP_GN(256, 1);
+  else if (gw <= 1024 * VEC) MLOP_GN(256, 4);
+  else MLOP_GN(256, 0);
+#undef MLOP_GN
 }
 
 void launch_gated_norm(const GatedNormArgs& a, bool f32, hipStream_t st) {

@@ -303,6 +303,31 @@ def test_latent_store(gpu, dtype, R, lead):
     assert R == pad_dim(R) or float(cache[..., R:].abs().max()) == 0
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("n,H,N,K", [(1, 3, 64, 64), (16, 2, 130, 128), (17, 4, 23, 192), (33, 2, 128, 512), (70, 3, 320, 64),
+                                     (150, 2, 28, 128)])
+def test_head_mm(gpu, dtype, n, H, N, K):
+    """Per-head products of the step's one-token tiles: from tokens to tiles and back, with and without a
+    gate, portions beside them."""
+    step = Step([1] * n + [5, 2], [7 + i for i in range(n)] + [9, 30], gpu)
+    m, T = step.meta, step.T
+    x, w, g = rnd(T, H * K + 8, seed=1, dtype=dtype), rnd(H, N, K, seed=2, dtype=dtype, gain=K ** -0.5), rnd(T, H * N + 8, seed=3, dtype=dtype)
+    tok = (m.q_start[m.tile_seq.long()] + m.tile_q0).cpu().long()
+    want = torch.einsum("thk,hnk->thn", x[:, :H * K].double().view(T, H, K), w.double())
+    op, lists = torch.ops.mlop.head_mm, (m.tile_seq, m.tile_q0, m.q_start, m.q_len)
+    xd, wd, gd = x.to(gpu)[:, :H * K].unflatten(1, (H, K)), w.to(gpu), g.to(gpu)[:, :H * N]
+    out = torch.empty(n, H, N, dtype=dtype, device=gpu)
+    op(out, xd, wd, *lists, True, False, None)
+    assert rel_err(out, want[tok]) < TOL[dtype]
+    back = torch.full((T, H, N), 7.0, dtype=dtype, device=gpu)
+    op(back, xd[tok.to(gpu)].contiguous(), wd, *lists, False, True, gd)
+    gate = torch.sigmoid(g[:, :H * N].double()).view(T, H, N)
+    assert rel_err(back.cpu()[tok], (want * gate)[tok]) < TOL[dtype]
+    rest = torch.ones(T, dtype=torch.bool)
+    rest[tok] = False
+    assert torch.all(back.cpu()[rest] == 7.0)
+
+
 def _latent_case(gpu, dtype, H, D, V, R, window, q_lens, ctx, min_part=None, spike=False, sink=True, gate=True, seed=0):
     """Max relative error of a latent-attention step against the oracle.  ``spike``: every query asks for
     one key whose score stands out: the first token, the last one inside the window, the first one
