@@ -45,7 +45,7 @@ __device__ __forceinline__ float log2_decay(const DeltaArgs& a, float z) { retur
 
 // NR: key rows of a strip that a thread keeps in registers from their loads, in front of everything else,
 // to the stores (one strip per thread, then); 0: the state is read twice.
-template <typename E, int VEC, int BT, int NR>
+template <typename E, int VEC, int BT, int NR, bool NT>
 __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r, const int* __restrict__ rows) {
   extern __shared__ float sm[];
   __shared__ float scratch[3][BT / 64];
@@ -77,7 +77,7 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
 #pragma unroll
         for (int e = 0; e < VEC; ++e) v[e] = 0.f;
       } else {
-        ldn<VEC>(S + strip * VEC + (size_t)d * dv, v);
+        ld_state<NT>(S + strip * VEC + (size_t)d * dv, v);
       }
     };
     if constexpr (NR > 0) {
@@ -195,7 +195,7 @@ __global__ void __launch_bounds__(BT) delta_rows_kernel(DeltaArgs a, StepRows r,
           const float w = wv[d], k = kv[d], ad = au[d];
 #pragma unroll
           for (int e = 0; e < VEC; ++e) xx[e] = fmaf(w, xx[e], fmaf(k, v[e], -ad * zz[e]));
-          stn<VEC>(S + strip * VEC + (size_t)d * dv, xx);
+          st_state<NT>(S + strip * VEC + (size_t)d * dv, xx);
         };
         if constexpr (NR > 0) {
 #pragma unroll
@@ -549,10 +549,16 @@ static void delta_rows_nr(const DeltaArgs& a, const StepRows& s, const int* rows
   const int per = std::min(a.dv / VEC, BT), rg = BT / per, nr = cdiv(a.dk, rg);
   const size_t lds = (size_t)(a.rank + 5 * a.dk + 3 * BT * VEC) * 4;
   const dim3 grid(n, a.H);
-  if (a.dv / VEC > BT) delta_rows_kernel<E, VEC, BT, 0><<<grid, BT, lds, st>>>(a, s, rows);
-  else if (nr <= 4) delta_rows_kernel<E, VEC, BT, 4><<<grid, BT, lds, st>>>(a, s, rows);
-  else if (nr <= 16) delta_rows_kernel<E, VEC, BT, 16><<<grid, BT, lds, st>>>(a, s, rows);
-  else delta_rows_kernel<E, VEC, BT, 0><<<grid, BT, lds, st>>>(a, s, rows);
+  const bool nt = (size_t)n * a.H * a.dk * a.dv * 4 >= kStreamBytes;
+#define MLOP_ROWS(NR)                                                                       \
+  do {                                                                                      \
+    if (nt) delta_rows_kernel<E, VEC, BT, NR, true><<<grid, BT, lds, st>>>(a, s, rows);     \
+    else delta_rows_kernel<E, VEC, BT, NR, false><<<grid, BT, lds, st>>>(a, s, rows);       \
+  } while (0)
+  if (nr > 16 || a.dv / VEC > BT) MLOP_ROWS(0);
+  else if (nr <= 4) MLOP_ROWS(4);
+  else MLOP_ROWS(16);
+#undef MLOP_ROWS
 }
 
 template <typename E>

@@ -65,4 +65,26 @@ __device__ __forceinline__ void stn(uint16_t* p, const float (&v)[N]) {
   }
 }
 
+// four (or one) floats that stream through: read or written once per launch, not kept in the caches
+template <int N>
+__device__ __forceinline__ void ldn_nt(const float* p, float (&v)[N]) {
+  if constexpr (N == 4) {
+    const f32x4 t = __builtin_nontemporal_load(reinterpret_cast<const f32x4*>(p));
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = t[j];
+  } else {
+#pragma unroll
+    for (int j = 0; j < N; ++j) v[j] = __builtin_nontemporal_load(p + j);
+  }
+}
+template <int N>
+__device__ __forceinline__ void stn_nt(float* p, const float (&v)[N]) {
+  if constexpr (N == 4) {
+    __builtin_nontemporal_store(f32x4{v[0], v[1], v[2], v[3]}, reinterpret_cast<f32x4*>(p));
+  } else {
+#pragma unroll
+    for (int j = 0; j < N; ++j) __builtin_nontemporal_store(v[j], p + j);
+  }
+}
+
 }  // namespace mlop

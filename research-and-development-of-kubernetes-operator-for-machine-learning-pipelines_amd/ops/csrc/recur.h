@@ -33,6 +33,18 @@ __device__ __forceinline__ void split3(const f32x4& x, u32x2 (&p)[3]) {
   }
 }
 
+// A decode step's states at this size pass through the caches without staying there: they would not be
+// there at the next step, and written lines left behind are written back under the next kernel.
+constexpr size_t kStreamBytes = 100u << 20;
+template <bool NT, int N>
+__device__ __forceinline__ void ld_state(const float* p, float (&v)[N]) {
+  if constexpr (NT) ldn_nt<N>(p, v); else ldn<N>(p, v);
+}
+template <bool NT, int N>
+__device__ __forceinline__ void st_state(float* p, const float (&v)[N]) {
+  if constexpr (NT) stn_nt<N>(p, v); else stn<N>(p, v);
+}
+
 // workgroup barrier for LDS hand-offs: global loads and stores stay in flight across it
 __device__ __forceinline__ void lds_sync() {
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");

@@ -20,7 +20,7 @@
 
 namespace mlop {
 
-template <typename E, int VEC, int BT>
+template <typename E, int VEC, int BT, bool NT>
 __global__ void __launch_bounds__(BT) ssd_rows_kernel(SsdArgs a, StepRows r, const int* __restrict__ rows) {
   extern __shared__ float sm[];
   const int s = rows[blockIdx.x], h = blockIdx.y, tid = threadIdx.x;
@@ -64,7 +64,7 @@ __global__ void __launch_bounds__(BT) ssd_rows_kernel(SsdArgs a, StepRows r, con
 #pragma unroll
             for (int e = 0; e < VEC; ++e) x[e] = 0.f;
           } else {
-            ldn<VEC>(col + (size_t)d * V, x);
+            ld_state<NT>(col + (size_t)d * V, x);
           }
           const float bd = bv[d], cd = cv[d];
 #pragma unroll
@@ -72,7 +72,7 @@ __global__ void __launch_bounds__(BT) ssd_rows_kernel(SsdArgs a, StepRows r, con
             x[e] = fmaf(de, x[e], bd * v[e]);
             acc[e] = fmaf(cd, x[e], acc[e]);
           }
-          stn<VEC>(col + (size_t)d * V, x);
+          st_state<NT>(col + (size_t)d * V, x);
         }
       }
 #pragma unroll
@@ -314,8 +314,9 @@ template <typename E, int BT>
 static void ssd_rows_t(const SsdArgs& a, const StepRows& s, const int* rows, int n, hipStream_t st) {
   const bool v4 = a.V % 4 == 0;
   const size_t lds = (size_t)(2 * a.N + BT * (v4 ? 4 : 1)) * 4;
-  if (v4) ssd_rows_kernel<E, 4, BT><<<dim3(n, a.H), BT, lds, st>>>(a, s, rows);
-  else ssd_rows_kernel<E, 1, BT><<<dim3(n, a.H), BT, lds, st>>>(a, s, rows);
+  if (v4 && (size_t)n * a.H * a.N * a.V * 4 >= kStreamBytes) ssd_rows_kernel<E, 4, BT, true><<<dim3(n, a.H), BT, lds, st>>>(a, s, rows);
+  else if (v4) ssd_rows_kernel<E, 4, BT, false><<<dim3(n, a.H), BT, lds, st>>>(a, s, rows);
+  else ssd_rows_kernel<E, 1, BT, false><<<dim3(n, a.H), BT, lds, st>>>(a, s, rows);
 }
 
 template <typename E>
