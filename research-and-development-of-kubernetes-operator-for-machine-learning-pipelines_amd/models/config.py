@@ -120,22 +120,56 @@ class GLASpec:
 
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """Stretched rotary frequencies: pairs that turn less than ``slow`` times in ``original`` positions turn
+    ``factor`` times slower, pairs that turn more than ``fast`` times as before, a ramp between them; cos
+    and sin times 0.1 ln(factor) + 1."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class RotarySpec:
+    """Rotary positions of ``dims`` dimensions in pairs (2i, 2i + 1)."""
+    base: float
+    dims: int
+    scaling: YarnSpec | None = None
+
+
+@dataclass(frozen=True)
 class LatentAttentionSpec:
-    """Softmax-attention mixer over cached latents, without positions."""
+    """Softmax-attention mixer over cached latents."""
     heads: int
-    dim: int                 # query / key head size
+    dim: int                 # query / key head size (without a rotated part)
     vdim: int                # value head size
-    rank: int                # latent size (all that is cached)
+    rank: int                # latent size
     scale: float             # score scale
     window: int = 0          # a token sees itself and the window - 1 tokens before it (0: all)
+    sink: bool = True        # a number per head joins the softmax's denominator
+    gate: bool = True        # output gate, one per value element
+    q_rank: int = 0          # queries through a normed latent of this size (0: straight from the input)
+    rot: RotarySpec | None = None  # rotated part of queries and keys; a key's is one for all heads, cached
+    kv_from: int = -1        # layer whose cached latents and rotated keys this one reads (-1: its own)
+
+    @property
+    def rot_dim(self) -> int:
+        return self.rot.dims if self.rot else 0
+
+    @property
+    def cached(self) -> int:
+        """Values kept per token."""
+        return 0 if self.kv_from >= 0 else self.rank + self.rot_dim
 
     def params(self, width: int) -> int:
-        hq, hv = self.heads * self.dim, self.heads * self.vdim
-        return width * (hq + self.rank + 2 * hv) + self.rank * (hq + hv + 1) + self.heads
+        n = self.macs(width) + self.q_rank + self.heads * self.sink
+        return n + (self.rank if self.kv_from < 0 else 0)
 
     def macs(self, width: int) -> int:
-        hq, hv = self.heads * self.dim, self.heads * self.vdim
-        return width * (hq + self.rank + 2 * hv) + self.rank * (hq + hv)
+        hq, hv = self.heads * (self.dim + self.rot_dim), self.heads * self.vdim
+        q = self.q_rank * (width + hq) if self.q_rank else width * hq
+        return q + width * (self.cached + hv * (1 + self.gate)) + self.rank * (self.heads * self.dim + hv)
 
 
 @dataclass(frozen=True)
@@ -191,10 +225,27 @@ class DeltaSpec:
 
 
 @dataclass(frozen=True)
+class MoESpec:
+    """Mixture of gated experts, each token through the ``top`` with the largest sigmoid scores, its input
+    times the score; beside them a shared expert (``shared`` 0: none) with a sigmoid gate per token."""
+    experts: int
+    top: int
+    ff: int
+    shared: int = 0
+
+    def params(self, width: int) -> int:
+        return width * (self.experts * (3 * self.ff + 1) + 3 * self.shared + bool(self.shared))
+
+    def macs(self, width: int) -> int:
+        return width * (self.experts + 3 * self.top * self.ff + 3 * self.shared + bool(self.shared))
+
+
+@dataclass(frozen=True)
 class LayerSpec:
     mixer: AttentionSpec | GLASpec | LatentAttentionSpec | SSDSpec | DeltaSpec
     ff: int = 0              # feed-forward width (0: none)
     limit: float = 0.0       # clamp of a gated feed-forward (designs that have one)
+    moe: MoESpec | None = None  # experts instead of the feed-forward
 
 
 @dataclass(frozen=True)
@@ -221,7 +272,7 @@ class HybridConfig(ModelConfig):
         return self.num_params()
 
     def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
-        return sum(m.rank if isinstance(m, LatentAttentionSpec) else m.kv_heads * (m.dim + m.vdim)
+        return sum(m.cached if isinstance(m, LatentAttentionSpec) else m.kv_heads * (m.dim + m.vdim)
                    for m in self.attention) * dtype_bytes
 
     def state_bytes_per_seq(self) -> int:
@@ -266,12 +317,49 @@ class RegesunConfig(HybridConfig):
         return 2 * (self.vocab_size * W + sum(la.mixer.macs(W) + 3 * W * la.ff for la in self.layers))
 
 
+@dataclass(frozen=True)
+class NafazenConfig(HybridConfig):
+    """Nafazen: latent attention with a rotated key part, on layers' own or an earlier layer's latents, dense
+    (xIELU) and mixture-of-experts feed-forwards, norms behind the sublayers only, soft-capped logits."""
+    embed_scale: float = 1.0
+    logit_softcap: float = 0.0
+
+    def __post_init__(self):
+        super().__post_init__()
+        for i, m in enumerate(self.attention):
+            if m.kv_from < 0:
+                continue
+            src = self.layers[m.kv_from].mixer if m.kv_from < i else None
+            if src is None or src.kv_from >= 0 or (src.rank, src.rot) != (m.rank, m.rot):
+                raise ValueError(f"layer {i}: layer {m.kv_from} has no latents of its own for it")
+
+    def _count(self, moe) -> int:
+        W = self.hidden_size
+        n = 2 * self.vocab_size * W + 1
+        for la in self.layers:
+            n += la.mixer.params(W) + 1 + bool(la.ff or la.moe)
+            n += moe(la.moe) if la.moe else 2 * W * la.ff + 2 * bool(la.ff)
+        return n
+
+    def num_params(self) -> int:
+        return self._count(lambda e: e.params(self.hidden_size))
+
+    def active_params(self) -> int:
+        return self._count(lambda e: e.macs(self.hidden_size))
+
+    def flops_per_token(self) -> int:
+        W = self.hidden_size
+        return 2 * (self.vocab_size * W + sum(la.mixer.macs(W) + (la.moe.macs(W) if la.moe else 2 * W * la.ff)
+                                              for la in self.layers))
+
+
 def _hybrid(cls, name: str, vocab: int, width: int, layers, eps: float, **kw):
     """``cls`` over listed layers, the uniform fields from the largest attention layer."""
     layers = tuple(layers)
     att = [la.mixer for la in layers if isinstance(la.mixer, (AttentionSpec, LatentAttentionSpec))]
     return cls(
-        name=name, vocab_size=vocab, hidden_size=width, intermediate_size=max((la.ff for la in layers), default=0),
+        name=name, vocab_size=vocab, hidden_size=width,
+        intermediate_size=max((la.moe.ff if la.moe else la.ff for la in layers), default=0),
         num_layers=len(layers), num_heads=max((m.heads for m in att), default=1),
         num_kv_heads=max((getattr(m, "kv_heads", 1) for m in att), default=1),
         head_dim=max((m.dim for m in att), default=64), rms_eps=eps, layers=layers,
@@ -286,6 +374,11 @@ def kosesun_config(name: str, vocab: int, width: int, layers, streams: int, embe
 
 def regesun_config(name: str, vocab: int, width: int, layers, max_position: int, eps: float = 1e-5, **kw) -> RegesunConfig:
     return _hybrid(RegesunConfig, name, vocab, width, layers, eps, max_position=max_position, **kw)
+
+
+def nafazen_config(name: str, vocab: int, width: int, layers, embed_scale: float, logit_softcap: float, eps: float = 1e-5,
+                   **kw) -> NafazenConfig:
+    return _hybrid(NafazenConfig, name, vocab, width, layers, eps, embed_scale=embed_scale, logit_softcap=logit_softcap, **kw)
 
 
 LLAMA3_8B = ModelConfig(
@@ -362,9 +455,34 @@ TINY_REGESUN = _regesun("tiny-regesun", width=256, ff=320, n_layers=4, vocab=512
                         latent=LatentAttentionSpec(heads=5, dim=24, vdim=32, rank=72, scale=0.2, window=40),
                         delta=DeltaSpec(heads=3, dim=56, rank=12), limit=2.0, max_position=2048)
 
+
+def _nafazen(name: str, width: int, ff: int, n_layers: int, vocab: int, heads: int, dim: int, rot_dim: int, vdim: int,
+             rank: int, q_rank: int, moe: MoESpec, **kw) -> NafazenConfig:
+    """Four layers in turn: stretched positions and a dense feed-forward, plain positions and experts, twice;
+    the last reads the second's latents."""
+    def att(scaling=None, kv_from=-1):
+        return LatentAttentionSpec(heads=heads, dim=dim, vdim=vdim, rank=rank, scale=(dim + rot_dim) ** -0.5, sink=False,
+                                   gate=False, q_rank=q_rank, rot=RotarySpec(500000.0, rot_dim, scaling), kv_from=kv_from)
+
+    yarn = YarnSpec(factor=4.0, original=4096, fast=32.0, slow=1.0)
+    turn = lambda i: (LayerSpec(att(yarn), ff), LayerSpec(att(), moe=moe), LayerSpec(att(yarn), ff),  # noqa: E731
+                      LayerSpec(att(kv_from=i - 2), moe=moe))[i % 4]
+    return nafazen_config(name, vocab, width, [turn(i) for i in range(n_layers)], embed_scale=width ** 0.5,
+                          logit_softcap=30.0, **kw)
+
+
+# attention and feed-forward sizes of the Regesun presets' order
+NAFAZEN_8B = _nafazen("nafazen-8b", width=4096, ff=14336, n_layers=32, vocab=128256, heads=32, dim=128, rot_dim=64, vdim=128,
+                      rank=512, q_rank=1536, moe=MoESpec(experts=8, top=2, ff=1792, shared=3584))
+NAFAZEN_1B = _nafazen("nafazen-1b", width=2048, ff=8192, n_layers=16, vocab=128256, heads=16, dim=64, rot_dim=64, vdim=64,
+                      rank=256, q_rank=768, moe=MoESpec(experts=16, top=2, ff=768, shared=1536))
+TINY_NAFAZEN = _nafazen("tiny-nafazen", width=192, ff=200, n_layers=4, vocab=512, heads=5, dim=24, rot_dim=16, vdim=40,
+                        rank=72, q_rank=56, moe=MoESpec(experts=6, top=2, ff=40, shared=72), max_position=2048)
+
 PRESETS = {c.name: c for c in (LLAMA3_8B, LLAMA3_70B, LLAMA31_8B, LLAMA31_70B, MIXTRAL_8X7B, TINY_LLAMA,
                                 TINY_MIXTRAL, TINY_LLAMA_8H, TINY_MIXTRAL_8E, KOSESUN_8B, KOSESUN_1B,
-                                TINY_KOSESUN, REGESUN_8B, REGESUN_1B, TINY_REGESUN)}
+                                TINY_KOSESUN, REGESUN_8B, REGESUN_1B, TINY_REGESUN, NAFAZEN_8B, NAFAZEN_1B,
+                                TINY_NAFAZEN)}
 # accepted aliases (MLflow tags / CR annotations use HF-ish names)
 ALIASES = {
     "meta-llama/Meta-Llama-3-8B": "llama3-8b", "llama-3-8b": "llama3-8b", "Llama-3-8B": "llama3-8b",

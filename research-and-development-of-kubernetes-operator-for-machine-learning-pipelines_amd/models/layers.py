@@ -43,6 +43,27 @@ def rope_table(head_dim: int, max_pos: int, theta: float, scaling: dict | None =
     return torch.cat([f.cos(), f.sin()], dim=-1).float().to(device)
 
 
+def rotary_table(rot, max_pos: int, device=None) -> torch.Tensor:
+    """[max_pos, dims] fp32 of a ``RotarySpec``: cos of the dims / 2 pairs, then sin (angles in fp64 on the
+    host)."""
+    inv, mult = rope_inv_freq(rot.dims, rot.base), 1.0
+    if rot.scaling is not None:
+        y = rot.scaling
+        # the pair that turns t times in the original range
+        pair = lambda t: rot.dims * math.log(y.original / (2 * math.pi * t)) / (2 * math.log(rot.base))  # noqa: E731
+        lo, hi = max(math.floor(pair(y.fast)), 0), min(math.ceil(pair(y.slow)), rot.dims - 1)
+        ramp = ((torch.arange(rot.dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 1e-3)).clamp(0, 1)
+        inv, mult = inv / y.factor * ramp + inv * (1 - ramp), 0.1 * math.log(y.factor) + 1
+    f = torch.outer(torch.arange(max_pos, dtype=torch.float64), inv)
+    return (torch.cat([f.cos(), f.sin()], dim=-1) * mult).float().to(device)
+
+
+def pad_rows(w: torch.Tensor, heads: int, rows: int) -> torch.Tensor:
+    """[heads * d, K] -> [heads * rows, K], every head's rows padded with zeros."""
+    v = w.view(heads, -1, w.shape[1])
+    return F.pad(v, (0, 0, 0, rows - v.shape[1])).reshape(heads * rows, w.shape[1])
+
+
 def init_weight(shape, device, dtype=torch.bfloat16, std: float = 0.02, gen: torch.Generator | None = None):
     w = torch.empty(*shape, device=device, dtype=dtype)
     w.normal_(0.0, std, generator=gen)

@@ -18,8 +18,8 @@ Layout mapping (HF name -> ours; TP sharding then reuses ``load_shard_from``):
   Mixtral: block_sparse_moe.gate | mlp.gate      -> router
            experts.{e}.w1 / w3 (legacy) or experts.gate_up_proj (fused) -> w13 (interleaved)
            experts.{e}.w2 or experts.down_proj   -> w2
-Kosesun and Regesun checkpoints (``"architecture"`` in config.json; tensors ``l<i>.mix.*`` ...) are read
-by the model itself as it is built (models/kosesun.py, models/regesun.py).
+Kosesun, Regesun and Nafazen checkpoints (``"architecture"`` in config.json; tensors ``l<i>.mix.*`` ...) are
+read by the model itself as it is built (models/kosesun.py, models/regesun.py, models/nafazen.py).
 Tensors are read lazily, one layer at a time (safetensors memory map), so a 141 GB
 checkpoint never sits in host memory at once.
 """
@@ -32,8 +32,8 @@ from pathlib import Path
 
 import torch
 
-from .config import (AttentionSpec, DeltaSpec, GLASpec, LatentAttentionSpec, LayerSpec, ModelConfig, PRESETS, SSDSpec,
-                     kosesun_config, regesun_config)
+from .config import (AttentionSpec, DeltaSpec, GLASpec, LatentAttentionSpec, LayerSpec, ModelConfig, MoESpec, PRESETS,
+                     RotarySpec, SSDSpec, YarnSpec, kosesun_config, nafazen_config, regesun_config)
 
 _ARCH_NAMES = {"LlamaForCausalLM": "llama", "MixtralForCausalLM": "mixtral", "MistralForCausalLM": "llama"}
 
@@ -182,8 +182,62 @@ def config_from_regesun(d: dict, shape_of, name: str | None = None) -> ModelConf
                           float(d["norm"]["eps"]))
 
 
+def _rotary(d: dict, where: str) -> RotarySpec:
+    _only(d, {"base", "dims", "scaling"}, where)
+    sc, yarn = d.get("scaling"), None
+    if sc is not None:
+        _only(sc, {"factor", "fast", "original", "slow"}, where + " scaling")
+        yarn = YarnSpec(*(float(sc[k]) for k in ("factor", "original", "fast", "slow")))
+        if min(yarn.factor, yarn.original, yarn.fast, yarn.slow) <= 0:
+            raise ValueError(f"{where}: unsupported scaling {sc}")
+    rot = RotarySpec(float(d["base"]), int(d["dims"]), yarn)
+    if rot.dims < 2 or rot.dims % 2 or rot.base <= 1:
+        raise ValueError(f"{where}: unsupported rotation {d}")
+    return rot
+
+
+def _nafazen_mlp(mlp: dict, where: str) -> dict:
+    """Feed-forward fields of a LayerSpec."""
+    if mlp.get("kind", "dense") == "dense":
+        _only(mlp, {"ff", "kind"}, where)
+        return {"ff": int(mlp["ff"])}
+    if mlp["kind"] != "moe":
+        raise ValueError(f"{where}: unsupported feed-forward {mlp['kind']!r}")
+    _only(mlp, {"expert", "kind", "router", "shared"}, where)
+    ex, ro, sh = mlp["expert"], mlp["router"], mlp.get("shared") or {"ff": 0}
+    _only(ex, {"ff"}, where + " expert"), _only(sh, {"ff"}, where + " shared"), _only(ro, {"experts", "top"}, where + " router")
+    moe = MoESpec(experts=int(ro["experts"]), top=int(ro["top"]), ff=int(ex["ff"]), shared=int(sh["ff"]))
+    if not 1 <= moe.top <= moe.experts or moe.ff < 1 or moe.shared < 0:
+        raise ValueError(f"{where}: unsupported expert sizes {mlp}")
+    return {"moe": moe}
+
+
+def config_from_nafazen(d: dict, shape_of, name: str | None = None) -> ModelConfig:
+    """NafazenConfig from a Nafazen ``config.json`` dict.  Settings this runtime does not know are rejected,
+    never dropped."""
+    _only(d, {"architecture", "embedding", "layers", "logit_softcap", "norm", "vocab", "width"}, "config")
+    _only(d["norm"], {"eps"}, "norm"), _only(d["embedding"], {"scale"}, "embedding")
+    layers = []
+    for i, la in enumerate(d["layers"]):
+        _only(la, {"type", "mixer", "mlp"}, f"layer {i}")
+        # the two kinds differ in whether the rotation is stretched, which the rotation itself tells
+        if la["type"] not in ("latent_attention", "latent_attention_2"):
+            raise ValueError(f"layer {i}: unknown mixer type {la['type']!r}")
+        m = {k: v for k, v in la["mixer"].items() if v is not None}
+        _only(m, {"dim", "heads", "kv_from", "kv_rank", "q_rank", "rot", "rot_dim", "scale", "vdim"}, f"layer {i} mixer")
+        mixer = LatentAttentionSpec(
+            heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), rank=int(m["kv_rank"]), scale=float(m["scale"]),
+            sink=False, gate=False, q_rank=int(m["q_rank"]) if "q_rank" in m else int(shape_of(f"l{i}.mix.dq")[0]),
+            rot=_rotary(m["rot"], f"layer {i} rotation"), kv_from=int(m.get("kv_from", -1)))
+        if mixer.scale <= 0 or int(m["rot_dim"]) != mixer.rot_dim or mixer.q_rank < 1:
+            raise ValueError(f"layer {i}: unsupported attention settings {m}")
+        layers.append(LayerSpec(mixer, **(_nafazen_mlp(la["mlp"], f"layer {i} mlp") if la.get("mlp") is not None else {})))
+    return nafazen_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers, float(d["embedding"]["scale"]),
+                          float(d["logit_softcap"]), float(d["norm"]["eps"]))
+
+
 # config.json's "architecture" -> its reader
-_HYBRIDS = {"Kosesun": config_from_kosesun, "Regesun": config_from_regesun}
+_HYBRIDS = {"Kosesun": config_from_kosesun, "Regesun": config_from_regesun, "Nafazen": config_from_nafazen}
 
 
 class _Tensors:
@@ -274,7 +328,7 @@ class HFWeights:
 def load_pretrained(path: str | os.PathLike, device="cuda", dtype=torch.bfloat16, pstate=None,
                     name: str | None = None, fold_norms: bool = True):
     """Build our model for the checkpoint in ``path`` and copy its (TP-sharded) weights in.  The
-    model class follows from config.json: ``architecture`` (Kosesun, Regesun) or HF's ``architectures``."""
+    model class follows from config.json: ``architecture`` (Kosesun, Regesun, Nafazen) or HF's ``architectures``."""
     from . import build_model
 
     path = Path(path)

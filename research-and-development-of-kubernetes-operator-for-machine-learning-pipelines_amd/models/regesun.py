@@ -28,18 +28,12 @@ from .. import ops
 from ..parallel.comm import ParallelState, single
 from ..runtime.kv_cache import KVLayer, pad_dim
 from .config import DeltaSpec, LatentAttentionSpec, RegesunConfig, SSDSpec
-from .layers import ParamSource, fuse_rows, linear
+from .layers import ParamSource, fuse_rows, linear, pad_rows
 
 CHUNK = 64                         # granule of the recurrent layers' prompt lists
 GLU_ALPHA = 1.702                  # of the feed-forward's gate
 DELTA_DECAY = math.exp(-0.5)       # largest log decay of the delta rule
 UNIT_EPS = 1e-6                    # in the delta rule's unit keys
-
-
-def _pad_rows(w: torch.Tensor, heads: int, rows: int) -> torch.Tensor:
-    """[heads * d, K] -> [heads * rows, K], every head's rows padded with zeros."""
-    v = w.view(heads, -1, w.shape[1])
-    return torch.nn.functional.pad(v, (0, 0, 0, rows - v.shape[1])).reshape(heads * rows, w.shape[1])
 
 
 class RegesunModel:
@@ -98,10 +92,10 @@ class RegesunModel:
         uk, uv = src(p + "uk", H * m.dim, R), src(p + "uv", H * m.vdim, R)
         pad_r = lambda w: torch.nn.functional.pad(w, (0, RP - R))  # noqa: E731
         # a head's query rows and the latent's rows padded to the kernels' row sizes with zeros
-        L = {"proj": fuse_rows([_pad_rows(src(p + "q", H * m.dim, W), H, KP), _pad_rows(src(p + "dkv", R, W), 1, RP),
+        L = {"proj": fuse_rows([pad_rows(src(p + "q", H * m.dim, W), H, KP), pad_rows(src(p + "dkv", R, W), 1, RP),
                                 src(p + "g", H * m.vdim, W)]),
              "c_norm": src(p + "dkv.norm", R, dtype=torch.float32, mean=1.0, std=0.0),
-             "w_kv": pad_r(torch.cat([_pad_rows(uk, H, KP), _pad_rows(uv, H, VP)])).contiguous(),
+             "w_kv": pad_r(torch.cat([pad_rows(uk, H, KP), pad_rows(uv, H, VP)])).contiguous(),
              "w_qk": torch.nn.functional.pad(uk.view(H, m.dim, R).transpose(1, 2), (0, KP - m.dim, 0, RP - R)).contiguous(),
              "w_vo": pad_r(uv.view(H, m.vdim, R)).contiguous(),
              "sink": src(p + "sink", H, dtype=torch.float32, std=1.0), "o": src(p + "o", W, H * m.vdim),

@@ -11,6 +11,7 @@ from __future__ import annotations
 
 import math
 import os
+from dataclasses import dataclass
 from pathlib import Path
 
 import torch
@@ -179,16 +180,18 @@ def paged_attention(q, k_cache, v_cache, meta, out: torch.Tensor | None = None):
     return out
 
 
-EPI_NONE, EPI_SILU_MUL, EPI_RELU2 = 0, 1, 6
+EPI_NONE, EPI_SILU_MUL, EPI_RELU2, EPI_XIELU = 0, 1, 6, 7
 
 
 def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi: int = EPI_NONE,
-         glu: tuple | None = None):
+         glu: tuple | None = None, xielu: tuple | None = None):
     """y = epi(x @ w^T), w [N, K] bf16.  EPI_SILU_MUL expects gate/up rows
     interleaved in groups of 16 (``interleave_gate_up``) and returns N/2 columns; with ``glu`` =
     (alpha, limit) it is the clamped gated unit g sigmoid(alpha g) (u + 1) of g = min(gate, limit),
-    u = clamp(up, -limit, limit) instead.  EPI_RELU2 is max(y, 0)^2."""
+    u = clamp(up, -limit, limit) instead.  EPI_RELU2 is max(y, 0)^2; EPI_XIELU with ``xielu`` = (a, b) is
+    y / 2 + a y^2 for y > 0 and y / 2 + b (exp(y) - 1 - y) otherwise."""
     N = w.shape[0]
+    glu = xielu or glu  # (two numbers either way)
     out_n = N // 2 if epi == EPI_SILU_MUL else N
     if not x.is_cuda:
         y = torch.nn.functional.linear(x, w) if x.dtype != torch.bfloat16 else \
@@ -198,6 +201,8 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
             y = ref.silu_mul(y) if glu is None else ref.clamp_glu(y, *glu)
         elif epi == EPI_RELU2:
             y = ref.relu2(y)
+        elif epi == EPI_XIELU:
+            y = ref.xielu(y, *glu)
         if out is not None:
             out.copy_(y.view_as(out))
             return out
@@ -209,7 +214,7 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
         x2 = x2.contiguous()
     M, K = x2.shape
     o2 = torch.empty(M, out_n, dtype=x.dtype, device=x.device) if out is None else out.view(M, out_n)
-    if x.dtype == torch.float32 and (epi != EPI_SILU_MUL or glu):  # true fp32 (library product; no reduced-precision mode)
+    if x.dtype == torch.float32:  # true fp32 (library product; no reduced-precision mode)
         _gemm_hipblaslt(x2, w, o2, epi, glu)
         return o2.view(*lead, out_n) if out is None else out
     _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi, glu)
@@ -234,8 +239,10 @@ def _gemm_hipblaslt(x2, w, o2, epi, glu=None):
         torch.matmul(x2, w.t(), out=o2)
         if epi == EPI_RELU2:
             torch.ops.mlop.relu2(o2)
-    elif glu is not None:
-        torch.ops.mlop.clamp_glu(o2, torch.matmul(x2, w.t()), *glu)
+        elif epi == EPI_XIELU:
+            torch.ops.mlop.xielu(o2, *glu)
+    elif glu is not None or x2.dtype == torch.float32:
+        torch.ops.mlop.clamp_glu(o2, torch.matmul(x2, w.t()), *(glu or (0.0, 0.0)))
     else:
         torch.ops.mlop.silu_mul(o2, torch.matmul(x2, w.t()), 1)
 
@@ -762,6 +769,15 @@ def relu2(x):
     return x
 
 
+def xielu(x, a: float, b: float):
+    """x / 2 + a x^2 for x > 0, x / 2 + b (exp(x) - 1 - x) otherwise, in place."""
+    if not x.is_cuda:
+        return x.copy_(ref.xielu(x, a, b))
+    _need_gpu()
+    torch.ops.mlop.xielu(x, a, b)
+    return x
+
+
 def softcap(x, cap: float):
     """cap * tanh(x / cap), fp32."""
     if not x.is_cuda:
@@ -814,26 +830,30 @@ def gla(proj, n_heads: int, dim: int, vdim: int, a2, a2_b, norm_w, tau: float, e
     return out
 
 
-def residual_begin(ids, table, scale: float, pos_table, positions, norm_w, eps: float):
+def residual_begin(ids, table, scale: float, pos_table, positions, norm_w, eps: float, width: int | None = None):
     """fp32 residual x = scale table[id] + pos_table[position] (``pos_table`` None: none) and the first
-    sublayer's input norm_w x / rms(x) in the table's dtype."""
+    sublayer's input norm_w x / rms(x) in the table's dtype (``norm_w`` [W] or one number; None: x itself).
+    ``width``: columns the mean square is over, where zeros pad the rows."""
     if not table.is_cuda:
-        return ref.residual_begin(ids, table, scale, pos_table, positions, norm_w, eps)
+        return ref.residual_begin(ids, table, scale, pos_table, positions, norm_w, eps, width)
     _need_gpu()
     x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=table.device)
     xn = torch.empty(x.shape, dtype=table.dtype, device=table.device)
-    torch.ops.mlop.residual_begin(xn, x, ids, table, scale, pos_table, positions, norm_w, eps)
+    torch.ops.mlop.residual_begin(xn, x, ids, table, scale, pos_table, positions, norm_w, eps, width or 0)
     return x, xn
 
 
-def residual_step(x, y, post_w, norm_w, eps: float, store: bool = True):
-    """x <- x + post_w y / rms(y) (``post_w`` None: x + y), in place unless ``store`` is off (nothing reads it
-    again); returns the next sublayer's input norm_w x / rms(x)."""
-    if not y.is_cuda:
-        return ref.residual_step(x, y, post_w, norm_w, eps)
+def residual_step(x, y, post_w, norm_w, eps: float, store: bool = True, width: int | None = None, experts=None):
+    """x <- x + post_w y / rms(y) (``post_w`` [W] or one number; None: x + y), in place unless ``store`` is off
+    (nothing reads it again); returns the next sublayer's input norm_w x / rms(x) (None: x itself).
+    ``experts`` = (rows [R, W], inv [T, k], gate [T] or None): gate[t] y[t] + sum_j rows[inv[t, j]] stands in
+    y's place (y None: the sum alone).  ``width`` as in residual_begin."""
+    if not x.is_cuda:
+        return ref.residual_step(x, y, post_w, norm_w, eps, width, experts)
     _need_gpu()
-    xn = torch.empty_like(y)
-    torch.ops.mlop.residual_step(xn, x, y, post_w, norm_w, eps, store)
+    rows, inv, gate = experts or (None, None, None)
+    xn = torch.empty(x.shape, dtype=(rows if y is None else y).dtype, device=x.device)
+    torch.ops.mlop.residual_step(xn, x, y, post_w, norm_w, eps, store, width or 0, rows, inv, gate)
     return xn
 
 
@@ -886,23 +906,41 @@ def delta(proj, w2, w0, a_b, decay_scale: float, unit_eps: float, state, meta):
     return o
 
 
-def latent_store(latents, w, eps: float, slots, cache):
-    """w l / rms(l) of the step's latents [T, R] into their cache slots ([NB, 1, BS, RP])."""
+def latent_store(latents, w, eps: float, slots, cache, rope=None, query=None):
+    """w l / rms(l) of the step's latents [T, R] into their cache slots ([NB, 1, BS, RP]).  ``rope`` = (keys
+    [T, n], table, positions, offset): the rotated key part to the row's dims offset .. offset + n.  ``query`` =
+    (x [T, r], weight [r], size): returns ``latent_query`` of them, from the same launch."""
     if not latents.is_cuda:
-        return ref.latent_store(latents, w, eps, slots, cache)
+        return ref.latent_store(latents, w, eps, slots, cache, rope, query)
     _need_gpu()
-    torch.ops.mlop.latent_store(cache, latents, w, eps, slots)
+    k, table, pos, off = rope or (None, None, None, 0)
+    x, qw, size = query or (None, None, 0)
+    out = None if x is None else torch.empty(x.shape[0], size, dtype=x.dtype, device=x.device)
+    torch.ops.mlop.latent_store(cache, latents, w, eps, slots, k, table, pos, off, out, x, qw)
+    return out
 
 
-def latent_attention(q, gate, cache, w_kv, w_qk, w_vo, vdim: int, scale: float, window: int, sink, meta):
+def latent_query(x, w, size: int, eps: float):
+    """w x / rms(x) of x [T, r], zeros up to ``size`` columns."""
+    if not x.is_cuda:
+        return ref.latent_query(x, w, eps, size)
+    _need_gpu()
+    out = torch.empty(x.shape[0], size, dtype=x.dtype, device=x.device)
+    torch.ops.mlop.latent_query(out, x, w, eps)
+    return out
+
+
+def latent_attention(q, gate, cache, w_kv, w_qk, w_vo, vdim: int, scale: float, window: int, sink, meta, rope=None):
     """Ragged attention over cached latents: q [T, H, KP] -> [T, H vdim].  A head's keys and values are linear
     in a latent row: ``w_kv`` [H (KP + VP), RP] expands a portion's keys and values; decoded tokens stay in the
-    latent space, with ``w_qk`` [H, RP, KP] (the keys' map, transposed) on the query and ``w_vo`` [H, vdim,
-    RP] (the values' map) on the result.  ``window``: tokens a token sees (0: all); ``sink`` [H] joins each
-    head's denominator; ``gate`` [T, H vdim]: the result times sigmoid(gate)."""
+    latent space, with ``w_qk`` [H, N, K] (the keys' map, transposed) on the query's first K dims and ``w_vo``
+    [H, vdim, RV] (the values' map) on the result's first RV.  ``window``: tokens a token sees (0: all);
+    ``sink`` [H] joins each head's denominator; ``gate`` [T, H vdim]: the result times sigmoid(gate).
+    ``rope`` = (table, n, q_off, k_off): dims q_off .. q_off + n of a query turn by its token's position, and
+    meet dims k_off .. k_off + n of the cached rows (N = k_off) as they are."""
     T, H, KP = q.shape
     if not q.is_cuda:
-        return ref.latent_attention(q, gate, cache, w_kv, H, vdim, scale, window, sink, meta)
+        return ref.latent_attention(q, gate, cache, w_kv, H, vdim, scale, window, sink, meta, rope)
     _need_gpu()
     from ..runtime.attn_meta import plan_partitions
 
@@ -910,11 +948,13 @@ def latent_attention(q, gate, cache, w_kv, w_qk, w_vo, vdim: int, scale: float, 
     out = torch.empty(T, H * vdim, dtype=q.dtype, device=dev)
     step = (meta.q_start, meta.q_len, meta.ctx_len)
     none = meta.tile_seq[:0]
-    nt, RP = meta.tile_seq.numel(), cache.shape[3]
+    nt, RP, RV = meta.tile_seq.numel(), cache.shape[3], w_vo.shape[2]
+    table, n_rot, q_off, _ = rope or (None, 0, 0, 0)
     if nt:
         ql = torch.empty(nt, H, RP, dtype=q.dtype, device=dev)
-        op.head_mm(ql, q, w_qk, meta.tile_seq, meta.tile_q0, meta.q_start, meta.q_len, True, False, None)
-        ol = torch.empty_like(ql)
+        op.head_mm(ql, q, w_qk, meta.tile_seq, meta.tile_q0, meta.q_start, meta.q_len, True, False, None, table,
+                   meta.positions, q_off)
+        ol = torch.empty(nt, H, RV, dtype=q.dtype, device=dev)
         keys = meta.part_tokens * meta.nparts
         part, nparts = plan_partitions(nt, -(-H // 32), min(keys, window + 31) if window else keys,
                                        target_wgs=512)
@@ -929,7 +969,8 @@ def latent_attention(q, gate, cache, w_kv, w_qk, w_vo, vdim: int, scale: float, 
         VP = kv.shape[1] // H - KP
         k, v = kv[:, :H * KP].unflatten(1, (H, KP)), kv[:, H * KP:].unflatten(1, (H, VP))
         op.attention_hd(out.view(T, H, vdim), meta.part_o, meta.part_ml, meta.part_sem, q, k, v, meta.block_tables, none,
-                        none, meta.ptile_seq, meta.ptile_q0, *step, KP, scale, sink, gate, 32, 1, window, meta.xbase, False)
+                        none, meta.ptile_seq, meta.ptile_q0, *step, KP, scale, sink, gate, 32, 1, window, meta.xbase, False,
+                        table, q_off)
     return out
 
 
@@ -947,6 +988,46 @@ def moe_route(logits: torch.Tensor, top_k: int):
     idx = torch.empty(T, top_k, dtype=torch.int32, device=logits.device)
     torch.ops.mlop.moe_route(w, idx, logits.contiguous())
     return w, idx
+
+
+@dataclass
+class Dispatched:
+    """A step's tokens dealt to experts.  Permuted row r (offsets[e] <= r < offsets[e + 1]: expert e's) is row r
+    of ``x`` or, with ``a_rows``, row a_rows[r] times row_w[r]; inv [T, k]: a token's permuted rows."""
+    x: torch.Tensor
+    offsets: torch.Tensor
+    inv: torch.Tensor
+    gate: torch.Tensor | None   # sigmoid of the row behind the router's experts, per token
+    a_rows: torch.Tensor | None = None
+    row_w: torch.Tensor | None = None
+
+
+def moe_dispatch_input(x, router, n_experts: int, top_k: int) -> Dispatched:
+    """Mixture of experts with sigmoid scores on the experts' inputs: each token goes to the ``top_k`` experts of
+    largest sigmoid(router row . x) (fp32), its row times that score.  ``router`` [E or E + 1, W]: a last row
+    behind the experts' gives every token a gate."""
+    T, dev, gated = x.shape[0], x.device, router.shape[0] > n_experts
+    if not x.is_cuda:
+        topw, topi, gate = ref.moe_route_sigmoid(x.float() @ router.float().t(), n_experts, top_k)
+        xp, offsets, src, inv = ref.moe_permute(x, topi, 0, n_experts)
+        return Dispatched((xp.float() * topw.reshape(-1)[src.long()][:, None]).to(x.dtype), offsets, inv.view(T, top_k), gate)
+    _need_gpu()
+    _sk_reserve(dev)  # the launch's ticket counter lives in the stream-K scratch
+    i32 = lambda *n: torch.empty(*n, dtype=torch.int32, device=dev)  # noqa: E731
+    topi, offsets, inv = i32(T, top_k), i32(n_experts + 1), i32(T, top_k)
+    topw = torch.empty(T, top_k, dtype=torch.float32, device=dev)
+    gate = torch.empty(T, dtype=torch.float32, device=dev) if gated else None
+    if x.dtype == torch.float32 or T <= 16:  # rows gathered, times their scores
+        xp, src = torch.empty(T * top_k, x.shape[1], dtype=x.dtype, device=dev), i32(T * top_k)
+        if x.dtype == torch.float32:
+            torch.ops.mlop.moe_route_sigmoid(topw, topi, gate, gemm(x, router), n_experts)
+            torch.ops.mlop.moe_permute_scaled(xp, offsets, src, inv, x, topi, topw, n_experts)
+        else:
+            torch.ops.mlop.moe_dispatch_small_sigmoid(topw, topi, xp, offsets, src, inv, gate, x, router, n_experts)
+        return Dispatched(xp, offsets, inv, gate)
+    a_rows, row_w = i32(T * top_k), torch.empty(T * top_k, dtype=torch.float32, device=dev)
+    torch.ops.mlop.moe_dispatch_mid_sigmoid(topw, topi, offsets, a_rows, row_w, inv, gate, x, router, n_experts)
+    return Dispatched(x, offsets, inv, gate, a_rows, row_w)
 
 
 def moe_permute(x, topi, e0: int, n_local: int):
@@ -1057,10 +1138,11 @@ def moe_combine(y, inv, topw):
     return out
 
 
-def grouped_gemm(xp, w, offsets, epi: int = EPI_NONE, avg_rows: int | None = None, a_rows=None):
+def grouped_gemm(xp, w, offsets, epi: int = EPI_NONE, avg_rows: int | None = None, a_rows=None, row_scale=None):
     """Per group e: rows offsets[e]:offsets[e+1] of xp times w[e]^T in ONE launch
     (tiles enumerate (group, m-tile) pairs on device: no host sync, graph-safe).  ``a_rows``
-    [R]: permuted row r is row a_rows[r] of xp (R output rows; moe_dispatch_mid)."""
+    [R]: permuted row r is row a_rows[r] of xp (R output rows; moe_dispatch_mid); ``row_scale`` [R], with
+    ``a_rows``: times that."""
     if a_rows is not None and not xp.is_cuda:
         xp = xp[a_rows.long()]
         a_rows = None
@@ -1075,5 +1157,11 @@ def grouped_gemm(xp, w, offsets, epi: int = EPI_NONE, avg_rows: int | None = Non
         return out
     rows = avg_rows if avg_rows is not None else max(1, R // max(1, w.shape[0]))
     _sk_reserve(xp.device)
-    torch.ops.mlop.grouped_gemm(out, xp, w, offsets, rows, epi, a_rows)
+    if xp.dtype == torch.float32:
+        wide = out if epi == EPI_NONE else torch.empty(R, N, dtype=xp.dtype, device=xp.device)
+        torch.ops.mlop.grouped_plain(wide, xp, w, offsets)
+        if epi == EPI_SILU_MUL:
+            torch.ops.mlop.clamp_glu(out, wide, 0.0, 0.0)
+        return out
+    torch.ops.mlop.grouped_gemm(out, xp, w, offsets, rows, epi, a_rows, row_scale)
     return out

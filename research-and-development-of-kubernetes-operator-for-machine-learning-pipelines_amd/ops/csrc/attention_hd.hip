@@ -13,7 +13,8 @@
 //   * sink: a number per head that joins the softmax's denominator once, with no key and no value;
 //   * gate: head h's output times sigmoid(gate[t, h]), or an element's with its own gate, in the epilogue;
 //   * window: a token sees itself and the window - 1 tokens before it; pages in front are not read;
-//   * a prompt's keys and values may also come from dense rows (latent attention's expanded keys).
+//   * a prompt's keys and values may also come from dense rows (latent attention's expanded keys);
+//   * rot: a part of a prompt's query heads may turn by the position as it is read.
 // The sizes above 256 and fp32 operands take attn_any_kernel (one wave per query and head).
 //
 // REQUIREMENT: the cache is zero-initialised at allocation (as attention.hip's) and the pad
@@ -48,6 +49,22 @@ __device__ __forceinline__ float gate_of(const AttnHdArgs& a, int tok, int head)
   if (!a.gate || a.gate_elem) return 1.f;
   const float g = bf2f(reinterpret_cast<const uint16_t*>(a.gate)[(size_t)tok * a.gate_stride + head]);
   return 1.f / (1.f + __expf(-g));
+}
+
+// dims c .. c + 7 of a query head, the rotated ones among them turned by position p
+__device__ __forceinline__ bf16x8 turn8(const AttnHdArgs& a, bf16x8 x, int c, int p) {
+  const int d0 = c - a.rot_lo, half = a.n_rot >> 1;
+  if (d0 + 8 <= 0 || d0 >= a.n_rot) return x;
+  const float* cs = a.rot + (size_t)min(max(p, 0), a.n_pos - 1) * a.n_rot;
+#pragma unroll
+  for (int e = 0; e < 8; e += 2) {
+    if (d0 + e < 0 || d0 + e >= a.n_rot) continue;
+    const float co = cs[(d0 + e) >> 1], si = cs[half + ((d0 + e) >> 1)];
+    const float u = bf2f_s(x[e]), v = bf2f_s(x[e + 1]);
+    x[e] = (short)f2bf(u * co - v * si);
+    x[e + 1] = (short)f2bf(v * co + u * si);
+  }
+  return x;
 }
 
 // an element's own gate
@@ -324,7 +341,7 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
 // attention.hip's flash32 scheme (32x32x16 MFMA, softmax on the lane, 3-deep LDS-DMA ring of page
 // pairs, counted vmcnt, one raw barrier per pair, deferred rescale).
 template <int NKB, int NVB>
-__global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel(AttnHdArgs a,
+__global__ void __launch_bounds__(256, (NKB + NVB) <= 5 ? 2 : 1) flash_hd_kernel(AttnHdArgs a,
                                                                                 const int* __restrict__ ptile_seq,
                                                                                 const int* __restrict__ ptile_q0) {
   constexpr int KP = 64 * NKB, VP = 64 * NVB, NQ = 4 * NKB, ND = 2 * NVB;
@@ -361,7 +378,8 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 4 ? 2 : 1) flash_hd_kernel
     const uint16_t* qrow = reinterpret_cast<const uint16_t*>(a.q) + (size_t)(qs + (q_ok ? qi : 0)) * a.q_row + head * a.q_head + 8 * h;
 #pragma unroll
     for (int t = 0; t < NQ; ++t) {
-      const bf16x8 v = *reinterpret_cast<const bf16x8*>(qrow + 16 * t);
+      bf16x8 v = *reinterpret_cast<const bf16x8*>(qrow + 16 * t);
+      if (a.rot) v = turn8(a, v, 16 * t + 8 * h, pos_r);
       qf[t] = q_ok ? v : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
     }
   }
@@ -585,7 +603,16 @@ __global__ void __launch_bounds__(256) attn_any_kernel(AttnHdArgs a, const int* 
   const E* vc = reinterpret_cast<const E*>(a.v_cache);
   const E* q = reinterpret_cast<const E*>(a.q) + (size_t)orow * a.q_row + head * a.q_head;
   float* qs = sm_q + wid * a.D;
-  for (int d = lane; d < a.D; d += 64) qs[d] = ld1(q + d);
+  const float* cs = a.rot ? a.rot + (size_t)min(max(n_keys - 1, 0), a.n_pos - 1) * a.n_rot : nullptr;
+  for (int d = lane; d < a.D; d += 64) {
+    const int r = d - a.rot_lo;
+    float v = ld1(q + d);
+    if (a.rot && r >= 0 && r < a.n_rot) {
+      const float co = cs[r >> 1], si = cs[(a.n_rot >> 1) + (r >> 1)];
+      v = r & 1 ? v * co + ld1(q + d - 1) * si : v * co - ld1(q + d + 1) * si;
+    }
+    qs[d] = v;
+  }
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
   __builtin_amdgcn_wave_barrier();
   const int* bt = a.bt + (size_t)s * a.bt_stride;

@@ -61,6 +61,14 @@ void hyper_step(Tensor xn, Tensor streams, Tensor y, Tensor mix, Tensor w_out, T
   mlop::launch_hyper(a, f32, cur());
 }
 
+void xielu(Tensor x, double a, double b) {
+  const bool f32 = model_f32(x, "x");
+  TORCH_CHECK(x.is_contiguous(), "x must be contiguous");
+  aligned16(x, "x");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_xielu(x.data_ptr(), x.numel(), (float)a, (float)b, f32, cur());
+}
+
 void relu2(Tensor x) {
   const bool f32 = model_f32(x, "x");
   TORCH_CHECK(x.is_contiguous(), "x must be contiguous");
@@ -144,7 +152,7 @@ void qk_norm_rope(Tensor q_out, Tensor k_cache, Tensor v_cache, Tensor proj, int
 void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Tensor q, Tensor k_cache, Tensor v_cache,
                   Tensor block_tables, Tensor tile_seq, Tensor tile_q0, Tensor ptile_seq, Tensor ptile_q0,
                   Tensor q_start, Tensor q_len, Tensor ctx_len, int64_t D, double scale, OptT sink, OptT gate,
-                  int64_t part_tokens, int64_t nparts, int64_t window, OptT xbase, bool by_tile) {
+                  int64_t part_tokens, int64_t nparts, int64_t window, OptT xbase, bool by_tile, OptT rot, int64_t rot_lo) {
   mlop::AttnHdArgs a{};
   const bool f32 = model_f32(q, "q");
   like(out, q, "out");
@@ -211,6 +219,15 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
     a.gate = gate->data_ptr();
     a.gate_stride = gate->stride(0);
     a.gate_elem = gate->size(1) != a.H;
+  }
+  if (rot) {
+    a.n_rot = (int)rot->size(1);
+    a.n_pos = (int)rot->size(0);
+    a.rot = f32_of(*rot, rot->numel(), "rot");
+    a.rot_lo = (int)rot_lo;
+    TORCH_CHECK(num_tiles == 0 && rot->dim() == 2 && a.n_pos >= 1 && a.n_rot % 2 == 0 && rot_lo >= 0 && rot_lo % 8 == 0 &&
+                    rot_lo + a.n_rot <= a.D,
+                "rot [positions, rotated dims] of prompt tiles");
   }
   a.scale_log2 = (float)(scale * 1.4426950408889634);
   a.num_blocks = (int)k_cache.size(0);
@@ -302,6 +319,7 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
   m.def("hyper_step(Tensor(a!) xn, Tensor(b!) streams, Tensor y, Tensor mix, Tensor w_out, Tensor w_in, "
         "Tensor norm_w, float eps, bool store) -> ()");
   m.def("relu2(Tensor(a!) x) -> ()");
+  m.def("xielu(Tensor(a!) x, float a, float b) -> ()");
   m.def("softcap(Tensor(a!) out, Tensor x, float cap) -> ()");
   m.def("qk_norm_rope(Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor proj, int D, int V, "
         "Tensor? q_w, Tensor? k_w, float eps, Tensor cos_sin, Tensor pos, Tensor slots, Tensor? v_first, Tensor? lam) "
@@ -309,7 +327,8 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
   m.def("attention_hd(Tensor(a!) out, Tensor(b!) part_o, Tensor(c!) part_ml, Tensor(d!) part_sem, Tensor q, "
         "Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_q0, Tensor ptile_seq, "
         "Tensor ptile_q0, Tensor q_start, Tensor q_len, Tensor ctx_len, int D, float scale, Tensor? sink, Tensor? gate, "
-        "int part_tokens, int nparts, int window=0, Tensor? xbase=None, bool by_tile=False) -> ()");
+        "int part_tokens, int nparts, int window=0, Tensor? xbase=None, bool by_tile=False, "
+        "Tensor? rot=None, int rot_lo=0) -> ()");
   m.def("gla(Tensor(a!) out, Tensor(b!) state, Tensor proj, int H, int dk, int dv, Tensor a2, Tensor a2_b, "
         "Tensor norm_w, float tau, float eps, Tensor q_start, Tensor q_len, Tensor ctx_len, Tensor rows, "
         "Tensor item_seq, Tensor item_t0, Tensor crow_seq, Tensor crow_item0, int chunk) -> ()");
@@ -319,6 +338,7 @@ TORCH_LIBRARY_IMPL(mlop, CUDA, m) {
   m.impl("hyper_begin", &hyper_begin);
   m.impl("hyper_step", &hyper_step);
   m.impl("relu2", &relu2);
+  m.impl("xielu", &xielu);
   m.impl("softcap", &softcap);
   m.impl("qk_norm_rope", &qk_norm_rope);
   m.impl("attention_hd", &attention_hd);

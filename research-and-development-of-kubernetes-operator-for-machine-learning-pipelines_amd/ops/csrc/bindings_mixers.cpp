@@ -3,6 +3,7 @@
 #include <cmath>
 
 #include "bind_util.h"
+#include "launch.h"
 #include "mixers.h"
 
 namespace {
@@ -31,7 +32,14 @@ mlop::StepRows step_rows(const Tensor& q_start, const Tensor& q_len, const Tenso
   return s;
 }
 
-void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, const Tensor& norm_w, double eps) {
+// [n] or one number
+const float* vec_or_one(const Tensor& t, int64_t n, bool& one, const char* name) {
+  one = t.numel() == 1 && n != 1;
+  aligned16(t, name);
+  return f32_of(t, one ? 1 : n, name);
+}
+
+void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, const OptT& norm_w, double eps, int64_t width) {
   TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.is_cuda() && x.scalar_type() == at::kFloat, "x must be [T, W] fp32");
   a.T = (int)x.size(0);
   a.W = (int)x.size(1);
@@ -39,17 +47,19 @@ void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, c
   TORCH_CHECK(xn.is_contiguous() && xn.numel() == x.numel(), "xn must be [T, W]");
   a.x = x.data_ptr<float>();
   a.xn = xn.data_ptr();
-  a.norm_w = f32_of(norm_w, a.W, "norm_w");
+  if (norm_w) a.norm_w = vec_or_one(*norm_w, a.W, a.norm_one, "norm_w");
   a.eps = (float)eps;
-  for (const Tensor* t : {&x, &xn, &norm_w}) aligned16(*t, "residual operand");
+  TORCH_CHECK(width >= 0 && width <= a.W, "width");
+  a.n = width ? (int)width : a.W;
+  for (const Tensor* t : {&x, &xn}) aligned16(*t, "residual operand");
 }
 
-void residual_begin(Tensor xn, Tensor x, Tensor ids, Tensor table, double scale, OptT pos_table, Tensor pos, Tensor norm_w,
-                    double eps) {
+void residual_begin(Tensor xn, Tensor x, Tensor ids, Tensor table, double scale, OptT pos_table, Tensor pos, OptT norm_w,
+                    double eps, int64_t width) {
   mlop::ResidualArgs a{};
   const bool f32 = model_f32(table, "table");
   like(xn, table, "xn");
-  residual_common(a, xn, x, norm_w, eps);
+  residual_common(a, xn, x, norm_w, eps, width);
   TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.numel() == a.T, "ids int64 [T]");
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && table.size(1) == a.W, "table must be [vocab, W]");
   aligned16(table, "table");
@@ -71,20 +81,31 @@ void residual_begin(Tensor xn, Tensor x, Tensor ids, Tensor table, double scale,
   mlop::launch_residual(a, f32, cur());
 }
 
-void residual_step(Tensor xn, Tensor x, Tensor y, OptT post_w, Tensor norm_w, double eps, bool store) {
+void residual_step(Tensor xn, Tensor x, OptT y, OptT post_w, OptT norm_w, double eps, bool store, int64_t width, OptT rows,
+                   OptT inv, OptT gate) {
   mlop::ResidualArgs a{};
-  const bool f32 = model_f32(y, "y");
-  like(xn, y, "xn");
-  residual_common(a, xn, x, norm_w, eps);
-  TORCH_CHECK(y.is_contiguous() && y.numel() == x.numel(), "y must be [T, W]");
-  aligned16(y, "y");
-  a.y = y.data_ptr();
-  if (post_w) {
-    a.post_w = f32_of(*post_w, a.W, "post_w");
-    aligned16(*post_w, "post_w");
+  TORCH_CHECK(y || rows, "residual_step needs a sublayer output");
+  const bool f32 = model_f32(xn, "xn");
+  residual_common(a, xn, x, norm_w, eps, width);
+  if (y) {
+    like(*y, xn, "y");
+    TORCH_CHECK(y->is_contiguous() && y->numel() == x.numel(), "y must be [T, W]");
+    aligned16(*y, "y");
+    a.y = y->data_ptr();
   }
+  if (rows) {
+    like(*rows, xn, "rows");
+    TORCH_CHECK(rows->dim() == 2 && rows->is_contiguous() && rows->size(1) == a.W, "rows must be [R, W]");
+    aligned16(*rows, "rows");
+    a.rows = rows->data_ptr();
+    TORCH_CHECK(inv && inv->dim() == 2 && inv->size(0) == a.T && inv->numel() <= rows->size(0), "inv must be [T, k]");
+    a.inv = i32_of(*inv, "inv");
+    a.top = (int)inv->size(1);
+    if (gate) a.gate = f32_of(*gate, a.T, "gate");
+  }
+  if (post_w) a.post_w = vec_or_one(*post_w, a.W, a.post_one, "post_w");
   a.store = store;
-  c10::DeviceGuard g(y.device());
+  c10::DeviceGuard g(xn.device());
   mlop::launch_residual(a, f32, cur());
 }
 
@@ -225,16 +246,67 @@ void delta(Tensor o, Tensor state, Tensor proj, Tensor w2, Tensor w0, Tensor a_b
   mlop::launch_delta(a, s, ws.defined() ? ws.data_ptr<float>() : nullptr, f32, cur());
 }
 
-void latent_store(Tensor cache, Tensor l, Tensor w, double eps, Tensor slots) {
+// the query latents' part of the arguments
+void query_part(mlop::LatentStoreArgs& a, const Tensor& out, const Tensor& x, const Tensor& w) {
+  like(out, x, "q_out");
+  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && out.is_contiguous() && out.size(0) == x.size(0) && out.size(1) >= x.size(1),
+              "query latents must be [T, r], out [T, >= r]");
+  aligned16(out, "q_out");
+  a.q_out = out.data_ptr();
+  a.q = x.data_ptr();
+  a.ldq = x.stride(0);
+  a.QR = (int)x.size(1);
+  a.QP = (int)out.size(1);
+  a.q_w = f32_of(w, a.QR, "q_w");
+  a.T = (int)x.size(0);
+}
+
+void latent_store(Tensor cache, Tensor l, Tensor w, double eps, Tensor slots, OptT k, OptT table, OptT pos, int64_t off,
+                  OptT q_out, OptT q, OptT q_w) {
+  mlop::LatentStoreArgs a{};
   const bool f32 = model_f32(l, "l");
   like(cache, l, "cache");
   TORCH_CHECK(cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == 1, "cache must be [NB, 1, BS, RP]");
   TORCH_CHECK(l.dim() == 2 && l.size(1) <= cache.size(3) && slots.numel() == l.size(0), "latents must be [T, R]");
   aligned16(cache, "cache");
+  if (q) {
+    TORCH_CHECK(q_out && q_w && q->size(0) == l.size(0), "query latents");
+    like(*q, l, "q");
+    query_part(a, *q_out, *q, *q_w);
+  }
+  a.cache = cache.data_ptr();
+  a.l = l.data_ptr();
+  a.ldl = l.stride(0);
+  a.R = (int)l.size(1);
+  a.RP = (int)cache.size(3);
+  a.w = f32_of(w, a.R, "w");
+  a.slots = i32_of(slots, "slots");
+  a.eps = (float)eps;
+  a.T = (int)l.size(0);
+  if (k) {
+    like(*k, l, "k");
+    TORCH_CHECK(table && pos && table->dim() == 2 && k->dim() == 2 && k->size(0) == a.T, "rotated keys");
+    a.n_rot = (int)table->size(1);
+    a.n_pos = (int)table->size(0);
+    TORCH_CHECK(k->size(1) == a.n_rot && a.n_rot % 2 == 0 && a.n_pos >= 1 && off >= a.R && off + a.n_rot <= a.RP, "rotated key size");
+    a.k = k->data_ptr();
+    a.ldk = k->stride(0);
+    a.table = f32_of(*table, table->numel(), "table");
+    a.pos = i32_of(*pos, "pos");
+    TORCH_CHECK(pos->numel() == a.T, "pos length");
+    a.off = (int)off;
+  }
   c10::DeviceGuard g(l.device());
-  mlop::launch_latent_store(cache.data_ptr(), l.data_ptr(), l.stride(0), f32_of(w, l.size(1), "w"), (float)eps,
-                            i32_of(slots, "slots"), (int)l.size(0), (int)l.size(1), (int)cache.size(3), (int)cache.size(2),
-                            f32, cur());
+  mlop::launch_latent_store(a, f32, cur());
+}
+
+void latent_query(Tensor out, Tensor x, Tensor w, double eps) {
+  mlop::LatentStoreArgs a{};
+  const bool f32 = model_f32(x, "x");
+  query_part(a, out, x, w);
+  a.eps = (float)eps;
+  c10::DeviceGuard g(x.device());
+  mlop::launch_latent_store(a, f32, cur());
 }
 
 void latent_gather(Tensor out, Tensor cache, Tensor block_tables, Tensor xbase, Tensor q_len, Tensor ctx_len,
@@ -268,7 +340,7 @@ void latent_gather(Tensor out, Tensor cache, Tensor block_tables, Tensor xbase, 
 }
 
 void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Tensor q_start, Tensor q_len, bool x_tok,
-             bool out_tok, OptT gate) {
+             bool out_tok, OptT gate, OptT table, OptT pos, int64_t x_off) {
   mlop::HeadMmArgs a{};
   const bool f32 = model_f32(x, "x");
   like(out, x, "out");
@@ -277,7 +349,9 @@ void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Te
   a.H = (int)w.size(0);
   a.N = (int)w.size(1);
   a.K = (int)w.size(2);
-  TORCH_CHECK(a.K % 64 == 0 && x.size(1) == a.H && x.size(2) == a.K && out.size(1) == a.H && out.size(2) == a.N, "head_mm sizes");
+  TORCH_CHECK(a.K % 64 == 0 && x.size(1) == a.H && x.size(2) >= a.K && out.size(1) == a.H &&
+                  (table ? out.size(2) > a.N && (out.size(2) - a.N) % 2 == 0 : out.size(2) == a.N),
+              "head_mm sizes");
   a.n_tiles = (int)tile_seq.numel();
   TORCH_CHECK((x_tok || x.size(0) >= a.n_tiles) && (out_tok || out.size(0) >= a.n_tiles) && a.n_tiles <= 65535, "head_mm rows");
   a.out = out.data_ptr();
@@ -296,6 +370,17 @@ void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Te
   a.q_len = i32_of(q_len, "q_len");
   a.x_tok = x_tok;
   a.out_tok = out_tok;
+  if (table) {
+    a.n_rot = (int)table->size(1);
+    a.n_pos = (int)table->size(0);
+    a.extra = (int)out.size(2) - a.N;
+    TORCH_CHECK(pos && table->dim() == 2 && a.n_pos >= 1 && a.n_rot % 2 == 0 && a.n_rot <= a.extra && x_off >= 0 &&
+                    x_off + a.n_rot <= x.size(2),
+                "rotated query part");
+    a.table = f32_of(*table, table->numel(), "table");
+    a.pos = i32_of(*pos, "pos");
+    a.x_off = (int)x_off;
+  }
   if (gate) {
     like(*gate, x, "gate");
     TORCH_CHECK(gate->dim() == 2 && gate->size(1) == (int64_t)a.H * a.N, "gate must be [T, H * N]");
@@ -306,6 +391,89 @@ void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Te
   mlop::launch_head_mm(a, f32, cur());
 }
 
+// operands common to the sigmoid routing's forms
+struct SigShape {
+  int T, E, rows, k, H;
+  float *topw, *gate;
+  int *topi, *inv;
+};
+SigShape sig_shape(const Tensor& topw, const Tensor& topi, const Tensor& inv, const OptT& gate, int64_t T, int64_t H, int64_t rows,
+                   int64_t E) {
+  SigShape s{};
+  const int64_t k = topi.dim() == 2 ? topi.size(1) : 0;
+  TORCH_CHECK(E >= 1 && E <= mlop::kSigMaxE && k >= 1 && k <= E && k <= mlop::kSigMaxTop, "1 .. ", mlop::kSigMaxE, " experts, top 1 .. ",
+              mlop::kSigMaxTop);
+  TORCH_CHECK(rows == E + (gate ? 1 : 0), "router rows: the experts', then the gate's");
+  TORCH_CHECK(topi.size(0) == T && inv.numel() == T * k && T * k < (1 << 28), "topi, inv must be [T, k]");
+  s.T = (int)T, s.E = (int)E, s.rows = (int)rows, s.k = (int)k, s.H = (int)H;
+  s.topw = const_cast<float*>(f32_of(topw, T * k, "topw"));
+  s.topi = const_cast<int*>(i32_of(topi, "topi"));
+  s.inv = const_cast<int*>(i32_of(inv, "inv"));
+  if (gate) s.gate = const_cast<float*>(f32_of(*gate, T, "gate"));
+  return s;
+}
+int* offsets_of(const Tensor& offsets, int64_t E) {
+  TORCH_CHECK(offsets.numel() == E + 1, "offsets must be [E + 1]");
+  return const_cast<int*>(i32_of(offsets, "offsets"));
+}
+void router_rows(const Tensor& x, const Tensor& w) {
+  TORCH_CHECK(x.is_cuda() && x.scalar_type() == at::kBFloat16 && w.is_cuda() && w.scalar_type() == at::kBFloat16, "bf16 x, router");
+  TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && w.dim() == 2 && w.is_contiguous() && w.size(1) == x.size(1) && x.size(1) % 8 == 0,
+              "x must be [T, H], router [rows, H], H a multiple of 8");
+  aligned16(x, "x");
+  aligned16(w, "router");
+}
+
+void moe_dispatch_small_sigmoid(Tensor topw, Tensor topi, Tensor xp, Tensor offsets, Tensor src, Tensor inv, OptT gate, Tensor x,
+                                Tensor w, int64_t E) {
+  router_rows(x, w);
+  const auto s = sig_shape(topw, topi, inv, gate, x.size(0), x.size(1), w.size(0), E);
+  TORCH_CHECK(s.T >= 1 && s.T <= 16, "1 .. 16 tokens");
+  like(xp, x, "xp");
+  TORCH_CHECK(xp.is_contiguous() && xp.dim() == 2 && xp.size(0) == s.T * s.k && xp.size(1) == s.H && src.numel() == s.T * s.k, "xp [T * k, H]");
+  aligned16(xp, "xp");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_moe_dispatch_small_sigmoid(s.topw, s.topi, xp.data_ptr(), offsets_of(offsets, E), const_cast<int*>(i32_of(src, "src")),
+                                          s.inv, s.gate, x.data_ptr(), w.data_ptr(), s.T, s.E, s.rows, s.k, s.H, cur());
+}
+
+void moe_dispatch_mid_sigmoid(Tensor topw, Tensor topi, Tensor offsets, Tensor a_rows, Tensor row_w, Tensor inv, OptT gate, Tensor x,
+                              Tensor w, int64_t E) {
+  router_rows(x, w);
+  const auto s = sig_shape(topw, topi, inv, gate, x.size(0), x.size(1), w.size(0), E);
+  TORCH_CHECK(s.T >= 1 && a_rows.numel() == s.T * s.k, "a_rows must be [T * k]");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_moe_dispatch_mid_sigmoid(s.topw, s.topi, offsets_of(offsets, E), const_cast<int*>(i32_of(a_rows, "a_rows")),
+                                        const_cast<float*>(f32_of(row_w, (int64_t)s.T * s.k, "row_w")), s.inv, s.gate, x.data_ptr(),
+                                        w.data_ptr(), s.T, s.E, s.rows, s.k, s.H, cur());
+}
+
+void moe_route_sigmoid(Tensor topw, Tensor topi, OptT gate, Tensor logits, int64_t E) {
+  TORCH_CHECK(logits.dim() == 2, "logits must be [T, rows]");
+  const auto s = sig_shape(topw, topi, topi, gate, logits.size(0), 0, logits.size(1), E);
+  c10::DeviceGuard g(logits.device());
+  mlop::launch_moe_route_sigmoid(s.topw, s.topi, s.gate, f32_of(logits, logits.numel(), "logits"), s.T, s.E, s.rows, s.k, cur());
+}
+
+void moe_permute_scaled(Tensor xp, Tensor offsets, Tensor src, Tensor inv, Tensor x, Tensor topi, Tensor topw, int64_t E) {
+  TORCH_CHECK(x.dim() == 2, "x must be [T, H]");
+  const auto s = sig_shape(topw, topi, inv, std::nullopt, x.size(0), x.size(1), E, E);
+  TORCH_CHECK(src.numel() == s.T * s.k, "src must be [T * k]");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_moe_permute_scaled(const_cast<float*>(f32_of(xp, (int64_t)s.T * s.k * s.H, "xp")), offsets_of(offsets, E),
+                                  const_cast<int*>(i32_of(src, "src")), s.inv, f32_of(x, x.numel(), "x"), s.topi, s.topw, s.T, s.k,
+                                  s.H, s.E, cur());
+}
+
+void grouped_plain(Tensor out, Tensor a, Tensor w, Tensor offsets) {
+  TORCH_CHECK(a.dim() == 2 && w.dim() == 3 && out.dim() == 2 && w.size(2) == a.size(1) && out.size(0) == a.size(0) &&
+                  out.size(1) == w.size(1) && a.size(0) < (1 << 20),
+              "a [R, K], w [G, N, K], out [R, N]");
+  c10::DeviceGuard g(a.device());
+  mlop::launch_grouped_plain(const_cast<float*>(f32_of(out, out.numel(), "out")), f32_of(a, a.numel(), "a"), f32_of(w, w.numel(), "w"),
+                             offsets_of(offsets, w.size(0)), (int)w.size(0), (int)a.size(0), (int)w.size(1), (int)w.size(2), cur());
+}
+
 }  // namespace
 
 #define MLOP_ROWS                                                                                                \
@@ -314,8 +482,9 @@ void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Te
 
 TORCH_LIBRARY_FRAGMENT(mlop, m) {
   m.def("residual_begin(Tensor(a!) xn, Tensor(b!) x, Tensor ids, Tensor table, float scale, Tensor? pos_table, Tensor pos, "
-        "Tensor norm_w, float eps) -> ()");
-  m.def("residual_step(Tensor(a!) xn, Tensor(b!) x, Tensor y, Tensor? post_w, Tensor norm_w, float eps, bool store) -> ()");
+        "Tensor? norm_w, float eps, int width=0) -> ()");
+  m.def("residual_step(Tensor(a!) xn, Tensor(b!) x, Tensor? y, Tensor? post_w, Tensor? norm_w, float eps, bool store, "
+        "int width=0, Tensor? rows=None, Tensor? inv=None, Tensor? gate=None) -> ()");
   m.def("gated_norm(Tensor(a!) out, Tensor y, Tensor gate, Tensor w, int groups, float eps, int act, bool gate_first) -> ()");
   m.def("clamp_glu(Tensor(a!) out, Tensor x, float alpha, float limit) -> ()");
   m.def("short_conv(Tensor(a!) out, Tensor(b!) tail, Tensor x, Tensor w, Tensor? b, " MLOP_ROWS ") -> ()");
@@ -323,11 +492,21 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
         MLOP_ROWS ") -> ()");
   m.def("delta(Tensor(a!) o, Tensor(b!) state, Tensor proj, Tensor w2, Tensor w0, Tensor a_b, float decay_scale, "
         "float unit_eps, " MLOP_ROWS ") -> ()");
-  m.def("latent_store(Tensor(a!) cache, Tensor l, Tensor w, float eps, Tensor slots) -> ()");
+  m.def("latent_store(Tensor(a!) cache, Tensor l, Tensor w, float eps, Tensor slots, Tensor? k=None, Tensor? table=None, "
+        "Tensor? pos=None, int off=0, Tensor(b!)? q_out=None, Tensor? q=None, Tensor? q_w=None) -> ()");
+  m.def("latent_query(Tensor(a!) out, Tensor x, Tensor w, float eps) -> ()");
   m.def("latent_gather(Tensor(a!) out, Tensor cache, Tensor block_tables, Tensor xbase, Tensor q_len, Tensor ctx_len, "
         "Tensor crow_seq, int rows, int x_max, int window) -> ()");
   m.def("head_mm(Tensor(a!) out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Tensor q_start, Tensor q_len, "
-        "bool x_tok, bool out_tok, Tensor? gate) -> ()");
+        "bool x_tok, bool out_tok, Tensor? gate, Tensor? table=None, Tensor? pos=None, int x_off=0) -> ()");
+  m.def("moe_dispatch_small_sigmoid(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!) xp, Tensor(d!) offsets, Tensor(e!) src, "
+        "Tensor(f!) inv, Tensor(g!)? gate, Tensor x, Tensor router, int n_experts) -> ()");
+  m.def("moe_dispatch_mid_sigmoid(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!) offsets, Tensor(d!) a_rows, Tensor(e!) row_w, "
+        "Tensor(f!) inv, Tensor(g!)? gate, Tensor x, Tensor router, int n_experts) -> ()");
+  m.def("moe_route_sigmoid(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!)? gate, Tensor logits, int n_experts) -> ()");
+  m.def("moe_permute_scaled(Tensor(a!) xp, Tensor(b!) offsets, Tensor(c!) src, Tensor(d!) inv, Tensor x, Tensor topi, Tensor topw, "
+        "int n_experts) -> ()");
+  m.def("grouped_plain(Tensor(a!) out, Tensor a, Tensor w, Tensor offsets) -> ()");
 }
 
 TORCH_LIBRARY_IMPL(mlop, CUDA, m) {
@@ -339,6 +518,12 @@ TORCH_LIBRARY_IMPL(mlop, CUDA, m) {
   m.impl("ssd", &ssd);
   m.impl("delta", &delta);
   m.impl("latent_store", &latent_store);
+  m.impl("latent_query", &latent_query);
   m.impl("latent_gather", &latent_gather);
   m.impl("head_mm", &head_mm);
+  m.impl("moe_dispatch_small_sigmoid", &moe_dispatch_small_sigmoid);
+  m.impl("moe_dispatch_mid_sigmoid", &moe_dispatch_mid_sigmoid);
+  m.impl("moe_route_sigmoid", &moe_route_sigmoid);
+  m.impl("moe_permute_scaled", &moe_permute_scaled);
+  m.impl("grouped_plain", &grouped_plain);
 }

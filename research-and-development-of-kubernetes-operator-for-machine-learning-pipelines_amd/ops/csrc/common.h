@@ -137,6 +137,11 @@ __device__ __forceinline__ float relu2_f(float x) {
   return r * r;
 }
 
+// xIELU: x / 2 + a x^2 for x > 0, x / 2 + b (exp(x) - 1 - x) otherwise
+__device__ __forceinline__ float xielu_f(float x, float a, float b) {
+  return fmaf(0.5f, x, x > 0.f ? a * x * x : b * (__expf(x) - 1.f - x));
+}
+
 __host__ __device__ constexpr int cdiv(int a, int b) { return (a + b - 1) / b; }
 
 }  // namespace mlop

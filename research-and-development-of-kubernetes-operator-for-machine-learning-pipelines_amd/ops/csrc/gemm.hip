@@ -27,7 +27,7 @@
 // (launch-boundary reduce, §5 "Projection GEMM at M = 256" item 2).
 //
 // Epilogues (fp32 LDS copy of the tile, 16-B coalesced stores):
-//   EPI_NONE      C = bf16(acc), or bf16(max(acc, 0)^2) (RopeEpi::relu2)
+//   EPI_NONE      C = bf16(acc), or an activation of acc (RopeEpi::act)
 //   EPI_SILU_MUL  B rows gate/up interleaved in groups of 16, C[:, j] = silu(g_j) * u_j (N/2 cols)
 //   EPI_ROPE      QKV projection: RoPE on q/k heads + q_out / paged K,V cache stores from the
 //                 staged tile (RopeEpi, launch.h); needs whole 128-wide heads per staged chunk
@@ -376,7 +376,7 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
         u32x4 o;
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-          o[j] = re.relu2 ? pack2(relu2_f(s[2 * j]), relu2_f(s[2 * j + 1])) : pack2(s[2 * j], s[2 * j + 1]);
+          o[j] = pack2(act_out(re, s[2 * j]), act_out(re, s[2 * j + 1]));
         *reinterpret_cast<u32x4*>(C + (size_t)(m0 + r) * ldc + n0 + c0 + c) = o;
       }
     } else {
@@ -389,7 +389,8 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
         const float* u = g + 16;
         // mid norm chain (re.ss_in: the producer's row totals): the row's RMSNorm factor scales
         // the accumulators first (W4_RS's order)
-        const float f = re.ss_in != nullptr ? rsqrtf(re.ss_in[m0 + r] * re.ss_inv_k + re.ss_eps) : 1.f;
+        float f = re.ss_in != nullptr ? rsqrtf(re.ss_in[m0 + r] * re.ss_inv_k + re.ss_eps) : 1.f;
+        if constexpr (GROUPED) f = re.row_scale != nullptr ? re.row_scale[m0 + r] : 1.f;
         u32x4 o;
 #pragma unroll
         for (int j = 0; j < 4; ++j)
@@ -405,14 +406,10 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
 template <int EPI>
 __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict__ C, int ldc,
                                                            const float* __restrict__ ws, int M,
-                                                           int N, int splits, int relu2 = 0, float glu_alpha = 0.f,
-                                                           float glu_limit = 0.f) {
+                                                           int N, int splits, RopeEpi re = RopeEpi{}) {
   const int outw = EPI == EPI_NONE ? N : N / 2;
   const int vpr = outw / 8;
   const long total = (long)M * vpr;
-  RopeEpi re{};
-  re.glu_alpha = glu_alpha;
-  re.glu_limit = glu_limit;
   for (long v = blockIdx.x * (long)blockDim.x + threadIdx.x; v < total;
        v += (long)gridDim.x * blockDim.x) {
     const int r = (int)(v / vpr), j0 = (int)(v % vpr) * 8;
@@ -430,11 +427,16 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict
         b[4] += w.x; b[5] += w.y; b[6] += w.z; b[7] += w.w;
       }
     }
+    if (EPI == EPI_SILU_MUL && re.row_scale != nullptr) {
+      const float f = re.row_scale[r];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) a[j] *= f, b[j] *= f;
+    }
     u32x4 o;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if (EPI == EPI_NONE)
-        o[j] = relu2 ? pack2(relu2_f(a[2 * j]), relu2_f(a[2 * j + 1])) : pack2(a[2 * j], a[2 * j + 1]);
+        o[j] = pack2(act_out(re, a[2 * j]), act_out(re, a[2 * j + 1]));
       else
         o[j] = pack2(glu_out(re, a[2 * j], b[2 * j]), glu_out(re, a[2 * j + 1], b[2 * j + 1]));
     }
@@ -1109,11 +1111,14 @@ __global__ void __launch_bounds__(512, 1) gemm_pp_kernel(
         if constexpr (EPI == EPI_NONE) {
 #pragma unroll
           for (int j = 0; j < 4; ++j)
-            sC[row * LD + j * 16 + (lane & 15)] = f2bf(re.relu2 ? relu2_f(acc[i][j][r]) : acc[i][j][r]);
+            sC[row * LD + j * 16 + (lane & 15)] = f2bf(act_out(re, acc[i][j][r]));
         } else {
+          float f = 1.f;
+          if constexpr (GROUPED)
+            if (re.row_scale != nullptr) f = re.row_scale[min(m0 + grp * 128 + row, m_end - 1)];
 #pragma unroll
           for (int jp = 0; jp < 2; ++jp) {
-            const float g = acc[i][2 * jp][r], u = acc[i][2 * jp + 1][r];
+            const float g = acc[i][2 * jp][r] * f, u = acc[i][2 * jp + 1][r] * f;
             sC[row * LD + jp * 16 + (lane & 15)] = f2bf(glu_out(re, g, u));
           }
         }
@@ -1718,22 +1723,23 @@ bool launch_mid_rs(const void* A, int lda, const void* B, void* out, int ldo, in
 }
 
 long gemm_workspace_floats(int M, int N, int K, int epi) {
-  if (epi == kEpiRelu2) epi = EPI_NONE;
+  if (epi_act(epi)) epi = EPI_NONE;
   if (gemv_takes(M, N, K, epi)) return 0;
   const Plan p = plan(M, N, K, false, 0, 0);
   return p.splits > 1 ? (long)p.splits * M * N : 0;
 }
 
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
-                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float glu_alpha, float glu_limit) {
+                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float p0, float p1) {
   if (M == 0) return;
   RopeEpi re{};
-  re.glu_alpha = glu_alpha;
-  re.glu_limit = glu_limit;
-  re.relu2 = epi == kEpiRelu2;
-  if (re.relu2) epi = EPI_NONE;
+  re.p0 = p0;
+  re.p1 = p1;
+  re.act = epi_act(epi);
+  const int epi0 = epi;
+  if (re.act) epi = EPI_NONE;
   if (gemv_takes(M, N, K, epi) && lda % 8 == 0 && ldb % 8 == 0) {
-    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, re.relu2 ? kEpiRelu2 : epi, st, glu_alpha, glu_limit);
+    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, epi0, st, p0, p1);
     return;
   }
   Plan p = plan(M, N, K, false, 0, 0);
@@ -1749,9 +1755,9 @@ void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ld
     const long total = (long)M * (outw / 8);
     const int g = (int)std::min<long>((total + 255) / 256, 4096);
     if (epi == EPI_NONE)
-      splitk_reduce_kernel<EPI_NONE><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, re.relu2);
+      splitk_reduce_kernel<EPI_NONE><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, re);
     else
-      splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, 0, glu_alpha, glu_limit);
+      splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, ldc, ws, M, N, p.splits, re);
   }
 }
 
@@ -1794,10 +1800,10 @@ bool launch_gemm_add_rmsnorm(const void* A, int lda, const void* B, void* out, v
 
 void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offsets, int n_groups,
                          int M, int N, int K, int max_rows, int epi, hipStream_t st, const int* a_rows,
-                         float** defer_ws, int* defer_splits) {
+                         float** defer_ws, int* defer_splits, const float* row_scale) {
   if (defer_splits) *defer_splits = 1;
   if (M == 0) return;
-  if (a_rows == nullptr && defer_splits == nullptr && gemv_grouped_takes(M, N, K, epi)) {  // MoE decode: stream only the routed experts' weights
+  if (a_rows == nullptr && row_scale == nullptr && defer_splits == nullptr && gemv_grouped_takes(M, N, K, epi)) {  // MoE decode: stream only the routed experts' weights
     launch_gemv_grouped(A, B, C, offsets, n_groups, M, N, K, epi, st);
     return;
   }
@@ -1823,6 +1829,7 @@ void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offse
   }
   RopeEpi re{};
   re.a_rows = a_rows;
+  re.row_scale = row_scale;
   if (epi == EPI_NONE)
     launch_plan<EPI_NONE, true>(p, (const uint16_t*)A, K, (const uint16_t*)B, K, (uint16_t*)C, N,
                                 ws, M, N, K, offsets, n_groups, st, re);
@@ -1839,7 +1846,7 @@ void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offse
     if (epi == EPI_NONE)
       splitk_reduce_kernel<EPI_NONE><<<g, 256, 0, st>>>((uint16_t*)C, N, ws, M, N, p.splits);
     else
-      splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, N / 2, ws, M, N, p.splits);
+      splitk_reduce_kernel<EPI_SILU_MUL><<<g, 256, 0, st>>>((uint16_t*)C, N / 2, ws, M, N, p.splits, re);
   }
 }
 

@@ -301,7 +301,7 @@ __global__ void __launch_bounds__(256) gemv_kernel(const uint16_t* __restrict__ 
 #pragma unroll
       for (int r = 0; r < R; ++r)
         if (lane == m * R + r && m < mc)
-          C[(size_t)m * ldc + set * R + r] = f2bf(re.relu2 ? relu2_f(acc[r][m]) : acc[r][m]);
+          C[(size_t)m * ldc + set * R + r] = f2bf(act_out(re, acc[r][m]));
   }
 }
 
@@ -376,14 +376,14 @@ bool gemv_takes(int M, int N, int K, int epi) {
 }
 
 void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ldc, int M, int N, int K,
-                 int epi, hipStream_t st, float glu_alpha, float glu_limit) {
+                 int epi, hipStream_t st, float p0, float p1) {
   auto* a = (const uint16_t*)A;
   auto* b = (const uint16_t*)B;
   auto* c = (uint16_t*)C;
   RopeEpi none{};
-  none.relu2 = epi == kEpiRelu2;
-  none.glu_alpha = glu_alpha;
-  none.glu_limit = glu_limit;
+  none.act = epi_act(epi);
+  none.p0 = p0;
+  none.p1 = p1;
   if (epi == EPI_SILU_MUL) run_gemv<EPI_SILU_MUL>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
   else run_gemv<EPI_NONE>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
 }

@@ -69,6 +69,10 @@ struct AttnHdArgs {
   bool gate_elem;        // one gate per head and value element (H x V); else one per head
   bool by_tile;          // q and out rows are decode tiles, not tokens
   int window;            // a token sees itself and the window - 1 tokens before it (0: all)
+  // prompt tiles: dims rot_lo .. rot_lo + n_rot of a query head turn by the token's position as they are
+  // read (null: none); [n_pos, n_rot]: cos of the pairs (2i, 2i + 1), then sin
+  const float* rot;
+  int rot_lo, n_rot, n_pos;
   int H, G, D, V, KP, VP;
   float scale_log2;
   int num_blocks;
@@ -77,10 +81,10 @@ struct AttnHdArgs {
 void launch_paged_hd(const AttnHdArgs& a, bool f32, float* part_o, float* part_ml, int* sem, const int* tile_seq,
                      const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st);
 // the same with keys and values the same latent rows (latent_decode.hip): by_tile, one head of KP = VP <=
-// 512 elements; partials per 16 heads
+// 576 elements, the first V of them values; partials per 16 heads
 void launch_latent_decode(const AttnHdArgs& a, float* part_o, float* part_ml, const int* tile_seq, const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st);
 inline bool latent_decode_ok(const AttnHdArgs& a, bool f32) {
-  return !f32 && a.by_tile && a.G == 1 && a.k_cache == a.v_cache && a.KP == a.VP && a.V == a.VP && a.KP <= 512;
+  return !f32 && a.by_tile && a.G == 1 && a.k_cache == a.v_cache && a.KP == a.VP && a.V % 64 == 0 && a.KP <= 576;
 }
 // tiles of up to 128 query tokens of one head
 void launch_flash_hd(const AttnHdArgs& a, bool f32, const int* tile_seq, const int* tile_q0, int num_tiles,
@@ -114,6 +118,7 @@ constexpr int kGlaMaxDk = 256;    // key size of the chunked kernel
 
 // ---- elementwise (hyper.hip)
 void launch_relu2(void* x, long n, bool f32, hipStream_t st);                       // in place
+void launch_xielu(void* x, long n, float a, float b, bool f32, hipStream_t st);     // in place
 void launch_softcap(float* out, const void* x, long n, float cap, bool f32, hipStream_t st);
 
 }  // namespace mlop

@@ -149,6 +149,18 @@ __global__ void __launch_bounds__(256) relu2_kernel(E* __restrict__ x, long n) {
   stn<VEC>(x + i, v);
 }
 
+// xIELU in place
+template <typename E, int VEC>
+__global__ void __launch_bounds__(256) xielu_kernel(E* __restrict__ x, long n, float a, float b) {
+  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (i >= n) return;
+  float v[VEC];
+  ldn<VEC>(x + i, v);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) v[e] = 0.5f * v[e] + (v[e] > 0.f ? a * v[e] * v[e] : b * (expm1f(v[e]) - v[e]));
+  stn<VEC>(x + i, v);
+}
+
 // out <- cap * tanh(x / cap), fp32
 template <typename E, int VEC>
 __global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ out, const E* __restrict__ x, long n,
@@ -172,6 +184,19 @@ void launch_relu2(void* x, long n, bool f32, hipStream_t st) {
   } else {
     if (v8) relu2_kernel<uint16_t, 8><<<grid, 256, 0, st>>>((uint16_t*)x, n);
     else relu2_kernel<uint16_t, 1><<<grid, 256, 0, st>>>((uint16_t*)x, n);
+  }
+}
+
+void launch_xielu(void* x, long n, float a, float b, bool f32, hipStream_t st) {
+  if (n == 0) return;
+  const bool v8 = n % 8 == 0;
+  const long grid = (n / (v8 ? 8 : 1) + 255) / 256;
+  if (f32) {
+    if (v8) xielu_kernel<float, 8><<<grid, 256, 0, st>>>((float*)x, n, a, b);
+    else xielu_kernel<float, 1><<<grid, 256, 0, st>>>((float*)x, n, a, b);
+  } else {
+    if (v8) xielu_kernel<uint16_t, 8><<<grid, 256, 0, st>>>((uint16_t*)x, n, a, b);
+    else xielu_kernel<uint16_t, 1><<<grid, 256, 0, st>>>((uint16_t*)x, n, a, b);
   }
 }
 

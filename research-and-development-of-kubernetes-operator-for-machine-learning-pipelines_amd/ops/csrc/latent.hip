@@ -1,7 +1,8 @@
 // Latent attention around attention_hd.hip's softmax: only a normed latent row c [R] per token is cached,
 // and every head's keys and values are linear in it (k = U_k c, v = U_v c).
 //
-//   latent_store    the token's latent, RMS-normed, into its cache slot;
+//   latent_store    the token's latent, RMS-normed, into its cache slot, a key part shared by all heads,
+//                   turned by the position, behind it; the queries' latent is normed beside them;
 //   prompts         latent_gather copies the latents of a portion's keys (cached ones and its own) to one
 //                   dense matrix, a GEMM expands them to keys and values, flash_hd reads those;
 //   decode          head_mm takes the query to the latent space (q U_k per head), the paged kernel
@@ -12,49 +13,79 @@
 
 namespace mlop {
 
-// a wave per token
+// the pair (u, v) turned by position p; n: rotated dims
+__device__ __forceinline__ void turn(const float* table, int p, int n_pos, int n, int pair, float& u, float& v) {
+  const float* cs = table + (size_t)min(max(p, 0), n_pos - 1) * n + pair;
+  const float c = cs[0], s = cs[n >> 1], x = u;
+  u = x * c - v * s;
+  v = v * c + x * s;
+}
+
+// one wave: out = w * x / rms(x), zeros from n to n_pad
 template <typename E, int VEC>
-__global__ void __launch_bounds__(256) latent_store_kernel(E* __restrict__ cache, const E* __restrict__ l, long ldl,
-                                                           const float* __restrict__ w, float eps,
-                                                           const int* __restrict__ slots, int T, int R, int RP) {
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (t >= T) return;
-  const int slot = slots[t];
-  if (slot < 0) return;
-  const E* x = l + (size_t)t * ldl;
+__device__ __forceinline__ void norm_row(E* out, const E* x, const float* w, int n, int n_pad, float eps, int lane) {
   float v[VEC], ss = 0.f;
-  for (int c = lane * VEC; c < R; c += 64 * VEC) {
+  for (int c = lane * VEC; c < n; c += 64 * VEC) {
     ldn<VEC>(x + c, v);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) ss = fmaf(v[e], v[e], ss);
   }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)R + eps);
-  E* out = cache + (size_t)slot * RP;
-  for (int c = lane * VEC; c < R; c += 64 * VEC) {
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)n + eps);
+  for (int c = lane * VEC; c < n_pad; c += 64 * VEC) {
     float wv[VEC];
-    ldn<VEC>(x + c, v);
-    ldn<VEC>(w + c, wv);
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) v[e] *= inv * wv[e];
+    for (int e = 0; e < VEC; ++e) v[e] = 0.f;
+    if (c < n) {
+      ldn<VEC>(x + c, v);
+      ldn<VEC>(w + c, wv);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] *= inv * wv[e];
+    }
     stn<VEC>(out + c, v);
   }
 }
 
-template <typename E>
-static void latent_store_t(void* cache, const void* l, long ldl, const float* w, float eps, const int* slots, int T, int R,
-                           int RP, hipStream_t st) {
-  const bool al = ((reinterpret_cast<uintptr_t>(l) | reinterpret_cast<uintptr_t>(w)) & 15) == 0 && ldl % 8 == 0;
-  const int grid = cdiv(T, 4);
-  if (al && R % 8 == 0) latent_store_kernel<E, 8><<<grid, 256, 0, st>>>((E*)cache, (const E*)l, ldl, w, eps, slots, T, R, RP);
-  else latent_store_kernel<E, 1><<<grid, 256, 0, st>>>((E*)cache, (const E*)l, ldl, w, eps, slots, T, R, RP);
+// a wave per token and job (its latent and rotated key; its query latent)
+template <typename E, int VEC>
+__global__ void __launch_bounds__(256) latent_store_kernel(LatentStoreArgs a) {
+  const int lane = threadIdx.x & 63, jobs = (a.l ? 1 : 0) + (a.q ? 1 : 0);
+  const int unit = blockIdx.x * 4 + (threadIdx.x >> 6), t = unit / jobs;
+  if (t >= a.T) return;
+  if (!a.l || unit % jobs) {
+    norm_row<E, VEC>(reinterpret_cast<E*>(a.q_out) + (size_t)t * a.QP, reinterpret_cast<const E*>(a.q) + (size_t)t * a.ldq,
+                     a.q_w, a.QR, a.QP, a.eps, lane);
+    return;
+  }
+  const int slot = a.slots[t];
+  if (slot < 0) return;
+  E* row = reinterpret_cast<E*>(a.cache) + (size_t)slot * a.RP;
+  if (a.k) {
+    const E* k = reinterpret_cast<const E*>(a.k) + (size_t)t * a.ldk;
+    const int p = a.pos[t];
+    for (int i = lane; i < a.n_rot >> 1; i += 64) {
+      float u = ld1(k + 2 * i), v = ld1(k + 2 * i + 1);
+      turn(a.table, p, a.n_pos, a.n_rot, i, u, v);
+      st1(row + a.off + 2 * i, u);
+      st1(row + a.off + 2 * i + 1, v);
+    }
+  }
+  norm_row<E, VEC>(row, reinterpret_cast<const E*>(a.l) + (size_t)t * a.ldl, a.w, a.R, a.R, a.eps, lane);
 }
 
-void launch_latent_store(void* cache, const void* l, long ldl, const float* w, float eps, const int* slots, int T, int R,
-                         int RP, int BS, bool f32, hipStream_t st) {
-  (void)BS;  // one latent head: a slot is a row of the page array
-  if (T == 0) return;
-  if (f32) latent_store_t<float>(cache, l, ldl, w, eps, slots, T, R, RP, st);
-  else latent_store_t<uint16_t>(cache, l, ldl, w, eps, slots, T, R, RP, st);
+template <typename E>
+static void latent_store_t(const LatentStoreArgs& a, hipStream_t st) {
+  auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool v8 = (!a.l || (al(a.l) && al(a.w) && a.ldl % 8 == 0 && a.R % 8 == 0)) &&
+                  (!a.q || (al(a.q) && al(a.q_w) && a.ldq % 8 == 0 && a.QR % 8 == 0 && a.QP % 8 == 0));
+  const int grid = cdiv(a.T * ((a.l ? 1 : 0) + (a.q ? 1 : 0)), 4);
+  if (v8) latent_store_kernel<E, 8><<<grid, 256, 0, st>>>(a);
+  else latent_store_kernel<E, 1><<<grid, 256, 0, st>>>(a);
+}
+
+void launch_latent_store(const LatentStoreArgs& a, bool f32, hipStream_t st) {
+  if (a.T == 0 || (!a.l && !a.q)) return;
+  if (f32) latent_store_t<float>(a, st);
+  else latent_store_t<uint16_t>(a, st);
 }
 
 // 16 threads per row, 16 rows per workgroup; blockIdx.x = n_crows: the zero rows behind the last one
@@ -94,11 +125,33 @@ __device__ __forceinline__ float gate_f(float g) { return 1.f / (1.f + __expf(-g
 
 }  // namespace
 
-// A workgroup: one head, 64 NT output columns (16 NT per wave), 16 MT tiles.
+// the columns behind a head's products: the rotated query part, then zeros (n tiles from m0)
+template <typename E>
+__device__ __forceinline__ void head_rot(const HeadMmArgs& a, int h, int m0, int n) {
+  const int pairs = a.extra >> 1;
+  for (int x = threadIdx.x; x < n * pairs; x += 256) {
+    const int i = m0 + x / pairs, p = x % pairs;
+    if (i >= a.n_tiles) return;
+    const int tok = tile_token(a, i);
+    float u = 0.f, v = 0.f;
+    if (2 * p < a.n_rot) {
+      const E* src = reinterpret_cast<const E*>(a.x) + (size_t)(a.x_tok ? tok : i) * a.ldx + h * a.hx + a.x_off + 2 * p;
+      u = ld1(src), v = ld1(src + 1);
+      turn(a.table, a.pos[tok], a.n_pos, a.n_rot, p, u, v);
+    }
+    E* out = reinterpret_cast<E*>(a.out) + (size_t)(a.out_tok ? tok : i) * a.ldo + h * a.ho + a.N + 2 * p;
+    st1(out, u);
+    st1(out + 1, v);
+  }
+}
+
+// A workgroup: one head, 64 NT output columns (16 NT per wave), 16 MT tiles; with a table, the last of a
+// head's workgroups has the columns behind the products.
 template <int MT, int NT>
 __global__ void __launch_bounds__(256) head_mm_kernel(HeadMmArgs a) {
   const int h = blockIdx.x, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l15 = lane & 15, g4 = lane >> 4;
   const int n0 = (blockIdx.y * 4 + wid) * 16 * NT, m0 = blockIdx.z * 16 * MT;
+  if (a.table && blockIdx.y == gridDim.y - 1) return head_rot<uint16_t>(a, h, m0, 16 * MT);
   if (n0 >= a.N) return;
   const uint16_t* w[NT];
 #pragma unroll
@@ -165,6 +218,7 @@ __global__ void __launch_bounds__(256) head_mm_kernel(HeadMmArgs a) {
 // plain form (fp32): one thread per output
 __global__ void __launch_bounds__(256) head_mm_plain_kernel(HeadMmArgs a) {
   const int h = blockIdx.x, n = blockIdx.y * 256 + threadIdx.x, i = blockIdx.z;
+  if (a.table && blockIdx.y == gridDim.y - 1) return head_rot<float>(a, h, i, 1);
   if (n >= a.N) return;
   const int tok = tile_token(a, i);
   const float* x = reinterpret_cast<const float*>(a.x) + (size_t)(a.x_tok ? tok : i) * a.ldx + h * a.hx;
@@ -177,14 +231,15 @@ __global__ void __launch_bounds__(256) head_mm_plain_kernel(HeadMmArgs a) {
 
 void launch_head_mm(const HeadMmArgs& a, bool f32, hipStream_t st) {
   if (a.n_tiles == 0) return;
+  const int more = a.table ? 1 : 0;
   if (f32) {
-    head_mm_plain_kernel<<<dim3(a.H, cdiv(a.N, 256), a.n_tiles), 256, 0, st>>>(a);
+    head_mm_plain_kernel<<<dim3(a.H, cdiv(a.N, 256) + more, a.n_tiles), 256, 0, st>>>(a);
   } else if (a.n_tiles > 64) {
-    head_mm_kernel<4, 2><<<dim3(a.H, cdiv(a.N, 128), cdiv(a.n_tiles, 64)), 256, 0, st>>>(a);
+    head_mm_kernel<4, 2><<<dim3(a.H, cdiv(a.N, 128) + more, cdiv(a.n_tiles, 64)), 256, 0, st>>>(a);
   } else if (a.n_tiles > 16) {
-    head_mm_kernel<2, 1><<<dim3(a.H, cdiv(a.N, 64), cdiv(a.n_tiles, 32)), 256, 0, st>>>(a);
+    head_mm_kernel<2, 1><<<dim3(a.H, cdiv(a.N, 64) + more, cdiv(a.n_tiles, 32)), 256, 0, st>>>(a);
   } else {
-    head_mm_kernel<1, 1><<<dim3(a.H, cdiv(a.N, 64), 1), 256, 0, st>>>(a);
+    head_mm_kernel<1, 1><<<dim3(a.H, cdiv(a.N, 64) + more, 1), 256, 0, st>>>(a);
   }
 }
 

@@ -1,10 +1,11 @@
 // Decode attention over cached latents: one query token per tile, keys and values are the SAME rows of RP
-// elements (one latent head), so a step reads each latent once.
+// elements (one latent head), of which the first V are values, so a step reads each latent once.
 //
 // A workgroup takes one tile, up to 32 heads and a partition of the keys.  Its two teams of 4 waves take
 // the partition's page pairs (32 keys) in turn, each through two LDS stages (LDS-DMA, one pair ahead), and
 // join at the end.  Wave w of a team works on head group w & 1 (16 heads, the MFMA columns) and half w >> 1
-// of the RP dims:
+// of the RP dims (of an odd number of 64-dim blocks both halves hold the middle one; the second half's queries
+// are zero there):
 //   S^T = C . Q^T over its half, the halves' partial scores meet in LDS, both waves run the same softmax,
 //   O^T += C^T . P^T for its half of the dims (with a deferred rescale).
 // Every LDS row is read as K (ds_read_b128 along dims) and as V (ds_read_b64_tr_b16 along keys), so the
@@ -61,15 +62,14 @@ __device__ __forceinline__ int sw(int t) { return ((t & 2) << 1) | ((t >> 2) & 2
 
 }  // namespace
 
-// NB: 64-element blocks of a latent row
-template <int NB>
+// NB: 64-element blocks of a latent row, NV of values (at least a.V / 64)
+template <int NB, int NV>
 __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float* __restrict__ part_o,
                                                            float* __restrict__ part_ml,
                                                            const int* __restrict__ tile_seq,
                                                            const int* __restrict__ tile_q0, int part_tokens, int nparts) {
-  // an odd NB is rounded up: the last block is staged twice, and meets zero queries the second time
-  constexpr int RP = 64 * NB, NBE = NB + NB % 2, NH = NBE / 2, NK = 2 * NH, ND = 4 * NH;
-  constexpr uint32_t STAGE = NBE * 4096u;  // bytes
+  constexpr int RP = 64 * NB, NH = (NB + 1) / 2, NHV = (NV + 1) / 2, NK = 2 * NH, ND = 4 * NHV;
+  constexpr uint32_t STAGE = NB * 4096u;  // bytes
   __shared__ __attribute__((aligned(256))) uint16_t smem[4 * STAGE / 2];  // [stage][team]; the join's exchange
   __shared__ __attribute__((aligned(16))) f32x4 sx[2][2][2][2][64];       // partial scores [team][group][half][product]
   const uint16_t* cc = reinterpret_cast<const uint16_t*>(a.k_cache);
@@ -79,7 +79,8 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
   const int team = wid8 >> 2, wid = wid8 & 3;
   const int grp = wid & 1, half = wid >> 1, r = lane & 15, g4 = lane >> 4;
   const int head0 = blockIdx.y * 32 + 16 * grp, nh = min(16, a.H - head0);  // (<= 0: no such group)
-  const int b0 = half * NH, nb = min(NH, NB - b0);                          // blocks of this half
+  const int b0 = half * (NB - NH), v0 = half * (NV - NHV);                  // first key / value block of this half
+  const int V = a.V;
   // (uniform, so that the page table is read through the scalar cache, not behind the LDS-DMA)
   const int s = __builtin_amdgcn_readfirstlane(tile_seq[tile]), qi = __builtin_amdgcn_readfirstlane(tile_q0[tile]);
   const int ql = __builtin_amdgcn_readfirstlane(a.q_len[s]), ctx = __builtin_amdgcn_readfirstlane(a.ctx_len[s]);
@@ -90,10 +91,10 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
   const int p_begin = k_base + part * part_tokens;
   const int p_end = min(kv_end, p_begin + part_tokens);
   const int h_all = min(32, a.H - (int)blockIdx.y * 32);
-  uint16_t* orow = out + ((size_t)tile * a.H + blockIdx.y * 32) * RP;
+  uint16_t* orow = out + ((size_t)tile * a.H + blockIdx.y * 32) * V;
   if (p_begin >= p_end) {  // nothing here; an empty row (graph padding) gives zeros
     if (part == 0 && kv_end <= 0 && live)
-      for (int e = threadIdx.x; e < h_all * RP; e += 512) orow[e] = 0;
+      for (int e = threadIdx.x; e < h_all * V; e += 512) orow[e] = 0;
     return;
   }
 
@@ -105,7 +106,7 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
       bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (ok && (kk >> 1) < nb) v = *reinterpret_cast<const bf16x8*>(qrow + kk * 32);
+      if (ok && (half == 0 || b0 + (kk >> 1) >= NH)) v = *reinterpret_cast<const bf16x8*>(qrow + kk * 32);
       qf[kk] = v;
     }
   }
@@ -125,17 +126,18 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
     uint16_t* base = smem + (2 * buf + team) * (STAGE / 2) + wid * 512;
     const uint16_t* src = cc + (size_t)pg * (kPg * RP) + src_off;
 #pragma unroll
-    for (int b = 0; b < NBE; ++b)
-      __builtin_amdgcn_global_load_lds((const void*)(src + min(b, NB - 1) * 64), (lds_void_t*)(base + b * 2048), 16, 0, 0);
+    for (int b = 0; b < NB; ++b)
+      __builtin_amdgcn_global_load_lds((const void*)(src + b * 64), (lds_void_t*)(base + b * 2048), 16, 0, 0);
   };
-  const uint32_t lds0 = (uint32_t)(uintptr_t)smem + team * STAGE + 4096u * b0;
+  const uint32_t lds0 = (uint32_t)(uintptr_t)smem + team * STAGE + 4096u * b0;   // keys
+  const uint32_t ldsv = (uint32_t)(uintptr_t)smem + team * STAGE + 4096u * v0;   // values
   // K: MFMA row r is key 8 (r >> 2) + (r & 3) of the pair in the first product, + 4 in the second
   const int kt = 8 * (r >> 2) + (r & 3);
   const uint32_t ka0 = lds0 + 128u * kt + 16u * (g4 ^ sw(kt & 15)), kb0 = lds0 + 128u * (kt + 4) + 16u * (g4 ^ sw((kt + 4) & 15));
   // V: transposed reads of keys 8 g4 + q (first) and + 4 (second), 16 dims at a time
   const int q = (lane >> 2) & 3, p4 = lane & 3, vt = 8 * g4 + q;
-  const uint32_t va0 = lds0 + 128u * vt + 16u * ((p4 >> 1) ^ sw(vt & 15)) + 8u * (p4 & 1);
-  const uint32_t vb0 = lds0 + 128u * (vt + 4) + 16u * ((p4 >> 1) ^ sw((vt + 4) & 15)) + 8u * (p4 & 1);
+  const uint32_t va0 = ldsv + 128u * vt + 16u * ((p4 >> 1) ^ sw(vt & 15)) + 8u * (p4 & 1);
+  const uint32_t vb0 = ldsv + 128u * (vt + 4) + 16u * ((p4 >> 1) ^ sw((vt + 4) & 15)) + 8u * (p4 & 1);
   const uint32_t sx_own = (uint32_t)(uintptr_t)&sx[team][grp][half][0][lane],
                  sx_other = (uint32_t)(uintptr_t)&sx[team][grp][half ^ 1][0][lane];
 
@@ -258,6 +260,8 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
     for (int d = 0; d < ND; ++d) o[d] = o[d] * f0 + xo[d * 64] * f1;
   }
   const bool ok = r < nh;
+  // 64-dim block v0 + i of the values is this wave's to store
+  auto mine_v = [&](int i) { return (half == 0 || v0 + i >= NHV) && (v0 + i) * 64 < V; };
   const size_t slab = (((size_t)tile * ny + blockIdx.y) * 2 + grp) * nparts;  // 16 heads each
   if (nparts == 1) {
     float L = l, f = 1.f;
@@ -270,19 +274,19 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
     if (ok) {
 #pragma unroll
       for (int d = 0; d < ND; ++d)
-        if ((d >> 2) < nb) {
+        if (mine_v(d >> 2)) {
           const float v[4] = {o[d][0] * inv, o[d][1] * inv, o[d][2] * inv, o[d][3] * inv};
-          stn<4>(orow + (size_t)(16 * grp + r) * RP + b0 * 64 + 16 * d + 4 * g4, v);
+          stn<4>(orow + (size_t)(16 * grp + r) * V + v0 * 64 + 16 * d + 4 * g4, v);
         }
     }
     return;
   }
   // partial (O, m, l) of this key range
   if (ok) {
-    float* po = part_o + ((slab + part) * 16 + r) * RP + b0 * 64 + 4 * g4;
+    float* po = part_o + ((slab + part) * 16 + r) * V + v0 * 64 + 4 * g4;
 #pragma unroll
     for (int d = 0; d < ND; ++d)
-      if ((d >> 2) < nb) *reinterpret_cast<f32x4*>(po + 16 * d) = o[d];
+      if (mine_v(d >> 2)) *reinterpret_cast<f32x4*>(po + 16 * d) = o[d];
     if (half == 0 && g4 == 0) {
       float* ml = part_ml + ((slab + part) * 16 + r) * 2;
       ml[0] = m;
@@ -292,19 +296,19 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(AttnHdArgs a, float*
 }
 
 // the partitions of one (tile, head): 4 elements per thread
-__global__ void __launch_bounds__(128) latent_combine_kernel(AttnHdArgs a, const float* __restrict__ part_o,
+__global__ void __launch_bounds__(192) latent_combine_kernel(AttnHdArgs a, const float* __restrict__ part_o,
                                                              const float* __restrict__ part_ml,
                                                              const int* __restrict__ tile_seq,
                                                              const int* __restrict__ tile_q0, int part_tokens, int nparts) {
-  const int tile = blockIdx.x, head = blockIdx.y, c = threadIdx.x * 4, RP = a.KP;
+  const int tile = blockIdx.x, head = blockIdx.y, c = threadIdx.x * 4, V = a.V;
   const int s = tile_seq[tile], qi = tile_q0[tile], ql = a.q_len[s], ctx = a.ctx_len[s];
   const int kv_end = qi < ql ? max(0, ctx - ql + qi + 1) : 0;
-  if (kv_end == 0 || c >= RP) return;  // (an empty row was zeroed)
+  if (kv_end == 0 || c >= V) return;  // (an empty row was zeroed)
   const int k_base = (a.window > 0 ? max(0, kv_end - a.window) : 0) & ~31;
   const int nvalid = min(nparts, (kv_end - k_base + part_tokens - 1) / part_tokens);
   const size_t slab = ((size_t)tile * (cdiv(a.H, 32) * 2) + (head >> 4)) * nparts * 16 + (head & 15);
   const float* ml = part_ml + slab * 2;
-  const float* po = part_o + slab * RP + c;
+  const float* po = part_o + slab * V + c;
   const float s2 = a.sink ? a.sink[head] * kLog2e : kLow;
   float M = s2;
   for (int p = 0; p < nvalid; ++p) M = fmaxf(M, ml[p * 32]);
@@ -314,25 +318,31 @@ __global__ void __launch_bounds__(128) latent_combine_kernel(AttnHdArgs a, const
   for (int p = 0; p < nvalid; ++p) {
     const float f = exp2f(ml[p * 32] - M);
     L += f * ml[p * 32 + 1];
-    acc += f * *reinterpret_cast<const f32x4*>(po + (size_t)p * 16 * RP);
+    acc += f * *reinterpret_cast<const f32x4*>(po + (size_t)p * 16 * V);
   }
   const float inv = L > 0.f ? 1.f / L : 0.f;
   const float v[4] = {acc[0] * inv, acc[1] * inv, acc[2] * inv, acc[3] * inv};
-  stn<4>(reinterpret_cast<uint16_t*>(a.out) + ((size_t)tile * a.H + head) * RP + c, v);
+  stn<4>(reinterpret_cast<uint16_t*>(a.out) + ((size_t)tile * a.H + head) * V + c, v);
 }
 
 void launch_latent_decode(const AttnHdArgs& a, float* part_o, float* part_ml, const int* tile_seq,
                           const int* tile_q0, int num_tiles, int part_tokens, int nparts, hipStream_t st) {
   const dim3 grid(num_tiles, cdiv(a.H, 32), nparts);
-#define MLOP_LD(N) \
-  case N: latent_decode_kernel<N><<<grid, 512, 0, st>>>(a, part_o, part_ml, tile_seq, tile_q0, part_tokens, nparts); break;
+#define MLOP_LD_V(N, V) \
+  latent_decode_kernel<N, V><<<grid, 512, 0, st>>>(a, part_o, part_ml, tile_seq, tile_q0, part_tokens, nparts)
+#define MLOP_LD(N)                                                        \
+  case N:                                                                 \
+    if (N > 1 && a.V / 64 < N) MLOP_LD_V(N, (N > 1 ? N - 1 : 1));         \
+    else MLOP_LD_V(N, N);                                                 \
+    break;
   switch (a.KP / 64) {
-    MLOP_LD(1) MLOP_LD(2) MLOP_LD(3) MLOP_LD(4) MLOP_LD(5) MLOP_LD(6) MLOP_LD(7) MLOP_LD(8)
+    MLOP_LD(1) MLOP_LD(2) MLOP_LD(3) MLOP_LD(4) MLOP_LD(5) MLOP_LD(6) MLOP_LD(7) MLOP_LD(8) MLOP_LD(9)
     default: break;
   }
 #undef MLOP_LD
+#undef MLOP_LD_V
   if (nparts > 1)
-    latent_combine_kernel<<<dim3(num_tiles, a.H), cdiv(a.KP, 256) * 64, 0, st>>>(a, part_o, part_ml, tile_seq, tile_q0,
+    latent_combine_kernel<<<dim3(num_tiles, a.H), cdiv(a.V, 256) * 64, 0, st>>>(a, part_o, part_ml, tile_seq, tile_q0,
                                                                                 part_tokens, nparts);
 }
 

@@ -72,18 +72,29 @@ struct RopeEpi {
   // mid norm chain (gemm.hip mid_chain_finish): 1 = the finishing split reads the partials with
   // plain loads behind one agent acquire, 0 = with sc1 loads only (gemm_mid_chain op 2 / 1)
   int mid_acq = 0;
-  // plain epilogue only: C = bf16(max(acc, 0)^2) instead of bf16(acc) (EPI_RELU2 of launch_gemm)
-  int relu2 = 0;
-  // SiLU-mul epilogue: alpha > 0 makes it the clamped gated unit (common.h clamp_glu_f) instead
-  float glu_alpha = 0.f, glu_limit = 0.f;
+  // plain epilogue only: an activation of the accumulator (kAct*; EPI_RELU2, EPI_XIELU of launch_gemm)
+  int act = 0;
+  // SiLU-mul epilogue: p0 > 0 makes it the clamped gated unit (common.h clamp_glu_f) with alpha = p0,
+  // limit = p1 instead; kActXielu: a = p0, b = p1
+  float p0 = 0.f, p1 = 0.f;
+  // grouped SiLU-mul: permuted row r's accumulators times row_scale[r] before the unit (nullptr: 1)
+  const float* row_scale = nullptr;
 };
+enum { kActNone = 0, kActRelu2 = 1, kActXielu = 2 };
 #ifdef __HIP__
 // one output of the gate / up epilogue
 __device__ __forceinline__ float glu_out(const RopeEpi& re, float g, float u) {
-  return re.glu_alpha > 0.f ? clamp_glu_f(g, u, re.glu_alpha, re.glu_limit) : silu_bf(g) * bf2f(f2bf(u));
+  return re.p0 > 0.f ? clamp_glu_f(g, u, re.p0, re.p1) : silu_bf(g) * bf2f(f2bf(u));
+}
+// one output of the plain epilogue
+__device__ __forceinline__ float act_out(const RopeEpi& re, float x) {
+  if (re.act == kActRelu2) return relu2_f(x);
+  return re.act == kActXielu ? xielu_f(x, re.p0, re.p1) : x;
 }
 #endif
-constexpr int kEpiRelu2 = 6;  // launch_gemm: plain product with the squared-relu epilogue
+// launch_gemm: plain product with an activation in its epilogue
+constexpr int kEpiRelu2 = 6, kEpiXielu = 7;
+constexpr int epi_act(int epi) { return epi == kEpiRelu2 ? kActRelu2 : epi == kEpiXielu ? kActXielu : kActNone; }
 // RoPE + paged-cache stores from the QKV projection's fp32 split-K slabs ws[splits][T][N] (the
 // split-K reduce fused in: small-M launch_gemm_rope)
 void launch_rope_cache_slabs(const RopeEpi& re, const float* ws, int splits, int T, int N, hipStream_t st);
@@ -127,7 +138,7 @@ int gemm_sk_workgroups(int M, int N, int K);
 // K2 skinny GEMV (gemv.hip): decode projections at M <= 8 (epi 0 none, 1 silu-mul, 3 rope)
 bool gemv_takes(int M, int N, int K, int epi);
 void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ldc, int M, int N, int K,
-                 int epi, hipStream_t st, float glu_alpha = 0.f, float glu_limit = 0.f);
+                 int epi, hipStream_t st, float p0 = 0.f, float p1 = 0.f);
 void launch_gemv_rope(const void* A, int lda, const void* B, int M, int N, int K, const RopeEpi& re,
                       hipStream_t st);
 // the decode norm chain's row-scale prologue parameters (gemv.hip PRO_RS)
@@ -173,14 +184,15 @@ bool gemm_rope_supported(int M, int N, int K);
 bool launch_gemm_rope(const void* A, int lda, const void* B, int M, int N, int K, const RopeEpi& re,
                       hipStream_t st);
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
-                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float glu_alpha = 0.f,
-                 float glu_limit = 0.f);
+                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float p0 = 0.f,
+                 float p1 = 0.f);
 bool launch_gemm_add_rmsnorm(const void* A, int lda, const void* B, void* out, void* residual,
                              const void* w, float eps, float* ws, long ws_floats, int M, int N,
                              int K, hipStream_t st);
 void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offsets, int n_groups,
                          int M, int N, int K, int max_rows, int epi, hipStream_t st, const int* a_rows = nullptr,
-                         float** defer_ws = nullptr, int* defer_splits = nullptr);
+                         float** defer_ws = nullptr, int* defer_splits = nullptr,
+                         const float* row_scale = nullptr);
 bool launch_moe_down_combine_add_rmsnorm(void* out, void* residual, void* y, const void* a, const void* w2,
                                          const int* offsets, int n_groups, int R, int H, int I, int max_rows,
                                          const int* inv, const float* topw, const void* norm_w, float eps, int T,
@@ -193,6 +205,19 @@ int moe_mid_max_tokens(int set);
 void launch_moe_dispatch_mid(float* topw, int* topi, int* offsets, int* arow, int* inv, const void* x, const void* wr,
                              int T, int E, int k, int H, int e0, int n_local, const void* pro_y, void* pro_res,
                              const void* pro_w, float pro_eps, void* pro_xn, hipStream_t st);
+// sigmoid routing with the scores on the experts' inputs (moe.hip); router rows: E experts', then a gate's or none
+constexpr int kSigMaxE = 256, kSigMaxTop = 32;
+void launch_moe_dispatch_small_sigmoid(float* topw, int* topi, void* xp, int* offsets, int* src, int* inv, float* gate,
+                                       const void* x, const void* wr, int T, int E, int rows, int k, int H,
+                                       hipStream_t st);
+void launch_moe_dispatch_mid_sigmoid(float* topw, int* topi, int* offsets, int* arow, float* row_w, int* inv, float* gate,
+                                     const void* x, const void* wr, int T, int E, int rows, int k, int H, hipStream_t st);
+void launch_moe_route_sigmoid(float* topw, int* topi, float* gate, const float* logits, int T, int E, int rows, int k,
+                              hipStream_t st);
+void launch_moe_permute_scaled(float* xp, int* offsets, int* src, int* inv, const float* x, const int* topi,
+                               const float* topw, int T, int k, int H, int E, hipStream_t st);
+void launch_grouped_plain(float* out, const float* a, const float* w, const int* offsets, int G, int R, int N, int K,
+                          hipStream_t st);
 void launch_moe_route(float* topw, int* topi, const void* logits, int T, int E, int k,
                       hipStream_t st);
 void launch_moe_permute(void* xp, int* offsets, int* src, int* inv, const void* x, const int* topi,

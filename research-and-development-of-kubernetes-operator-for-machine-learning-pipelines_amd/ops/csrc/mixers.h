@@ -26,9 +26,14 @@ struct StepRows {
 struct ResidualArgs {
   float* x;               // [T, W]
   void* xn;               // [T, W] the next sublayer's input: norm_w * x / rms(x)
-  const void* y;          // [T, W] sublayer output
-  const float* post_w;    // [W] y is normed on its own, times this (null: added as it is)
-  const float* norm_w;    // [W]
+  const void* y;          // [T, W] sublayer output (null: the experts' alone)
+  const void* rows;       // [R, W] or null: sublayer output gate[t] y[t] + sum_j rows[inv[t, j]]
+  const int* inv;         // [T, top]
+  const float* gate;      // [T] or null
+  int top;
+  const float* post_w;    // [W] or, post_one, one number: y is normed on its own, times this (null: added as it is)
+  const float* norm_w;    // [W] or, norm_one, one number (null: xn = x)
+  bool post_one, norm_one;
   const long* ids;        // [T]  (start: x = scale * table[id] + pos_table[pos])
   const void* table;      // [vocab, W]
   const void* pos_table;  // [n_pos, W] or null
@@ -36,6 +41,7 @@ struct ResidualArgs {
   long vocab, n_pos;
   float embed_scale, eps;
   int T, W;
+  int n;                  // columns the mean square is over (the rest are zero)
   bool store;             // write x back
 };
 void launch_residual(const ResidualArgs& a, bool f32, hipStream_t st);
@@ -57,7 +63,7 @@ struct GatedNormArgs {
 void launch_gated_norm(const GatedNormArgs& a, bool f32, hipStream_t st);
 
 // ---- clamped gated unit of interleaved gate / up columns (residual.hip)
-// out[t, i] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
+// out[t, i] = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit); alpha 0: silu(gate) up
 void launch_clamp_glu(void* out, const void* x, int T, int I, float alpha, float limit, bool f32, hipStream_t st);
 
 // ---- short causal convolution + silu with its last inputs as state (short_conv.hip)
@@ -107,9 +113,29 @@ long delta_ws_floats(int n_items, int chunk, int H, int dk);
 bool delta_blocks_ok(int dk, float decay_scale);  // else portions run token by token, without workspace
 
 // ---- latent attention (latent.hip; attention_hd.hip runs the softmax)
-// c = w * l / rms(l) of latent rows l into the paged cache [NB, 1, BS, RP]
-void launch_latent_store(void* cache, const void* l, long ldl, const float* w, float eps, const int* slots, int T, int R,
-                         int RP, int BS, bool f32, hipStream_t st);
+// c = w * l / rms(l) of latent rows l into the paged cache [NB, 1, BS, RP], with a rotated key part behind
+// it; and / or the queries' latents, normed the same way, to rows of their own
+struct LatentStoreArgs {
+  void* cache;
+  const void* l;          // [T, ldl], first R columns (null: no latents)
+  long ldl;
+  const float* w;         // [R]
+  const int* slots;       // < 0: no cache write
+  int R, RP;
+  const void* k;          // [T, ldk], first n_rot columns: dims off .. off + n_rot of the row (null: none)
+  long ldk;
+  const float* table;     // [n_pos, n_rot]: cos of the pairs (2i, 2i + 1), then sin
+  const int* pos;
+  int n_rot, off, n_pos;
+  void* q_out;            // [T, QP], columns past QR zero
+  const void* q;          // [T, ldq], first QR columns (null: none)
+  long ldq;
+  const float* q_w;       // [QR]
+  int QR, QP;
+  float eps;
+  int T;
+};
+void launch_latent_store(const LatentStoreArgs& a, bool f32, hipStream_t st);
 // cached rows of every portion's keys, positions window_start .. context end, to out [rows, RP];
 // row of position p of sequence s: xbase[s] + p; the `pad` rows behind them are zeroed
 struct LatentGatherArgs {
@@ -130,6 +156,11 @@ struct HeadMmArgs {
   const void* gate;       // [T, ldg]: out times sigmoid(gate[token, h * N + n]) (null: none)
   long ldg;
   int n_tiles, H, N, K;   // K a multiple of 64
+  // columns N .. N + extra of out (table; null: none): x's dims x_off .. x_off + n_rot, turned by the
+  // token's position, then zeros
+  const float* table;     // [n_pos, n_rot]
+  const int* pos;
+  int extra, x_off, n_rot, n_pos;
 };
 void launch_head_mm(const HeadMmArgs& a, bool f32, hipStream_t st);
 

@@ -1,6 +1,10 @@
 // Mixture-of-experts routing kernels for gfx950 (K11 route, K12 permute, K14 combine).
 // The expert FFN itself is the grouped MFMA GEMM of gemm.hip (K13).
 //
+// Two kinds of routing: softmax over the router's logits, renormalised over the chosen experts, the weights on
+// the experts' outputs (moe_combine); or (SIG) fp32 logits, the chosen experts' sigmoid scores as they are, the
+// scores on the experts' INPUT rows, and possibly one row behind the experts' whose sigmoid is a gate per token.
+//
 // Everything stays on the device and has static shapes (T*k rows reserved, the
 // valid count lives in offsets[n_local]), so an MoE layer can be captured in
 // a hipGraph: no host sync to size the permuted batch.
@@ -148,15 +152,54 @@ struct MoePro {
 // (all of a lane's chunks in flight together) while the wave walks the T activation rows.
 constexpr int kSmallT = 16, kMaxE = 64, kDispWaves = 8;
 
-template <int CH>  // 16-B chunks per lane per row: H = CH * 512
+// SIG: `rows` router rows, the first E of them experts'
+struct SigArgs {
+  float* gate;   // [T] sigmoid of row E (nullptr: there is none)
+  float* row_w;  // [T * k] score of each permuted row (the gathered rows hold it already: nullptr)
+  int rows;
+};
+__device__ __forceinline__ float sigmoid_of(float z) { return 1.f / (1.f + __expf(-z)); }
+
+// the largest of n logits behind (v, i) in the order of falling value, then rising index
+__device__ __forceinline__ void next_best(const float* z, int n, float& v, int& i) {
+  float bv = -INFINITY;
+  int bi = n;
+  for (int e = 0; e < n; ++e) {
+    const float s = z[e];
+    if ((s < v || (s == v && e > i)) && s > bv) bv = s, bi = e;
+  }
+  v = bv;
+  i = min(bi, n - 1);
+}
+
+// router logits of two token rows, any row length (a multiple of 8)
+__device__ __forceinline__ void dot_rows2(const uint16_t* w, const uint16_t* x0, const uint16_t* x1, int H, int lane,
+                                          float& s0, float& s1) {
+  s0 = s1 = 0.f;
+  for (int c = lane * 8; c < H; c += 512) {
+    const u32x4 b = *reinterpret_cast<const u32x4*>(w + c), p = *reinterpret_cast<const u32x4*>(x0 + c),
+                q = *reinterpret_cast<const u32x4*>(x1 + c);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      s0 += lo_bf(p[j]) * lo_bf(b[j]) + hi_bf(p[j]) * hi_bf(b[j]);
+      s1 += lo_bf(q[j]) * lo_bf(b[j]) + hi_bf(q[j]) * hi_bf(b[j]);
+    }
+  }
+  s0 = wave_sum(s0);
+  s1 = wave_sum(s1);
+}
+
+template <int CH, bool SIG = false>  // 16-B chunks per lane per row: H = CH * 512 (0: any H)
 __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
     float* __restrict__ topw, int* __restrict__ topi, uint16_t* __restrict__ xp, int* __restrict__ offsets,
     int* __restrict__ src, int* __restrict__ inv, const uint16_t* __restrict__ x,
-    const uint16_t* __restrict__ wr, int T, int E, int k, int H, int e0, int n_local, MoePro pro) {
-  __shared__ float lg[kSmallT][kMaxE];
-  __shared__ int s_topi[kSmallT * 8];
-  __shared__ int cnt[kMaxE + 1];
-  __shared__ int base[kMaxE + 1];
+    const uint16_t* __restrict__ wr, int T, int E, int k, int H, int e0, int n_local, MoePro pro, SigArgs sig = SigArgs{}) {
+  constexpr int ME = SIG ? kSigMaxE : kMaxE, MK = SIG ? kSigMaxTop : 8;
+  __shared__ float lg[kSmallT][ME + SIG];
+  __shared__ int s_topi[kSmallT * MK];
+  __shared__ float s_topw[SIG ? kSmallT * MK : 1];
+  __shared__ int cnt[ME + 1];
+  __shared__ int base[ME + 1];
   __shared__ float red[16];
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   if (pro.y != nullptr) {
@@ -194,14 +237,24 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
     x = pro.xn;
   }
   // 1. router logits: lg[t][e] = bf16(x[t] . wr[e])
-  for (int e = wv; e < E; e += kDispWaves) {
+  for (int e = wv; e < (SIG ? sig.rows : E); e += kDispWaves) {
+    if constexpr (CH == 0) {
+      for (int t = 0; t < T; t += 2) {
+        float s0, s1;
+        dot_rows2(wr + (size_t)e * H, x + (size_t)t * H, x + (size_t)min(t + 1, T - 1) * H, H, lane, s0, s1);
+        if (lane == 0) lg[t][e] = s0;
+        if (lane == 0 && t + 1 < T) lg[t + 1][e] = s1;
+      }
+      continue;
+    }
     const uint16_t* we = wr + (size_t)e * H + lane * 8;
-    u32x4 b[CH];
+    constexpr int CN = CH ? CH : 1;
+    u32x4 b[CN];
 #pragma unroll
     for (int i = 0; i < CH; ++i) b[i] = *reinterpret_cast<const u32x4*>(we + i * 512);
     for (int t = 0; t < T; ++t) {
       const uint16_t* xt = x + (size_t)t * H + lane * 8;
-      u32x4 a[CH];
+      u32x4 a[CN];
 #pragma unroll
       for (int i = 0; i < CH; ++i) a[i] = *reinterpret_cast<const u32x4*>(xt + i * 512);
       float acc = 0.f;
@@ -210,13 +263,23 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
 #pragma unroll
         for (int q = 0; q < 4; ++q) acc += lo_bf(a[i][q]) * lo_bf(b[i][q]) + hi_bf(a[i][q]) * hi_bf(b[i][q]);
       acc = wave_sum(acc);
-      if (lane == 0) lg[t][e] = bf2f(f2bf(acc));
+      if (lane == 0) lg[t][e] = SIG ? acc : bf2f(f2bf(acc));
     }
   }
   for (int e = threadIdx.x; e <= n_local; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
   // 2. softmax -> top-k -> renormalise (moe_route_kernel's math), one thread per token
-  if (threadIdx.x < T) {
+  if (SIG && threadIdx.x < T) {
+    const int t = threadIdx.x;
+    float v = INFINITY;
+    int e = -1;
+    for (int j = 0; j < k; ++j) {
+      next_best(lg[t], E, v, e);
+      s_topi[t * k + j] = topi[t * k + j] = e;
+      s_topw[t * k + j] = topw[t * k + j] = sigmoid_of(v);
+    }
+    if (sig.gate) sig.gate[t] = sigmoid_of(lg[t][E]);
+  } else if (threadIdx.x < T) {
     const int t = threadIdx.x;
     float mx = -INFINITY;
     for (int e = 0; e < E; ++e) mx = fmaxf(mx, lg[t][e]);
@@ -280,9 +343,13 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
   for (int i = threadIdx.x; i < n_slots * vpr; i += blockDim.x) {
     const int s = i / vpr, c = (i % vpr) * 8;
     const int row = s_topi[s];
-    if (row >= 0)
-      *reinterpret_cast<u32x4*>(xp + (size_t)row * H + c) =
-          *reinterpret_cast<const u32x4*>(x + (size_t)(s / k) * H + c);
+    if (row < 0) continue;
+    u32x4 v = *reinterpret_cast<const u32x4*>(x + (size_t)(s / k) * H + c);
+    if constexpr (SIG) {
+#pragma unroll
+      for (int q = 0; q < 4; ++q) v[q] = pack2(s_topw[s] * lo_bf(v[q]), s_topw[s] * hi_bf(v[q]));
+    }
+    *reinterpret_cast<u32x4*>(xp + (size_t)row * H + c) = v;
   }
 }
 
@@ -303,6 +370,24 @@ void launch_moe_dispatch_small(float* topw, int* topi, void* xp, int* offsets, i
     case 2048: MLOP_DISP(4); break;
     case 4096: MLOP_DISP(8); break;
     default: MLOP_DISP(16); break;
+  }
+#undef MLOP_DISP
+}
+
+void launch_moe_dispatch_small_sigmoid(float* topw, int* topi, void* xp, int* offsets, int* src, int* inv, float* gate,
+                                       const void* x, const void* wr, int T, int E, int rows, int k, int H,
+                                       hipStream_t st) {
+  const SigArgs sig{gate, nullptr, rows};
+#define MLOP_DISP(CH)                                                                                             \
+  moe_dispatch_small_kernel<CH, true><<<1, 64 * kDispWaves, 0, st>>>(topw, topi, (uint16_t*)xp, offsets, src, inv, \
+                                                                     (const uint16_t*)x, (const uint16_t*)wr, T, E, k, \
+                                                                     H, 0, E, MoePro{}, sig)
+  switch (H) {
+    case 1024: MLOP_DISP(2); break;
+    case 2048: MLOP_DISP(4); break;
+    case 4096: MLOP_DISP(8); break;
+    case 8192: MLOP_DISP(16); break;
+    default: MLOP_DISP(0); break;
   }
 #undef MLOP_DISP
 }
@@ -338,14 +423,15 @@ int moe_mid_max_tokens(int set) {
   return g_mid_max_t;
 }
 
-template <int CH, int kMidTok>
+template <int CH, int kMidTok, bool SIG = false>  // CH 0: any H (SIG)
 __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
     float* __restrict__ topw, int* __restrict__ topi, int* __restrict__ offsets, int* __restrict__ arow,
     int* __restrict__ inv, const uint16_t* __restrict__ x, const uint16_t* __restrict__ wr, int T, int E, int k,
-    int H, int e0, int n_local, MoePro pro, int* __restrict__ ticket) {
-  __shared__ float lg[kMidTok][kMaxE];
-  __shared__ int cnt[kMaxE + 1];
-  __shared__ int base[kMaxE + 1];
+    int H, int e0, int n_local, MoePro pro, int* __restrict__ ticket, SigArgs sig = SigArgs{}) {
+  constexpr int ME = SIG ? kSigMaxE : kMaxE;
+  __shared__ float lg[kMidTok][ME + SIG];
+  __shared__ int cnt[ME + 1];
+  __shared__ int base[ME + 1];
   __shared__ float red[16];
   __shared__ int last;
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
@@ -385,16 +471,26 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
     x = pro.xn;
   }
   // router logits of this workgroup's tokens
-  for (int e = wv; e < E; e += kDispWaves) {
+  for (int e = wv; e < (SIG ? sig.rows : E); e += kDispWaves) {
+    if constexpr (CH == 0) {
+      for (int tp = 0; tp < nt; tp += 2) {
+        float s0, s1;
+        dot_rows2(wr + (size_t)e * H, x + (size_t)(t0 + tp) * H, x + (size_t)(t0 + min(tp + 1, nt - 1)) * H, H, lane, s0, s1);
+        if (lane == 0) lg[tp][e] = s0;
+        if (lane == 0 && tp + 1 < nt) lg[tp + 1][e] = s1;
+      }
+      continue;
+    }
     const uint16_t* we = wr + (size_t)e * H + lane * 8;
-    u32x4 b[CH];
+    constexpr int CN = CH ? CH : 1;
+    u32x4 b[CN];
 #pragma unroll
     for (int i = 0; i < CH; ++i) b[i] = *reinterpret_cast<const u32x4*>(we + i * 512);
     // token rows two at a time, both rows' chunks in flight together (with the router row's
     // on the first pair: one latency, not three)
 #pragma unroll 1
     for (int tp = 0; tp < kMidTok; tp += 2) {
-      u32x4 a[2][CH];
+      u32x4 a[2][CN];
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -409,13 +505,25 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
           for (int q = 0; q < 4; ++q)
             acc += lo_bf(a[t][i][q]) * lo_bf(b[i][q]) + hi_bf(a[t][i][q]) * hi_bf(b[i][q]);
         acc = wave_sum(acc);
-        if (lane == 0 && tp + t < nt) lg[tp + t][e] = bf2f(f2bf(acc));
+        if (lane == 0 && tp + t < nt) lg[tp + t][e] = SIG ? acc : bf2f(f2bf(acc));
       }
     }
   }
   __syncthreads();
   const auto rs_topi = __builtin_amdgcn_make_buffer_rsrc((void*)topi, 0, T * k * 4, 0x00020000);
-  if (threadIdx.x < nt) {  // moe_route_kernel's math
+  const auto rs_topw = __builtin_amdgcn_make_buffer_rsrc((void*)topw, 0, T * k * 4, 0x00020000);
+  if (SIG && threadIdx.x < nt) {
+    const int t = threadIdx.x;
+    float v = INFINITY;
+    int e = -1;
+    for (int j = 0; j < k; ++j) {
+      next_best(lg[t], E, v, e);
+      const uint32_t at = (uint32_t)(((t0 + t) * k + j) * 4);
+      __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(sigmoid_of(v)), rs_topw, at, 0, 16 /* sc1 */);
+      __builtin_amdgcn_raw_buffer_store_b32(e, rs_topi, at, 0, 16 /* sc1 */);
+    }
+    if (sig.gate) sig.gate[t0 + t] = sigmoid_of(lg[t][E]);
+  } else if (threadIdx.x < nt) {  // moe_route_kernel's math
     const int t = threadIdx.x;
     float mx = -INFINITY;
     for (int e = 0; e < E; ++e) mx = fmaxf(mx, lg[t][e]);
@@ -498,6 +606,13 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
       const int s = s0 + j * (int)blockDim.x + (int)threadIdx.x;
       rk[j] = s < n_slots ? inv[s] : -1;
     }
+    float wt[kSortChunk];
+    if constexpr (SIG) {
+#pragma unroll
+      for (int j = 0; j < kSortChunk; ++j)
+        wt[j] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(
+            rs_topw, (uint32_t)((s0 + j * (int)blockDim.x + (int)threadIdx.x) * 4), 0, 16 /* sc1 */));
+    }
 #pragma unroll
     for (int j = 0; j < kSortChunk; ++j) {
       const int s = s0 + j * (int)blockDim.x + (int)threadIdx.x, e = ev[j];
@@ -505,6 +620,7 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
         const int row = base[e] + rk[j];
         inv[s] = row;
         arow[row] = s / k;
+        if constexpr (SIG) sig.row_w[row] = wt[j];
       }
     }
   }
@@ -538,6 +654,120 @@ void launch_moe_dispatch_mid(float* topw, int* topi, int* offsets, int* arow, in
   }
 #undef MLOP_DISP
 #undef MLOP_DISP_T
+}
+
+void launch_moe_dispatch_mid_sigmoid(float* topw, int* topi, int* offsets, int* arow, float* row_w, int* inv, float* gate,
+                                     const void* x, const void* wr, int T, int E, int rows, int k, int H, hipStream_t st) {
+  float* ws = nullptr;
+  int* ticket = nullptr;
+  int cus = 0;
+  if (!gemm_sk_scratch(&ws, &ticket, &cus)) throw std::runtime_error("moe_dispatch_mid: stream-K scratch not reserved");
+  const SigArgs sig{gate, row_w, rows};
+  const int tok = T >= 2048 ? 8 : T >= 512 ? 4 : 2, grid = (T + tok - 1) / tok;
+#define MLOP_DISP_T(CH, TOK)                                                                                           \
+  moe_dispatch_mid_kernel<CH, TOK, true><<<grid, 64 * kDispWaves, 0, st>>>(topw, topi, offsets, arow, inv,               \
+                                                                           (const uint16_t*)x, (const uint16_t*)wr, T, E, \
+                                                                           k, H, 0, E, MoePro{}, ticket, sig)
+#define MLOP_DISP(CH)                       \
+  if (tok == 8) MLOP_DISP_T(CH, 8);         \
+  else if (tok == 4) MLOP_DISP_T(CH, 4);    \
+  else MLOP_DISP_T(CH, 2);
+  switch (H) {
+    case 1024: MLOP_DISP(2); break;
+    case 2048: MLOP_DISP(4); break;
+    case 4096: MLOP_DISP(8); break;
+    case 8192: MLOP_DISP(16); break;
+    default: MLOP_DISP(0); break;
+  }
+#undef MLOP_DISP
+#undef MLOP_DISP_T
+}
+
+// fp32 forms of the sigmoid routing: one thread per token over its logits, the counting sort, a gather that
+// weights the rows, and the experts' products on fp32 FMAs
+__global__ void __launch_bounds__(128) moe_route_sigmoid_kernel(float* __restrict__ topw, int* __restrict__ topi,
+                                                               float* __restrict__ gate, const float* __restrict__ logits,
+                                                               int T, int E, int rows, int k) {
+  const int t = blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= T) return;
+  const float* l = logits + (size_t)t * rows;
+  float v = INFINITY;
+  int e = -1;
+  for (int j = 0; j < k; ++j) {
+    next_best(l, E, v, e);
+    topi[t * k + j] = e;
+    topw[t * k + j] = 1.f / (1.f + expf(-v));
+  }
+  if (gate) gate[t] = 1.f / (1.f + expf(-l[E]));
+}
+
+void launch_moe_route_sigmoid(float* topw, int* topi, float* gate, const float* logits, int T, int E, int rows, int k,
+                              hipStream_t st) {
+  if (T == 0) return;
+  moe_route_sigmoid_kernel<<<(T + 127) / 128, 128, 0, st>>>(topw, topi, gate, logits, T, E, rows, k);
+}
+
+__global__ void __launch_bounds__(256) moe_gather_scaled_kernel(float* __restrict__ xp, const float* __restrict__ x,
+                                                               const int* __restrict__ src, const float* __restrict__ topw,
+                                                               const int* __restrict__ offsets, int n_local, int k, int H) {
+  const int r = blockIdx.x;
+  if (r >= offsets[n_local]) return;
+  const int s = src[r];
+  const float w = topw[s];
+  for (int c = threadIdx.x; c < H; c += blockDim.x) xp[(size_t)r * H + c] = w * x[(size_t)(s / k) * H + c];
+}
+
+void launch_moe_permute_scaled(float* xp, int* offsets, int* src, int* inv, const float* x, const int* topi,
+                               const float* topw, int T, int k, int H, int E, hipStream_t st) {
+  moe_sort_kernel<<<1, 1024, 0, st>>>(offsets, src, inv, topi, T * k, 0, E);
+  if (T * k > 0) moe_gather_scaled_kernel<<<T * k, 256, 0, st>>>(xp, x, src, topw, offsets, E, k, H);
+}
+
+// a 32 x 64 tile of one expert's rows (blockIdx.y: the tile among all experts'), 8 outputs per thread
+__global__ void __launch_bounds__(256) grouped_plain_kernel(float* __restrict__ out, const float* __restrict__ a,
+                                                           const float* __restrict__ w, const int* __restrict__ offsets,
+                                                           int G, int N, int K) {
+  __shared__ float sa[32][33], sb[64][33];
+  int t = blockIdx.y, e = 0;
+  for (; e < G; ++e) {
+    const int tiles = (offsets[e + 1] - offsets[e] + 31) / 32;
+    if (t < tiles) break;
+    t -= tiles;
+  }
+  if (e >= G) return;
+  const int m0 = offsets[e] + 32 * t, m_end = offsets[e + 1], n0 = blockIdx.x * 64, tid = threadIdx.x;
+  const int tm = tid >> 5, tn = tid & 31;  // rows tm + 8 i, columns tn + 32 j
+  const float* we = w + (size_t)e * N * K;
+  float acc[4][2] = {};
+  for (int k0 = 0; k0 < K; k0 += 32) {
+    __syncthreads();
+    for (int i = tid; i < 32 * 32; i += 256) {
+      const int r = i >> 5, c = i & 31;
+      sa[r][c] = m0 + r < m_end && k0 + c < K ? a[(size_t)(m0 + r) * K + k0 + c] : 0.f;
+    }
+    for (int i = tid; i < 64 * 32; i += 256) {
+      const int r = i >> 5, c = i & 31;
+      sb[r][c] = n0 + r < N && k0 + c < K ? we[(size_t)(n0 + r) * K + k0 + c] : 0.f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int c = 0; c < 32; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = fmaf(sa[tm + 8 * i][c], sb[tn + 32 * j][c], acc[i][j]);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+      if (m0 + tm + 8 * i < m_end && n0 + tn + 32 * j < N) out[(size_t)(m0 + tm + 8 * i) * N + n0 + tn + 32 * j] = acc[i][j];
+}
+
+void launch_grouped_plain(float* out, const float* a, const float* w, const int* offsets, int G, int R, int N, int K,
+                          hipStream_t st) {
+  if (R == 0) return;
+  grouped_plain_kernel<<<dim3(cdiv(N, 64), cdiv(R, 32) + G), 256, 0, st>>>(out, a, w, offsets, G, N, K);
 }
 
 // combine fused with the decoder's residual add + RMSNorm (one workgroup per token row, 8

@@ -1,7 +1,8 @@
 // The fp32 residual stream of a decoder with a norm before and behind every sublayer, and two
 // elementwise steps such decoders use:
 //
-//   residual    x <- x + post_w * y / rms(y)   (or x + y),   xn = norm_w * x / rms(x)
+//   residual    x <- x + post_w * y / rms(y)   (or x + y),   xn = norm_w * x / rms(x)   (or x)
+//               where y may be a token's expert rows summed, beside a gated shared row
 //   gated norm  group norm of y with a gate before or behind it
 //   clamp_glu   clamped gated unit of a feed-forward's [gate | up] columns
 //
@@ -14,10 +15,14 @@
 
 namespace mlop {
 
-template <typename E, int VEC, int NI, bool START>
+enum { kStart = 0, kStep = 1, kExperts = 2 };  // residual_kernel: where y comes from
+
+template <typename E, int VEC, int NI, int KIND>
 __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
   __shared__ float scratch[16];
+  constexpr bool START = KIND == kStart;
   const int row = blockIdx.x, W = a.W, tid = threadIdx.x, BT = blockDim.x;
+  const float post1 = a.post_one ? *a.post_w : 1.f, norm1 = a.norm_one ? *a.norm_w : 1.f;
   float* xr = a.x + (size_t)row * W;
   float x[NI][VEC], y[NI][VEC], pw[NI][VEC], nw[NI][VEC];
   const E* yr;
@@ -26,15 +31,18 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
     yr = reinterpret_cast<const E*>(a.table) + (size_t)min(max(a.ids[row], 0l), a.vocab - 1) * W;
     if (a.pos_table) pr = reinterpret_cast<const E*>(a.pos_table) + (size_t)min((long)max(a.pos[row], 0), a.n_pos - 1) * W;
   } else {
-    yr = reinterpret_cast<const E*>(a.y) + (size_t)row * W;
+    yr = reinterpret_cast<const E*>(a.y) + (a.y ? (size_t)row * W : 0);
   }
+  const bool post_v = a.post_w && !a.post_one, norm_v = a.norm_w && !a.norm_one;
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int c = (tid + BT * i) * VEC;
     if (c < W) {
-      ldn<VEC>(yr + c, y[i]);
-      ldn<VEC>(a.norm_w + c, nw[i]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) pw[i][e] = post1, nw[i][e] = norm1, y[i][e] = 0.f;
+      if (KIND != kExperts || a.y) ldn<VEC>(yr + c, y[i]);
+      if (norm_v) ldn<VEC>(a.norm_w + c, nw[i]);
       if constexpr (START) {
         float p[VEC];
 #pragma unroll
@@ -44,7 +52,31 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
         for (int e = 0; e < VEC; ++e) x[i][e] = fmaf(a.embed_scale, y[i][e], p[e]);
       } else {
         ldn<VEC>(xr + c, x[i]);
-        if (a.post_w) ldn<VEC>(a.post_w + c, pw[i]);
+        if (post_v) ldn<VEC>(a.post_w + c, pw[i]);
+      }
+    }
+  }
+  if constexpr (KIND == kExperts) {
+    if (a.gate) {
+      const float g = a.gate[row];
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) y[i][e] *= g;
+    }
+    const int* inv = a.inv + (size_t)row * a.top;
+#pragma unroll 2
+    for (int j = 0; j < a.top; ++j) {
+      const E* er = reinterpret_cast<const E*>(a.rows) + (size_t)inv[j] * W;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int c = (tid + BT * i) * VEC;
+        if (c < W) {
+          float v[VEC];
+          ldn<VEC>(er + c, v);
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) y[i][e] += v[e];
+        }
       }
     }
   }
@@ -57,7 +89,7 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
 #pragma unroll
           for (int e = 0; e < VEC; ++e) ss = fmaf(y[i][e], y[i][e], ss);
         }
-      inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + a.eps);
+      inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)a.n + a.eps);
     }
 #pragma unroll
     for (int i = 0; i < NI; ++i)
@@ -74,7 +106,7 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
       for (int e = 0; e < VEC; ++e) ss = fmaf(x[i][e], x[i][e], ss);
     }
   }
-  const float inv = 1.f / sqrtf(block_sum(ss, scratch) / (float)W + a.eps);
+  const float inv = a.norm_w ? 1.f / sqrtf(block_sum(ss, scratch) / (float)a.n + a.eps) : 1.f;
   E* xn = reinterpret_cast<E*>(a.xn) + (size_t)row * W;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
@@ -89,8 +121,9 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
 
 template <typename E, int VEC, int NI>
 static void residual_ni(const ResidualArgs& a, int block, hipStream_t st) {
-  if (a.ids) residual_kernel<E, VEC, NI, true><<<a.T, block, 0, st>>>(a);
-  else residual_kernel<E, VEC, NI, false><<<a.T, block, 0, st>>>(a);
+  if (a.ids) residual_kernel<E, VEC, NI, kStart><<<a.T, block, 0, st>>>(a);
+  else if (a.rows) residual_kernel<E, VEC, NI, kExperts><<<a.T, block, 0, st>>>(a);
+  else residual_kernel<E, VEC, NI, kStep><<<a.T, block, 0, st>>>(a);
 }
 
 template <typename E, int VEC>
@@ -233,7 +266,7 @@ __global__ void __launch_bounds__(256) clamp_glu_kernel(E* __restrict__ out, con
     ldn<4>(row, g);
     ldn<4>(row + 16, u);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) g[e] = clamp_glu_f(g[e], u[e], alpha, limit);
+    for (int e = 0; e < 4; ++e) g[e] = alpha > 0.f ? clamp_glu_f(g[e], u[e], alpha, limit) : g[e] / (1.f + expf(-g[e])) * u[e];
     stn<4>(out + t * I + c, g);
   }
 }

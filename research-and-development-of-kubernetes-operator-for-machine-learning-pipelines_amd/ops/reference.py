@@ -128,6 +128,11 @@ def relu2(x):
     return torch.relu(x.float()).square().to(x.dtype)
 
 
+def xielu(x, a, b):
+    z = x.float()
+    return (torch.where(z > 0, a * z * z, b * (torch.expm1(z.clamp(max=0)) - z)) + 0.5 * z).to(x.dtype)
+
+
 def softcap(x, cap):
     return cap * torch.tanh(x.float() / cap)
 
@@ -208,16 +213,28 @@ def gla(proj, H, D, V, a2, a2_b, norm_w, tau, eps, state, meta):
     return o.to(proj.dtype)
 
 
-def residual_begin(ids, table, scale, pos_table, positions, norm_w, eps):
+def _unit_n(x, eps, width):
+    """x over the root mean square of its first ``width`` columns (the rest are zero)."""
+    return x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) / (width or x.shape[-1]) + eps)
+
+
+def residual_begin(ids, table, scale, pos_table, positions, norm_w, eps, width=None):
     x = table[ids.reshape(-1).long()].float() * scale
     if pos_table is not None:
         x = x + pos_table[positions.long()].float()
-    return x, (_unit(x, eps) * norm_w).to(table.dtype)
+    return x, (x if norm_w is None else _unit_n(x, eps, width) * norm_w).to(table.dtype)
 
 
-def residual_step(x, y, post_w, norm_w, eps):
-    x.add_(_unit(y.float(), eps) * post_w if post_w is not None else y.float())
-    return (_unit(x, eps) * norm_w).to(y.dtype)
+def residual_step(x, y, post_w, norm_w, eps, width=None, experts=None):
+    dtype = y.dtype if experts is None else experts[0].dtype
+    out = y.float() if y is not None else torch.zeros_like(x)
+    if experts is not None:
+        rows, inv, gate = experts
+        if gate is not None:
+            out = out * gate[:, None]
+        out = out + rows.float()[inv.long()].sum(1)
+    x.add_(_unit_n(out, eps, width) * post_w if post_w is not None else out)
+    return (x if norm_w is None else _unit_n(x, eps, width) * norm_w).to(dtype)
 
 
 def gated_norm(y, gate, w, groups, eps, silu, gate_first):
@@ -290,16 +307,32 @@ def delta(proj, w2, w0, a_b, decay_scale, unit_eps, state, meta):
     return o.reshape(T, hv).to(proj.dtype)
 
 
-def latent_store(latents, w, eps, slots, cache):
+def latent_query(x, w, eps, size):
+    return torch.nn.functional.pad(_unit(x.float(), eps) * w, (0, size - x.shape[1])).to(x.dtype)
+
+
+def latent_store(latents, w, eps, slots, cache, rope=None, query=None):
     c = (_unit(latents.float(), eps) * w).to(cache.dtype)
     keep = slots >= 0
-    cache.view(-1, cache.shape[-1])[slots[keep].long(), :c.shape[1]] = c[keep]
+    rows = cache.view(-1, cache.shape[-1])
+    rows[slots[keep].long(), :c.shape[1]] = c[keep]
+    if rope is not None:
+        k, table, positions, off = rope
+        cs, half = table[positions.long()], table.shape[1] // 2
+        k = rotate_pairs(k.float()[:, None], cs[:, :half], cs[:, half:])[:, 0].to(cache.dtype)
+        rows[slots[keep].long(), off:off + k.shape[1]] = k[keep]
+    return latent_query(*query[:2], eps, query[2]) if query is not None else None
 
 
-def latent_attention(q, gate, cache, w_kv, H, V, scale, window, sink, meta):
+def latent_attention(q, gate, cache, w_kv, H, V, scale, window, sink, meta, rope=None):
     """q [T, H, KP]; w_kv [H (KP + VP), RP]: a head's keys, then values, of a latent row."""
     T, KP = q.shape[0], q.shape[2]
     VP = w_kv.shape[0] // H - KP
+    if rope is not None:
+        table, n, off, _ = rope
+        cs = table[meta.positions.long()]
+        turned = rotate_pairs(q[:, :, off:off + n].float(), cs[:, :n // 2], cs[:, n // 2:]).to(q.dtype)
+        q = torch.cat([q[:, :, :off], turned, q[:, :, off + n:]], 2)
     out = torch.zeros(T, H, V, dtype=torch.float32, device=q.device)
     for row, s, n, ctx in _live_rows(meta):
         c, _ = gather_kv(cache, cache, meta.block_tables[row], ctx)
@@ -329,6 +362,14 @@ def moe_route(logits, top_k):
     w, idx = torch.topk(p, top_k, dim=-1)
     w = w / w.sum(-1, keepdim=True)
     return w, idx.to(torch.int32)
+
+
+def moe_route_sigmoid(logits, E, top_k):
+    """fp32 logits [T, E] or, with a gate behind them, [T, E + 1] -> (scores of the top_k largest, experts,
+    sigmoid of the gate or None)."""
+    s = torch.sigmoid(logits.float())
+    w, idx = torch.topk(s[:, :E], top_k, dim=-1)
+    return w, idx.to(torch.int32), s[:, E].contiguous() if s.shape[1] > E else None
 
 
 def moe_permute(x, topi, e0, n_local):
