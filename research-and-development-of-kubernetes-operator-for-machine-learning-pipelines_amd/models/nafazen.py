@@ -30,6 +30,7 @@ from .config import LatentAttentionSpec, NafazenConfig
 from .layers import ParamSource, fuse_rows, linear, pad_rows, rotary_table
 
 CHUNK = 64  # granule of the step's list of prompt portions
+MAX_EXPERTS, MAX_TOP = 256, 64  # of the routing kernels
 
 
 def _up8(n: int) -> int:
@@ -67,6 +68,8 @@ class NafazenModel:
             self.layers.append(L)
             subs.append((self._attention, i, number(p + "norm1")))
             if la.moe:
+                if la.moe.experts > MAX_EXPERTS or la.moe.top > MAX_TOP:
+                    raise ValueError(f"layer {i}: at most {MAX_EXPERTS} experts, {MAX_TOP} of them per token")
                 L.update(self._init_experts(src, p + "mlp.", la.moe))
                 subs.append((self._experts, i, number(p + "norm2")))
             elif la.ff:

@@ -206,7 +206,7 @@ void launch_moe_dispatch_mid(float* topw, int* topi, int* offsets, int* arow, in
                              int T, int E, int k, int H, int e0, int n_local, const void* pro_y, void* pro_res,
                              const void* pro_w, float pro_eps, void* pro_xn, hipStream_t st);
 // sigmoid routing with the scores on the experts' inputs (moe.hip); router rows: E experts', then a gate's or none
-constexpr int kSigMaxE = 256, kSigMaxTop = 32;
+constexpr int kSigMaxE = 256, kSigMaxTop = 64;
 void launch_moe_dispatch_small_sigmoid(float* topw, int* topi, void* xp, int* offsets, int* src, int* inv, float* gate,
                                        const void* x, const void* wr, int T, int E, int rows, int k, int H,
                                        hipStream_t st);

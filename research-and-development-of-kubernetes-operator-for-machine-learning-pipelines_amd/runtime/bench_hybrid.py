@@ -1,8 +1,9 @@
 """Prefill and decode throughput of the hybrid designs beside the closest models of the package, at
 equal layer sizes (``bench.py --hybrid``).
 
-Each size has a Regesun and a Kosesun preset cut to a few layers and a Llama, all of the same width,
-layer count, vocabulary and feed-forward parameters.  Both run through the engine's own scheduler
+Each size has a Nafazen, a Regesun and a Kosesun preset cut to a few layers, a Mixtral with the Nafazen's
+experts and a Llama, all of the same width, layer count and vocabulary, the dense ones of the same
+feed-forward parameters.  All run through the engine's own scheduler
 (``add_request`` / ``step``; decode replays the captured graphs), random weights, random prompts,
 greedy sampling.  One JSON line per (model, workload); ``--hybrid-kernels`` adds each kernel's share
 of a profiled run.
@@ -17,7 +18,7 @@ from dataclasses import replace
 import torch
 
 from ..models import build_model
-from ..models.config import LLAMA3_8B, get_config
+from ..models.config import LLAMA3_8B, MIXTRAL_8X7B, get_config
 from .engine import Engine, EngineConfig
 from .sampler import SamplingParams
 
@@ -33,8 +34,17 @@ def sizes() -> list:
     l1 = replace(LLAMA3_8B, name="llama-1b", num_layers=LAYERS, hidden_size=2048, intermediate_size=5376, num_heads=16,
                  num_kv_heads=4)
     r8, r1 = get_config("regesun-8b", num_layers=LAYERS), get_config("regesun-1b", num_layers=LAYERS)
-    return [("8b", *(replace(c, max_position=16384) for c in (r8, k8, l8))),
-            ("1b", *(replace(c, max_position=16384) for c in (r1, k1, l1)))]
+    n8, n1 = get_config("nafazen-8b", num_layers=LAYERS), get_config("nafazen-1b", num_layers=LAYERS)
+
+    def mixtral(name, like, of):  # the experts of ``like`` in every layer, attention and vocabulary of ``of``
+        e = like.layers[1].moe
+        return replace(MIXTRAL_8X7B, name=name, num_layers=LAYERS, hidden_size=of.hidden_size, vocab_size=of.vocab_size,
+                       num_heads=of.num_heads, num_kv_heads=of.num_kv_heads, intermediate_size=e.ff, num_experts=e.experts,
+                       top_k=e.top)
+
+    m8, m1 = mixtral("mixtral-8b", n8, l8), mixtral("mixtral-1b", n1, l1)
+    return [("8b", *(replace(c, max_position=16384) for c in (n8, r8, k8, m8, l8))),
+            ("1b", *(replace(c, max_position=16384) for c in (n1, r1, k1, m1, l1)))]
 
 
 def _kernels(fn) -> list:
