@@ -233,7 +233,7 @@ def config_from_nafazen(d: dict, shape_of, name: str | None = None) -> ModelConf
             raise ValueError(f"layer {i}: unsupported attention settings {m}")
         layers.append(LayerSpec(mixer, **(_nafazen_mlp(la["mlp"], f"layer {i} mlp") if la.get("mlp") is not None else {})))
     return nafazen_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers, float(d["embedding"]["scale"]),
-                          float(d["logit_softcap"]), float(d["norm"]["eps"]))
+                          float(d.get("logit_softcap") or 0.0), float(d["norm"]["eps"]))
 
 
 # config.json's "architecture" -> its reader

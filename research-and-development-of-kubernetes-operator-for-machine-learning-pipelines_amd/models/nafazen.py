@@ -196,8 +196,9 @@ class NafazenModel:
         return x
 
     def logits_local(self, hidden: torch.Tensor) -> torch.Tensor:
-        """[n, padded width] -> soft-capped logits [n, vocab] in fp32."""
-        return ops.softcap(linear(hidden, self.head), self.cfg.logit_softcap)[:, :self.cfg.vocab_size]
+        """[n, padded width] -> logits [n, vocab], soft-capped in fp32 (no cap: as the product leaves them)."""
+        lg = linear(hidden, self.head)
+        return (ops.softcap(lg, self.cfg.logit_softcap) if self.cfg.logit_softcap else lg)[:, :self.cfg.vocab_size]
 
     logits = logits_local
 

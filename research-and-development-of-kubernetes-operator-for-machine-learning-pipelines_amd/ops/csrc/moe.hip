@@ -176,6 +176,7 @@ __device__ __forceinline__ void next_best(const float* z, int n, float& v, int& 
 __device__ __forceinline__ void dot_rows2(const uint16_t* w, const uint16_t* x0, const uint16_t* x1, int H, int lane,
                                           float& s0, float& s1) {
   s0 = s1 = 0.f;
+#pragma unroll 4
   for (int c = lane * 8; c < H; c += 512) {
     const u32x4 b = *reinterpret_cast<const u32x4*>(w + c), p = *reinterpret_cast<const u32x4*>(x0 + c),
                 q = *reinterpret_cast<const u32x4*>(x1 + c);
@@ -471,7 +472,19 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
     x = pro.xn;
   }
   // router logits of this workgroup's tokens
-  for (int e = wv; e < (SIG ? sig.rows : E); e += kDispWaves) {
+  // SIG: the rows past a whole round of the waves (a gate behind 8 experts, say) are dealt to them by token pairs
+  const int n_rounds = SIG ? sig.rows / kDispWaves * kDispWaves : E;
+  if constexpr (SIG) {
+    const int pairs = (nt + 1) >> 1;
+    for (int u = wv; u < (sig.rows - n_rounds) * pairs; u += kDispWaves) {
+      const int e = n_rounds + u / pairs, tp = u % pairs * 2;
+      float s0, s1;
+      dot_rows2(wr + (size_t)e * H, x + (size_t)(t0 + tp) * H, x + (size_t)(t0 + min(tp + 1, nt - 1)) * H, H, lane, s0, s1);
+      if (lane == 0) lg[tp][e] = s0;
+      if (lane == 0 && tp + 1 < nt) lg[tp + 1][e] = s1;
+    }
+  }
+  for (int e = wv; e < n_rounds; e += kDispWaves) {
     if constexpr (CH == 0) {
       for (int tp = 0; tp < nt; tp += 2) {
         float s0, s1;
