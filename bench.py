@@ -126,7 +126,7 @@ def parse(argv=None):
     ap.add_argument("--phase-child", choices=("tp", "ep"), default=None, help=argparse.SUPPRESS)
     ap.add_argument("--hybrid", action="store_true",
                     help="instead of the headline: prefill / decode throughput of the hybrid designs beside a "
-                         "Llama of equal layer sizes, one JSON line each (mlopamd/runtime/bench_hybrid.py)")
+                         "Mixtral and a Llama of equal layer sizes, one JSON line each (mlopamd/runtime/bench_hybrid.py)")
     ap.add_argument("--hybrid-kernels", action="store_true", help="with --hybrid: each workload's kernel times")
     ap.add_argument("--hybrid-only", default="", help="with --hybrid: models whose size and name contain this")
     ap.add_argument("--cr-ready-samples", type=int, default=3,
