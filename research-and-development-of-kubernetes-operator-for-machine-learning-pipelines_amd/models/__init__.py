@@ -1,10 +1,10 @@
-"""Model zoo: Llama-3 (8B / 70B), Mixtral-8x7B (MoE), Kosesun, Regesun and Nafazen (hybrids), random-init bf16.
+"""Model zoo: Llama-3 (8B / 70B), Mixtral-8x7B (MoE), Kosesun, Regesun, Nafazen and Dibedra (hybrids), random-init bf16.
 
 The configs import without torch (the operator image's placement planner reads them);
 ``build_model`` pulls in torch and the model code on first use."""
 from __future__ import annotations
 
-from .config import HybridConfig, KosesunConfig, ModelConfig, NafazenConfig, RegesunConfig, get_config, PRESETS  # noqa: F401
+from .config import DibedraConfig, HybridConfig, KosesunConfig, ModelConfig, NafazenConfig, RegesunConfig, get_config, PRESETS  # noqa: F401
 
 
 def build_model(name_or_cfg, device="cuda", dtype=None, pstate=None, seed: int = 0, weights=None):
@@ -21,6 +21,10 @@ def build_model(name_or_cfg, device="cuda", dtype=None, pstate=None, seed: int =
         from .nafazen import NafazenModel
 
         return NafazenModel(cfg, device=device, dtype=dtype, pstate=pstate, seed=seed, weights=weights)
+    if isinstance(cfg, DibedraConfig):
+        from .dibedra import DibedraModel
+
+        return DibedraModel(cfg, device=device, dtype=dtype, pstate=pstate, seed=seed, weights=weights)
     if isinstance(cfg, KosesunConfig):
         from .kosesun import KosesunModel
 

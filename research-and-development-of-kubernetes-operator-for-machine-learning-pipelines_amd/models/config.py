@@ -79,6 +79,25 @@ class ModelConfig:
 
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """Stretched rotary frequencies: pairs that turn less than ``slow`` times in ``original`` positions turn
+    ``factor`` times slower, pairs that turn more than ``fast`` times as before, a ramp between them; cos
+    and sin times 0.1 ln(factor) + 1."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class RotarySpec:
+    """Rotary positions of ``dims`` dimensions in pairs (2i, 2i + 1)."""
+    base: float
+    dims: int
+    scaling: YarnSpec | None = None
+
+
+@dataclass(frozen=True)
 class AttentionSpec:
     """Softmax-attention mixer of a hybrid decoder layer."""
     heads: int
@@ -89,13 +108,25 @@ class AttentionSpec:
     rot_base: float
     rot_dims: int            # leading dims of a head that rotate (pairs 2i, 2i + 1)
     v_mix: bool = False      # values mixed with the first v_mix layer's
+    scaling: YarnSpec | None = None
+    window: int = 0          # a token sees itself and the window - 1 tokens before it (0: all)
+    head_norm: bool = False  # query / key norm per head, one weight for all heads (else over the whole rows)
+    tied_kv: bool = False    # the values are the projected keys (before norm and rotation)
+    sink: bool = True        # a number per head joins the softmax's denominator
+    gate_elem: bool = False  # output gate per value element (else per head)
+
+    @property
+    def rot(self) -> RotarySpec:
+        return RotarySpec(self.rot_base, self.rot_dims, self.scaling)
 
     def params(self, width: int) -> int:
-        qk, v = (self.heads + self.kv_heads) * self.dim, self.kv_heads * self.vdim
-        return width * (qk + v + self.heads + self.heads * self.vdim) + qk + self.heads + int(self.v_mix)
+        norms = 2 * self.dim if self.head_norm else (self.heads + self.kv_heads) * self.dim
+        return self.macs(width) + norms + self.heads * self.sink + int(self.v_mix)
 
     def macs(self, width: int) -> int:
-        return width * ((self.heads + self.kv_heads) * self.dim + (self.kv_heads + self.heads) * self.vdim + self.heads)
+        qk, v = (self.heads + self.kv_heads) * self.dim, 0 if self.tied_kv else self.kv_heads * self.vdim
+        gates = self.heads * (self.vdim if self.gate_elem else 1)
+        return width * (qk + v + gates + self.heads * self.vdim)
 
 
 @dataclass(frozen=True)
@@ -117,25 +148,6 @@ class GLASpec:
 
     def state_elems(self) -> int:
         return self.heads * self.dim * self.vdim
-
-
-@dataclass(frozen=True)
-class YarnSpec:
-    """Stretched rotary frequencies: pairs that turn less than ``slow`` times in ``original`` positions turn
-    ``factor`` times slower, pairs that turn more than ``fast`` times as before, a ramp between them; cos
-    and sin times 0.1 ln(factor) + 1."""
-    factor: float
-    original: float
-    fast: float
-    slow: float
-
-
-@dataclass(frozen=True)
-class RotarySpec:
-    """Rotary positions of ``dims`` dimensions in pairs (2i, 2i + 1)."""
-    base: float
-    dims: int
-    scaling: YarnSpec | None = None
 
 
 @dataclass(frozen=True)
@@ -226,18 +238,37 @@ class DeltaSpec:
 
 @dataclass(frozen=True)
 class MoESpec:
-    """Mixture of gated experts, each token through the ``top`` with the largest sigmoid scores, its input
-    times the score; beside them a shared expert (``shared`` 0: none) with a sigmoid gate per token."""
+    """Mixture of gated experts.
+
+    ``scores`` "sigmoid": each token goes through the ``top`` experts with the largest sigmoid scores, its input
+    times the score; beside them a shared expert (``shared`` 0: none) with a sigmoid gate per token.
+    "softmax": scores over all experts, the weights on the experts' outputs as they are.  The last ``identity``
+    of the scored outputs give the token itself back.  A number per output (``correction``) joins the score where
+    experts are chosen, and only there; the outputs form ``groups`` equal groups of neighbours, and the choice is
+    from the ``keep`` groups with the largest best one."""
     experts: int
     top: int
     ff: int
     shared: int = 0
+    scores: str = "sigmoid"
+    identity: int = 0
+    groups: int = 1
+    keep: int = 1
+    correction: bool = False
+    limit: float = 0.0       # clamped gated unit with this bound (0: silu(gate) up)
+
+    @property
+    def outputs(self) -> int:
+        """Router outputs that are experts."""
+        return self.experts + self.identity
 
     def params(self, width: int) -> int:
-        return width * (self.experts * (3 * self.ff + 1) + 3 * self.shared + bool(self.shared))
+        return (width * (self.outputs + 3 * self.experts * self.ff + 3 * self.shared + bool(self.shared)) +
+                self.outputs * self.correction)
 
     def macs(self, width: int) -> int:
-        return width * (self.experts + 3 * self.top * self.ff + 3 * self.shared + bool(self.shared))
+        used = 3 * self.top * self.ff * self.experts // self.outputs
+        return width * (self.outputs + used + 3 * self.shared + bool(self.shared))
 
 
 @dataclass(frozen=True)
@@ -246,6 +277,7 @@ class LayerSpec:
     ff: int = 0              # feed-forward width (0: none)
     limit: float = 0.0       # clamp of a gated feed-forward (designs that have one)
     moe: MoESpec | None = None  # experts instead of the feed-forward
+    weights_of: int = -1     # layer whose weights this one uses (-1: its own); its cache is its own
 
 
 @dataclass(frozen=True)
@@ -353,6 +385,38 @@ class NafazenConfig(HybridConfig):
                                               for la in self.layers))
 
 
+@dataclass(frozen=True)
+class DibedraConfig(HybridConfig):
+    """Dibedra: windowed attention whose values are its keys, beside the feed-forward (dense or experts in groups,
+    some of them the identity) on one normed input; dynamic-tanh norms; layers may use another's weights."""
+    logit_scale: float = 1.0
+
+    def __post_init__(self):
+        super().__post_init__()
+        for i, la in enumerate(self.layers):
+            j = la.weights_of
+            if j >= 0 and (j >= len(self.layers) or self.layers[j].weights_of >= 0 or replace(self.layers[j], weights_of=j) != la):
+                raise ValueError(f"layer {i}: layer {j} has no weights of its own for it")
+
+    def _count(self, layer) -> int:
+        # embedding, head, last norm
+        return (2 * self.vocab_size + 2) * self.hidden_size + 1 + sum(layer(la) for la in self.layers)
+
+    def num_params(self) -> int:
+        W = self.hidden_size
+        return self._count(lambda la: 0 if la.weights_of >= 0 else la.mixer.params(W) + 2 * W + 1 +
+                           (la.moe.params(W) if la.moe else 2 * W * la.ff))
+
+    def active_params(self) -> int:
+        W = self.hidden_size
+        return self._count(lambda la: la.mixer.params(W) + 2 * W + 1 + (la.moe.macs(W) if la.moe else 2 * W * la.ff))
+
+    def flops_per_token(self) -> int:
+        W = self.hidden_size
+        return 2 * (self.vocab_size * W + sum(la.mixer.macs(W) + (la.moe.macs(W) if la.moe else 2 * W * la.ff)
+                                              for la in self.layers))
+
+
 def _hybrid(cls, name: str, vocab: int, width: int, layers, eps: float, **kw):
     """``cls`` over listed layers, the uniform fields from the largest attention layer."""
     layers = tuple(layers)
@@ -379,6 +443,10 @@ def regesun_config(name: str, vocab: int, width: int, layers, max_position: int,
 def nafazen_config(name: str, vocab: int, width: int, layers, embed_scale: float, logit_softcap: float, eps: float = 1e-5,
                    **kw) -> NafazenConfig:
     return _hybrid(NafazenConfig, name, vocab, width, layers, eps, embed_scale=embed_scale, logit_softcap=logit_softcap, **kw)
+
+
+def dibedra_config(name: str, vocab: int, width: int, layers, logit_scale: float = 1.0, eps: float = 1e-5, **kw) -> DibedraConfig:
+    return _hybrid(DibedraConfig, name, vocab, width, layers, eps, logit_scale=logit_scale, **kw)
 
 
 LLAMA3_8B = ModelConfig(
@@ -479,10 +547,34 @@ NAFAZEN_1B = _nafazen("nafazen-1b", width=2048, ff=8192, n_layers=16, vocab=1282
 TINY_NAFAZEN = _nafazen("tiny-nafazen", width=192, ff=200, n_layers=4, vocab=512, heads=5, dim=24, rot_dim=16, vdim=40,
                         rank=72, q_rank=56, moe=MoESpec(experts=6, top=2, ff=40, shared=72), max_position=2048)
 
+
+def _dibedra(name: str, width: int, ff: int, n_layers: int, vocab: int, heads: int, kv_heads: int, dim: int, window: int,
+             moe: MoESpec, **kw) -> DibedraConfig:
+    """Four layers in turn: a dense feed-forward, experts, the same dense layer, and the experts' once more."""
+    att = AttentionSpec(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5, rot_base=500000.0, rot_dims=dim,
+                        scaling=YarnSpec(factor=4.0, original=4096, fast=32.0, slow=1.0), window=window, head_norm=True,
+                        tied_kv=True, sink=False, gate_elem=True)
+    turn = lambda i: LayerSpec(att, *(() if i % 2 else (ff,)), moe=moe if i % 2 else None,  # noqa: E731
+                               weights_of=i - 2 if i % 4 > 1 else -1)
+    return dibedra_config(name, vocab, width, [turn(i) for i in range(n_layers)], logit_scale=0.5, **kw)
+
+
+# head sizes of the Llama's, feed-forwards of the Kosesun presets' and experts of the Nafazen presets' sizes (two of
+# them per token where the scores are even)
+DIBEDRA_8B = _dibedra("dibedra-8b", width=4096, ff=21504, n_layers=32, vocab=128256, heads=32, kv_heads=8, dim=128, window=4096,
+                      moe=MoESpec(experts=8, top=3, ff=1792, scores="softmax", identity=4, groups=3, keep=2, correction=True,
+                                  limit=7.0))
+DIBEDRA_1B = _dibedra("dibedra-1b", width=2048, ff=8192, n_layers=16, vocab=128256, heads=16, kv_heads=4, dim=128, window=1024,
+                      moe=MoESpec(experts=16, top=3, ff=768, scores="softmax", identity=8, groups=6, keep=3, correction=True,
+                                  limit=7.0))
+TINY_DIBEDRA = _dibedra("tiny-dibedra", width=192, ff=200, n_layers=5, vocab=512, heads=6, kv_heads=2, dim=24, window=40,
+                        moe=MoESpec(experts=5, top=2, ff=40, scores="softmax", identity=1, groups=3, keep=2, correction=True,
+                                    limit=2.0), max_position=2048)
+
 PRESETS = {c.name: c for c in (LLAMA3_8B, LLAMA3_70B, LLAMA31_8B, LLAMA31_70B, MIXTRAL_8X7B, TINY_LLAMA,
                                 TINY_MIXTRAL, TINY_LLAMA_8H, TINY_MIXTRAL_8E, KOSESUN_8B, KOSESUN_1B,
                                 TINY_KOSESUN, REGESUN_8B, REGESUN_1B, TINY_REGESUN, NAFAZEN_8B, NAFAZEN_1B,
-                                TINY_NAFAZEN)}
+                                TINY_NAFAZEN, DIBEDRA_8B, DIBEDRA_1B, TINY_DIBEDRA)}
 # accepted aliases (MLflow tags / CR annotations use HF-ish names)
 ALIASES = {
     "meta-llama/Meta-Llama-3-8B": "llama3-8b", "llama-3-8b": "llama3-8b", "Llama-3-8B": "llama3-8b",

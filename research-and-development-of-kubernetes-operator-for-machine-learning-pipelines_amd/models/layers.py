@@ -58,6 +58,11 @@ def rotary_table(rot, max_pos: int, device=None) -> torch.Tensor:
     return (torch.cat([f.cos(), f.sin()], dim=-1) * mult).float().to(device)
 
 
+def pad_to(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
+    """[n, K] with zero rows and columns up to [rows, cols]."""
+    return F.pad(w, (0, cols - w.shape[1], 0, rows - w.shape[0])).contiguous()
+
+
 def pad_rows(w: torch.Tensor, heads: int, rows: int) -> torch.Tensor:
     """[heads * d, K] -> [heads * rows, K], every head's rows padded with zeros."""
     v = w.view(heads, -1, w.shape[1])

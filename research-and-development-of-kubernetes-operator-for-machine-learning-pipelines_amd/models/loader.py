@@ -18,8 +18,8 @@ Layout mapping (HF name -> ours; TP sharding then reuses ``load_shard_from``):
   Mixtral: block_sparse_moe.gate | mlp.gate      -> router
            experts.{e}.w1 / w3 (legacy) or experts.gate_up_proj (fused) -> w13 (interleaved)
            experts.{e}.w2 or experts.down_proj   -> w2
-Kosesun, Regesun and Nafazen checkpoints (``"architecture"`` in config.json; tensors ``l<i>.mix.*`` ...) are
-read by the model itself as it is built (models/kosesun.py, models/regesun.py, models/nafazen.py).
+Kosesun, Regesun, Nafazen and Dibedra checkpoints (``"architecture"`` in config.json; tensors ``l<i>.mix.*`` ...)
+are read by the model itself as it is built (models/kosesun.py, regesun.py, nafazen.py, dibedra.py).
 Tensors are read lazily, one layer at a time (safetensors memory map), so a 141 GB
 checkpoint never sits in host memory at once.
 """
@@ -33,7 +33,7 @@ from pathlib import Path
 import torch
 
 from .config import (AttentionSpec, DeltaSpec, GLASpec, LatentAttentionSpec, LayerSpec, ModelConfig, MoESpec, PRESETS,
-                     RotarySpec, SSDSpec, YarnSpec, kosesun_config, nafazen_config, regesun_config)
+                     RotarySpec, SSDSpec, YarnSpec, dibedra_config, kosesun_config, nafazen_config, regesun_config)
 
 _ARCH_NAMES = {"LlamaForCausalLM": "llama", "MixtralForCausalLM": "mixtral", "MistralForCausalLM": "llama"}
 
@@ -236,8 +236,63 @@ def config_from_nafazen(d: dict, shape_of, name: str | None = None) -> ModelConf
                           float(d.get("logit_softcap") or 0.0), float(d["norm"]["eps"]))
 
 
+def _dibedra_mlp(mlp: dict, where: str) -> dict:
+    """Feed-forward fields of a LayerSpec."""
+    if mlp.get("kind", "dense") == "dense":
+        _only(mlp, {"ff", "kind"}, where)
+        return {"ff": int(mlp["ff"])}
+    if mlp["kind"] != "moe":
+        raise ValueError(f"{where}: unsupported feed-forward {mlp['kind']!r}")
+    _only(mlp, {"expert", "kind", "router"}, where)
+    ex, ro = mlp["expert"], mlp["router"]
+    groups = ro.get("groups") or {"count": 1, "keep": 1}
+    _only(ex, {"ff", "limit"}, where + " expert"), _only(ro, {"experts", "groups", "identity", "top"}, where + " router")
+    _only(groups, {"count", "keep"}, where + " groups")
+    moe = MoESpec(experts=int(ro["experts"]), top=int(ro["top"]), ff=int(ex["ff"]), scores="softmax",
+                  identity=int(ro.get("identity") or 0), groups=int(groups["count"]), keep=int(groups["keep"]), correction=True,
+                  limit=float(ex["limit"]))
+    if (min(moe.experts, moe.top, moe.ff, moe.groups) < 1 or moe.identity < 0 or moe.outputs % moe.groups or
+            not 1 <= moe.keep <= moe.groups or moe.top > moe.outputs // moe.groups * moe.keep or moe.limit <= 0):
+        raise ValueError(f"{where}: unsupported expert settings {mlp}")
+    return {"moe": moe}
+
+
+def config_from_dibedra(d: dict, shape_of, name: str | None = None) -> ModelConfig:
+    """DibedraConfig from a Dibedra ``config.json`` dict.  Settings this runtime does not know are rejected,
+    never dropped."""
+    _only(d, {"architecture", "layers", "logit_scale", "norm", "vocab", "width"}, "config")
+    _only(d["norm"], {"eps"}, "norm")
+    layers = []
+    for i, la in enumerate(d["layers"]):
+        _only(la, {"type", "mixer", "mlp", "weights_of"}, f"layer {i}")
+        if la["type"] != "attention":
+            raise ValueError(f"layer {i}: unknown mixer type {la['type']!r}")
+        m = la["mixer"]
+        _only(m, {"dim", "heads", "kv_heads", "mask", "rot", "scale", "vdim"}, f"layer {i} mixer")
+        mask = m.get("mask") or {"size": 0}
+        _only(mask, {"size"}, f"layer {i} mask")
+        rot = _rotary(m["rot"], f"layer {i} rotation")
+        mixer = AttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                              scale=float(m["scale"]), rot_base=rot.base, rot_dims=rot.dims, scaling=rot.scaling,
+                              window=int(mask["size"]), head_norm=True, tied_kv=True, sink=False, gate_elem=True)
+        if (mixer.scale <= 0 or mixer.window < 0 or mixer.vdim != mixer.dim or mixer.heads % mixer.kv_heads or
+                rot.dims > mixer.dim):
+            raise ValueError(f"layer {i}: unsupported attention settings {m}")
+        j = la.get("weights_of")
+        j = -1 if j is None else int(j)
+        for _ in d["layers"]:  # the layer that holds the tensors
+            if 0 <= j < len(d["layers"]) and d["layers"][j].get("weights_of") is not None:
+                j = int(d["layers"][j]["weights_of"])
+        layers.append(LayerSpec(mixer, **(_dibedra_mlp(la["mlp"], f"layer {i} mlp") if la.get("mlp") is not None else {}),
+                                weights_of=j))
+    scale = d.get("logit_scale")
+    return dibedra_config(name or d["architecture"], int(d["vocab"]), int(d["width"]), layers,
+                          1.0 if scale is None else float(scale), float(d["norm"]["eps"]))
+
+
 # config.json's "architecture" -> its reader
-_HYBRIDS = {"Kosesun": config_from_kosesun, "Regesun": config_from_regesun, "Nafazen": config_from_nafazen}
+_HYBRIDS = {"Kosesun": config_from_kosesun, "Regesun": config_from_regesun, "Nafazen": config_from_nafazen,
+            "Dibedra": config_from_dibedra}
 
 
 class _Tensors:
@@ -328,7 +383,7 @@ class HFWeights:
 def load_pretrained(path: str | os.PathLike, device="cuda", dtype=torch.bfloat16, pstate=None,
                     name: str | None = None, fold_norms: bool = True):
     """Build our model for the checkpoint in ``path`` and copy its (TP-sharded) weights in.  The
-    model class follows from config.json: ``architecture`` (Kosesun, Regesun, Nafazen) or HF's ``architectures``."""
+    model class follows from config.json: ``architecture`` (Kosesun, Regesun, Nafazen, Dibedra) or HF's ``architectures``."""
     from . import build_model
 
     path = Path(path)

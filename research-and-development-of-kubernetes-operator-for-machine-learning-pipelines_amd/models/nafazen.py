@@ -27,7 +27,7 @@ from .. import ops
 from ..parallel.comm import ParallelState, single
 from ..runtime.kv_cache import KVLayer, pad_dim
 from .config import LatentAttentionSpec, NafazenConfig
-from .layers import ParamSource, fuse_rows, linear, pad_rows, rotary_table
+from .layers import ParamSource, fuse_rows, linear, pad_rows, pad_to, rotary_table
 
 CHUNK = 64  # granule of the step's list of prompt portions
 MAX_EXPERTS, MAX_TOP = 256, 64  # of the routing kernels
@@ -35,10 +35,6 @@ MAX_EXPERTS, MAX_TOP = 256, 64  # of the routing kernels
 
 def _up8(n: int) -> int:
     return -(-n // 8) * 8
-
-
-def _pad_to(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
-    return F.pad(w, (0, cols - w.shape[1], 0, rows - w.shape[0])).contiguous()
 
 
 class NafazenModel:
@@ -54,7 +50,7 @@ class NafazenModel:
         self.width = pad_dim(W)  # of every row as stored
         src = ParamSource(weights, self.device, dtype, seed * 1000)
         number = lambda name: src(name, dtype=torch.float32, mean=1.0, std=0.0).reshape(1)  # noqa: E731
-        self.embed = _pad_to(src("embed", cfg.vocab_size, W), cfg.vocab_size, self.width)
+        self.embed = pad_to(src("embed", cfg.vocab_size, W), cfg.vocab_size, self.width)
         self.layers, self.cache_layout, self.state_shapes = [], [], []
         self._tables, self._table_len = {}, 0
         # decode work units per token: groups of 16 heads; partials hold latents
@@ -76,7 +72,7 @@ class NafazenModel:
                 L.update(self._init_dense(src, p + "mlp.", la.ff))
                 subs.append((self._dense, i, number(p + "norm2")))
         self.final_norm = number("final.norm")
-        self.head = fuse_rows([_pad_to(src("head", cfg.vocab_size, W), cfg.vocab_size, self.width)])
+        self.head = fuse_rows([pad_to(src("head", cfg.vocab_size, W), cfg.vocab_size, self.width)])
         # decode graphs only where every product is a kernel of this package: a library product may
         # record memory-set nodes, which have replayed wrongly
         ws = [self.head] + [v for L in self.layers for k, v in L.items() if k in ("down_q", "uq", "o", "up", "down", "s_gate_up",
@@ -97,12 +93,12 @@ class NafazenModel:
         VH = _up8(m.vdim)
         while H * VH % 64:
             VH += 8
-        down = [_pad_to(src(p + "dq", m.q_rank, W), QP, Wp)]
+        down = [pad_to(src(p + "dq", m.q_rank, W), QP, Wp)]
         L = {"q_norm": src(p + "dq.norm", m.q_rank, dtype=torch.float32, mean=1.0, std=0.0), "QP": QP, "KP": KP, "VH": VH,
              "q_off": q_off, "k_off": k_off}
         if m.kv_from < 0:
             dkv = src(p + "dkv", R + rot, W)
-            down += [_pad_to(dkv[:R], k_off, Wp), _pad_to(dkv[R:], rot, Wp)]
+            down += [pad_to(dkv[:R], k_off, Wp), pad_to(dkv[R:], rot, Wp)]
             L["c_norm"] = src(p + "dkv.norm", R, dtype=torch.float32, mean=1.0, std=0.0)
             L["cache"] = len(self.cache_layout)
             self.cache_layout.append(KVLayer(1, RP, 0))
@@ -115,11 +111,11 @@ class NafazenModel:
         same = torch.zeros(H, KP, RP, device=self.device, dtype=self.dtype)
         same[:, :m.dim, :R] = uk.view(H, m.dim, R)
         same[:, q_off:q_off + rot, k_off:k_off + rot] = torch.eye(rot, device=self.device, dtype=self.dtype)
-        L.update(down_q=fuse_rows(down), uq=_pad_to(uq.reshape(H * KP, m.q_rank), H * KP, QP),
-                 w_kv=torch.cat([same.view(H * KP, RP), _pad_to(pad_rows(uv, H, pad_dim(VH)), H * pad_dim(VH), RP)]).contiguous(),
+        L.update(down_q=fuse_rows(down), uq=pad_to(uq.reshape(H * KP, m.q_rank), H * KP, QP),
+                 w_kv=torch.cat([same.view(H * KP, RP), pad_to(pad_rows(uv, H, pad_dim(VH)), H * pad_dim(VH), RP)]).contiguous(),
                  w_qk=F.pad(uk.view(H, m.dim, R).transpose(1, 2), (0, KD - m.dim, 0, k_off - R)).contiguous(),
                  w_vo=F.pad(uv.view(H, m.vdim, R), (0, pad_dim(R) - R, 0, VH - m.vdim)).contiguous(),
-                 o=_pad_to(F.pad(src(p + "o", W, H * m.vdim).view(W, H, m.vdim), (0, VH - m.vdim)).reshape(W, H * VH), Wp, H * VH))
+                 o=pad_to(F.pad(src(p + "o", W, H * m.vdim).view(W, H, m.vdim), (0, VH - m.vdim)).reshape(W, H * VH), Wp, H * VH))
         self._tables.setdefault(m.rot, None)
         self.n_kv, self.part_dim = max(self.n_kv, -(-H // 16)), max(self.part_dim, RP)
         return L
@@ -127,13 +123,13 @@ class NafazenModel:
     def _init_dense(self, src, p, ff):
         W, Wp, fp = self.cfg.hidden_size, self.width, pad_dim(ff)
         a, b = F.softplus(src(p + "act", 2, dtype=torch.float32, std=0.5).double()).tolist()
-        return {"up": _pad_to(src(p + "up", ff, W), fp, Wp), "down": _pad_to(src(p + "down", W, ff), Wp, fp), "act": (a, b + 0.5)}
+        return {"up": pad_to(src(p + "up", ff, W), fp, Wp), "down": pad_to(src(p + "down", W, ff), Wp, fp), "act": (a, b + 0.5)}
 
     def _gated(self, src, p, ff):
         """(gate and up rows interleaved, down) of a gated feed-forward, in whole tiles."""
         W, Wp, fp = self.cfg.hidden_size, self.width, pad_dim(ff)
-        gate, up = (_pad_to(src(p + n, ff, W), fp, Wp) for n in ("gate", "up"))
-        return ops.interleave_gate_up(gate, up).contiguous(), _pad_to(src(p + "down", W, ff), Wp, fp)
+        gate, up = (pad_to(src(p + n, ff, W), fp, Wp) for n in ("gate", "up"))
+        return ops.interleave_gate_up(gate, up).contiguous(), pad_to(src(p + "down", W, ff), Wp, fp)
 
     def _init_experts(self, src, p, m):
         W, Wp, fp = self.cfg.hidden_size, self.width, pad_dim(m.ff)
@@ -145,7 +141,7 @@ class NafazenModel:
         if m.shared:
             L["s_gate_up"], L["s_down"] = self._gated(src, p + "shared.", m.shared)
             router.append(src(p + "shared.sg", 1, W))  # rides behind the router's rows
-        L["router"] = _pad_to(torch.cat(router), sum(r.shape[0] for r in router), Wp)
+        L["router"] = pad_to(torch.cat(router), sum(r.shape[0] for r in router), Wp)
         return L
 
     def reserve_positions(self, n: int) -> None:

@@ -180,16 +180,18 @@ def paged_attention(q, k_cache, v_cache, meta, out: torch.Tensor | None = None):
     return out
 
 
-EPI_NONE, EPI_SILU_MUL, EPI_RELU2, EPI_XIELU = 0, 1, 6, 7
+EPI_NONE, EPI_SILU_MUL, EPI_RELU2, EPI_XIELU, EPI_GELU = 0, 1, 6, 7, 8
 
 
 def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi: int = EPI_NONE,
-         glu: tuple | None = None, xielu: tuple | None = None):
+         glu: tuple | None = None, xielu: tuple | None = None, act_from: int = 0):
     """y = epi(x @ w^T), w [N, K] bf16.  EPI_SILU_MUL expects gate/up rows
     interleaved in groups of 16 (``interleave_gate_up``) and returns N/2 columns; with ``glu`` =
     (alpha, limit) it is the clamped gated unit g sigmoid(alpha g) (u + 1) of g = min(gate, limit),
     u = clamp(up, -limit, limit) instead.  EPI_RELU2 is max(y, 0)^2; EPI_XIELU with ``xielu`` = (a, b) is
-    y / 2 + a y^2 for y > 0 and y / 2 + b (exp(y) - 1 - y) otherwise."""
+    y / 2 + a y^2 for y > 0 and y / 2 + b (exp(y) - 1 - y) otherwise; EPI_GELU is the tanh gelu.
+    ``act_from`` (a multiple of 128): EPI_RELU2 / EPI_XIELU / EPI_GELU from that column on, the columns before it
+    as they are."""
     N = w.shape[0]
     glu = xielu or glu  # (two numbers either way)
     out_n = N // 2 if epi == EPI_SILU_MUL else N
@@ -199,10 +201,9 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
         if epi == EPI_SILU_MUL:
             y = deinterleave_cols(y)
             y = ref.silu_mul(y) if glu is None else ref.clamp_glu(y, *glu)
-        elif epi == EPI_RELU2:
-            y = ref.relu2(y)
-        elif epi == EPI_XIELU:
-            y = ref.xielu(y, *glu)
+        elif epi != EPI_NONE:
+            act = {EPI_RELU2: ref.relu2, EPI_XIELU: ref.xielu, EPI_GELU: ref.gelu_tanh}[epi]
+            y = torch.cat([y[..., :act_from], act(y[..., act_from:], *(glu or ()))], -1)
         if out is not None:
             out.copy_(y.view_as(out))
             return out
@@ -215,32 +216,27 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor | None = None, epi:
     M, K = x2.shape
     o2 = torch.empty(M, out_n, dtype=x.dtype, device=x.device) if out is None else out.view(M, out_n)
     if x.dtype == torch.float32:  # true fp32 (library product; no reduced-precision mode)
-        _gemm_hipblaslt(x2, w, o2, epi, glu)
+        _gemm_hipblaslt(x2, w, o2, epi, glu, act_from)
         return o2.view(*lead, out_n) if out is None else out
-    _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi, glu)
+    _GEMM_IMPL[_gemm_backend(M, N, K, epi, x2, w, o2)](x2, w, o2, epi, glu, act_from)
     return o2.view(*lead, out_n) if out is None else out
 
 
-def _gemm_mlop(x2, w, o2, epi, glu=None):
+def _gemm_mlop(x2, w, o2, epi, glu=None, act_from=0):
     _sk_reserve(x2.device)
     M, K = x2.shape
     nws = torch.ops.mlop.gemm_workspace(M, w.shape[0], K, epi)
     ws = torch.empty(max(nws, 1), dtype=torch.float32, device=x2.device) if nws else _EMPTY.get(x2.device)
-    if glu is None:
-        torch.ops.mlop.gemm(o2, x2, w, ws, epi)
-    else:
-        torch.ops.mlop.gemm(o2, x2, w, ws, epi, *glu)
+    torch.ops.mlop.gemm(o2, x2, w, ws, epi, *(glu or (0.0, 0.0)), act_from)
 
 
-def _gemm_hipblaslt(x2, w, o2, epi, glu=None):
+def _gemm_hipblaslt(x2, w, o2, epi, glu=None, act_from=0):
     """Plain library GEMM (hipBLASLt via torch.matmul); the SiLU-mul epilogue (or the clamped gated
-    unit) then runs as a separate kernel on the interleaved columns."""
+    unit) then runs as a separate kernel on the interleaved columns, an activation in place."""
     if epi != EPI_SILU_MUL:
         torch.matmul(x2, w.t(), out=o2)
-        if epi == EPI_RELU2:
-            torch.ops.mlop.relu2(o2)
-        elif epi == EPI_XIELU:
-            torch.ops.mlop.xielu(o2, *glu)
+        if epi != EPI_NONE:
+            torch.ops.mlop.act_columns(o2, act_from, epi, *(glu or (0.0, 0.0)))
     elif glu is not None or x2.dtype == torch.float32:
         torch.ops.mlop.clamp_glu(o2, torch.matmul(x2, w.t()), *(glu or (0.0, 0.0)))
     else:
@@ -778,6 +774,15 @@ def xielu(x, a: float, b: float):
     return x
 
 
+def gelu_tanh(x):
+    """x / 2 (1 + tanh(sqrt(2 / pi) (x + 0.044715 x^3))), in place."""
+    if not x.is_cuda:
+        return x.copy_(ref.gelu_tanh(x))
+    _need_gpu()
+    torch.ops.mlop.act_columns(x, 0, EPI_GELU, 0.0, 0.0)
+    return x
+
+
 def softcap(x, cap: float):
     """cap * tanh(x / cap), fp32."""
     if not x.is_cuda:
@@ -803,17 +808,38 @@ def qk_norm_rope(proj, n_heads: int, dim: int, vdim: int, q_w, k_w, eps: float, 
     return q
 
 
-def attention_hd(q, k_cache, v_cache, meta, dim: int, vdim: int, scale: float, sink=None, gate=None):
-    """Ragged causal paged attention of any head sizes: q [T, H, KP] -> [T, H, vdim].  ``sink`` [H] joins
-    each head's softmax denominator; ``gate`` [T, H]: the head's output times sigmoid(gate).  (Windows,
-    gates per element and dense keys: ``latent_attention``.)"""
+def qk_head_norm(q, k, v, n_heads: int, dim: int, vdim: int, q_w, k_w, eps: float, cos_sin, positions, slots, k_cache,
+                 v_cache):
+    """q [T, H dim], k [T, G dim] (row strides of their own) -> q [T, H, KP]: RMS norm of each head, weight q_w or k_w
+    [dim] for all of them, then rotation of the first cos_sin.shape[1] dims in pairs (2i, 2i + 1); k into its paged
+    cache, and v [T, G vdim] as it is into its own.  ``v`` None: the values are k as given."""
     if not q.is_cuda:
-        return ref.attention_hd(q, k_cache, v_cache, meta, dim, vdim, scale, sink, gate)
+        return ref.qk_head_norm(q, k, v, n_heads, dim, vdim, q_w, k_w, eps, cos_sin, positions, slots, k_cache, v_cache)
     _need_gpu()
-    out = torch.empty(q.shape[0], q.shape[1], vdim, dtype=q.dtype, device=q.device)
+    out = torch.empty(q.shape[0], n_heads, k_cache.shape[3], dtype=q.dtype, device=q.device)
+    torch.ops.mlop.qk_head_norm(out, k_cache, v_cache, q, k, v, dim, vdim, q_w, k_w, eps, cos_sin, positions, slots)
+    return out
+
+
+def attention_hd(q, k_cache, v_cache, meta, dim: int, vdim: int, scale: float, sink=None, gate=None, window: int = 0, out=None):
+    """Ragged causal paged attention of any head sizes: q [T, H, KP] -> [T, H, vdim] (``out``: where to, rows of any
+    stride).  ``sink`` [H] joins each head's softmax denominator; ``gate``: [T, H], the head's output times
+    sigmoid(gate), or [T, H vdim], each element's; ``window``: tokens a token sees (0: all).  (Dense keys:
+    ``latent_attention``.)"""
+    if not q.is_cuda:
+        o = ref.attention_hd(q, k_cache, v_cache, meta, dim, vdim, scale, sink, gate, window)
+        return o if out is None else out.copy_(o)
+    _need_gpu()
+    out = torch.empty(q.shape[0], q.shape[1], vdim, dtype=q.dtype, device=q.device) if out is None else out
+    part, nparts = meta.part_tokens, meta.nparts
+    if window and nparts > 1:
+        from ..runtime.attn_meta import plan_partitions
+
+        G = k_cache.shape[1]
+        part, nparts = plan_partitions(meta.tile_seq.numel(), G * -(-(q.shape[1] // G) // 16), min(part * nparts, window + 31))
     torch.ops.mlop.attention_hd(out, meta.part_o, meta.part_ml, meta.part_sem, q, k_cache, v_cache, meta.block_tables,
                                 meta.tile_seq, meta.tile_q0, meta.ptile_seq, meta.ptile_q0, meta.q_start, meta.q_len,
-                                meta.ctx_len, dim, scale, sink, gate, meta.part_tokens, meta.nparts)
+                                meta.ctx_len, dim, scale, sink, gate, part, nparts, window)
     return out
 
 
@@ -830,30 +856,34 @@ def gla(proj, n_heads: int, dim: int, vdim: int, a2, a2_b, norm_w, tau: float, e
     return out
 
 
-def residual_begin(ids, table, scale: float, pos_table, positions, norm_w, eps: float, width: int | None = None):
+def residual_begin(ids, table, scale: float, pos_table, positions, norm_w, eps: float, width: int | None = None, tanh=None):
     """fp32 residual x = scale table[id] + pos_table[position] (``pos_table`` None: none) and the first
     sublayer's input norm_w x / rms(x) in the table's dtype (``norm_w`` [W] or one number; None: x itself).
-    ``width``: columns the mean square is over, where zeros pad the rows."""
+    ``width``: columns the mean square is over, where zeros pad the rows.  ``tanh`` = (alpha, b): the input is
+    norm_w tanh(alpha x) + b instead (one number, and [W])."""
     if not table.is_cuda:
-        return ref.residual_begin(ids, table, scale, pos_table, positions, norm_w, eps, width)
+        return ref.residual_begin(ids, table, scale, pos_table, positions, norm_w, eps, width, tanh)
     _need_gpu()
     x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=table.device)
     xn = torch.empty(x.shape, dtype=table.dtype, device=table.device)
-    torch.ops.mlop.residual_begin(xn, x, ids, table, scale, pos_table, positions, norm_w, eps, width or 0)
+    torch.ops.mlop.residual_begin(xn, x, ids, table, scale, pos_table, positions, norm_w, eps, width or 0, *(tanh or (None, None)))
     return x, xn
 
 
-def residual_step(x, y, post_w, norm_w, eps: float, store: bool = True, width: int | None = None, experts=None):
+def residual_step(x, y, post_w, norm_w, eps: float, store: bool = True, width: int | None = None, experts=None, share=None,
+                  tanh=None):
     """x <- x + post_w y / rms(y) (``post_w`` [W] or one number; None: x + y), in place unless ``store`` is off
     (nothing reads it again); returns the next sublayer's input norm_w x / rms(x) (None: x itself).
     ``experts`` = (rows [R, W], inv [T, k], gate [T] or None): gate[t] y[t] + sum_j rows[inv[t, j]] stands in
-    y's place (y None: the sum alone).  ``width`` as in residual_begin."""
+    y's place (y None: the sum alone; inv < 0: no row).  ``share`` = (w [T, k], h [T, W] or None, u [T] or None): rows
+    times w[t, j], and u[t] h[t] joins the sum.  ``width`` and ``tanh`` as in residual_begin."""
     if not x.is_cuda:
-        return ref.residual_step(x, y, post_w, norm_w, eps, width, experts)
+        return ref.residual_step(x, y, post_w, norm_w, eps, width, experts, share, tanh)
     _need_gpu()
     rows, inv, gate = experts or (None, None, None)
     xn = torch.empty(x.shape, dtype=(rows if y is None else y).dtype, device=x.device)
-    torch.ops.mlop.residual_step(xn, x, y, post_w, norm_w, eps, store, width or 0, rows, inv, gate)
+    torch.ops.mlop.residual_step(xn, x, y, post_w, norm_w, eps, store, width or 0, rows, inv, gate, *(share or (None, None, None)),
+                                 *(tanh or (None, None)))
     return xn
 
 
@@ -1000,6 +1030,8 @@ class Dispatched:
     gate: torch.Tensor | None   # sigmoid of the row behind the router's experts, per token
     a_rows: torch.Tensor | None = None
     row_w: torch.Tensor | None = None
+    top_w: torch.Tensor | None = None   # [T, k] weights of a token's rows (moe_dispatch_groups)
+    self_w: torch.Tensor | None = None  # [T] weight of the token itself
 
 
 def moe_dispatch_input(x, router, n_experts: int, top_k: int) -> Dispatched:
@@ -1028,6 +1060,37 @@ def moe_dispatch_input(x, router, n_experts: int, top_k: int) -> Dispatched:
     a_rows, row_w = i32(T * top_k), torch.empty(T * top_k, dtype=torch.float32, device=dev)
     torch.ops.mlop.moe_dispatch_mid_sigmoid(topw, topi, offsets, a_rows, row_w, inv, gate, x, router, n_experts)
     return Dispatched(x, offsets, inv, gate, a_rows, row_w)
+
+
+def moe_dispatch_groups(x, router, correction, n_experts: int, top_k: int, groups: int = 1, keep: int = 1) -> Dispatched:
+    """Mixture of experts with softmax scores (fp32, over all router rows) as weights of the experts' outputs, not
+    renormalized.  Choice scores are scores + ``correction`` [rows] (None: none): the rows form ``groups`` equal groups
+    of neighbours, and a token's ``top_k`` are the largest in the ``keep`` groups with the largest best one.  ``router``
+    [E + I, W]: rows past the E experts are identity experts; a token's inv is -1 there, their weights add up in
+    ``self_w``."""
+    T, dev, n = x.shape[0], x.device, router.shape[0]
+    if not x.is_cuda:
+        topw, topi, self_w = ref.moe_route_groups(x.float() @ router.float().t(), correction, n_experts, top_k, groups, keep)
+        xp, offsets, _, inv = ref.moe_permute(x, topi, 0, n_experts)
+        return Dispatched(xp, offsets, inv.view(T, top_k), None, top_w=topw, self_w=self_w)
+    _need_gpu()
+    _sk_reserve(dev)  # the launch's ticket counter lives in the stream-K scratch
+    i32 = lambda *n: torch.empty(*n, dtype=torch.int32, device=dev)  # noqa: E731
+    topi, offsets, inv = i32(T, top_k), i32(n_experts + 1), i32(T, top_k)
+    topw = torch.empty(T, top_k, dtype=torch.float32, device=dev)
+    self_w = torch.empty(T, dtype=torch.float32, device=dev) if n > n_experts else None
+    choice = (correction, n_experts, groups, keep)
+    if x.dtype == torch.float32 or T <= 16:  # rows gathered
+        xp, src = torch.empty(T * top_k, x.shape[1], dtype=x.dtype, device=dev), i32(T * top_k)
+        if x.dtype == torch.float32:
+            torch.ops.mlop.moe_route_groups(topw, topi, self_w, gemm(x, router), *choice)
+            torch.ops.mlop.moe_permute_scaled(xp, offsets, src, inv, x, topi, None, n_experts)
+        else:
+            torch.ops.mlop.moe_dispatch_small_groups(topw, topi, xp, offsets, src, inv, self_w, x, router, *choice)
+        return Dispatched(xp, offsets, inv, None, top_w=topw, self_w=self_w)
+    a_rows = i32(T * top_k)
+    torch.ops.mlop.moe_dispatch_mid_groups(topw, topi, offsets, a_rows, inv, self_w, x, router, *choice)
+    return Dispatched(x, offsets, inv, None, a_rows, top_w=topw, self_w=self_w)
 
 
 def moe_permute(x, topi, e0: int, n_local: int):
@@ -1138,17 +1201,19 @@ def moe_combine(y, inv, topw):
     return out
 
 
-def grouped_gemm(xp, w, offsets, epi: int = EPI_NONE, avg_rows: int | None = None, a_rows=None, row_scale=None):
+def grouped_gemm(xp, w, offsets, epi: int = EPI_NONE, avg_rows: int | None = None, a_rows=None, row_scale=None, glu=None):
     """Per group e: rows offsets[e]:offsets[e+1] of xp times w[e]^T in ONE launch
     (tiles enumerate (group, m-tile) pairs on device: no host sync, graph-safe).  ``a_rows``
     [R]: permuted row r is row a_rows[r] of xp (R output rows; moe_dispatch_mid); ``row_scale`` [R], with
-    ``a_rows``: times that."""
+    ``a_rows``: times that.  ``glu`` = (alpha, limit): EPI_SILU_MUL is the clamped gated unit (see gemm)."""
     if a_rows is not None and not xp.is_cuda:
         xp = xp[a_rows.long()]
         a_rows = None
     if not xp.is_cuda:
         y = ref.grouped_gemm(xp, w, offsets)
-        return ref.silu_mul(deinterleave_cols(y)) if epi == EPI_SILU_MUL else y
+        if epi != EPI_SILU_MUL:
+            return y
+        return ref.silu_mul(deinterleave_cols(y)) if glu is None else ref.clamp_glu(deinterleave_cols(y), *glu)
     _need_gpu()
     N = w.shape[1]
     R = xp.shape[0] if a_rows is None else a_rows.numel()
@@ -1161,7 +1226,7 @@ def grouped_gemm(xp, w, offsets, epi: int = EPI_NONE, avg_rows: int | None = Non
         wide = out if epi == EPI_NONE else torch.empty(R, N, dtype=xp.dtype, device=xp.device)
         torch.ops.mlop.grouped_plain(wide, xp, w, offsets)
         if epi == EPI_SILU_MUL:
-            torch.ops.mlop.clamp_glu(out, wide, 0.0, 0.0)
+            torch.ops.mlop.clamp_glu(out, wide, *(glu or (0.0, 0.0)))
         return out
-    torch.ops.mlop.grouped_gemm(out, xp, w, offsets, rows, epi, a_rows, row_scale)
+    torch.ops.mlop.grouped_gemm(out, xp, w, offsets, rows, epi, a_rows, row_scale, *(glu or (0.0, 0.0)))
     return out

@@ -75,6 +75,18 @@ __device__ __forceinline__ float gate_at(const AttnHdArgs& a, int tok, int head,
 template <int N>
 __device__ __forceinline__ void gate_elems(const AttnHdArgs& a, int tok, int head, int c, float (&v)[N]) {
   if (!a.gate || !a.gate_elem) return;
+  if (a.gate_vec) {  // V a multiple of 4
+    const uint16_t* g = reinterpret_cast<const uint16_t*>(a.gate) + (size_t)tok * a.gate_stride + head * a.V + c;
+#pragma unroll
+    for (int j = 0; j < N; j += 4) {
+      if (c + j >= a.V) continue;
+      float z[4];
+      ldn<4>(g + j, z);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[j + i] *= __builtin_amdgcn_rcpf(1.f + __expf(-z[i]));
+    }
+    return;
+  }
 #pragma unroll
   for (int j = 0; j < N; ++j)
     if (c + j < a.V) v[j] *= gate_at(a, tok, head, c + j);
@@ -129,7 +141,7 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
     // no partition of an empty row (graph padding) draws the last ticket: partition 0 zeroes it
     if (part == 0 && kv_end <= 0 && live) {
       for (int e = threadIdx.x; e < nh * a.V; e += 256)
-        out[((size_t)orow * a.H + head0 + e / a.V) * a.V + e % a.V] = 0;
+        out[(size_t)orow * a.out_row + (head0 + e / a.V) * a.V + e % a.V] = 0;
     }
     return;
   }
@@ -271,7 +283,7 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
 #pragma unroll
       for (int j = 0; j < 8; ++j) acc[j] *= inv;
       gate_elems(a, tok, head0 + rr, c, acc);
-      store8(out + ((size_t)orow * a.H + head0 + rr) * a.V, c, a.V, acc);
+      store8(out + (size_t)orow * a.out_row + (head0 + rr) * a.V, c, a.V, acc);
     } else {
       // partial (O, m, l) of this key range, stored through to the memory side (sc1) so that the
       // ticket below needs no release fence
@@ -333,7 +345,7 @@ __global__ void __launch_bounds__(256) paged_hd_kernel(AttnHdArgs a, float* __re
 #pragma unroll
     for (int j = 0; j < 8; ++j) acc[j] *= inv;
     gate_elems(a, tok, head0 + rr, c, acc);
-    store8(out + ((size_t)orow * a.H + head0 + rr) * a.V, c, a.V, acc);
+    store8(out + (size_t)orow * a.out_row + (head0 + rr) * a.V, c, a.V, acc);
   }
 }
 
@@ -565,7 +577,7 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 5 ? 2 : 1) flash_hd_kernel
   }
   const float inv = l > 0.f ? f * gate_of(a, qs + qi, head) / l : 0.f;
   // O^T element e of dim block d is dim 32 d + 8 (e >> 2) + 4 h + (e & 3) of this lane's row
-  uint16_t* orow = reinterpret_cast<uint16_t*>(a.out) + ((size_t)(qs + qi) * a.H + head) * a.V;
+  uint16_t* orow = reinterpret_cast<uint16_t*>(a.out) + (size_t)(qs + qi) * a.out_row + head * a.V;
   const bool v4 = a.V % 4 == 0;
 #pragma unroll
   for (int d = 0; d < ND; ++d)
@@ -651,7 +663,7 @@ __global__ void __launch_bounds__(256) attn_any_kernel(AttnHdArgs a, const int* 
   float inv = l > 0.f ? f / l : 0.f;
   const E* gate = reinterpret_cast<const E*>(a.gate) + (size_t)tok * a.gate_stride;
   if (a.gate && !a.gate_elem) inv /= 1.f + expf(-ld1(gate + head));
-  E* dst = reinterpret_cast<E*>(a.out) + ((size_t)orow * a.H + head) * a.V;
+  E* dst = reinterpret_cast<E*>(a.out) + (size_t)orow * a.out_row + head * a.V;
 #pragma unroll
   for (int i = 0; i < kHdMaxV / 64; ++i) {
     const int c = i * 64 + lane;

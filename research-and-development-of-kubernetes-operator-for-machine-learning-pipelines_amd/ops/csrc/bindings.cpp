@@ -264,7 +264,7 @@ int64_t gemm_workspace(int64_t M, int64_t N, int64_t K, int64_t epi) {
 }
 
 // out[M, N or N/2] = epi(a[M, K] . w[N, K]^T)
-void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi, double p0, double p1) {
+void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi, double p0, double p1, int64_t act_from) {
   TORCH_CHECK(a.is_cuda() && a.scalar_type() == at::kBFloat16 && a.dim() == 2 && a.stride(1) == 1,
               "a must be bf16 [M, K] with unit inner stride");
   check_bf16(w, "w");
@@ -274,7 +274,8 @@ void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi, double p0, dou
   TORCH_CHECK(w.dim() == 2 && w.size(1) == K, "w must be [N, K]");
   TORCH_CHECK(K % 64 == 0, "K must be a multiple of 64");
   TORCH_CHECK(N % 8 == 0 && a.stride(0) % 8 == 0 && out.stride(0) % 8 == 0, "16-B aligned rows");
-  TORCH_CHECK(epi == 0 || epi == 1 || epi == mlop::kEpiRelu2 || epi == mlop::kEpiXielu, "epi");
+  TORCH_CHECK(epi == 0 || epi == 1 || mlop::epi_act((int)epi), "epi");
+  TORCH_CHECK(act_from >= 0 && act_from % 128 == 0 && (act_from == 0 || mlop::epi_act((int)epi)), "act_from: whole 128 columns");
   TORCH_CHECK(epi != 1 || N % 32 == 0, "silu_mul epilogue needs N % 32 == 0");
   TORCH_CHECK(out.size(0) == M && out.size(1) == (epi == 1 ? N / 2 : N), "out shape");
   TORCH_CHECK(reinterpret_cast<uintptr_t>(a.data_ptr()) % 16 == 0 &&
@@ -289,7 +290,7 @@ void gemm(Tensor out, Tensor a, Tensor w, Tensor ws, int64_t epi, double p0, dou
   c10::DeviceGuard g(a.device());
   mlop::launch_gemm(a.data_ptr(), (int)a.stride(0), w.data_ptr(), (int)K, out.data_ptr(),
                     (int)out.stride(0), wsp, wsn, (int)M, (int)N, (int)K, (int)epi, cur_stream(), (float)p0,
-                    (float)p1);
+                    (float)p1, (int)act_from);
 }
 
 // QKV projection with RoPE + paged-cache stores in the GEMM epilogue; false = this M
@@ -516,7 +517,7 @@ int64_t decode_chain_max_m() { return mlop::decode_chain_max_m(); }
 
 // grouped (MoE): rows of a sorted by group, offsets [G+1]; w [G, N, K]
 void grouped_gemm(Tensor out, Tensor a, Tensor w, Tensor offsets, int64_t max_rows, int64_t epi,
-                  std::optional<Tensor> a_rows, std::optional<Tensor> row_scale) {
+                  std::optional<Tensor> a_rows, std::optional<Tensor> row_scale, double p0, double p1) {
   check_bf16(out, "out"); check_bf16(a, "a"); check_bf16(w, "w"); check_i32(offsets, "offsets");
   TORCH_CHECK(a.dim() == 2 && w.dim() == 3 && w.size(2) == a.size(1), "a [M, K], w [G, N, K]");
   // with a_rows the permuted rows are out's (M = out rows) and a holds the token rows they name
@@ -536,7 +537,7 @@ void grouped_gemm(Tensor out, Tensor a, Tensor w, Tensor offsets, int64_t max_ro
   mlop::launch_grouped_gemm(a.data_ptr(), w.data_ptr(), out.data_ptr(), offsets.data_ptr<int>(),
                             (int)G, (int)M, (int)N, (int)K, (int)max_rows, (int)epi, cur_stream(),
                             a_rows ? a_rows->data_ptr<int>() : nullptr, nullptr, nullptr,
-                            row_scale ? row_scale->data_ptr<float>() : nullptr);
+                            row_scale ? row_scale->data_ptr<float>() : nullptr, (float)p0, (float)p1);
 }
 
 void moe_route(Tensor topw, Tensor topi, Tensor logits) {
@@ -934,9 +935,9 @@ TORCH_LIBRARY(mlop, m) {
         "Tensor pos, Tensor cos_sin, Tensor slots, Tensor ss_in, float eps) -> bool");
   m.def("gemm_rope_cache(Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor a, Tensor w, "
         "Tensor pos, Tensor cos_sin, Tensor slots) -> bool");
-  m.def("gemm(Tensor(a!) out, Tensor a, Tensor w, Tensor(b!) ws, int epi, float p0=0., float p1=0.) -> ()");
+  m.def("gemm(Tensor(a!) out, Tensor a, Tensor w, Tensor(b!) ws, int epi, float p0=0., float p1=0., int act_from=0) -> ()");
   m.def("grouped_gemm(Tensor(a!) out, Tensor a, Tensor w, Tensor offsets, int max_rows, "
-        "int epi, Tensor? a_rows=None, Tensor? row_scale=None) -> ()");
+        "int epi, Tensor? a_rows=None, Tensor? row_scale=None, float p0=0., float p1=0.) -> ()");
   m.def("gemm_add_rmsnorm(Tensor(a!) out, Tensor(b!) residual, Tensor a, Tensor w, Tensor norm_w, "
         "Tensor(c!) ws, float eps) -> bool");
   m.def("gemv_chain_supported(int M, int N, int K, int epi) -> bool", &gemv_chain_supported);

@@ -5,6 +5,7 @@
 
 #include "bind_util.h"
 #include "hybrid.h"
+#include "launch.h"
 
 namespace {
 
@@ -61,20 +62,15 @@ void hyper_step(Tensor xn, Tensor streams, Tensor y, Tensor mix, Tensor w_out, T
   mlop::launch_hyper(a, f32, cur());
 }
 
-void xielu(Tensor x, double a, double b) {
+void act_columns(Tensor x, int64_t n0, int64_t epi, double a, double b) {
   const bool f32 = model_f32(x, "x");
-  TORCH_CHECK(x.is_contiguous(), "x must be contiguous");
+  TORCH_CHECK(x.is_contiguous() && x.dim() >= 1, "x must be contiguous");
+  const int64_t N = x.size(-1);
+  TORCH_CHECK(n0 >= 0 && n0 <= N && N < (1 << 30) && mlop::epi_act((int)epi), "columns, activation");
   aligned16(x, "x");
   c10::DeviceGuard g(x.device());
-  mlop::launch_xielu(x.data_ptr(), x.numel(), (float)a, (float)b, f32, cur());
-}
-
-void relu2(Tensor x) {
-  const bool f32 = model_f32(x, "x");
-  TORCH_CHECK(x.is_contiguous(), "x must be contiguous");
-  aligned16(x, "x");
-  c10::DeviceGuard g(x.device());
-  mlop::launch_relu2(x.data_ptr(), x.numel(), f32, cur());
+  mlop::launch_act_columns(x.data_ptr(), N ? x.numel() / N : 0, (int)N, (int)n0, mlop::epi_act((int)epi), (float)a, (float)b, f32,
+                           cur());
 }
 
 void softcap(Tensor out, Tensor x, double cap) {
@@ -146,6 +142,64 @@ void qk_norm_rope(Tensor q_out, Tensor k_cache, Tensor v_cache, Tensor proj, int
   mlop::launch_qk_norm(a, f32, cur());
 }
 
+void qk_head_norm(Tensor q_out, Tensor k_cache, Tensor v_cache, Tensor q, Tensor k, OptT v, int64_t D, int64_t V, Tensor q_w,
+                  Tensor k_w, double eps, Tensor cos_sin, Tensor pos, Tensor slots) {
+  mlop::QkHeadNormArgs a{};
+  const bool f32 = model_f32(q, "q");
+  like(k, q, "k");
+  like(q_out, q, "q_out");
+  like(k_cache, q, "k_cache");
+  like(v_cache, q, "v_cache");
+  TORCH_CHECK(q_out.dim() == 3 && q_out.is_contiguous() && k_cache.dim() == 4 && k_cache.is_contiguous() &&
+                  v_cache.dim() == 4 && v_cache.is_contiguous() && q.dim() == 2 && k.dim() == 2,
+              "qk_head_norm ranks");
+  a.T = (int)q_out.size(0);
+  a.H = (int)q_out.size(1);
+  a.KP = (int)q_out.size(2);
+  a.G = (int)k_cache.size(1);
+  a.BS = (int)k_cache.size(2);
+  a.VP = (int)v_cache.size(3);
+  a.D = (int)D;
+  a.V = (int)V;
+  TORCH_CHECK(k_cache.size(3) == a.KP && v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == a.G && v_cache.size(2) == a.BS,
+              "caches must be [NB, G, BS, KP] and [NB, G, BS, VP]");
+  TORCH_CHECK(D >= 1 && D <= a.KP && V >= 1 && V <= a.VP && a.KP % 8 == 0, "head sizes");
+  TORCH_CHECK(q.size(0) == a.T && q.size(1) == a.H * D && k.size(0) == a.T && k.size(1) == a.G * D, "q [T, H * D], k [T, G * D]");
+  a.q = q.data_ptr();
+  a.k = k.data_ptr();
+  a.ldq = q.stride(0);
+  a.ldk = k.stride(0);
+  if (v) {
+    like(*v, q, "v");
+    TORCH_CHECK(v->dim() == 2 && v->size(0) == a.T && v->size(1) == a.G * V, "v [T, G * V]");
+    a.v = v->data_ptr();
+    a.ldv = v->stride(0);
+  } else {
+    TORCH_CHECK(V == D, "keys as values have the keys' size");
+  }
+  aligned16(q_out, "q_out");
+  aligned16(k_cache, "k_cache");
+  aligned16(v_cache, "v_cache");
+  a.q_w = f32_of(q_w, D, "q_w");
+  a.k_w = f32_of(k_w, D, "k_w");
+  aligned16(q_w, "q_w");
+  aligned16(k_w, "k_w");
+  a.eps = (float)eps;
+  TORCH_CHECK(cos_sin.dim() == 2, "cos_sin must be [max_pos, R]");
+  a.cos_sin = f32_of(cos_sin, cos_sin.numel(), "cos_sin");
+  aligned16(cos_sin, "cos_sin");
+  a.R = (int)cos_sin.size(1);
+  TORCH_CHECK(a.R % 2 == 0 && a.R <= D, "rotated dims must be even and at most the head size");
+  a.pos = i32_of(pos, "pos");
+  a.slots = i32_of(slots, "slots");
+  TORCH_CHECK(pos.numel() == a.T && slots.numel() == a.T, "pos / slots length");
+  a.q_out = q_out.data_ptr();
+  a.k_cache = k_cache.data_ptr();
+  a.v_cache = v_cache.data_ptr();
+  c10::DeviceGuard g(q.device());
+  mlop::launch_qk_head_norm(a, f32, cur());
+}
+
 // decode tiles (one query token each) and prompt tiles (128 tokens of a head) of one step.  k, v: paged
 // caches [NB, G, 16, KP]; or, with xbase, dense rows [rows, G, KP] of prompt tiles.  by_tile: q [tiles, H,
 // KP] and out by decode tile
@@ -159,7 +213,9 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
   like(k_cache, q, "k_cache");
   like(v_cache, q, "v_cache");
   const int64_t num_tiles = tile_seq.numel(), num_ptiles = ptile_seq.numel();
-  TORCH_CHECK(q.dim() == 3 && out.dim() == 3 && out.is_contiguous(), "q, out ranks");
+  TORCH_CHECK(q.dim() == 3 && out.dim() == 3 && out.stride(1) == out.size(2), "q, out ranks");
+  a.out_row = out.stride(0);
+  TORCH_CHECK(a.out_row >= out.size(1) * out.size(2) && (a.out_row % 8 == 0 || out.is_contiguous()), "out rows");
   a.H = (int)q.size(1);
   a.KP = (int)q.size(2);
   a.V = (int)out.size(2);
@@ -219,6 +275,7 @@ void attention_hd(Tensor out, Tensor part_o, Tensor part_ml, Tensor part_sem, Te
     a.gate = gate->data_ptr();
     a.gate_stride = gate->stride(0);
     a.gate_elem = gate->size(1) != a.H;
+    a.gate_vec = a.V % 4 == 0 && a.gate_stride % 4 == 0 && reinterpret_cast<uintptr_t>(a.gate) % 8 == 0;
   }
   if (rot) {
     a.n_rot = (int)rot->size(1);
@@ -318,12 +375,13 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
         "Tensor norm_w, float eps) -> ()");
   m.def("hyper_step(Tensor(a!) xn, Tensor(b!) streams, Tensor y, Tensor mix, Tensor w_out, Tensor w_in, "
         "Tensor norm_w, float eps, bool store) -> ()");
-  m.def("relu2(Tensor(a!) x) -> ()");
-  m.def("xielu(Tensor(a!) x, float a, float b) -> ()");
+  m.def("act_columns(Tensor(a!) x, int n0, int epi, float a, float b) -> ()");
   m.def("softcap(Tensor(a!) out, Tensor x, float cap) -> ()");
   m.def("qk_norm_rope(Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor proj, int D, int V, "
         "Tensor? q_w, Tensor? k_w, float eps, Tensor cos_sin, Tensor pos, Tensor slots, Tensor? v_first, Tensor? lam) "
         "-> ()");
+  m.def("qk_head_norm(Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor q, Tensor k, Tensor? v, int D, int V, "
+        "Tensor q_w, Tensor k_w, float eps, Tensor cos_sin, Tensor pos, Tensor slots) -> ()");
   m.def("attention_hd(Tensor(a!) out, Tensor(b!) part_o, Tensor(c!) part_ml, Tensor(d!) part_sem, Tensor q, "
         "Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tile_seq, Tensor tile_q0, Tensor ptile_seq, "
         "Tensor ptile_q0, Tensor q_start, Tensor q_len, Tensor ctx_len, int D, float scale, Tensor? sink, Tensor? gate, "
@@ -337,10 +395,10 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
 TORCH_LIBRARY_IMPL(mlop, CUDA, m) {
   m.impl("hyper_begin", &hyper_begin);
   m.impl("hyper_step", &hyper_step);
-  m.impl("relu2", &relu2);
-  m.impl("xielu", &xielu);
+  m.impl("act_columns", &act_columns);
   m.impl("softcap", &softcap);
   m.impl("qk_norm_rope", &qk_norm_rope);
+  m.impl("qk_head_norm", &qk_head_norm);
   m.impl("attention_hd", &attention_hd);
   m.impl("gla", &gla);
 }

@@ -39,7 +39,8 @@ const float* vec_or_one(const Tensor& t, int64_t n, bool& one, const char* name)
   return f32_of(t, one ? 1 : n, name);
 }
 
-void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, const OptT& norm_w, double eps, int64_t width) {
+void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, const OptT& norm_w, double eps, int64_t width,
+                     const OptT& tanh_a, const OptT& tanh_b) {
   TORCH_CHECK(x.dim() == 2 && x.is_contiguous() && x.is_cuda() && x.scalar_type() == at::kFloat, "x must be [T, W] fp32");
   a.T = (int)x.size(0);
   a.W = (int)x.size(1);
@@ -49,17 +50,23 @@ void residual_common(mlop::ResidualArgs& a, const Tensor& xn, const Tensor& x, c
   a.xn = xn.data_ptr();
   if (norm_w) a.norm_w = vec_or_one(*norm_w, a.W, a.norm_one, "norm_w");
   a.eps = (float)eps;
+  TORCH_CHECK(tanh_a.has_value() == tanh_b.has_value() && (!tanh_a || norm_w), "a dynamic tanh has alpha, weight and b");
+  if (tanh_a) {
+    a.tanh_a = f32_of(*tanh_a, 1, "tanh alpha");
+    a.tanh_b = f32_of(*tanh_b, a.W, "tanh b");
+    aligned16(*tanh_b, "tanh b");
+  }
   TORCH_CHECK(width >= 0 && width <= a.W, "width");
   a.n = width ? (int)width : a.W;
   for (const Tensor* t : {&x, &xn}) aligned16(*t, "residual operand");
 }
 
 void residual_begin(Tensor xn, Tensor x, Tensor ids, Tensor table, double scale, OptT pos_table, Tensor pos, OptT norm_w,
-                    double eps, int64_t width) {
+                    double eps, int64_t width, OptT tanh_a, OptT tanh_b) {
   mlop::ResidualArgs a{};
   const bool f32 = model_f32(table, "table");
   like(xn, table, "xn");
-  residual_common(a, xn, x, norm_w, eps, width);
+  residual_common(a, xn, x, norm_w, eps, width, tanh_a, tanh_b);
   TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.numel() == a.T, "ids int64 [T]");
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && table.size(1) == a.W, "table must be [vocab, W]");
   aligned16(table, "table");
@@ -82,11 +89,11 @@ void residual_begin(Tensor xn, Tensor x, Tensor ids, Tensor table, double scale,
 }
 
 void residual_step(Tensor xn, Tensor x, OptT y, OptT post_w, OptT norm_w, double eps, bool store, int64_t width, OptT rows,
-                   OptT inv, OptT gate) {
+                   OptT inv, OptT gate, OptT row_w, OptT self, OptT self_w, OptT tanh_a, OptT tanh_b) {
   mlop::ResidualArgs a{};
   TORCH_CHECK(y || rows, "residual_step needs a sublayer output");
   const bool f32 = model_f32(xn, "xn");
-  residual_common(a, xn, x, norm_w, eps, width);
+  residual_common(a, xn, x, norm_w, eps, width, tanh_a, tanh_b);
   if (y) {
     like(*y, xn, "y");
     TORCH_CHECK(y->is_contiguous() && y->numel() == x.numel(), "y must be [T, W]");
@@ -102,6 +109,14 @@ void residual_step(Tensor xn, Tensor x, OptT y, OptT post_w, OptT norm_w, double
     a.inv = i32_of(*inv, "inv");
     a.top = (int)inv->size(1);
     if (gate) a.gate = f32_of(*gate, a.T, "gate");
+    if (row_w) a.row_w = f32_of(*row_w, inv->numel(), "row_w");
+    if (self) {
+      like(*self, xn, "self");
+      TORCH_CHECK(self->is_contiguous() && self->numel() == x.numel() && self_w, "self must be [T, W], with weights");
+      aligned16(*self, "self");
+      a.self = self->data_ptr();
+      a.self_w = f32_of(*self_w, a.T, "self_w");
+    }
   }
   if (post_w) a.post_w = vec_or_one(*post_w, a.W, a.post_one, "post_w");
   a.store = store;
@@ -391,7 +406,7 @@ void head_mm(Tensor out, Tensor x, Tensor w, Tensor tile_seq, Tensor tile_q0, Te
   mlop::launch_head_mm(a, f32, cur());
 }
 
-// operands common to the sigmoid routing's forms
+// operands common to the forms of the routing kinds
 struct SigShape {
   int T, E, rows, k, H;
   float *topw, *gate;
@@ -455,14 +470,70 @@ void moe_route_sigmoid(Tensor topw, Tensor topi, OptT gate, Tensor logits, int64
   mlop::launch_moe_route_sigmoid(s.topw, s.topi, s.gate, f32_of(logits, logits.numel(), "logits"), s.T, s.E, s.rows, s.k, cur());
 }
 
-void moe_permute_scaled(Tensor xp, Tensor offsets, Tensor src, Tensor inv, Tensor x, Tensor topi, Tensor topw, int64_t E) {
-  TORCH_CHECK(x.dim() == 2, "x must be [T, H]");
-  const auto s = sig_shape(topw, topi, inv, std::nullopt, x.size(0), x.size(1), E, E);
-  TORCH_CHECK(src.numel() == s.T * s.k, "src must be [T * k]");
+// the choice among all of the router's outputs, the first E of them experts
+mlop::ChooseArgs choose_args(const OptT& correction, const OptT& self_w, int64_t T, int64_t n, int64_t E, int64_t k, int64_t groups,
+                             int64_t keep) {
+  TORCH_CHECK(n >= E && n <= mlop::kSigMaxE, "router outputs: E .. ", mlop::kSigMaxE);
+  TORCH_CHECK(groups >= 1 && n % groups == 0 && keep >= 1 && keep <= groups && k <= n / groups * keep,
+              "groups must divide the outputs, the kept ones hold the choice");
+  TORCH_CHECK(self_w.has_value() == (n > E), "self_w comes with identity experts");
+  mlop::ChooseArgs c{};
+  c.n = (int)n, c.groups = (int)groups, c.keep = (int)keep;
+  if (correction) c.correction = f32_of(*correction, n, "correction");
+  if (self_w) c.self_w = const_cast<float*>(f32_of(*self_w, T, "self_w"));
+  return c;
+}
+// as sig_shape; top may exceed the experts where identity experts are chosen beside them
+SigShape group_shape(const Tensor& topw, const Tensor& topi, const Tensor& inv, int64_t T, int64_t H, int64_t rows, int64_t E) {
+  TORCH_CHECK(E >= 1 && E <= rows, "1 .. rows experts");
+  SigShape s = sig_shape(topw, topi, inv, std::nullopt, T, H, rows, rows);
+  s.E = (int)E;
+  return s;
+}
+
+void moe_dispatch_small_groups(Tensor topw, Tensor topi, Tensor xp, Tensor offsets, Tensor src, Tensor inv, OptT self_w, Tensor x,
+                               Tensor w, OptT correction, int64_t E, int64_t groups, int64_t keep) {
+  router_rows(x, w);
+  const auto s = group_shape(topw, topi, inv, x.size(0), x.size(1), w.size(0), E);
+  const auto c = choose_args(correction, self_w, s.T, s.rows, E, s.k, groups, keep);
+  TORCH_CHECK(s.T >= 1 && s.T <= 16, "1 .. 16 tokens");
+  like(xp, x, "xp");
+  TORCH_CHECK(xp.is_contiguous() && xp.dim() == 2 && xp.size(0) == s.T * s.k && xp.size(1) == s.H && src.numel() == s.T * s.k, "xp [T * k, H]");
+  aligned16(xp, "xp");
   c10::DeviceGuard g(x.device());
-  mlop::launch_moe_permute_scaled(const_cast<float*>(f32_of(xp, (int64_t)s.T * s.k * s.H, "xp")), offsets_of(offsets, E),
-                                  const_cast<int*>(i32_of(src, "src")), s.inv, f32_of(x, x.numel(), "x"), s.topi, s.topw, s.T, s.k,
-                                  s.H, s.E, cur());
+  mlop::launch_moe_dispatch_small_groups(s.topw, s.topi, xp.data_ptr(), offsets_of(offsets, E), const_cast<int*>(i32_of(src, "src")),
+                                         s.inv, x.data_ptr(), w.data_ptr(), s.T, s.E, s.k, s.H, c, cur());
+}
+
+void moe_dispatch_mid_groups(Tensor topw, Tensor topi, Tensor offsets, Tensor a_rows, Tensor inv, OptT self_w, Tensor x, Tensor w,
+                             OptT correction, int64_t E, int64_t groups, int64_t keep) {
+  router_rows(x, w);
+  const auto s = group_shape(topw, topi, inv, x.size(0), x.size(1), w.size(0), E);
+  const auto c = choose_args(correction, self_w, s.T, s.rows, E, s.k, groups, keep);
+  TORCH_CHECK(s.T >= 1 && a_rows.numel() == s.T * s.k, "a_rows must be [T * k]");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_moe_dispatch_mid_groups(s.topw, s.topi, offsets_of(offsets, E), const_cast<int*>(i32_of(a_rows, "a_rows")), s.inv,
+                                       x.data_ptr(), w.data_ptr(), s.T, s.E, s.k, s.H, c, cur());
+}
+
+void moe_route_groups(Tensor topw, Tensor topi, OptT self_w, Tensor logits, OptT correction, int64_t E, int64_t groups, int64_t keep) {
+  TORCH_CHECK(logits.dim() == 2, "logits must be [T, rows]");
+  const auto s = group_shape(topw, topi, topi, logits.size(0), 0, logits.size(1), E);
+  const auto c = choose_args(correction, self_w, s.T, s.rows, E, s.k, groups, keep);
+  c10::DeviceGuard g(logits.device());
+  mlop::launch_moe_route_groups(s.topw, s.topi, f32_of(logits, logits.numel(), "logits"), s.T, s.E, s.k, c, cur());
+}
+
+// fp32: the experts' rows gathered, times their scores (topw; none: as they are)
+void moe_permute_scaled(Tensor xp, Tensor offsets, Tensor src, Tensor inv, Tensor x, Tensor topi, OptT topw, int64_t E) {
+  TORCH_CHECK(x.dim() == 2 && topi.dim() == 2 && topi.size(0) == x.size(0) && E >= 1 && E <= mlop::kSigMaxE, "x [T, H], topi [T, k]");
+  const int64_t T = x.size(0), k = topi.size(1), H = x.size(1);
+  TORCH_CHECK(src.numel() == T * k && inv.numel() == T * k && T * k < (1 << 28), "src, inv must be [T * k]");
+  c10::DeviceGuard g(x.device());
+  mlop::launch_moe_permute_scaled(const_cast<float*>(f32_of(xp, T * k * H, "xp")), offsets_of(offsets, E),
+                                  const_cast<int*>(i32_of(src, "src")), const_cast<int*>(i32_of(inv, "inv")), f32_of(x, x.numel(), "x"),
+                                  i32_of(topi, "topi"), topw ? f32_of(*topw, T * k, "topw") : nullptr, (int)T, (int)k, (int)H, (int)E,
+                                  cur());
 }
 
 void grouped_plain(Tensor out, Tensor a, Tensor w, Tensor offsets) {
@@ -482,9 +553,10 @@ void grouped_plain(Tensor out, Tensor a, Tensor w, Tensor offsets) {
 
 TORCH_LIBRARY_FRAGMENT(mlop, m) {
   m.def("residual_begin(Tensor(a!) xn, Tensor(b!) x, Tensor ids, Tensor table, float scale, Tensor? pos_table, Tensor pos, "
-        "Tensor? norm_w, float eps, int width=0) -> ()");
+        "Tensor? norm_w, float eps, int width=0, Tensor? tanh_a=None, Tensor? tanh_b=None) -> ()");
   m.def("residual_step(Tensor(a!) xn, Tensor(b!) x, Tensor? y, Tensor? post_w, Tensor? norm_w, float eps, bool store, "
-        "int width=0, Tensor? rows=None, Tensor? inv=None, Tensor? gate=None) -> ()");
+        "int width=0, Tensor? rows=None, Tensor? inv=None, Tensor? gate=None, Tensor? row_w=None, Tensor? self_x=None, "
+        "Tensor? self_w=None, Tensor? tanh_a=None, Tensor? tanh_b=None) -> ()");
   m.def("gated_norm(Tensor(a!) out, Tensor y, Tensor gate, Tensor w, int groups, float eps, int act, bool gate_first) -> ()");
   m.def("clamp_glu(Tensor(a!) out, Tensor x, float alpha, float limit) -> ()");
   m.def("short_conv(Tensor(a!) out, Tensor(b!) tail, Tensor x, Tensor w, Tensor? b, " MLOP_ROWS ") -> ()");
@@ -504,7 +576,13 @@ TORCH_LIBRARY_FRAGMENT(mlop, m) {
   m.def("moe_dispatch_mid_sigmoid(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!) offsets, Tensor(d!) a_rows, Tensor(e!) row_w, "
         "Tensor(f!) inv, Tensor(g!)? gate, Tensor x, Tensor router, int n_experts) -> ()");
   m.def("moe_route_sigmoid(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!)? gate, Tensor logits, int n_experts) -> ()");
-  m.def("moe_permute_scaled(Tensor(a!) xp, Tensor(b!) offsets, Tensor(c!) src, Tensor(d!) inv, Tensor x, Tensor topi, Tensor topw, "
+  m.def("moe_dispatch_small_groups(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!) xp, Tensor(d!) offsets, Tensor(e!) src, "
+        "Tensor(f!) inv, Tensor(g!)? self_w, Tensor x, Tensor router, Tensor? correction, int n_experts, int groups, int keep) -> ()");
+  m.def("moe_dispatch_mid_groups(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!) offsets, Tensor(d!) a_rows, Tensor(e!) inv, "
+        "Tensor(f!)? self_w, Tensor x, Tensor router, Tensor? correction, int n_experts, int groups, int keep) -> ()");
+  m.def("moe_route_groups(Tensor(a!) topw, Tensor(b!) topi, Tensor(c!)? self_w, Tensor logits, Tensor? correction, int n_experts, "
+        "int groups, int keep) -> ()");
+  m.def("moe_permute_scaled(Tensor(a!) xp, Tensor(b!) offsets, Tensor(c!) src, Tensor(d!) inv, Tensor x, Tensor topi, Tensor? topw, "
         "int n_experts) -> ()");
   m.def("grouped_plain(Tensor(a!) out, Tensor a, Tensor w, Tensor offsets) -> ()");
 }
@@ -524,6 +602,9 @@ TORCH_LIBRARY_IMPL(mlop, CUDA, m) {
   m.impl("moe_dispatch_small_sigmoid", &moe_dispatch_small_sigmoid);
   m.impl("moe_dispatch_mid_sigmoid", &moe_dispatch_mid_sigmoid);
   m.impl("moe_route_sigmoid", &moe_route_sigmoid);
+  m.impl("moe_dispatch_small_groups", &moe_dispatch_small_groups);
+  m.impl("moe_dispatch_mid_groups", &moe_dispatch_mid_groups);
+  m.impl("moe_route_groups", &moe_route_groups);
   m.impl("moe_permute_scaled", &moe_permute_scaled);
   m.impl("grouped_plain", &grouped_plain);
 }

@@ -132,6 +132,12 @@ __device__ __forceinline__ float clamp_glu_f(float g, float u, float alpha, floa
   return g * (u + 1.f) / (1.f + __expf(-alpha * g));
 }
 
+// tanh gelu: x / 2 (1 + tanh(u)) = x / (1 + exp(-2 u)), u = sqrt(2 / pi) (x + 0.044715 x^3)
+__device__ __forceinline__ float gelu_tanh_f(float x) {
+  const float u = 0.7978845608028654f * fmaf(0.044715f * x * x, x, x);
+  return x * __builtin_amdgcn_rcpf(1.f + __expf(-2.f * u));
+}
+
 __device__ __forceinline__ float relu2_f(float x) {
   const float r = fmaxf(x, 0.f);
   return r * r;

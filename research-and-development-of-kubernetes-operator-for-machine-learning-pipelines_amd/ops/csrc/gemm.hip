@@ -27,7 +27,7 @@
 // (launch-boundary reduce, §5 "Projection GEMM at M = 256" item 2).
 //
 // Epilogues (fp32 LDS copy of the tile, 16-B coalesced stores):
-//   EPI_NONE      C = bf16(acc), or an activation of acc (RopeEpi::act)
+//   EPI_NONE      C = bf16(acc), or an activation of acc (RopeEpi::act, act_n0)
 //   EPI_SILU_MUL  B rows gate/up interleaved in groups of 16, C[:, j] = silu(g_j) * u_j (N/2 cols)
 //   EPI_ROPE      QKV projection: RoPE on q/k heads + q_out / paged K,V cache stores from the
 //                 staged tile (RopeEpi, launch.h); needs whole 128-wide heads per staged chunk
@@ -376,7 +376,7 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
         u32x4 o;
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-          o[j] = pack2(act_out(re, s[2 * j]), act_out(re, s[2 * j + 1]));
+          o[j] = pack2(act_out(re, s[2 * j], n0 + c0 + c), act_out(re, s[2 * j + 1], n0 + c0 + c));
         *reinterpret_cast<u32x4*>(C + (size_t)(m0 + r) * ldc + n0 + c0 + c) = o;
       }
     } else {
@@ -436,7 +436,7 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if (EPI == EPI_NONE)
-        o[j] = pack2(act_out(re, a[2 * j]), act_out(re, a[2 * j + 1]));
+        o[j] = pack2(act_out(re, a[2 * j], j0), act_out(re, a[2 * j + 1], j0));
       else
         o[j] = pack2(glu_out(re, a[2 * j], b[2 * j]), glu_out(re, a[2 * j + 1], b[2 * j + 1]));
     }
@@ -1111,7 +1111,7 @@ __global__ void __launch_bounds__(512, 1) gemm_pp_kernel(
         if constexpr (EPI == EPI_NONE) {
 #pragma unroll
           for (int j = 0; j < 4; ++j)
-            sC[row * LD + j * 16 + (lane & 15)] = f2bf(act_out(re, acc[i][j][r]));
+            sC[row * LD + j * 16 + (lane & 15)] = f2bf(act_out(re, acc[i][j][r], n0 + wc * 64));
         } else {
           float f = 1.f;
           if constexpr (GROUPED)
@@ -1730,16 +1730,17 @@ long gemm_workspace_floats(int M, int N, int K, int epi) {
 }
 
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
-                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float p0, float p1) {
+                 long ws_floats, int M, int N, int K, int epi, hipStream_t st, float p0, float p1, int act_n0) {
   if (M == 0) return;
   RopeEpi re{};
+  re.act_n0 = act_n0;
   re.p0 = p0;
   re.p1 = p1;
   re.act = epi_act(epi);
   const int epi0 = epi;
   if (re.act) epi = EPI_NONE;
   if (gemv_takes(M, N, K, epi) && lda % 8 == 0 && ldb % 8 == 0) {
-    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, epi0, st, p0, p1);
+    launch_gemv(A, lda, B, ldb, C, ldc, M, N, K, epi0, st, p0, p1, act_n0);
     return;
   }
   Plan p = plan(M, N, K, false, 0, 0);
@@ -1800,11 +1801,11 @@ bool launch_gemm_add_rmsnorm(const void* A, int lda, const void* B, void* out, v
 
 void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offsets, int n_groups,
                          int M, int N, int K, int max_rows, int epi, hipStream_t st, const int* a_rows,
-                         float** defer_ws, int* defer_splits, const float* row_scale) {
+                         float** defer_ws, int* defer_splits, const float* row_scale, float p0, float p1) {
   if (defer_splits) *defer_splits = 1;
   if (M == 0) return;
   if (a_rows == nullptr && row_scale == nullptr && defer_splits == nullptr && gemv_grouped_takes(M, N, K, epi)) {  // MoE decode: stream only the routed experts' weights
-    launch_gemv_grouped(A, B, C, offsets, n_groups, M, N, K, epi, st);
+    launch_gemv_grouped(A, B, C, offsets, n_groups, M, N, K, epi, st, p0, p1);
     return;
   }
   Plan p = plan(M, N, K, true, n_groups, max_rows);
@@ -1830,6 +1831,8 @@ void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offse
   RopeEpi re{};
   re.a_rows = a_rows;
   re.row_scale = row_scale;
+  re.p0 = p0;
+  re.p1 = p1;
   if (epi == EPI_NONE)
     launch_plan<EPI_NONE, true>(p, (const uint16_t*)A, K, (const uint16_t*)B, K, (uint16_t*)C, N,
                                 ws, M, N, K, offsets, n_groups, st, re);

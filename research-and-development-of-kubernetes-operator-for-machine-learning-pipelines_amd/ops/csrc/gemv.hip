@@ -301,7 +301,7 @@ __global__ void __launch_bounds__(256) gemv_kernel(const uint16_t* __restrict__ 
 #pragma unroll
       for (int r = 0; r < R; ++r)
         if (lane == m * R + r && m < mc)
-          C[(size_t)m * ldc + set * R + r] = f2bf(act_out(re, acc[r][m]));
+          C[(size_t)m * ldc + set * R + r] = f2bf(act_out(re, acc[r][m], set * R + r));
   }
 }
 
@@ -376,12 +376,13 @@ bool gemv_takes(int M, int N, int K, int epi) {
 }
 
 void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ldc, int M, int N, int K,
-                 int epi, hipStream_t st, float p0, float p1) {
+                 int epi, hipStream_t st, float p0, float p1, int act_n0) {
   auto* a = (const uint16_t*)A;
   auto* b = (const uint16_t*)B;
   auto* c = (uint16_t*)C;
   RopeEpi none{};
   none.act = epi_act(epi);
+  none.act_n0 = act_n0;
   none.p0 = p0;
   none.p1 = p1;
   if (epi == EPI_SILU_MUL) run_gemv<EPI_SILU_MUL>(a, lda, b, ldb, c, ldc, M, N, K, none, st);
@@ -395,7 +396,7 @@ void launch_gemv_rope(const void* A, int lda, const void* B, int M, int N, int K
 
 template <int M, int EPI>
 void run_gemv_grouped_m(const uint16_t* A, const uint16_t* B, uint16_t* C, int ldc, int N, int K,
-                        const int* offsets, int n_groups, hipStream_t st) {
+                        const int* offsets, int n_groups, const RopeEpi& re, hipStream_t st) {
   constexpr int U = M <= 2 ? 4 : 2;
   const int pairs = N / 2;
   const int rp = pairs / 2 >= 2048 ? 2 : 1;
@@ -407,7 +408,7 @@ void run_gemv_grouped_m(const uint16_t* A, const uint16_t* B, uint16_t* C, int l
     const int sets = spg * slots;                                                                  \
     const int blocks = KW == 1 ? cdiv(sets, 4) : sets;                                             \
     gemv_kernel<M, RP, EPI, KW, U, PRO_NONE, true><<<blocks, 256, 0, st>>>(A, K, B, K, C, ldc, N, K,  \
-                                                                          RopeEpi{}, NormPro{}, ga); \
+                                                                          re, NormPro{}, ga); \
   } while (0)
   if (rp == 2) {
     if (kw4) MLOP_GEMV_G(2, 4); else MLOP_GEMV_G(2, 1);
@@ -424,15 +425,18 @@ bool gemv_grouped_takes(int M, int N, int K, int epi) {
 }
 
 void launch_gemv_grouped(const void* A, const void* B, void* C, const int* offsets, int n_groups, int M, int N,
-                         int K, int epi, hipStream_t st) {
+                         int K, int epi, hipStream_t st, float p0, float p1) {
+  RopeEpi re{};
+  re.p0 = p0;
+  re.p1 = p1;
   auto* a = (const uint16_t*)A;
   auto* b = (const uint16_t*)B;
   auto* c = (uint16_t*)C;
   const int ldc = epi == EPI_SILU_MUL ? N / 2 : N;
 #define MLOP_GG(MM)                                                                       \
   case MM:                                                                                \
-    if (epi == EPI_SILU_MUL) run_gemv_grouped_m<MM, EPI_SILU_MUL>(a, b, c, ldc, N, K, offsets, n_groups, st); \
-    else run_gemv_grouped_m<MM, EPI_NONE>(a, b, c, ldc, N, K, offsets, n_groups, st);          \
+    if (epi == EPI_SILU_MUL) run_gemv_grouped_m<MM, EPI_SILU_MUL>(a, b, c, ldc, N, K, offsets, n_groups, re, st); \
+    else run_gemv_grouped_m<MM, EPI_NONE>(a, b, c, ldc, N, K, offsets, n_groups, re, st);          \
     break;
   switch (M) {
     MLOP_GG(1) MLOP_GG(2) MLOP_GG(3) MLOP_GG(4) MLOP_GG(5) MLOP_GG(6) MLOP_GG(7) MLOP_GG(8)

@@ -1,5 +1,5 @@
-// Launchers of the hybrid-decoder kernels (hyper-connections, whole-projection query / key norm
-// with partial rotary positions, paged attention of any head sizes with a softmax sink and an
+// Launchers of the hybrid-decoder kernels (hyper-connections, whole-projection or per-head query / key
+// norm with partial rotary positions, paged attention of any head sizes with a softmax sink and an
 // output gate, gated linear attention).  `f32` selects float operands; otherwise bf16.
 #pragma once
 
@@ -49,9 +49,27 @@ struct QkNormArgs {
 };
 void launch_qk_norm(const QkNormArgs& a, bool f32, hipStream_t st);
 
+// ---- per-head query / key norm + rotary + paged stores (qk_norm.hip)
+struct QkHeadNormArgs {
+  void* q_out;           // [T, H, KP], dims past D zero
+  void* k_cache;         // [NB, G, BS, KP]
+  void* v_cache;         // [NB, G, BS, VP]
+  const void *q, *k, *v; // [T, H x D], [T, G x D], [T, G x V]; v null: the values are k as given (V = D)
+  long ldq, ldk, ldv;
+  const float *q_w, *k_w;  // [D]: one weight for all heads, each divided by its own root mean square
+  float eps;
+  const float* cos_sin;  // [max_pos, R]: cos of the R / 2 pairs, then sin
+  int R;                 // rotated dims of a head (even; pairs 2i, 2i + 1)
+  const int* pos;
+  const int* slots;      // < 0: no cache write
+  int T, H, G, D, V, KP, VP, BS;
+};
+void launch_qk_head_norm(const QkHeadNormArgs& a, bool f32, hipStream_t st);
+
 // ---- paged attention of any head sizes (attention_hd.hip)
 struct AttnHdArgs {
-  void* out;             // [T, H, V] (by_tile: [tiles, H, V])
+  void* out;             // [T, H, V] (by_tile: [tiles, H, V]), rows out_row elements apart
+  long out_row;
   const void* q;         // rows of KP per token (by_tile: per tile) and head
   long q_row, q_head;    // strides of q (elements)
   // keys and values, 16-token pages: row t of page p, head g at p * 16 * pitch + t * row + g * head.  Paged
@@ -67,6 +85,7 @@ struct AttnHdArgs {
   const void* gate;      // [T, gate_stride] pre-sigmoid, or null
   long gate_stride;
   bool gate_elem;        // one gate per head and value element (H x V); else one per head
+  bool gate_vec;         // element gates are read 4 at a time (aligned rows)
   bool by_tile;          // q and out rows are decode tiles, not tokens
   int window;            // a token sees itself and the window - 1 tokens before it (0: all)
   // prompt tiles: dims rot_lo .. rot_lo + n_rot of a query head turn by the token's position as they are
@@ -117,8 +136,8 @@ bool gla_chunks_need_o32(int dv);
 constexpr int kGlaMaxDk = 256;    // key size of the chunked kernel
 
 // ---- elementwise (hyper.hip)
-void launch_relu2(void* x, long n, bool f32, hipStream_t st);                       // in place
-void launch_xielu(void* x, long n, float a, float b, bool f32, hipStream_t st);     // in place
+// an activation (launch.h kAct*) of columns n0 .. N, in place
+void launch_act_columns(void* x, long rows, int N, int n0, int act, float a, float b, bool f32, hipStream_t st);
 void launch_softcap(float* out, const void* x, long n, float cap, bool f32, hipStream_t st);
 
 }  // namespace mlop

@@ -10,6 +10,7 @@
 // The first pass of a step starts every stream from the scaled embedding row instead.
 #include "elem.h"
 #include "hybrid.h"
+#include "launch.h"
 
 namespace mlop {
 
@@ -134,31 +135,23 @@ void launch_hyper(const HyperArgs& a, bool f32, hipStream_t st) {
   }
 }
 
-// x <- max(x, 0)^2 in place
+// an activation of columns n0 .. N of the rows, in place
 template <typename E, int VEC>
-__global__ void __launch_bounds__(256) relu2_kernel(E* __restrict__ x, long n) {
+__global__ void __launch_bounds__(256) act_columns_kernel(E* __restrict__ x, long total, int N, int n0, int act, float a, float b) {
   const long i = ((long)blockIdx.x * 256 + threadIdx.x) * VEC;
-  if (i >= n) return;
+  if (i >= total) return;
+  const int w = N - n0;
+  E* p = x + i / w * N + n0 + i % w;
   float v[VEC];
-  ldn<VEC>(x + i, v);
+  ldn<VEC>(p, v);
 #pragma unroll
   for (int e = 0; e < VEC; ++e) {
-    const float r = fmaxf(v[e], 0.f);
-    v[e] = r * r;
+    const float z = v[e];
+    if (act == kActGelu) v[e] = z / (1.f + expf(-1.5957691216057308f * fmaf(0.044715f * z * z, z, z)));
+    else if (act == kActXielu) v[e] = 0.5f * z + (z > 0.f ? a * z * z : b * (expm1f(z) - z));
+    else v[e] = relu2_f(z);
   }
-  stn<VEC>(x + i, v);
-}
-
-// xIELU in place
-template <typename E, int VEC>
-__global__ void __launch_bounds__(256) xielu_kernel(E* __restrict__ x, long n, float a, float b) {
-  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * VEC;
-  if (i >= n) return;
-  float v[VEC];
-  ldn<VEC>(x + i, v);
-#pragma unroll
-  for (int e = 0; e < VEC; ++e) v[e] = 0.5f * v[e] + (v[e] > 0.f ? a * v[e] * v[e] : b * (expm1f(v[e]) - v[e]));
-  stn<VEC>(x + i, v);
+  stn<VEC>(p, v);
 }
 
 // out <- cap * tanh(x / cap), fp32
@@ -174,29 +167,17 @@ __global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ out, c
   stn<VEC>(out + i, v);
 }
 
-void launch_relu2(void* x, long n, bool f32, hipStream_t st) {
-  if (n == 0) return;
-  const bool v8 = n % 8 == 0;
-  const long grid = (n / (v8 ? 8 : 1) + 255) / 256;
+void launch_act_columns(void* x, long rows, int N, int n0, int act, float a, float b, bool f32, hipStream_t st) {
+  const long total = rows * (N - n0);
+  if (total == 0) return;
+  const bool v8 = N % 8 == 0 && n0 % 8 == 0;
+  const long grid = (total / (v8 ? 8 : 1) + 255) / 256;
   if (f32) {
-    if (v8) relu2_kernel<float, 8><<<grid, 256, 0, st>>>((float*)x, n);
-    else relu2_kernel<float, 1><<<grid, 256, 0, st>>>((float*)x, n);
+    if (v8) act_columns_kernel<float, 8><<<grid, 256, 0, st>>>((float*)x, total, N, n0, act, a, b);
+    else act_columns_kernel<float, 1><<<grid, 256, 0, st>>>((float*)x, total, N, n0, act, a, b);
   } else {
-    if (v8) relu2_kernel<uint16_t, 8><<<grid, 256, 0, st>>>((uint16_t*)x, n);
-    else relu2_kernel<uint16_t, 1><<<grid, 256, 0, st>>>((uint16_t*)x, n);
-  }
-}
-
-void launch_xielu(void* x, long n, float a, float b, bool f32, hipStream_t st) {
-  if (n == 0) return;
-  const bool v8 = n % 8 == 0;
-  const long grid = (n / (v8 ? 8 : 1) + 255) / 256;
-  if (f32) {
-    if (v8) xielu_kernel<float, 8><<<grid, 256, 0, st>>>((float*)x, n, a, b);
-    else xielu_kernel<float, 1><<<grid, 256, 0, st>>>((float*)x, n, a, b);
-  } else {
-    if (v8) xielu_kernel<uint16_t, 8><<<grid, 256, 0, st>>>((uint16_t*)x, n, a, b);
-    else xielu_kernel<uint16_t, 1><<<grid, 256, 0, st>>>((uint16_t*)x, n, a, b);
+    if (v8) act_columns_kernel<uint16_t, 8><<<grid, 256, 0, st>>>((uint16_t*)x, total, N, n0, act, a, b);
+    else act_columns_kernel<uint16_t, 1><<<grid, 256, 0, st>>>((uint16_t*)x, total, N, n0, act, a, b);
   }
 }
 

@@ -72,29 +72,36 @@ struct RopeEpi {
   // mid norm chain (gemm.hip mid_chain_finish): 1 = the finishing split reads the partials with
   // plain loads behind one agent acquire, 0 = with sc1 loads only (gemm_mid_chain op 2 / 1)
   int mid_acq = 0;
-  // plain epilogue only: an activation of the accumulator (kAct*; EPI_RELU2, EPI_XIELU of launch_gemm)
-  int act = 0;
+  // plain epilogue only: an activation of the accumulator (kAct*; EPI_RELU2, EPI_XIELU, EPI_GELU of launch_gemm)
+  // from column act_n0 on (a multiple of 128)
+  int act = 0, act_n0 = 0;
   // SiLU-mul epilogue: p0 > 0 makes it the clamped gated unit (common.h clamp_glu_f) with alpha = p0,
   // limit = p1 instead; kActXielu: a = p0, b = p1
   float p0 = 0.f, p1 = 0.f;
   // grouped SiLU-mul: permuted row r's accumulators times row_scale[r] before the unit (nullptr: 1)
   const float* row_scale = nullptr;
 };
-enum { kActNone = 0, kActRelu2 = 1, kActXielu = 2 };
+enum { kActNone = 0, kActRelu2 = 1, kActXielu = 2, kActGelu = 3 };
 #ifdef __HIP__
 // one output of the gate / up epilogue
 __device__ __forceinline__ float glu_out(const RopeEpi& re, float g, float u) {
   return re.p0 > 0.f ? clamp_glu_f(g, u, re.p0, re.p1) : silu_bf(g) * bf2f(f2bf(u));
 }
-// one output of the plain epilogue
-__device__ __forceinline__ float act_out(const RopeEpi& re, float x) {
-  if (re.act == kActRelu2) return relu2_f(x);
-  return re.act == kActXielu ? xielu_f(x, re.p0, re.p1) : x;
+__device__ __forceinline__ float act_f(int act, float x, float p0, float p1) {
+  if (act == kActGelu) return gelu_tanh_f(x);
+  if (act == kActRelu2) return relu2_f(x);
+  return act == kActXielu ? xielu_f(x, p0, p1) : x;
+}
+// one output of the plain epilogue, of column col
+__device__ __forceinline__ float act_out(const RopeEpi& re, float x, int col) {
+  return col < re.act_n0 ? x : act_f(re.act, x, re.p0, re.p1);
 }
 #endif
 // launch_gemm: plain product with an activation in its epilogue
-constexpr int kEpiRelu2 = 6, kEpiXielu = 7;
-constexpr int epi_act(int epi) { return epi == kEpiRelu2 ? kActRelu2 : epi == kEpiXielu ? kActXielu : kActNone; }
+constexpr int kEpiRelu2 = 6, kEpiXielu = 7, kEpiGelu = 8;
+constexpr int epi_act(int epi) {
+  return epi == kEpiRelu2 ? kActRelu2 : epi == kEpiXielu ? kActXielu : epi == kEpiGelu ? kActGelu : kActNone;
+}
 // RoPE + paged-cache stores from the QKV projection's fp32 split-K slabs ws[splits][T][N] (the
 // split-K reduce fused in: small-M launch_gemm_rope)
 void launch_rope_cache_slabs(const RopeEpi& re, const float* ws, int splits, int T, int N, hipStream_t st);
@@ -138,7 +145,7 @@ int gemm_sk_workgroups(int M, int N, int K);
 // K2 skinny GEMV (gemv.hip): decode projections at M <= 8 (epi 0 none, 1 silu-mul, 3 rope)
 bool gemv_takes(int M, int N, int K, int epi);
 void launch_gemv(const void* A, int lda, const void* B, int ldb, void* C, int ldc, int M, int N, int K,
-                 int epi, hipStream_t st, float p0 = 0.f, float p1 = 0.f);
+                 int epi, hipStream_t st, float p0 = 0.f, float p1 = 0.f, int act_n0 = 0);
 void launch_gemv_rope(const void* A, int lda, const void* B, int M, int N, int K, const RopeEpi& re,
                       hipStream_t st);
 // the decode norm chain's row-scale prologue parameters (gemv.hip PRO_RS)
@@ -179,20 +186,20 @@ void launch_gemv_rs(const void* A, int lda, const void* B, void* C, int ldc, int
 void launch_gemv_res(const void* A, int lda, const void* B, void* residual, int M, int N, int K, hipStream_t st);
 bool gemv_grouped_takes(int M, int N, int K, int epi);
 void launch_gemv_grouped(const void* A, const void* B, void* C, const int* offsets, int n_groups, int M, int N,
-                         int K, int epi, hipStream_t st);
+                         int K, int epi, hipStream_t st, float p0 = 0.f, float p1 = 0.f);
 bool gemm_rope_supported(int M, int N, int K);
 bool launch_gemm_rope(const void* A, int lda, const void* B, int M, int N, int K, const RopeEpi& re,
                       hipStream_t st);
 void launch_gemm(const void* A, int lda, const void* B, int ldb, void* C, int ldc, float* ws,
                  long ws_floats, int M, int N, int K, int epi, hipStream_t st, float p0 = 0.f,
-                 float p1 = 0.f);
+                 float p1 = 0.f, int act_n0 = 0);
 bool launch_gemm_add_rmsnorm(const void* A, int lda, const void* B, void* out, void* residual,
                              const void* w, float eps, float* ws, long ws_floats, int M, int N,
                              int K, hipStream_t st);
 void launch_grouped_gemm(const void* A, const void* B, void* C, const int* offsets, int n_groups,
                          int M, int N, int K, int max_rows, int epi, hipStream_t st, const int* a_rows = nullptr,
                          float** defer_ws = nullptr, int* defer_splits = nullptr,
-                         const float* row_scale = nullptr);
+                         const float* row_scale = nullptr, float p0 = 0.f, float p1 = 0.f);
 bool launch_moe_down_combine_add_rmsnorm(void* out, void* residual, void* y, const void* a, const void* w2,
                                          const int* offsets, int n_groups, int R, int H, int I, int max_rows,
                                          const int* inv, const float* topw, const void* norm_w, float eps, int T,
@@ -205,6 +212,18 @@ int moe_mid_max_tokens(int set);
 void launch_moe_dispatch_mid(float* topw, int* topi, int* offsets, int* arow, int* inv, const void* x, const void* wr,
                              int T, int E, int k, int H, int e0, int n_local, const void* pro_y, void* pro_res,
                              const void* pro_w, float pro_eps, void* pro_xn, hipStream_t st);
+// grouped routing (moe.hip): the choice among n router outputs, in `keep` of `groups` equal groups
+struct ChooseArgs {
+  int n, groups, keep;
+  const float* correction;  // [n] or null
+  float* self_w;            // [T] weight of the outputs behind the experts', or null (there are none)
+};
+void launch_moe_dispatch_small_groups(float* topw, int* topi, void* xp, int* offsets, int* src, int* inv, const void* x,
+                                      const void* wr, int T, int E, int k, int H, const ChooseArgs& cho, hipStream_t st);
+void launch_moe_dispatch_mid_groups(float* topw, int* topi, int* offsets, int* arow, int* inv, const void* x, const void* wr,
+                                    int T, int E, int k, int H, const ChooseArgs& cho, hipStream_t st);
+void launch_moe_route_groups(float* topw, int* topi, const float* logits, int T, int E, int k, const ChooseArgs& cho,
+                             hipStream_t st);
 // sigmoid routing with the scores on the experts' inputs (moe.hip); router rows: E experts', then a gate's or none
 constexpr int kSigMaxE = 256, kSigMaxTop = 64;
 void launch_moe_dispatch_small_sigmoid(float* topw, int* topi, void* xp, int* offsets, int* src, int* inv, float* gate,

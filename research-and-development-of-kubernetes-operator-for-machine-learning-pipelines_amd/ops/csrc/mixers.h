@@ -27,13 +27,17 @@ struct ResidualArgs {
   float* x;               // [T, W]
   void* xn;               // [T, W] the next sublayer's input: norm_w * x / rms(x)
   const void* y;          // [T, W] sublayer output (null: the experts' alone)
-  const void* rows;       // [R, W] or null: sublayer output gate[t] y[t] + sum_j rows[inv[t, j]]
-  const int* inv;         // [T, top]
+  const void* rows;       // [R, W] or null: sublayer output gate[t] y[t] + sum_j row_w[t, j] rows[inv[t, j]] + self_w[t] self[t]
+  const int* inv;         // [T, top], < 0: no row
   const float* gate;      // [T] or null
+  const float* row_w;     // [T, top] or null: ones
+  const void* self;       // [T, W] or null
+  const float* self_w;    // [T]
   int top;
   const float* post_w;    // [W] or, post_one, one number: y is normed on its own, times this (null: added as it is)
   const float* norm_w;    // [W] or, norm_one, one number (null: xn = x)
   bool post_one, norm_one;
+  const float *tanh_a, *tanh_b;  // one number, [W], or null: xn = norm_w * tanh(a x) + b instead
   const long* ids;        // [T]  (start: x = scale * table[id] + pos_table[pos])
   const void* table;      // [vocab, W]
   const void* pos_table;  // [n_pos, W] or null

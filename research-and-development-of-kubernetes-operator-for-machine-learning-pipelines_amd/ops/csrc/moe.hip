@@ -1,9 +1,14 @@
 // Mixture-of-experts routing kernels for gfx950 (K11 route, K12 permute, K14 combine).
 // The expert FFN itself is the grouped MFMA GEMM of gemm.hip (K13).
 //
-// Two kinds of routing: softmax over the router's logits, renormalised over the chosen experts, the weights on
-// the experts' outputs (moe_combine); or (SIG) fp32 logits, the chosen experts' sigmoid scores as they are, the
-// scores on the experts' INPUT rows, and possibly one row behind the experts' whose sigmoid is a gate per token.
+// Three kinds of routing:
+//   kSoftmax  softmax over the router's logits, renormalised over the chosen experts, the weights on the experts'
+//             outputs (moe_combine);
+//   kSigmoid  fp32 logits, the chosen experts' sigmoid scores as they are, the scores on the experts' INPUT rows, and
+//             possibly one row behind the experts' whose sigmoid is a gate per token;
+//   kGroups   fp32 logits, softmax over all of them, scores as they are on the experts' outputs (residual.hip sums
+//             them); a correction per output and a choice of groups decide who is chosen; outputs behind the experts'
+//             are identity experts, which have no row.
 //
 // Everything stays on the device and has static shapes (T*k rows reserved, the
 // valid count lives in offsets[n_local]), so an MoE layer can be captured in
@@ -152,7 +157,9 @@ struct MoePro {
 // (all of a lane's chunks in flight together) while the wave walks the T activation rows.
 constexpr int kSmallT = 16, kMaxE = 64, kDispWaves = 8;
 
-// SIG: `rows` router rows, the first E of them experts'
+enum { kSoftmax = 0, kSigmoid = 1, kGroups = 2 };
+
+// kSigmoid: `rows` router rows, the first E of them experts'
 struct SigArgs {
   float* gate;   // [T] sigmoid of row E (nullptr: there is none)
   float* row_w;  // [T * k] score of each permuted row (the gathered rows hold it already: nullptr)
@@ -170,6 +177,81 @@ __device__ __forceinline__ void next_best(const float* z, int n, float& v, int& 
   }
   v = bv;
   i = min(bi, n - 1);
+}
+
+// kGroups, one wave: scores of one token's n logits z (in LDS, overwritten by the choice scores), the top k of them
+// through put(j, output, score).  gm: LDS, groups floats.  Returns the weights of outputs from E on, added up.
+template <typename F>
+__device__ __forceinline__ float choose_groups(const ChooseArgs& c, float* z, float* gm, int E, int k, int lane, F&& put) {
+  constexpr int PER = kSigMaxE / 64;
+  auto lds_fence = [] {
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+    __builtin_amdgcn_wave_barrier();
+  };
+  float s[PER], ch[PER], mx = -INFINITY, sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = e < c.n ? z[e] : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
+  mx = wave_max(mx);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    s[i] = expf(s[i] - mx);
+    sum += s[i];
+  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = lane + 64 * i;
+    s[i] /= sum;
+    ch[i] = e < c.n ? s[i] + (c.correction ? c.correction[e] : 0.f) : -INFINITY;
+  }
+  if (c.keep < c.groups) {
+    const int size = c.n / c.groups;
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (lane + 64 * i < c.n) z[lane + 64 * i] = ch[i];
+    lds_fence();
+    for (int g = lane; g < c.groups; g += 64) {
+      float m = -INFINITY;
+      for (int e = 0; e < size; ++e) m = fmaxf(m, z[g * size + e]);
+      gm[g] = m;
+    }
+    lds_fence();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int e = lane + 64 * i;
+      if (e >= c.n) continue;
+      const int g = e / size;
+      int before = 0;  // groups ahead of this output's
+      for (int o = 0; o < c.groups; ++o) before += gm[o] > gm[g] || (gm[o] == gm[g] && o < g);
+      if (before >= c.keep) ch[i] = -INFINITY;
+    }
+  }
+  float own = 0.f;
+  for (int j = 0; j < k; ++j) {
+    float bv = -INFINITY;
+    int be = c.n;
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (ch[i] > bv) bv = ch[i], be = lane + 64 * i;
+    for (int o = 1; o < 64; o <<= 1) {
+      const float v = __shfl_xor(bv, o);
+      const int e = __shfl_xor(be, o);
+      if (v > bv || (v == bv && e < be)) bv = v, be = e;
+    }
+    be = min(be, c.n - 1);
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (be == lane + 64 * i) {
+        put(j, be, s[i]);
+        if (be >= E) own += s[i];
+        ch[i] = -INFINITY;
+      }
+  }
+  return wave_sum(own);
 }
 
 // router logits of two token rows, any row length (a multiple of 8)
@@ -190,13 +272,15 @@ __device__ __forceinline__ void dot_rows2(const uint16_t* w, const uint16_t* x0,
   s1 = wave_sum(s1);
 }
 
-template <int CH, bool SIG = false>  // 16-B chunks per lane per row: H = CH * 512 (0: any H)
+template <int CH, int KIND = kSoftmax>  // 16-B chunks per lane per row: H = CH * 512 (0: any H)
 __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
     float* __restrict__ topw, int* __restrict__ topi, uint16_t* __restrict__ xp, int* __restrict__ offsets,
     int* __restrict__ src, int* __restrict__ inv, const uint16_t* __restrict__ x,
-    const uint16_t* __restrict__ wr, int T, int E, int k, int H, int e0, int n_local, MoePro pro, SigArgs sig = SigArgs{}) {
-  constexpr int ME = SIG ? kSigMaxE : kMaxE, MK = SIG ? kSigMaxTop : 8;
+    const uint16_t* __restrict__ wr, int T, int E, int k, int H, int e0, int n_local, MoePro pro, SigArgs sig = SigArgs{}, ChooseArgs cho = ChooseArgs{}) {
+  constexpr bool SIG = KIND == kSigmoid;
+  constexpr int ME = KIND != kSoftmax ? kSigMaxE : kMaxE, MK = KIND != kSoftmax ? kSigMaxTop : 8;
   __shared__ float lg[kSmallT][ME + SIG];
+  __shared__ float s_gm[KIND == kGroups ? kDispWaves : 1][KIND == kGroups ? kSigMaxE : 1];
   __shared__ int s_topi[kSmallT * MK];
   __shared__ float s_topw[SIG ? kSmallT * MK : 1];
   __shared__ int cnt[ME + 1];
@@ -238,7 +322,7 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
     x = pro.xn;
   }
   // 1. router logits: lg[t][e] = bf16(x[t] . wr[e])
-  for (int e = wv; e < (SIG ? sig.rows : E); e += kDispWaves) {
+  for (int e = wv; e < (KIND == kGroups ? cho.n : SIG ? sig.rows : E); e += kDispWaves) {
     if constexpr (CH == 0) {
       for (int t = 0; t < T; t += 2) {
         float s0, s1;
@@ -264,13 +348,21 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
 #pragma unroll
         for (int q = 0; q < 4; ++q) acc += lo_bf(a[i][q]) * lo_bf(b[i][q]) + hi_bf(a[i][q]) * hi_bf(b[i][q]);
       acc = wave_sum(acc);
-      if (lane == 0) lg[t][e] = SIG ? acc : bf2f(f2bf(acc));
+      if (lane == 0) lg[t][e] = KIND != kSoftmax ? acc : bf2f(f2bf(acc));
     }
   }
   for (int e = threadIdx.x; e <= n_local; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
   // 2. softmax -> top-k -> renormalise (moe_route_kernel's math), one thread per token
-  if (SIG && threadIdx.x < T) {
+  if constexpr (KIND == kGroups) {
+    for (int t = wv; t < T; t += kDispWaves) {
+      const float own = choose_groups(cho, lg[t], s_gm[wv], E, k, lane, [&](int j, int e, float s) {
+        s_topi[t * k + j] = topi[t * k + j] = e;
+        topw[t * k + j] = s;
+      });
+      if (cho.self_w && lane == 0) cho.self_w[t] = own;
+    }
+  } else if (SIG && threadIdx.x < T) {
     const int t = threadIdx.x;
     float v = INFINITY;
     int e = -1;
@@ -380,7 +472,7 @@ void launch_moe_dispatch_small_sigmoid(float* topw, int* topi, void* xp, int* of
                                        hipStream_t st) {
   const SigArgs sig{gate, nullptr, rows};
 #define MLOP_DISP(CH)                                                                                             \
-  moe_dispatch_small_kernel<CH, true><<<1, 64 * kDispWaves, 0, st>>>(topw, topi, (uint16_t*)xp, offsets, src, inv, \
+  moe_dispatch_small_kernel<CH, kSigmoid><<<1, 64 * kDispWaves, 0, st>>>(topw, topi, (uint16_t*)xp, offsets, src, inv, \
                                                                      (const uint16_t*)x, (const uint16_t*)wr, T, E, k, \
                                                                      H, 0, E, MoePro{}, sig)
   switch (H) {
@@ -424,13 +516,15 @@ int moe_mid_max_tokens(int set) {
   return g_mid_max_t;
 }
 
-template <int CH, int kMidTok, bool SIG = false>  // CH 0: any H (SIG)
+template <int CH, int kMidTok, int KIND = kSoftmax>  // CH 0: any H (kSigmoid, kGroups)
 __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
     float* __restrict__ topw, int* __restrict__ topi, int* __restrict__ offsets, int* __restrict__ arow,
     int* __restrict__ inv, const uint16_t* __restrict__ x, const uint16_t* __restrict__ wr, int T, int E, int k,
-    int H, int e0, int n_local, MoePro pro, int* __restrict__ ticket, SigArgs sig = SigArgs{}) {
-  constexpr int ME = SIG ? kSigMaxE : kMaxE;
+    int H, int e0, int n_local, MoePro pro, int* __restrict__ ticket, SigArgs sig = SigArgs{}, ChooseArgs cho = ChooseArgs{}) {
+  constexpr bool SIG = KIND == kSigmoid;
+  constexpr int ME = KIND != kSoftmax ? kSigMaxE : kMaxE;
   __shared__ float lg[kMidTok][ME + SIG];
+  __shared__ float s_gm[KIND == kGroups ? kDispWaves : 1][KIND == kGroups ? kSigMaxE : 1];
   __shared__ int cnt[ME + 1];
   __shared__ int base[ME + 1];
   __shared__ float red[16];
@@ -472,11 +566,12 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
     x = pro.xn;
   }
   // router logits of this workgroup's tokens
-  // SIG: the rows past a whole round of the waves (a gate behind 8 experts, say) are dealt to them by token pairs
-  const int n_rounds = SIG ? sig.rows / kDispWaves * kDispWaves : E;
-  if constexpr (SIG) {
+  // rows past a whole round of the waves (a gate behind 8 experts, say) are dealt to them by token pairs
+  const int n_rows = KIND == kGroups ? cho.n : SIG ? sig.rows : E;
+  const int n_rounds = KIND != kSoftmax ? n_rows / kDispWaves * kDispWaves : E;
+  if constexpr (KIND != kSoftmax) {
     const int pairs = (nt + 1) >> 1;
-    for (int u = wv; u < (sig.rows - n_rounds) * pairs; u += kDispWaves) {
+    for (int u = wv; u < (n_rows - n_rounds) * pairs; u += kDispWaves) {
       const int e = n_rounds + u / pairs, tp = u % pairs * 2;
       float s0, s1;
       dot_rows2(wr + (size_t)e * H, x + (size_t)(t0 + tp) * H, x + (size_t)(t0 + min(tp + 1, nt - 1)) * H, H, lane, s0, s1);
@@ -518,14 +613,23 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
           for (int q = 0; q < 4; ++q)
             acc += lo_bf(a[t][i][q]) * lo_bf(b[i][q]) + hi_bf(a[t][i][q]) * hi_bf(b[i][q]);
         acc = wave_sum(acc);
-        if (lane == 0 && tp + t < nt) lg[tp + t][e] = SIG ? acc : bf2f(f2bf(acc));
+        if (lane == 0 && tp + t < nt) lg[tp + t][e] = KIND != kSoftmax ? acc : bf2f(f2bf(acc));
       }
     }
   }
   __syncthreads();
   const auto rs_topi = __builtin_amdgcn_make_buffer_rsrc((void*)topi, 0, T * k * 4, 0x00020000);
   const auto rs_topw = __builtin_amdgcn_make_buffer_rsrc((void*)topw, 0, T * k * 4, 0x00020000);
-  if (SIG && threadIdx.x < nt) {
+  if constexpr (KIND == kGroups) {
+    for (int t = wv; t < nt; t += kDispWaves) {
+      const float own = choose_groups(cho, lg[t], s_gm[wv], E, k, lane, [&](int j, int e, float s) {
+        const uint32_t at = (uint32_t)(((t0 + t) * k + j) * 4);
+        topw[(t0 + t) * k + j] = s;
+        __builtin_amdgcn_raw_buffer_store_b32(e, rs_topi, at, 0, 16 /* sc1 */);
+      });
+      if (cho.self_w && lane == 0) cho.self_w[t0 + t] = own;
+    }
+  } else if (SIG && threadIdx.x < nt) {
     const int t = threadIdx.x;
     float v = INFINITY;
     int e = -1;
@@ -678,7 +782,7 @@ void launch_moe_dispatch_mid_sigmoid(float* topw, int* topi, int* offsets, int* 
   const SigArgs sig{gate, row_w, rows};
   const int tok = T >= 2048 ? 8 : T >= 512 ? 4 : 2, grid = (T + tok - 1) / tok;
 #define MLOP_DISP_T(CH, TOK)                                                                                           \
-  moe_dispatch_mid_kernel<CH, TOK, true><<<grid, 64 * kDispWaves, 0, st>>>(topw, topi, offsets, arow, inv,               \
+  moe_dispatch_mid_kernel<CH, TOK, kSigmoid><<<grid, 64 * kDispWaves, 0, st>>>(topw, topi, offsets, arow, inv,               \
                                                                            (const uint16_t*)x, (const uint16_t*)wr, T, E, \
                                                                            k, H, 0, E, MoePro{}, ticket, sig)
 #define MLOP_DISP(CH)                       \
@@ -696,8 +800,72 @@ void launch_moe_dispatch_mid_sigmoid(float* topw, int* topi, int* offsets, int* 
 #undef MLOP_DISP_T
 }
 
-// fp32 forms of the sigmoid routing: one thread per token over its logits, the counting sort, a gather that
-// weights the rows, and the experts' products on fp32 FMAs
+void launch_moe_dispatch_small_groups(float* topw, int* topi, void* xp, int* offsets, int* src, int* inv, const void* x,
+                                      const void* wr, int T, int E, int k, int H, const ChooseArgs& cho, hipStream_t st) {
+#define MLOP_DISP(CH)                                                                                               \
+  moe_dispatch_small_kernel<CH, kGroups><<<1, 64 * kDispWaves, 0, st>>>(topw, topi, (uint16_t*)xp, offsets, src, inv, \
+                                                                        (const uint16_t*)x, (const uint16_t*)wr, T, E, k, \
+                                                                        H, 0, E, MoePro{}, SigArgs{}, cho)
+  switch (H) {
+    case 1024: MLOP_DISP(2); break;
+    case 2048: MLOP_DISP(4); break;
+    case 4096: MLOP_DISP(8); break;
+    case 8192: MLOP_DISP(16); break;
+    default: MLOP_DISP(0); break;
+  }
+#undef MLOP_DISP
+}
+
+void launch_moe_dispatch_mid_groups(float* topw, int* topi, int* offsets, int* arow, int* inv, const void* x, const void* wr,
+                                    int T, int E, int k, int H, const ChooseArgs& cho, hipStream_t st) {
+  float* ws = nullptr;
+  int* ticket = nullptr;
+  int cus = 0;
+  if (!gemm_sk_scratch(&ws, &ticket, &cus)) throw std::runtime_error("moe_dispatch_mid: stream-K scratch not reserved");
+  const int tok = T >= 2048 ? 8 : T >= 512 ? 4 : 2, grid = (T + tok - 1) / tok;
+#define MLOP_DISP_T(CH, TOK)                                                                                             \
+  moe_dispatch_mid_kernel<CH, TOK, kGroups><<<grid, 64 * kDispWaves, 0, st>>>(topw, topi, offsets, arow, inv,              \
+                                                                              (const uint16_t*)x, (const uint16_t*)wr, T, E, \
+                                                                              k, H, 0, E, MoePro{}, ticket, SigArgs{}, cho)
+#define MLOP_DISP(CH)                       \
+  if (tok == 8) MLOP_DISP_T(CH, 8);         \
+  else if (tok == 4) MLOP_DISP_T(CH, 4);    \
+  else MLOP_DISP_T(CH, 2);
+  switch (H) {
+    case 1024: MLOP_DISP(2); break;
+    case 2048: MLOP_DISP(4); break;
+    case 4096: MLOP_DISP(8); break;
+    case 8192: MLOP_DISP(16); break;
+    default: MLOP_DISP(0); break;
+  }
+#undef MLOP_DISP
+#undef MLOP_DISP_T
+}
+
+// fp32 forms of the sigmoid and the grouped routing: one thread (wave) per token over its logits, the counting sort, a
+// gather that may weight the rows, and the experts' products on fp32 FMAs
+__global__ void __launch_bounds__(256) moe_route_groups_kernel(float* __restrict__ topw, int* __restrict__ topi,
+                                                              const float* __restrict__ logits, int T, int E, int k,
+                                                              ChooseArgs cho) {
+  __shared__ float z[4][kSigMaxE], gm[4][kSigMaxE];
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, t = blockIdx.x * 4 + wv;
+  if (t >= T) return;  // whole waves; no barrier below
+  for (int e = lane; e < cho.n; e += 64) z[wv][e] = logits[(size_t)t * cho.n + e];
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+  __builtin_amdgcn_wave_barrier();
+  const float own = choose_groups(cho, z[wv], gm[wv], E, k, lane, [&](int j, int e, float s) {
+    topi[t * k + j] = e;
+    topw[t * k + j] = s;
+  });
+  if (cho.self_w && lane == 0) cho.self_w[t] = own;
+}
+
+void launch_moe_route_groups(float* topw, int* topi, const float* logits, int T, int E, int k, const ChooseArgs& cho,
+                             hipStream_t st) {
+  if (T == 0) return;
+  moe_route_groups_kernel<<<(T + 3) / 4, 256, 0, st>>>(topw, topi, logits, T, E, k, cho);
+}
+
 __global__ void __launch_bounds__(128) moe_route_sigmoid_kernel(float* __restrict__ topw, int* __restrict__ topi,
                                                                float* __restrict__ gate, const float* __restrict__ logits,
                                                                int T, int E, int rows, int k) {
@@ -726,7 +894,7 @@ __global__ void __launch_bounds__(256) moe_gather_scaled_kernel(float* __restric
   const int r = blockIdx.x;
   if (r >= offsets[n_local]) return;
   const int s = src[r];
-  const float w = topw[s];
+  const float w = topw ? topw[s] : 1.f;
   for (int c = threadIdx.x; c < H; c += blockDim.x) xp[(size_t)r * H + c] = w * x[(size_t)(s / k) * H + c];
 }
 

@@ -229,4 +229,149 @@ void launch_qk_norm(const QkNormArgs& a, bool f32, hipStream_t st) {
   else run_qk<uint16_t>(a, st);
 }
 
+// Per-head form: every query and key head divided by its own root mean square, one weight for all of them; the
+// values are columns of their own or the keys as given.  Vector kernel: LPH lanes of a wave hold a head's 8-element
+// vectors in registers from the sum of squares to the stores, HPT heads of one token in turn (fetched together).
+template <typename E, int LPH, int HPT>
+__global__ void __launch_bounds__(256) qk_head_norm_vec_kernel(QkHeadNormArgs a) {
+  const int units = cdiv(a.H + a.G, HPT), c = threadIdx.x % LPH * 8;
+  const long unit = (long)blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
+  if (unit >= (long)a.T * units) return;  // whole groups of lanes; no barrier below
+  const int t = (int)(unit / units), h0 = (int)(unit % units) * HPT;
+  const bool in = c < a.D;
+  const E* qr = reinterpret_cast<const E*>(a.q) + (size_t)t * a.ldq;
+  const E* kr = reinterpret_cast<const E*>(a.k) + (size_t)t * a.ldk;
+  float x[HPT][8];
+#pragma unroll
+  for (int i = 0; i < HPT; ++i) {
+    const int h = min(h0 + i, a.H + a.G - 1);
+    ldn<8>((h < a.H ? qr + h * a.D : kr + (h - a.H) * a.D) + (in ? c : 0), x[i]);
+  }
+  // the weights, cos and sin fetched beside the heads, unconditionally (clamped)
+  float qw[8], kw[8], co[4], si[4];
+  ldn<8>(a.q_w + (in ? c : 0), qw);
+  ldn<8>(a.k_w + (in ? c : 0), kw);
+  const int half = a.R >> 1;
+  const float* cs = a.cos_sin + (size_t)a.pos[t] * a.R;
+  if (a.R % 8 == 0) {
+    const int o = c < a.R ? c >> 1 : 0;
+    if (a.R) {
+      ldn<4>(cs + o, co);
+      ldn<4>(cs + half + o, si);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) co[e] = c < a.R ? co[e] : 1.f, si[e] = c < a.R ? si[e] : 0.f;
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const bool r = c + 2 * e < a.R;
+      co[e] = r ? cs[(c >> 1) + e] : 1.f;
+      si[e] = r ? cs[half + (c >> 1) + e] : 0.f;
+    }
+  }
+  const int slot = a.slots[t], blk = slot >= 0 ? slot / a.BS : 0, off = slot - blk * a.BS;
+#pragma unroll
+  for (int i = 0; i < HPT; ++i) {
+    const int h = h0 + i, g = h - a.H;
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s = fmaf(x[i][e], x[i][e], s);
+    s = in ? s : 0.f;
+    s += detail::dpp<0xB1>(s);
+    s += detail::dpp<0x4E>(s);
+    s += detail::dpp<0x141>(s);  // 8 lanes
+    if constexpr (LPH >= 16) s += detail::dpp<0x140>(s);
+    if constexpr (LPH >= 32) s += __shfl_xor(s, 16);
+    if constexpr (LPH >= 64) s += __shfl_xor(s, 32);
+    if (h >= a.H + a.G || (g >= 0 && slot < 0)) continue;
+    const float inv = 1.f / sqrtf(s / (float)a.D + a.eps);
+    float o[8];
+#pragma unroll
+    for (int e = 0; e < 8; e += 2) {
+      const float u = x[i][e] * inv * (g < 0 ? qw[e] : kw[e]), y = x[i][e + 1] * inv * (g < 0 ? qw[e + 1] : kw[e + 1]);
+      o[e] = u * co[e >> 1] - y * si[e >> 1];
+      o[e + 1] = y * co[e >> 1] + u * si[e >> 1];
+    }
+    if (g < 0) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[e] = in ? o[e] : 0.f;
+      if (c < a.KP) stn<8>(reinterpret_cast<E*>(a.q_out) + ((size_t)t * a.H + h) * a.KP + c, o);
+      continue;
+    }
+    const size_t line = ((size_t)blk * a.G + g) * a.BS + off;
+    if (in) stn<8>(reinterpret_cast<E*>(a.k_cache) + line * a.KP + c, o);
+    E* vo = reinterpret_cast<E*>(a.v_cache) + line * a.VP;
+    if (!a.v) {
+      if (in) stn<8>(vo + c, x[i]);
+    } else {
+      const E* vr = reinterpret_cast<const E*>(a.v) + (size_t)t * a.ldv + (size_t)g * a.V;
+      for (int e = threadIdx.x % LPH; e < a.V; e += LPH) st1(vo + e, ld1(vr + e));
+    }
+  }
+}
+
+// any head size and alignment: a wave per (token, head)
+template <typename E>
+__global__ void __launch_bounds__(256) qk_head_norm_any_kernel(QkHeadNormArgs a) {
+  const int lane = threadIdx.x & 63;
+  const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (unit >= (long)a.T * (a.H + a.G)) return;
+  const int t = (int)(unit / (a.H + a.G)), h = (int)(unit % (a.H + a.G)), g = h - a.H;
+  const E* src = g < 0 ? reinterpret_cast<const E*>(a.q) + (size_t)t * a.ldq + (size_t)h * a.D
+                       : reinterpret_cast<const E*>(a.k) + (size_t)t * a.ldk + (size_t)g * a.D;
+  float s = 0.f;
+  for (int d = lane; d < a.D; d += 64) {
+    const float x = ld1(src + d);
+    s = fmaf(x, x, s);
+  }
+  const float inv = 1.f / sqrtf(wave_sum(s) / (float)a.D + a.eps);
+  const float* w = g < 0 ? a.q_w : a.k_w;
+  const float* cs = a.cos_sin + (size_t)a.pos[t] * a.R;
+  auto turned = [&](int d) {
+    const float x = ld1(src + d) * inv * w[d];
+    if (d >= a.R) return x;
+    const float y = ld1(src + (d ^ 1)) * inv * w[d ^ 1], co = cs[d >> 1], si = cs[(a.R >> 1) + (d >> 1)];
+    return d & 1 ? x * co + y * si : x * co - y * si;
+  };
+  if (g < 0) {
+    E* q = reinterpret_cast<E*>(a.q_out) + ((size_t)t * a.H + h) * a.KP;
+    for (int d = lane; d < a.KP; d += 64) st1(q + d, d < a.D ? turned(d) : 0.f);
+    return;
+  }
+  const int slot = a.slots[t];
+  if (slot < 0) return;
+  const size_t line = ((size_t)(slot / a.BS) * a.G + g) * a.BS + slot % a.BS;
+  E* ko = reinterpret_cast<E*>(a.k_cache) + line * a.KP;
+  E* vo = reinterpret_cast<E*>(a.v_cache) + line * a.VP;
+  for (int d = lane; d < a.D; d += 64) st1(ko + d, turned(d));
+  const E* vr = a.v ? reinterpret_cast<const E*>(a.v) + (size_t)t * a.ldv + (size_t)g * a.V : src;
+  for (int d = lane; d < a.V; d += 64) st1(vo + d, ld1(vr + d));
+}
+
+template <typename E>
+static void run_qk_head(const QkHeadNormArgs& a, hipStream_t st) {
+  const bool al = ((reinterpret_cast<uintptr_t>(a.q) | reinterpret_cast<uintptr_t>(a.k)) & 15) == 0;
+  if (al && a.D % 8 == 0 && a.ldq % 8 == 0 && a.ldk % 8 == 0 && a.KP <= 512 && a.VP % 8 == 0) {
+    const int HPT = a.T >= 1024 ? 4 : 1;
+#define MLOP_QKH_N(LPH, N) \
+  qk_head_norm_vec_kernel<E, LPH, N><<<(int)(((long)a.T * cdiv(a.H + a.G, N) * LPH + 255) / 256), 256, 0, st>>>(a)
+#define MLOP_QKH(LPH) \
+  if (HPT == 4) MLOP_QKH_N(LPH, 4); else MLOP_QKH_N(LPH, 1)
+    if (a.KP <= 64) { MLOP_QKH(8); }
+    else if (a.KP <= 128) { MLOP_QKH(16); }
+    else if (a.KP <= 256) { MLOP_QKH(32); }
+    else { MLOP_QKH(64); }
+#undef MLOP_QKH
+#undef MLOP_QKH_N
+  } else {
+    qk_head_norm_any_kernel<E><<<(int)(((long)a.T * (a.H + a.G) + 3) / 4), 256, 0, st>>>(a);
+  }
+}
+
+void launch_qk_head_norm(const QkHeadNormArgs& a, bool f32, hipStream_t st) {
+  if (a.T == 0) return;
+  if (f32) run_qk_head<float>(a, st);
+  else run_qk_head<uint16_t>(a, st);
+}
+
 }  // namespace mlop

@@ -2,7 +2,8 @@
 // elementwise steps such decoders use:
 //
 //   residual    x <- x + post_w * y / rms(y)   (or x + y),   xn = norm_w * x / rms(x)   (or x)
-//               where y may be a token's expert rows summed, beside a gated shared row
+//               where y may be a token's expert rows summed (weighted, with the token's own input as one of
+//               them), beside a gated shared row; or xn = norm_w * tanh(alpha x) + b (dynamic tanh: no statistics)
 //   gated norm  group norm of y with a gate before or behind it
 //   clamp_glu   clamped gated unit of a feed-forward's [gate | up] columns
 //
@@ -56,6 +57,12 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
       }
     }
   }
+  float nb[NI][VEC];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int c = (tid + BT * i) * VEC;
+    if (a.tanh_a && c < W) ldn<VEC>(a.tanh_b + c, nb[i]);
+  }
   if constexpr (KIND == kExperts) {
     if (a.gate) {
       const float g = a.gate[row];
@@ -64,10 +71,7 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
 #pragma unroll
         for (int e = 0; e < VEC; ++e) y[i][e] *= g;
     }
-    const int* inv = a.inv + (size_t)row * a.top;
-#pragma unroll 2
-    for (int j = 0; j < a.top; ++j) {
-      const E* er = reinterpret_cast<const E*>(a.rows) + (size_t)inv[j] * W;
+    auto add = [&](const E* er, float w) {
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
         const int c = (tid + BT * i) * VEC;
@@ -75,9 +79,20 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
           float v[VEC];
           ldn<VEC>(er + c, v);
 #pragma unroll
-          for (int e = 0; e < VEC; ++e) y[i][e] += v[e];
+          for (int e = 0; e < VEC; ++e) y[i][e] = fmaf(w, v[e], y[i][e]);
         }
       }
+    };
+    const int* inv = a.inv + (size_t)row * a.top;
+    const float* row_w = a.row_w + (a.row_w ? (size_t)row * a.top : 0);
+#pragma unroll 2
+    for (int j = 0; j < a.top; ++j) {
+      if (inv[j] < 0) continue;
+      add(reinterpret_cast<const E*>(a.rows) + (size_t)inv[j] * W, a.row_w ? row_w[j] : 1.f);
+    }
+    if (a.self) {
+      const float w = a.self_w[row];
+      if (w != 0.f) add(reinterpret_cast<const E*>(a.self) + (size_t)row * W, w);
     }
   }
   if constexpr (!START) {
@@ -106,8 +121,21 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
       for (int e = 0; e < VEC; ++e) ss = fmaf(x[i][e], x[i][e], ss);
     }
   }
-  const float inv = a.norm_w ? 1.f / sqrtf(block_sum(ss, scratch) / (float)a.n + a.eps) : 1.f;
   E* xn = reinterpret_cast<E*>(a.xn) + (size_t)row * W;
+  if (a.tanh_a) {
+    const float alpha = *a.tanh_a;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int c = (tid + BT * i) * VEC;
+      if (c < W) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) x[i][e] = fmaf(tanhf(alpha * x[i][e]), nw[i][e], nb[i][e]);
+        stn<VEC>(xn + c, x[i]);
+      }
+    }
+    return;
+  }
+  const float inv = a.norm_w ? 1.f / sqrtf(block_sum(ss, scratch) / (float)a.n + a.eps) : 1.f;
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int c = (tid + BT * i) * VEC;

@@ -133,6 +133,11 @@ def xielu(x, a, b):
     return (torch.where(z > 0, a * z * z, b * (torch.expm1(z.clamp(max=0)) - z)) + 0.5 * z).to(x.dtype)
 
 
+def gelu_tanh(x):
+    v = x.float()
+    return (0.5 * v * (1 + torch.tanh(math.sqrt(2 / math.pi) * (v + 0.044715 * v ** 3)))).to(x.dtype)
+
+
 def softcap(x, cap):
     return cap * torch.tanh(x.float() / cap)
 
@@ -173,7 +178,20 @@ def _live_rows(meta):
     return [(r, qs[r], ql[r], cl[r]) for r in sorted(rows) if ql[r] and cl[r]]
 
 
-def attention_hd(q, k_cache, v_cache, meta, D, V, scale, sink, gate):
+def qk_head_norm(q, k, v, H, D, V, q_w, k_w, eps, cos_sin, positions, slots, k_cache, v_cache):
+    T, G, half = q.shape[0], k_cache.shape[1], cos_sin.shape[1] // 2
+    cs = cos_sin[positions.long()]
+    turn = lambda x, n, w: rotate_pairs(_unit(x.float().reshape(T, n, D), eps) * w, cs[:, :half], cs[:, half:]).to(q.dtype)  # noqa: E731
+    out = torch.zeros(T, H, k_cache.shape[3], dtype=q.dtype, device=q.device)
+    out[:, :, :D] = turn(q, H, q_w)
+    keep, BS = slots >= 0, k_cache.shape[2]
+    s = slots[keep].long()
+    k_cache[s // BS, :, s % BS, :D] = turn(k, G, k_w)[keep]
+    v_cache[s // BS, :, s % BS, :V] = (k if v is None else v).reshape(T, G, V)[keep].to(v_cache.dtype)
+    return out
+
+
+def attention_hd(q, k_cache, v_cache, meta, D, V, scale, sink, gate, window=0):
     T, H = q.shape[:2]
     G = k_cache.shape[1]
     out = torch.zeros(T, H, V, dtype=torch.float32, device=q.device)
@@ -183,13 +201,15 @@ def attention_hd(q, k_cache, v_cache, meta, D, V, scale, sink, gate):
         v = v[..., :V].float().repeat_interleave(H // G, 1)
         w = torch.einsum("qhd,khd->hqk", q[s:s + n, :, :D].float(), k) * scale
         pos = torch.arange(ctx - n, ctx, device=q.device)[:, None]
-        w = w.masked_fill((torch.arange(ctx, device=q.device)[None] > pos)[None], float("-inf"))
+        keys = torch.arange(ctx, device=q.device)[None]
+        hidden = (keys > pos) | (keys <= pos - window) if window else keys > pos
+        w = w.masked_fill(hidden[None], float("-inf"))
         if sink is not None:
             w = torch.cat([w, sink.float().view(H, 1, 1).expand(H, n, 1)], -1)
         p = torch.softmax(w, -1)[..., :ctx]
         out[s:s + n] = torch.einsum("hqk,khd->qhd", p, v)
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())[..., None]
+        out = out * torch.sigmoid(gate.float()).view(T, H, -1)
     return out.to(q.dtype)
 
 
@@ -218,23 +238,32 @@ def _unit_n(x, eps, width):
     return x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) / (width or x.shape[-1]) + eps)
 
 
-def residual_begin(ids, table, scale, pos_table, positions, norm_w, eps, width=None):
+def _next_input(x, norm_w, eps, width, tanh):
+    if tanh is not None:
+        return norm_w * torch.tanh(tanh[0] * x) + tanh[1]
+    return x if norm_w is None else _unit_n(x, eps, width) * norm_w
+
+
+def residual_begin(ids, table, scale, pos_table, positions, norm_w, eps, width=None, tanh=None):
     x = table[ids.reshape(-1).long()].float() * scale
     if pos_table is not None:
         x = x + pos_table[positions.long()].float()
-    return x, (x if norm_w is None else _unit_n(x, eps, width) * norm_w).to(table.dtype)
+    return x, _next_input(x, norm_w, eps, width, tanh).to(table.dtype)
 
 
-def residual_step(x, y, post_w, norm_w, eps, width=None, experts=None):
+def residual_step(x, y, post_w, norm_w, eps, width=None, experts=None, share=None, tanh=None):
     dtype = y.dtype if experts is None else experts[0].dtype
     out = y.float() if y is not None else torch.zeros_like(x)
     if experts is not None:
         rows, inv, gate = experts
         if gate is not None:
             out = out * gate[:, None]
-        out = out + rows.float()[inv.long()].sum(1)
+        w = (inv >= 0).float() if share is None else share[0] * (inv >= 0)
+        out = out + (rows.float()[inv.long().clamp(min=0)] * w[..., None]).sum(1)
+        if share is not None and share[1] is not None:
+            out = out + share[2][:, None] * share[1].float()
     x.add_(_unit_n(out, eps, width) * post_w if post_w is not None else out)
-    return (x if norm_w is None else _unit_n(x, eps, width) * norm_w).to(dtype)
+    return _next_input(x, norm_w, eps, width, tanh).to(dtype)
 
 
 def gated_norm(y, gate, w, groups, eps, silu, gate_first):
@@ -370,6 +399,19 @@ def moe_route_sigmoid(logits, E, top_k):
     s = torch.sigmoid(logits.float())
     w, idx = torch.topk(s[:, :E], top_k, dim=-1)
     return w, idx.to(torch.int32), s[:, E].contiguous() if s.shape[1] > E else None
+
+
+def moe_route_groups(logits, correction, E, top_k, groups, keep):
+    """fp32 logits [T, n] -> (weights, experts [T, k], weight of the outputs past the E experts per token or None)."""
+    T, n = logits.shape
+    s = torch.softmax(logits.float(), -1)
+    choice = s if correction is None else s + correction
+    best = choice.view(T, groups, -1).amax(-1)
+    kept = torch.zeros_like(best, dtype=torch.bool).scatter_(1, torch.topk(best, keep, -1).indices, True)
+    choice = choice.masked_fill(~kept.repeat_interleave(n // groups, 1), float("-inf"))
+    idx = torch.topk(choice, top_k, -1).indices
+    w = s.gather(1, idx)
+    return w, idx.to(torch.int32), (w * (idx >= E)).sum(-1) if n > E else None
 
 
 def moe_permute(x, topi, e0, n_local):
