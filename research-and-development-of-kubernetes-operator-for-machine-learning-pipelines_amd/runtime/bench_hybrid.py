@@ -1,8 +1,8 @@
 """Prefill and decode throughput of the hybrid designs beside the closest models of the package, at
 equal layer sizes (``bench.py --hybrid``).
 
-Each size has a Nafazen, a Regesun and a Kosesun preset cut to a few layers, a Mixtral with the Nafazen's
-experts and a Llama, all of the same width, layer count and vocabulary, the dense ones of the same
+Each size has a Dibedra, a Nafazen, a Regesun and a Kosesun preset cut to a few layers, a Mixtral with the
+Nafazen's experts and a Llama, all of the same width, layer count and vocabulary, the dense ones of the same
 feed-forward parameters.  All run through the engine's own scheduler
 (``add_request`` / ``step``; decode replays the captured graphs), random weights, random prompts,
 greedy sampling.  One JSON line per (model, workload); ``--hybrid-kernels`` adds each kernel's share
@@ -35,6 +35,7 @@ def sizes() -> list:
                  num_kv_heads=4)
     r8, r1 = get_config("regesun-8b", num_layers=LAYERS), get_config("regesun-1b", num_layers=LAYERS)
     n8, n1 = get_config("nafazen-8b", num_layers=LAYERS), get_config("nafazen-1b", num_layers=LAYERS)
+    d8, d1 = get_config("dibedra-8b", num_layers=LAYERS), get_config("dibedra-1b", num_layers=LAYERS)
 
     def mixtral(name, like, of):  # the experts of ``like`` in every layer, attention and vocabulary of ``of``
         e = like.layers[1].moe
@@ -43,8 +44,8 @@ def sizes() -> list:
                        top_k=e.top)
 
     m8, m1 = mixtral("mixtral-8b", n8, l8), mixtral("mixtral-1b", n1, l1)
-    return [("8b", *(replace(c, max_position=16384) for c in (n8, r8, k8, m8, l8))),
-            ("1b", *(replace(c, max_position=16384) for c in (n1, r1, k1, m1, l1)))]
+    return [("8b", *(replace(c, max_position=16384) for c in (d8, n8, r8, k8, m8, l8))),
+            ("1b", *(replace(c, max_position=16384) for c in (d1, n1, r1, k1, m1, l1)))]
 
 
 def _kernels(fn) -> list:
