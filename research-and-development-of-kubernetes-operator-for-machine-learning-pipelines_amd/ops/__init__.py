@@ -1080,7 +1080,7 @@ def moe_dispatch_groups(x, router, correction, n_experts: int, top_k: int, group
     topw = torch.empty(T, top_k, dtype=torch.float32, device=dev)
     self_w = torch.empty(T, dtype=torch.float32, device=dev) if n > n_experts else None
     choice = (correction, n_experts, groups, keep)
-    if x.dtype == torch.float32 or T <= 16:  # rows gathered
+    if x.dtype == torch.float32 or T * top_k <= 8:  # rows gathered
         xp, src = torch.empty(T * top_k, x.shape[1], dtype=x.dtype, device=dev), i32(T * top_k)
         if x.dtype == torch.float32:
             torch.ops.mlop.moe_route_groups(topw, topi, self_w, gemm(x, router), *choice)

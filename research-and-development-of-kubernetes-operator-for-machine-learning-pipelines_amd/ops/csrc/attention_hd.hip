@@ -578,14 +578,32 @@ __global__ void __launch_bounds__(256, (NKB + NVB) <= 5 ? 2 : 1) flash_hd_kernel
   const float inv = l > 0.f ? f * gate_of(a, qs + qi, head) / l : 0.f;
   // O^T element e of dim block d is dim 32 d + 8 (e >> 2) + 4 h + (e & 3) of this lane's row
   uint16_t* orow = reinterpret_cast<uint16_t*>(a.out) + (size_t)(qs + qi) * a.out_row + head * a.V;
-  const bool v4 = a.V % 4 == 0;
+  const bool v4 = a.V % 4 == 0, gv = a.gate && a.gate_elem && a.gate_vec;
+  // the gates of all elements are fetched together, ahead of the stores
+  u32x2 z[ND][4];
+  if (gv) {
+    const uint16_t* g = reinterpret_cast<const uint16_t*>(a.gate) + (size_t)(qs + qi) * a.gate_stride + head * a.V;
+#pragma unroll
+    for (int d = 0; d < ND; ++d)
+#pragma unroll
+      for (int b = 0; b < 4; ++b) {
+        const int c = 32 * d + 8 * b + 4 * h;
+        z[d][b] = *reinterpret_cast<const u32x2*>(g + (c < a.V ? c : 0));
+      }
+  }
 #pragma unroll
   for (int d = 0; d < ND; ++d)
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
       const int c = 32 * d + 8 * b + 4 * h;
       float v[4] = {o[d][4 * b] * inv, o[d][4 * b + 1] * inv, o[d][4 * b + 2] * inv, o[d][4 * b + 3] * inv};
-      gate_elems(a, qs + qi, head, c, v);
+      if (gv) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          v[j] *= __builtin_amdgcn_rcpf(1.f + __expf(-(j & 1 ? hi_bf(z[d][b][j >> 1]) : lo_bf(z[d][b][j >> 1]))));
+      } else {
+        gate_elems(a, qs + qi, head, c, v);
+      }
       if (v4) {
         if (c < a.V) stn<4>(orow + c, v);
       } else {

@@ -129,7 +129,15 @@ __device__ __forceinline__ float silu_bf(float g) {
 __device__ __forceinline__ float clamp_glu_f(float g, float u, float alpha, float limit) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
-  return g * (u + 1.f) / (1.f + __expf(-alpha * g));
+  return g * (u + 1.f) * __builtin_amdgcn_rcpf(1.f + __expf(-alpha * g));
+}
+
+// tanh to a few ulp: odd polynomial around zero, (1 - e) / (1 + e) with e = exp(-2 |x|) elsewhere
+__device__ __forceinline__ float tanh_f(float x) {
+  const float a = fabsf(x), q = x * x, e = __expf(-2.f * a);
+  const float p = fmaf(q, fmaf(q, fmaf(q, fmaf(q, fmaf(q, -8.863235529902197e-3f, 2.186948853615520e-2f), -5.396825396825397e-2f),
+                                       1.333333333333333e-1f), -3.333333333333333e-1f), 1.f);
+  return a < 0.4f ? x * p : copysignf((1.f - e) * __builtin_amdgcn_rcpf(1.f + e), x);
 }
 
 // tanh gelu: x / 2 (1 + tanh(u)) = x / (1 + exp(-2 u)), u = sqrt(2 / pi) (x + 0.044715 x^3)

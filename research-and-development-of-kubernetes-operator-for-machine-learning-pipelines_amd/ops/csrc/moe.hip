@@ -179,15 +179,10 @@ __device__ __forceinline__ void next_best(const float* z, int n, float& v, int& 
   i = min(bi, n - 1);
 }
 
-// kGroups, one wave: scores of one token's n logits z (in LDS, overwritten by the choice scores), the top k of them
-// through put(j, output, score).  gm: LDS, groups floats.  Returns the weights of outputs from E on, added up.
-template <typename F>
+// kGroups, one wave: scores of one token's n <= 64 PER logits z (LDS, overwritten by the choice scores if PER > 1), the
+// top k of them through put(j, output, score).  gm: LDS, groups floats.  Returns the weights of outputs from E on, added up.
+template <int PER, typename F>
 __device__ __forceinline__ float choose_groups(const ChooseArgs& c, float* z, float* gm, int E, int k, int lane, F&& put) {
-  constexpr int PER = kSigMaxE / 64;
-  auto lds_fence = [] {
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
-    __builtin_amdgcn_wave_barrier();
-  };
   float s[PER], ch[PER], mx = -INFINITY, sum = 0.f;
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
@@ -201,48 +196,69 @@ __device__ __forceinline__ float choose_groups(const ChooseArgs& c, float* z, fl
     s[i] = expf(s[i] - mx);
     sum += s[i];
   }
-  sum = wave_sum(sum);
+  const float inv = 1.f / wave_sum(sum);
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
     const int e = lane + 64 * i;
-    s[i] /= sum;
+    s[i] *= inv;
     ch[i] = e < c.n ? s[i] + (c.correction ? c.correction[e] : 0.f) : -INFINITY;
   }
   if (c.keep < c.groups) {
+    // an output stays if fewer than `keep` groups come ahead of its own (ties: the lower group)
     const int size = c.n / c.groups;
+    if constexpr (PER == 1) {
+      const int mine = lane / size;
+      float best = -INFINITY, own = -INFINITY;  // lane g: group g's best; and the own group's
+      for (int g = 0; g < c.groups; ++g) {
+        const float m = wave_max(mine == g ? ch[0] : -INFINITY);
+        best = lane == g ? m : best;
+        own = mine == g ? m : own;
+      }
+      int before = 0;
+      for (int g = 0; g < c.groups; ++g) {
+        const float m = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(best), g));
+        before += m > own || (m == own && g < mine);
+      }
+      if (before >= c.keep) ch[0] = -INFINITY;
+    } else {
+      auto lds_fence = [] {
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+        __builtin_amdgcn_wave_barrier();
+      };
 #pragma unroll
-    for (int i = 0; i < PER; ++i)
-      if (lane + 64 * i < c.n) z[lane + 64 * i] = ch[i];
-    lds_fence();
-    for (int g = lane; g < c.groups; g += 64) {
-      float m = -INFINITY;
-      for (int e = 0; e < size; ++e) m = fmaxf(m, z[g * size + e]);
-      gm[g] = m;
-    }
-    lds_fence();
+      for (int i = 0; i < PER; ++i)
+        if (lane + 64 * i < c.n) z[lane + 64 * i] = ch[i];
+      lds_fence();
+      for (int g = lane; g < c.groups; g += 64) {
+        float m = -INFINITY;
+        for (int e = 0; e < size; ++e) m = fmaxf(m, z[g * size + e]);
+        gm[g] = m;
+      }
+      lds_fence();
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int e = lane + 64 * i;
-      if (e >= c.n) continue;
-      const int g = e / size;
-      int before = 0;  // groups ahead of this output's
-      for (int o = 0; o < c.groups; ++o) before += gm[o] > gm[g] || (gm[o] == gm[g] && o < g);
-      if (before >= c.keep) ch[i] = -INFINITY;
+      for (int i = 0; i < PER; ++i) {
+        const int e = lane + 64 * i;
+        if (e >= c.n) continue;
+        const int g = e / size;
+        const float own = gm[g];
+        int before = 0;
+        for (int o = 0; o < c.groups; ++o) before += gm[o] > own || (gm[o] == own && o < g);
+        if (before >= c.keep) ch[i] = -INFINITY;
+      }
     }
   }
   float own = 0.f;
   for (int j = 0; j < k; ++j) {
-    float bv = -INFINITY;
-    int be = c.n;
+    float bv = ch[0];
 #pragma unroll
-    for (int i = 0; i < PER; ++i)
-      if (ch[i] > bv) bv = ch[i], be = lane + 64 * i;
-    for (int o = 1; o < 64; o <<= 1) {
-      const float v = __shfl_xor(bv, o);
-      const int e = __shfl_xor(be, o);
-      if (v > bv || (v == bv && e < be)) bv = v, be = e;
+    for (int i = 1; i < PER; ++i) bv = fmaxf(bv, ch[i]);
+    bv = wave_max(bv);
+    int be = j;  // (no number is the largest: any output)
+#pragma unroll
+    for (int i = PER - 1; i >= 0; --i) {
+      const unsigned long long at = __ballot(ch[i] == bv && lane + 64 * i < c.n);
+      if (at) be = 64 * i + __builtin_ctzll(at);
     }
-    be = min(be, c.n - 1);
 #pragma unroll
     for (int i = 0; i < PER; ++i)
       if (be == lane + 64 * i) {
@@ -252,6 +268,50 @@ __device__ __forceinline__ float choose_groups(const ChooseArgs& c, float* z, fl
       }
   }
   return wave_sum(own);
+}
+
+template <typename F>
+__device__ __forceinline__ float choose_groups(const ChooseArgs& c, float* z, float* gm, int E, int k, int lane, F&& put) {
+  return c.n <= 64 ? choose_groups<1>(c, z, gm, E, k, lane, put) : choose_groups<kSigMaxE / 64>(c, z, gm, E, k, lane, put);
+}
+
+// kGroups: logits lg [nt <= 16 tokens][n <= 16 NT outputs] on the matrix cores, rows of H (a multiple of 64) elements.
+// The waves take 64 columns in turn; their partial sums meet in red (LDS).  Ends with a barrier behind its last write.
+template <int NT, int LD>
+__device__ __forceinline__ void router_tile(const uint16_t* x, int nt, const uint16_t* w, int n, int H, float (*lg)[LD],
+                                            float (*red)[16][16 * NT + 1]) {
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, r = lane & 15, g = lane >> 4;
+  const uint16_t* xr = x + (size_t)min(r, nt - 1) * H + g * 8;
+  const uint16_t* wr[NT];
+  f32x4 acc[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) {
+    wr[i] = w + (size_t)min(16 * i + r, n - 1) * H + g * 8;
+    acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  constexpr int U = NT > 2 ? 1 : 4 / NT;  // loads of U x 64 columns in flight
+#pragma unroll U
+  for (int k = 64 * wv; k < H; k += 64 * kDispWaves) {
+#pragma unroll
+    for (int kk = 0; kk < 64; kk += 32) {
+      const bf16x8 a = *reinterpret_cast<const bf16x8*>(xr + k + kk);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) acc[i] = mfma16(a, *reinterpret_cast<const bf16x8*>(wr[i] + k + kk), acc[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) red[wv][4 * g + j][16 * i + r] = acc[i][j];
+  __syncthreads();
+  for (int u = threadIdx.x; u < nt * n; u += 64 * kDispWaves) {
+    const int t = u / n, e = u % n;
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < kDispWaves; ++i) sum += red[i][t][e];
+    lg[t][e] = sum;
+  }
+  __syncthreads();
 }
 
 // router logits of two token rows, any row length (a multiple of 8)
@@ -333,7 +393,7 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
       continue;
     }
     const uint16_t* we = wr + (size_t)e * H + lane * 8;
-    constexpr int CN = CH ? CH : 1;
+    constexpr int CN = CH > 0 ? CH : 1;
     u32x4 b[CN];
 #pragma unroll
     for (int i = 0; i < CH; ++i) b[i] = *reinterpret_cast<const u32x4*>(we + i * 512);
@@ -404,7 +464,35 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_small_kernel(
   __syncthreads();
   // 3. counting sort of the T*k slots by local expert (moe_sort_kernel), slot order kept
   const int n_slots = T * k;
-  if (threadIdx.x == 0) {
+  if constexpr (KIND == kGroups) {  // any order inside an expert: no value depends on it
+    constexpr int PER = kSmallT * kSigMaxTop / (64 * kDispWaves);
+    int rank[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int s = threadIdx.x + 64 * kDispWaves * i, e = s < n_slots ? s_topi[s] : E;
+      rank[i] = e < E ? atomicAdd(&cnt[e], 1) : -1;
+    }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+      int acc = 0;
+      for (int e = 0; e < E; ++e) {
+        base[e] = acc;
+        offsets[e] = acc;
+        acc += cnt[e];
+      }
+      offsets[E] = acc;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int s = threadIdx.x + 64 * kDispWaves * i;
+      if (s >= n_slots) continue;
+      const int row = rank[i] < 0 ? -1 : base[s_topi[s]] + rank[i];
+      inv[s] = row;
+      if (row >= 0) src[row] = s;
+      s_topi[s] = row;
+    }
+  } else if (threadIdx.x == 0) {
     for (int s = 0; s < n_slots; ++s) {
       const int e = s_topi[s] - e0;
       if (e >= 0 && e < n_local) ++cnt[e];
@@ -516,8 +604,8 @@ int moe_mid_max_tokens(int set) {
   return g_mid_max_t;
 }
 
-template <int CH, int kMidTok, int KIND = kSoftmax>  // CH 0: any H (kSigmoid, kGroups)
-__global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
+template <int CH, int kMidTok, int KIND = kSoftmax>  // CH 0: any H; < 0: router_tile of 16 * -CH outputs (kGroups)
+__global__ void __launch_bounds__(64 * kDispWaves, CH < 0 ? 4 : 1) moe_dispatch_mid_kernel(
     float* __restrict__ topw, int* __restrict__ topi, int* __restrict__ offsets, int* __restrict__ arow,
     int* __restrict__ inv, const uint16_t* __restrict__ x, const uint16_t* __restrict__ wr, int T, int E, int k,
     int H, int e0, int n_local, MoePro pro, int* __restrict__ ticket, SigArgs sig = SigArgs{}, ChooseArgs cho = ChooseArgs{}) {
@@ -568,8 +656,11 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
   // router logits of this workgroup's tokens
   // rows past a whole round of the waves (a gate behind 8 experts, say) are dealt to them by token pairs
   const int n_rows = KIND == kGroups ? cho.n : SIG ? sig.rows : E;
-  const int n_rounds = KIND != kSoftmax ? n_rows / kDispWaves * kDispWaves : E;
-  if constexpr (KIND != kSoftmax) {
+  const int n_rounds = CH < 0 ? 0 : KIND != kSoftmax ? n_rows / kDispWaves * kDispWaves : E;
+  if constexpr (CH < 0) {
+    __shared__ float part[kDispWaves][16][16 * -CH + 1];
+    router_tile<-CH>(x + (size_t)t0 * H, nt, wr, cho.n, H, lg, part);
+  } else if constexpr (KIND != kSoftmax) {
     const int pairs = (nt + 1) >> 1;
     for (int u = wv; u < (n_rows - n_rounds) * pairs; u += kDispWaves) {
       const int e = n_rounds + u / pairs, tp = u % pairs * 2;
@@ -590,7 +681,7 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
       continue;
     }
     const uint16_t* we = wr + (size_t)e * H + lane * 8;
-    constexpr int CN = CH ? CH : 1;
+    constexpr int CN = CH > 0 ? CH : 1;
     u32x4 b[CN];
 #pragma unroll
     for (int i = 0; i < CH; ++i) b[i] = *reinterpret_cast<const u32x4*>(we + i * 512);
@@ -682,12 +773,18 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
   if (!last) return;
   // counting sort of the T*k slots by local expert
   const int n_slots = T * k;
+  // kGroups: counters in kRep copies, a lane's by its number (few experts: lanes of a wave rarely meet)
+  constexpr int kRep = CH < 0 ? 8 : 1;
+  __shared__ int rep_cnt[kRep > 1 ? kRep * 64 : 1], rep_base[kRep > 1 ? kRep * 64 : 1];
+  const int rep = threadIdx.x % kRep;
   for (int e = threadIdx.x; e <= n_local; e += blockDim.x) cnt[e] = 0;
+  if (kRep > 1)
+    for (int e = threadIdx.x; e < kRep * 64; e += blockDim.x) rep_cnt[e] = 0;
   __syncthreads();
   // the sc1 loads in batches of kSortChunk per thread, all in flight before the first use: one
   // at a time, each load's latency was paid per slot (a 3,060-token mixed step: 12 slots per
   // thread and pass, ~40 of the launch's 52 us)
-  constexpr int kSortChunk = 8;
+  constexpr int kSortChunk = CH < 0 ? 24 : 8;
   auto load_chunk = [&](int s0, int (&ev)[kSortChunk]) {
 #pragma unroll
     for (int j = 0; j < kSortChunk; ++j) {
@@ -701,11 +798,35 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
 #pragma unroll
     for (int j = 0; j < kSortChunk; ++j) {
       const int s = s0 + j * (int)blockDim.x + (int)threadIdx.x, e = ev[j];
-      if (s < n_slots) inv[s] = (e >= 0 && e < n_local) ? atomicAdd(&cnt[e], 1) : -1;  // rank in its expert
+      // rank in its expert (in its copy's part of it)
+      if (s < n_slots) inv[s] = (e >= 0 && e < n_local) ? atomicAdd(kRep > 1 ? &rep_cnt[e * kRep + rep] : &cnt[e], 1) : -1;
     }
   }
   __syncthreads();
-  if (threadIdx.x == 0) {
+  if constexpr (kRep > 1) {
+    if (threadIdx.x < 64) {  // lane = expert
+      int n = 0, before;
+      if (lane < n_local)
+#pragma unroll
+        for (int r = 0; r < kRep; ++r) n += rep_cnt[lane * kRep + r];
+      before = n;
+      for (int o = 1; o < 64; o <<= 1) {
+        const int v = __shfl_up(before, o);
+        if (lane >= o) before += v;
+      }
+      const int total = __shfl(before, 63);
+      before -= n;
+      if (lane < n_local) {
+        offsets[lane] = before;
+#pragma unroll
+        for (int r = 0; r < kRep; ++r) {
+          rep_base[lane * kRep + r] = before;
+          before += rep_cnt[lane * kRep + r];
+        }
+      }
+      if (lane == 0) offsets[n_local] = total;
+    }
+  } else if (threadIdx.x == 0) {
     int acc = 0;
     for (int e = 0; e < n_local; ++e) {
       base[e] = acc;
@@ -734,7 +855,7 @@ __global__ void __launch_bounds__(64 * kDispWaves) moe_dispatch_mid_kernel(
     for (int j = 0; j < kSortChunk; ++j) {
       const int s = s0 + j * (int)blockDim.x + (int)threadIdx.x, e = ev[j];
       if (s < n_slots && e >= 0 && e < n_local) {
-        const int row = base[e] + rk[j];
+        const int row = (kRep > 1 ? rep_base[e * kRep + rep] : base[e]) + rk[j];
         inv[s] = row;
         arow[row] = s / k;
         if constexpr (SIG) sig.row_w[row] = wt[j];
@@ -822,24 +943,24 @@ void launch_moe_dispatch_mid_groups(float* topw, int* topi, int* offsets, int* a
   int* ticket = nullptr;
   int cus = 0;
   if (!gemm_sk_scratch(&ws, &ticket, &cus)) throw std::runtime_error("moe_dispatch_mid: stream-K scratch not reserved");
-  const int tok = T >= 2048 ? 8 : T >= 512 ? 4 : 2, grid = (T + tok - 1) / tok;
-#define MLOP_DISP_T(CH, TOK)                                                                                             \
-  moe_dispatch_mid_kernel<CH, TOK, kGroups><<<grid, 64 * kDispWaves, 0, st>>>(topw, topi, offsets, arow, inv,              \
-                                                                              (const uint16_t*)x, (const uint16_t*)wr, T, E, \
-                                                                              k, H, 0, E, MoePro{}, ticket, SigArgs{}, cho)
-#define MLOP_DISP(CH)                       \
-  if (tok == 8) MLOP_DISP_T(CH, 8);         \
-  else if (tok == 4) MLOP_DISP_T(CH, 4);    \
-  else MLOP_DISP_T(CH, 2);
-  switch (H) {
-    case 1024: MLOP_DISP(2); break;
-    case 2048: MLOP_DISP(4); break;
-    case 4096: MLOP_DISP(8); break;
-    case 8192: MLOP_DISP(16); break;
-    default: MLOP_DISP(0); break;
+#define MLOP_DISP(CH, TOK)                                                                                                \
+  moe_dispatch_mid_kernel<CH, TOK, kGroups><<<(T + TOK - 1) / TOK, 64 * kDispWaves, 0, st>>>(                               \
+      topw, topi, offsets, arow, inv, (const uint16_t*)x, (const uint16_t*)wr, T, E, k, H, 0, E, MoePro{}, ticket, SigArgs{}, \
+      cho)
+  if (T >= 2048 && H % 64 == 0 && cho.n <= 64) {  // tiles of 16 tokens
+    if (cho.n <= 16) MLOP_DISP(-1, 16);
+    else if (cho.n <= 32) MLOP_DISP(-2, 16);
+    else MLOP_DISP(-4, 16);
+  } else {
+    switch (H) {
+      case 1024: MLOP_DISP(2, 2); break;
+      case 2048: MLOP_DISP(4, 2); break;
+      case 4096: MLOP_DISP(8, 2); break;
+      case 8192: MLOP_DISP(16, 2); break;
+      default: MLOP_DISP(0, 2); break;
+    }
   }
 #undef MLOP_DISP
-#undef MLOP_DISP_T
 }
 
 // fp32 forms of the sigmoid and the grouped routing: one thread (wave) per token over its logits, the counting sort, a

@@ -10,6 +10,7 @@
 // A row's elements stay in registers between its sums of squares and the stores, so each pass reads
 // and writes every operand once (HBM-bound).
 #include <algorithm>
+#include <type_traits>
 
 #include "elem.h"
 #include "mixers.h"
@@ -43,7 +44,7 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
 #pragma unroll
       for (int e = 0; e < VEC; ++e) pw[i][e] = post1, nw[i][e] = norm1, y[i][e] = 0.f;
       if (KIND != kExperts || a.y) ldn<VEC>(yr + c, y[i]);
-      if (norm_v) ldn<VEC>(a.norm_w + c, nw[i]);
+      if (KIND != kExperts && norm_v) ldn<VEC>(a.norm_w + c, nw[i]);
       if constexpr (START) {
         float p[VEC];
 #pragma unroll
@@ -53,15 +54,9 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
         for (int e = 0; e < VEC; ++e) x[i][e] = fmaf(a.embed_scale, y[i][e], p[e]);
       } else {
         ldn<VEC>(xr + c, x[i]);
-        if (post_v) ldn<VEC>(a.post_w + c, pw[i]);
+        if (KIND != kExperts && post_v) ldn<VEC>(a.post_w + c, pw[i]);
       }
     }
-  }
-  float nb[NI][VEC];
-#pragma unroll
-  for (int i = 0; i < NI; ++i) {
-    const int c = (tid + BT * i) * VEC;
-    if (a.tanh_a && c < W) ldn<VEC>(a.tanh_b + c, nb[i]);
   }
   if constexpr (KIND == kExperts) {
     if (a.gate) {
@@ -71,28 +66,53 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
 #pragma unroll
         for (int e = 0; e < VEC; ++e) y[i][e] *= g;
     }
-    auto add = [&](const E* er, float w) {
-#pragma unroll
-      for (int i = 0; i < NI; ++i) {
-        const int c = (tid + BT * i) * VEC;
-        if (c < W) {
-          float v[VEC];
-          ldn<VEC>(er + c, v);
-#pragma unroll
-          for (int e = 0; e < VEC; ++e) y[i][e] = fmaf(w, v[e], y[i][e]);
-        }
-      }
-    };
     const int* inv = a.inv + (size_t)row * a.top;
     const float* row_w = a.row_w + (a.row_w ? (size_t)row * a.top : 0);
-#pragma unroll 2
-    for (int j = 0; j < a.top; ++j) {
-      if (inv[j] < 0) continue;
-      add(reinterpret_cast<const E*>(a.rows) + (size_t)inv[j] * W, a.row_w ? row_w[j] : 1.f);
-    }
-    if (a.self) {
-      const float w = a.self_w[row];
-      if (w != 0.f) add(reinterpret_cast<const E*>(a.self) + (size_t)row * W, w);
+    const E* self = reinterpret_cast<const E*>(a.self) + (a.self ? (size_t)row * W : 0);
+    const E* none = a.y ? yr : reinterpret_cast<const E*>(a.rows);  // read with weight 0 where there is no row
+    const int total = a.top + (a.self != nullptr);
+    // N rows at a time, all of them in flight before the first is added
+    auto add = [&](int j0, auto n_) {
+      constexpr int N = decltype(n_)::value;
+      struct alignas(sizeof(E) * VEC) Pack {
+        E e[VEC];
+      };
+      const E* er[N];
+      float w[N];
+      Pack v[N][NI];
+#pragma unroll
+      for (int k = 0; k < N; ++k) {
+        const int j = j0 + k, r = j < a.top ? inv[j] : -1;
+        er[k] = r >= 0 ? reinterpret_cast<const E*>(a.rows) + (size_t)r * W : none;
+        w[k] = r < 0 ? 0.f : a.row_w ? row_w[j] : 1.f;
+        if (j == a.top && a.self) er[k] = self, w[k] = a.self_w[row];
+      }
+#pragma unroll
+      for (int k = 0; k < N; ++k)
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+          const int c = (tid + BT * i) * VEC;
+          v[k][i] = *reinterpret_cast<const Pack*>(er[k] + (c < W ? c : 0));
+        }
+#pragma unroll
+      for (int k = 0; k < N; ++k)
+#pragma unroll
+        for (int i = 0; i < NI; ++i)
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) y[i][e] = fmaf(w[k], w[k] != 0.f ? ld1(&v[k][i].e[e]) : 0.f, y[i][e]);
+    };
+    int j = 0;
+    if (total != 2)
+      for (; j + 2 < total; j += 4) add(j, std::integral_constant<int, 4>{});
+    for (; j < total; j += 2) add(j, std::integral_constant<int, 2>{});
+    // (behind the rows: registers)
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int c = (tid + BT * i) * VEC;
+      if (c < W) {
+        if (norm_v) ldn<VEC>(a.norm_w + c, nw[i]);
+        if (post_v) ldn<VEC>(a.post_w + c, pw[i]);
+      }
     }
   }
   if constexpr (!START) {
@@ -128,8 +148,10 @@ __global__ void __launch_bounds__(1024) residual_kernel(ResidualArgs a) {
     for (int i = 0; i < NI; ++i) {
       const int c = (tid + BT * i) * VEC;
       if (c < W) {
+        float nb[VEC];
+        ldn<VEC>(a.tanh_b + c, nb);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) x[i][e] = fmaf(tanhf(alpha * x[i][e]), nw[i][e], nb[i][e]);
+        for (int e = 0; e < VEC; ++e) x[i][e] = fmaf(tanh_f(alpha * x[i][e]), nw[i][e], nb[e]);
         stn<VEC>(xn + c, x[i]);
       }
     }
@@ -158,7 +180,7 @@ template <typename E, int VEC>
 static void residual_vec(const ResidualArgs& a, hipStream_t st) {
   const int per = cdiv(a.W, VEC);
   // few rows: a row over up to 1024 threads (latency); many: 256 (several rows per CU)
-  int ni = a.T <= 256 ? 1 : std::min(4, cdiv(per, 256));
+  int ni = a.T <= 256 ? 1 : std::min(a.rows ? 2 : 4, cdiv(per, 256));
   if (cdiv(per, ni) > 1024) ni = cdiv(per, 1024);
   const int p2 = ni <= 1 ? 1 : ni <= 2 ? 2 : ni <= 4 ? 4 : 16;
   const int block = cdiv(cdiv(per, p2), 64) * 64;
@@ -294,7 +316,14 @@ __global__ void __launch_bounds__(256) clamp_glu_kernel(E* __restrict__ out, con
     ldn<4>(row, g);
     ldn<4>(row + 16, u);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) g[e] = alpha > 0.f ? clamp_glu_f(g[e], u[e], alpha, limit) : g[e] / (1.f + expf(-g[e])) * u[e];
+    for (int e = 0; e < 4; ++e) {
+      if (alpha > 0.f) {  // (in fp32 to the last bits: an exact quotient)
+        const float z = fminf(g[e], limit), up = fminf(fmaxf(u[e], -limit), limit);
+        g[e] = z * (up + 1.f) / (1.f + expf(-alpha * z));
+      } else {
+        g[e] = g[e] / (1.f + expf(-g[e])) * u[e];
+      }
+    }
     stn<4>(out + t * I + c, g);
   }
 }
