@@ -142,8 +142,8 @@ __device__ __forceinline__ float tanh_f(float x) {
 
 // tanh gelu: x / 2 (1 + tanh(u)) = x / (1 + exp(-2 u)), u = sqrt(2 / pi) (x + 0.044715 x^3)
 __device__ __forceinline__ float gelu_tanh_f(float x) {
-  const float u = 0.7978845608028654f * fmaf(0.044715f * x * x, x, x);
-  return x * __builtin_amdgcn_rcpf(1.f + __expf(-2.f * u));
+  constexpr float c = -2.f * 1.4426950408889634f * 0.7978845608028654f;  // to the base 2
+  return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * fmaf(c * 0.044715f, x * x, c)));
 }
 
 __device__ __forceinline__ float relu2_f(float x) {

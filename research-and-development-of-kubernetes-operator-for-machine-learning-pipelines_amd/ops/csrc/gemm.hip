@@ -372,11 +372,13 @@ __global__ void __launch_bounds__(WM * WN * 64) gemm_kernel(
       for (int v = tid; v < BM * VPR; v += T) {
         const int r = v / VPR, c = (v % VPR) * 8;
         if (r >= rows_here || n0 + c0 + c >= N) continue;
-        const float* s = sC + r * LDC + c;
+        float s[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) s[j] = sC[r * LDC + c + j];
+        act_outs(re, s, n0 + c0 + c);
         u32x4 o;
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          o[j] = pack2(act_out(re, s[2 * j], n0 + c0 + c), act_out(re, s[2 * j + 1], n0 + c0 + c));
+        for (int j = 0; j < 4; ++j) o[j] = pack2(s[2 * j], s[2 * j + 1]);
         *reinterpret_cast<u32x4*>(C + (size_t)(m0 + r) * ldc + n0 + c0 + c) = o;
       }
     } else {
@@ -432,11 +434,12 @@ __global__ void __launch_bounds__(256) splitk_reduce_kernel(uint16_t* __restrict
 #pragma unroll
       for (int j = 0; j < 8; ++j) a[j] *= f, b[j] *= f;
     }
+    if (EPI == EPI_NONE) act_outs(re, a, j0);
     u32x4 o;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if (EPI == EPI_NONE)
-        o[j] = pack2(act_out(re, a[2 * j], j0), act_out(re, a[2 * j + 1], j0));
+        o[j] = pack2(a[2 * j], a[2 * j + 1]);
       else
         o[j] = pack2(glu_out(re, a[2 * j], b[2 * j]), glu_out(re, a[2 * j + 1], b[2 * j + 1]));
     }
@@ -1109,9 +1112,10 @@ __global__ void __launch_bounds__(512, 1) gemm_pp_kernel(
       for (int r = 0; r < 4; ++r) {
         const int row = i * 16 + 4 * (lane >> 4) + r;
         if constexpr (EPI == EPI_NONE) {
+          float v[4] = {acc[i][0][r], acc[i][1][r], acc[i][2][r], acc[i][3][r]};
+          act_outs(re, v, n0 + wc * 64);
 #pragma unroll
-          for (int j = 0; j < 4; ++j)
-            sC[row * LD + j * 16 + (lane & 15)] = f2bf(act_out(re, acc[i][j][r], n0 + wc * 64));
+          for (int j = 0; j < 4; ++j) sC[row * LD + j * 16 + (lane & 15)] = f2bf(v[j]);
         } else {
           float f = 1.f;
           if constexpr (GROUPED)

@@ -92,6 +92,21 @@ __device__ __forceinline__ float act_f(int act, float x, float p0, float p1) {
   if (act == kActRelu2) return relu2_f(x);
   return act == kActXielu ? xielu_f(x, p0, p1) : x;
 }
+// N outputs of the plain epilogue, of columns from col on (one side of act_n0): one branch, not one per output
+template <int N>
+__device__ __forceinline__ void act_outs(const RopeEpi& re, float (&v)[N], int col) {
+  if (re.act == kActNone || col < re.act_n0) return;
+  if (re.act == kActGelu) {
+#pragma unroll
+    for (int e = 0; e < N; ++e) v[e] = gelu_tanh_f(v[e]);
+  } else if (re.act == kActRelu2) {
+#pragma unroll
+    for (int e = 0; e < N; ++e) v[e] = relu2_f(v[e]);
+  } else {
+#pragma unroll
+    for (int e = 0; e < N; ++e) v[e] = xielu_f(v[e], re.p0, re.p1);
+  }
+}
 // one output of the plain epilogue, of column col
 __device__ __forceinline__ float act_out(const RopeEpi& re, float x, int col) {
   return col < re.act_n0 ? x : act_f(re.act, x, re.p0, re.p1);
