@@ -11,7 +11,7 @@ The feed-forward is dense (tanh gelu), a mixture of experts, or absent:
       grouped down GEMM  ->  residual_step (sums a token's weighted expert rows, and its input for identity experts)
 
 Both sublayers of a dense layer are two products: their input projections side by side, and their output
-projections over the row [attention | gelu(up)].
+projections over the row [attention | gelu(up)].  In captured decode steps experts run beside attention.
 
 A layer may use another's weights; every layer has pages of its own (``cache_layout``).
 
@@ -31,6 +31,10 @@ from .layers import ParamSource, fuse_rows, linear, pad_to, rotary_table
 
 GLU_ALPHA = 1.702  # of the experts' gated unit
 MAX_OUTPUTS, MAX_TOP = 256, 64  # of the routing kernels
+# captured decode steps of so many tokens run a layer's experts beside its attention, on a stream of their own.  (One
+# token: joining the branches costs more than they gain.  Above 256 rows dense products may use the scratch that
+# the experts' products share; captured steps are the only ones where the two run at once.)
+SIDE_TOKENS = range(4, 257)
 
 
 def _up(n: int, m: int) -> int:
@@ -78,6 +82,7 @@ class DibedraModel:
         ws = [self.head] + [L[k] for L in self.weights.values() for k in ("proj", "out")]
         self.graph_safe = dtype == torch.bfloat16 and all(ops.gemm_is_native(*w.shape) for w in ws)
         self.n_q = self.n_kv
+        self._side = torch.cuda.Stream(self.device) if self.device.type == "cuda" else None
         # step metadata: one decode tile per one-token row, 128-token prompt tiles for every longer portion
         self.meta_kwargs = {"group": 16, "flash_tile": 128, "flash_min_q": 2, "part_dim": self.v_pad, "chunk": 0}
 
@@ -137,6 +142,14 @@ class DibedraModel:
         m, eps = la.mixer, self.cfg.rms_eps
         k_cache, v_cache = kv.k[i], kv.v[i]
         g0, q0, nq = L["g0"], L["q0"], m.heads * m.dim
+        side, experts = None, {}
+        if la.moe and x.is_cuda and x.shape[0] in SIDE_TOKENS and torch.cuda.is_current_stream_capturing():
+            side = self._side
+            side.wait_stream(torch.cuda.current_stream())
+            with torch.cuda.stream(side):
+                experts = self._experts(L, la.moe, x)
+        elif la.moe:
+            experts = self._experts(L, la.moe, x)
         proj = ops.gemm(x, L["proj"], epi=ops.EPI_GELU, act_from=L["u0"]) if la.ff else linear(x, L["proj"])
         heads = proj[:, q0:q0 + nq]
         q = ops.qk_head_norm(heads, proj[:, :m.kv_heads * m.dim], None, m.heads, m.dim, m.vdim, L["q_norm"], L["k_norm"], eps,
@@ -144,10 +157,10 @@ class DibedraModel:
         # the heads' outputs take the queries' place
         ops.attention_hd(q, k_cache, v_cache, meta, m.dim, m.vdim, m.scale, gate=proj[:, g0:g0 + nq], window=m.window,
                          out=heads.unflatten(1, (m.heads, m.dim)))
-        add = {"y": linear(proj[:, q0:L["end"]], L["out"])}
-        if la.moe:
-            add.update(self._experts(L, la.moe, x))
-        return add
+        y = linear(proj[:, q0:L["end"]], L["out"])
+        if side is not None:
+            torch.cuda.current_stream().wait_stream(side)
+        return {"y": y, **experts}
 
     def _experts(self, L, m, x):
         d = ops.moe_dispatch_groups(x, L["router"], L["correction"], m.experts, m.top, m.groups, m.keep)
