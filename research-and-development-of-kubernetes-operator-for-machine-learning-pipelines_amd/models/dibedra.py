@@ -2,8 +2,8 @@
 
 Layers are listed one by one in the configuration.  A layer's attention and its feed-forward read one normed
 input and are added to one fp32 residual together; norms are dynamic tanh (no statistics).  Attention is
-windowed, its queries and keys normed per head, its values the keys as projected, its output gated per element.
-The feed-forward is dense (tanh gelu), a mixture of experts, or absent:
+windowed, its queries and keys normed per head, its values the keys before norm and rotation, its output gated
+per element.  The feed-forward is dense (tanh gelu), a mixture of experts, or absent:
 
   residual_begin | residual_step  ->  [k | gate | q | up] GEMM (gelu on the last columns)  ->  qk_head_norm (norm,
       rotation, paged stores)  ->  attention_hd into q's columns  ->  [O | down] GEMM  ->  residual_step

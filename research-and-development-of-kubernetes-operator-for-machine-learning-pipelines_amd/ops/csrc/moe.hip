@@ -947,18 +947,21 @@ void launch_moe_dispatch_mid_groups(float* topw, int* topi, int* offsets, int* a
   moe_dispatch_mid_kernel<CH, TOK, kGroups><<<(T + TOK - 1) / TOK, 64 * kDispWaves, 0, st>>>(                               \
       topw, topi, offsets, arow, inv, (const uint16_t*)x, (const uint16_t*)wr, T, E, k, H, 0, E, MoePro{}, ticket, SigArgs{}, \
       cho)
-  if (T >= 2048 && H % 64 == 0 && cho.n <= 64) {  // tiles of 16 tokens
+  if (T > 1024 && H % 64 == 0 && cho.n <= 64) {  // tiles of 16 tokens
     if (cho.n <= 16) MLOP_DISP(-1, 16);
     else if (cho.n <= 32) MLOP_DISP(-2, 16);
     else MLOP_DISP(-4, 16);
   } else {
+#define MLOP_DISP_T(CH) \
+  if (T > 1024) MLOP_DISP(CH, 8); else MLOP_DISP(CH, 2)
     switch (H) {
-      case 1024: MLOP_DISP(2, 2); break;
-      case 2048: MLOP_DISP(4, 2); break;
-      case 4096: MLOP_DISP(8, 2); break;
-      case 8192: MLOP_DISP(16, 2); break;
-      default: MLOP_DISP(0, 2); break;
+      case 1024: MLOP_DISP_T(2); break;
+      case 2048: MLOP_DISP_T(4); break;
+      case 4096: MLOP_DISP_T(8); break;
+      case 8192: MLOP_DISP_T(16); break;
+      default: MLOP_DISP_T(0); break;
     }
+#undef MLOP_DISP_T
   }
 #undef MLOP_DISP
 }

@@ -7,9 +7,8 @@ import dibedra_cases as cases
 import dibedra_oracle as orc
 
 pytestmark = pytest.mark.gpu
-# rms error over the logits' spread (hybrid_util.logits_err); bf16 rounds every projection and sublayer
-# output, and these models' sharp attention amplifies it
-TOL = {torch.float32: 3e-4, torch.bfloat16: 0.16}
+# rms error over the logits' spread (hybrid_util.logits_err); bf16 rounds every projection and sublayer output
+TOL = {torch.float32: 3e-4, torch.bfloat16: 0.04}
 DTYPES = [torch.float32, torch.bfloat16]
 
 
@@ -82,7 +81,7 @@ def test_long_decoding(gpu, tmp_path, dtype):
 @pytest.mark.parametrize("tight", [False, True])
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_greedy_generation(gpu, tmp_path, dtype, tight):
-    eng = cases.greedy_generation(tmp_path, gpu, dtype, 1e-3 if dtype == torch.float32 else 0.3, tight=tight)
+    eng = cases.greedy_generation(tmp_path, gpu, dtype, 1e-3 if dtype == torch.float32 else 0.1, tight=tight)
     assert (eng.stats["graph_steps"] > 0) == (dtype == torch.bfloat16)  # fp32 products are the library's: no graphs
 
 

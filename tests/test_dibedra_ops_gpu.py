@@ -233,7 +233,7 @@ def test_other_activations_from_a_column_on(gpu, n0):
 
 # (experts, identity experts, chosen, groups, kept, width)
 ROUTES = [(5, 2, 3, 1, 1, 128), (1, 0, 1, 1, 1, 192), (9, 0, 9, 3, 3, 64), (12, 3, 4, 5, 2, 1024), (1, 7, 2, 2, 2, 72), (8, 4, 3, 3, 2, 4096),
-          (6, 6, 12, 1, 1, 320), (40, 8, 6, 4, 1, 384), (16, 8, 3, 6, 3, 2048), (250, 6, 24, 16, 5, 256), (63, 1, 20, 64, 40, 1000), (3, 5, 2, 8, 3, 8192)]
+          (6, 6, 12, 1, 1, 320), (40, 8, 6, 4, 1, 384), (16, 8, 3, 6, 3, 2048), (250, 6, 24, 16, 5, 256), (90, 10, 7, 5, 2, 2048), (63, 1, 20, 64, 40, 1000), (3, 5, 2, 8, 3, 8192)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -245,7 +245,7 @@ def test_grouped_routing(gpu, dtype, E, identity, top, groups, keep, W):
     router = (2.0 * torch.randn(n, W, generator=g) * W ** -0.5).to(torch.bfloat16)
     corr = 0.3 * torch.randn(n, generator=g)
     for correction in (corr, None):
-        for T in (1, 2, 16, 17, 70, 600, 2100) if correction is corr and n < 100 else (3, 40):
+        for T in (1, 2, 16, 17, 70, 600, 2100) if correction is corr and n < 100 else (3, 40, 1100):
             x = torch.randn(T, W, generator=g).to(torch.bfloat16)
             d = ops.moe_dispatch_groups(x.to(gpu, dtype), router.to(gpu, dtype), None if correction is None else corr.to(gpu), E, top,
                                         groups, keep)
